@@ -11,7 +11,8 @@
  *     argument, or a positive hipError_t from the launch; mi355_last_error()
  *     returns a thread-local message for the last non-zero return;
  *   - strides are in ELEMENTS; the innermost (head_dim) stride is always 1;
- *   - head_dim in {32, 64, 128}; GQA: query head h reads kv head h / (Hq / Hkv).
+ *   - head_dim in {32, 64, 128} (mi355_paged_attn_any_fwd: any multiple of 8 up to 512);
+ *     GQA: query head h reads kv head h / (Hq / Hkv).
  */
 #ifndef MI355_ATTN_H
 #define MI355_ATTN_H
@@ -34,7 +35,7 @@ enum {
 enum {
     MI355_BF16 = 0,         /* bfloat16 q/k/v/out and bf16 KV cache              */
     MI355_FP8_E4M3 = 1,     /* OCP fp8-e4m3 KV cache (max 448) + fp32 scales     */
-    MI355_FP32 = 2          /* float32 (RMSNorm weight only)                     */
+    MI355_FP32 = 2          /* float32 (norm weights; the entry points that name it) */
 };
 
 /* mask modes of the prefill entry point */
@@ -281,6 +282,66 @@ int mi355_paged_decode_fwd_static(const void* q, const void* k_cache, const void
                                   int B, int Hq, int Hkv, int D, int block_size, int64_t num_blocks, int max_ctx,
                                   float softmax_scale, int kv_dtype, void* stream);
 
+/*
+ * Attention with per-query-head terms: the three forward entry points above with
+ *   score(h, i, j) = softmax_scale * head_scale[h] * (q_i . k_j)
+ *   out_i = sum_j exp(score_ij) v_j / (exp(sink[h]) + sum_j exp(score_ij))
+ * head_scale, sink: fp32 (Hq), each optional (NULL: factor 1 / no sink).  A sink is a score that has neither key nor
+ * value: it is not scaled, is visible to every query and enters the denominator once, also when the keys are split over
+ * workgroups.  head_scale must not be negative in the prefill forms (fold a sign into q).  The mathematics of
+ * llm-core/llm_core/model.py:308-325 otherwise.
+ *   mi355_prefill_fwd_headwise        : mi355_prefill_fwd (mask modes NONE / CAUSAL) or, n_split > 1, _splitkv
+ *   mi355_prefill_paged_fwd_headwise  : mi355_prefill_paged_fwd
+ *   mi355_paged_decode_fwd_headwise   : mi355_paged_decode_fwd; q rows may be strided (q_row_stride elements, a
+ *                                       multiple of 8: e.g. a view of a merged projection), q 16-byte aligned
+ */
+int mi355_prefill_fwd_headwise(const void* q, const void* k, const void* v, void* out,
+                               const int64_t q_strides[3], const int64_t k_strides[3],
+                               const int64_t v_strides[3], const int64_t o_strides[3],
+                               const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k,
+                               const float* head_scale, const float* sink, int B, int Hq, int Hkv,
+                               int Sq_max, int Sk_max, int D, float softmax_scale, int mask_mode, int dtype,
+                               int n_split, int64_t total_q_rows, void* workspace, size_t workspace_bytes,
+                               void* stream);
+int mi355_prefill_paged_fwd_headwise(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                     int64_t q_token_stride, int64_t out_token_stride,
+                                     const int32_t* cu_seqlens_q, const int32_t* block_tables, int64_t table_stride,
+                                     int64_t max_blocks, const int32_t* context_lens, const float* head_scale,
+                                     const float* sink, int B, int Hq, int Hkv, int Sq_max, int D, int block_size,
+                                     int64_t num_blocks, float softmax_scale, int kv_dtype, int n_split,
+                                     int64_t total_q_rows, void* workspace, size_t workspace_bytes, void* stream);
+int mi355_paged_decode_fwd_headwise(const void* q, int64_t q_row_stride, const void* k_cache, const void* v_cache,
+                                    void* out, const int32_t* block_tables, int64_t bt_row_stride,
+                                    const int32_t* context_lens, const float* k_scale, const float* v_scale,
+                                    const float* head_scale, const float* sink, void* workspace,
+                                    size_t workspace_bytes, int B, int Hq, int Hkv, int D, int block_size,
+                                    int64_t num_blocks, int max_ctx, float softmax_scale, int kv_dtype, void* stream);
+
+/*
+ * Paged causal attention for any head size and for fp32 -- the general path: keys and values of different sizes Dk, Dv
+ * (multiples of 8 up to 512), caches (num_blocks,Hkv,16,Dk) and (num_blocks,Hkv,16,Dv) of the same element type as q
+ * and out (dtype MI355_BF16 or MI355_FP32; fp32 arithmetic either way).  With cu_seqlens_q the rows are chunks as in
+ * mi355_prefill_paged_fwd (n_rows = packed rows); without it sequence b owns row b, a decode step (n_rows = B).
+ * head_scale, sink as above (head_scale of any sign).  Table entries of visible keys only are read, clamped into the
+ * pool.  No MFMA: the 16-bit kernels above are the fast path where their head sizes fit.
+ */
+int mi355_paged_attn_any_fwd(const void* q, const void* k_cache, const void* v_cache, void* out, int64_t q_row_stride,
+                             int64_t out_row_stride, int64_t n_rows, const int32_t* cu_seqlens_q,
+                             const int32_t* block_tables, int64_t bt_row_stride, int64_t max_blocks,
+                             const int32_t* context_lens, const float* head_scale, const float* sink, int B, int Hq,
+                             int Hkv, int Dk, int Dv, int block_size, int64_t num_blocks, float softmax_scale,
+                             int dtype, void* stream);
+
+/*
+ * Unrotated keys and values of T new tokens into the paged cache (the producer for models without RoPE; with it:
+ * mi355_rope_and_cache).  k (T,Hkv,k_dim), v (T,Hkv,v_dim), heads contiguous, token strides in elements; caches
+ * (num_blocks,Hkv,16,k_dim) / (num_blocks,Hkv,16,v_dim) of the same dtype (MI355_BF16 or MI355_FP32); head rows and
+ * token strides are multiples of 16 bytes.  A slot outside [0, 16 * num_blocks) is not written.
+ */
+int mi355_kv_cache_write(const void* k, const void* v, void* k_cache, void* v_cache, const int64_t* slot_mapping,
+                         int64_t num_blocks, int64_t T, int Hkv, int k_dim, int v_dim, int64_t k_token_stride,
+                         int64_t v_token_stride, int dtype, void* stream);
+
 /* Tokens of one sequence handled by one workgroup of the split-K pass: grows with max_ctx (1024, 2048, 4096) and
  * shrinks again, down to 256, while a batch of contexts beyond 1024 tokens has fewer workgroups than the GPU has
  * compute units. */
@@ -369,6 +430,38 @@ int mi355_rms_norm_fwd(const void* x, const void* residual, const void* weight, 
  */
 int mi355_silu_mul_fwd(const void* gate, const void* up, void* out, int64_t n_rows, int n_cols,
                        int64_t gate_row_stride, int64_t up_row_stride, int64_t out_row_stride, void* stream);
+
+/*
+ * End of a sublayer in a model with Dynamic Tanh norms (tanh(alpha x) w + b, no statistics) and gated residuals, and the
+ * norm in front of the next sublayer, in one pass over (n_rows, n_cols):
+ *   s = (sub + sub_bias) * sigmoid(gate + gate_bias)
+ *   x = resid_in + (tanh(post_alpha s) post_weight + post_bias)
+ *   y = tanh(next_alpha x) next_weight + next_bias
+ * sub, gate, y: dtype MI355_BF16 or MI355_FP32, row strides in elements; resid_in / resid_out (may be the same) and all
+ * parameter vectors: fp32, contiguous.  Parts are optional: sub NULL -> x = resid_in (a plain norm); gate NULL -> no
+ * gate; post_weight NULL -> no norm on s; resid_out NULL -> x is not kept; next_weight NULL with y -> weight 1, bias 0;
+ * y NULL -> no norm of x.  The residual stays fp32 throughout.
+ */
+int mi355_dyt_residual_fwd(const void* sub, const float* sub_bias, const void* gate, const float* gate_bias,
+                           float post_alpha, const float* post_weight, const float* post_bias, const float* resid_in,
+                           float* resid_out, float next_alpha, const float* next_weight, const float* next_bias,
+                           void* y, int64_t n_rows, int n_cols, int64_t sub_row_stride, int64_t gate_row_stride,
+                           int64_t y_row_stride, int dtype, void* stream);
+
+/*
+ * PolyNorm activation: out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 with element-wise powers and
+ * N(v) = v / sqrt(mean(v^2) + eps) over the row; fp32 math, one rounding.  coeffs = {c0, c1, c2, c3} in HOST memory.
+ */
+int mi355_polynorm_fwd(const void* z, void* out, int64_t n_rows, int n_cols, int64_t z_row_stride,
+                       int64_t out_row_stride, const float coeffs[4], float eps, int dtype, void* stream);
+
+/*
+ * out[t] = embed[tokens[t]] + pos[positions[t]] in fp32 (n_rows, n_cols): token embedding plus learned position vector,
+ * the start of an fp32 residual stream.  embed (vocab, n_cols), pos (n_positions, n_cols) of dtype MI355_BF16 or
+ * MI355_FP32; ids outside their table are clamped into it.
+ */
+int mi355_embed_pos_fwd(const void* embed, const void* pos, const int64_t* tokens, const int32_t* positions, float* out,
+                        int64_t n_rows, int n_cols, int64_t vocab, int64_t n_positions, int dtype, void* stream);
 
 /*
  * Plain device-to-device copy of `bytes` bytes (16-byte aligned).  Measurement aid

@@ -2,6 +2,9 @@
 
 Usage: python build.py            (from anywhere; output lands next to the
 Python package so the built library travels with the source tree)
+       python build.py --serving  (libmi355attn_serving.so: what serving a model needs and no more --
+no training kernels, no checks of the compiler's output; the command line tools run this in a
+checkout that has no library yet)
 """
 from __future__ import annotations
 
@@ -16,8 +19,10 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 OUT_DIR = os.path.join(HERE, "mi355_attn")
 LIB_NAME = "libmi355attn.so"
+SERVING_LIB_NAME = "libmi355attn_serving.so"      # without the kernels that only training needs
+TRAINING_ONLY = ("prefill_bwd.hip",)
 SOURCES = ["api.hip", "paged_decode.hip", "prefill_fwd.hip", "prefill_fwd_w64.hip", "prefill_bwd.hip", "kv_cache_ops.hip",
-           "layer_ops.hip"]
+           "layer_ops.hip", "paged_attn_any.hip"]
 # prefill_fwd_w64.hip keeps its output accumulators in AGPRs that only its assembly statements touch: its builtin MFMAs
 # must therefore be selected in VGPR form, so that the compiler allocates no AGPR for them.
 # It is also compiled without the machine-code hoisting of loop invariants: hoisted out of the job loop, a few dozen
@@ -154,24 +159,42 @@ def check_scalar_address_hazards(src: str) -> str:
     return "%s: %d inline-assembly memory instructions, none reads a scalar register within five wait states of a vector write" % (src, n_checked)
 
 
+def _compile_all(srcs, tag=""):
+    """Objects of `srcs`, compiled in parallel: [(object, compiler messages)]."""
+    obj_dir = os.path.join(HERE, "build")
+    os.makedirs(obj_dir, exist_ok=True)
+
+    def compile_one(src):
+        obj = os.path.join(obj_dir, src.replace(".hip", tag + ".o"))
+        log = _run([HIPCC, *FLAGS, *EXTRA_FLAGS.get(src, []), "-c", os.path.join(CSRC, src), "-o", obj])
+        return obj, log
+
+    with ThreadPoolExecutor(max_workers=8) as ex:
+        return list(ex.map(compile_one, srcs))
+
+
+def build_serving_library() -> str:
+    tag = ".%d" % os.getpid()                      # (two first calls at once each build their own and the last one stays)
+    objs = [o for o, _ in _compile_all([s for s in SOURCES if s not in TRAINING_ONLY], tag)]
+    lib = os.path.join(OUT_DIR, SERVING_LIB_NAME)
+    _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", lib + tag, *objs])
+    os.replace(lib + tag, lib)
+    for o in objs:
+        os.remove(o)
+    return lib
+
+
 def build_library(verbose: bool = True) -> str:
     # the hand-scheduled assembly of prefill_fwd_w64.hip is generated text: regenerate it so that it cannot go stale
     _run([sys.executable, os.path.join(CSRC, "gen_prefill_w64_loop.py")])
-    obj_dir = os.path.join(HERE, "build")
-    os.makedirs(obj_dir, exist_ok=True)
     srcs = [s for s in SOURCES if os.path.exists(os.path.join(CSRC, s))]
-
-    def compile_one(src):
-        obj = os.path.join(obj_dir, src.replace(".hip", ".o"))
-        log = _run([HIPCC, *FLAGS, *EXTRA_FLAGS.get(src, []), "-c", os.path.join(CSRC, src), "-o", obj])
-        return obj, log
 
     # sources whose kernels issue memory instructions from inline assembly
     asm_dma = [s for s in ("prefill_fwd.hip", "prefill_fwd_w64.hip", "prefill_bwd.hip") if s in srcs]
     with ThreadPoolExecutor(max_workers=4) as ex:
         check = ex.submit(check_w64_registers)
         hazards = [ex.submit(check_scalar_address_hazards, s) for s in asm_dma]
-        results = list(ex.map(compile_one, srcs))
+        results = _compile_all(srcs)
         notes = [check.result()] + [h.result() for h in hazards]
     if verbose:
         print("\n".join(notes))
@@ -186,5 +209,8 @@ def build_library(verbose: bool = True) -> str:
 
 
 if __name__ == "__main__":
-    build_library()
+    if "--serving" in sys.argv[1:]:
+        build_serving_library()
+    else:
+        build_library()
     sys.exit(0)

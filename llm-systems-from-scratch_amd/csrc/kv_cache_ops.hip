@@ -419,6 +419,74 @@ extern "C" int mi355_rope_and_cache(const void* q_in, const void* k_in, const vo
     return MI355_OK;
 }
 
+namespace mi355 {
+
+// ---- new keys and values, unrotated, into the paged cache -------------------------------------------
+// A copy of whole head rows, whatever their element type: keys of k_row and values of v_row 16-byte pieces per head.
+// One thread per piece; consecutive threads own consecutive pieces of a token's keys, then of its values.
+struct KvWriteParams {
+    const unsigned char *k, *v;
+    unsigned char *k_cache, *v_cache;
+    const int64_t* slots;
+    int64_t k_tok, v_tok;            // token strides in bytes (heads are contiguous)
+    int64_t T, n_slots;
+    int Hkv, k_row, v_row;
+};
+
+__global__ __launch_bounds__(256) void kv_cache_write_kernel(KvWriteParams p) {
+    const int k_pieces = p.Hkv * p.k_row, per_tok = k_pieces + p.Hkv * p.v_row;
+    const int64_t total = p.T * per_tok;
+    for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t t = idx / per_tok;
+        const int64_t slot = p.slots[t];
+        if (slot < 0 || slot >= p.n_slots) continue;
+        int piece = (int)(idx % per_tok);
+        const bool is_v = piece >= k_pieces;
+        if (is_v) piece -= k_pieces;
+        const int row = is_v ? p.v_row : p.k_row, hk = piece / row, c = piece % row;
+        const unsigned char* src = (is_v ? p.v + t * p.v_tok : p.k + t * p.k_tok) + (int64_t)piece * 16;
+        unsigned char* dst = (is_v ? p.v_cache : p.k_cache) + ((((slot >> 4) * p.Hkv + hk) * 16 + (slot & 15)) * row + c) * 16;
+        *reinterpret_cast<u32x4*>(dst) = *reinterpret_cast<const u32x4*>(src);
+    }
+}
+
+}  // namespace mi355
+
+extern "C" int mi355_kv_cache_write(const void* k, const void* v, void* k_cache, void* v_cache, const int64_t* slot_mapping,
+                                    int64_t num_blocks, int64_t T, int Hkv, int k_dim, int v_dim, int64_t k_token_stride,
+                                    int64_t v_token_stride, int dtype, void* stream) {
+    if (!k || !v || !k_cache || !v_cache || !slot_mapping) return set_error(MI355_EINVAL, "kv_cache_write: null pointer argument");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32)
+        return set_error(MI355_EDTYPE, "kv_cache_write: dtype must be MI355_BF16 or MI355_FP32");
+    if (T < 0 || Hkv <= 0 || k_dim <= 0 || v_dim <= 0 || num_blocks <= 0)
+        return set_error(MI355_EINVAL, "kv_cache_write: T, Hkv, k_dim, v_dim, num_blocks out of range");
+    const int es = dtype == MI355_BF16 ? 2 : 4;
+    if ((k_dim * es) % 16 || (v_dim * es) % 16 || (k_token_stride * es) % 16 || (v_token_stride * es) % 16)
+        return set_error(MI355_EINVAL, "kv_cache_write: head rows and token strides must be multiples of 16 bytes");
+    if (((uintptr_t)k | (uintptr_t)v | (uintptr_t)k_cache | (uintptr_t)v_cache) & 15)
+        return set_error(MI355_EINVAL, "kv_cache_write: k, v and the caches must be 16-byte aligned");
+    if (T == 0) return MI355_OK;
+    KvWriteParams p;
+    p.k = (const unsigned char*)k;
+    p.v = (const unsigned char*)v;
+    p.k_cache = (unsigned char*)k_cache;
+    p.v_cache = (unsigned char*)v_cache;
+    p.slots = slot_mapping;
+    p.k_tok = k_token_stride * es;
+    p.v_tok = v_token_stride * es;
+    p.T = T;
+    p.n_slots = num_blocks * 16;
+    p.Hkv = Hkv;
+    p.k_row = k_dim * es / 16;
+    p.v_row = v_dim * es / 16;
+    const int64_t blocks = (T * Hkv * (p.k_row + p.v_row) + 255) / 256;
+    hipLaunchKernelGGL(kv_cache_write_kernel, dim3((unsigned)(blocks < 0x7fffffffLL ? blocks : 0x7fffffffLL)), dim3(256), 0,
+                       (hipStream_t)stream, p);
+    const int rc = (int)hipGetLastError();
+    if (rc != 0) return set_error(rc, hipGetErrorString((hipError_t)rc));
+    return MI355_OK;
+}
+
 extern "C" int mi355_quantize_kv_fp8(const void* cache_bf16, void* cache_fp8, float* scale, int64_t num_blocks, int Hkv,
                                      int D, int block_size, void* stream) {
     if (!cache_bf16 || !cache_fp8 || !scale) return set_error(MI355_EINVAL, "quantize_kv_fp8: null pointer argument");

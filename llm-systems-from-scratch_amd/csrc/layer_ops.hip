@@ -1,7 +1,9 @@
-// The two fused elementwise/normalisation ops that sit next to attention in a transformer
-// block: RMSNorm forward (optionally fused with the residual add in front of it) and
-// silu(gate) * up.  Both are streaming kernels: HBM-bound, 16-byte accesses, fp32 math,
-// one rounding to bf16 per stored value.
+// The fused elementwise/normalisation ops that sit next to attention in a transformer
+// block: RMSNorm forward (optionally fused with the residual add in front of it),
+// silu(gate) * up, the end of a sublayer in a model with Dynamic Tanh norms and gated
+// residuals, the PolyNorm activation, and the token + position embedding.  All are
+// streaming kernels: HBM-bound, 16-byte accesses, fp32 math, one rounding to bf16 per
+// stored value (the last three also exist with fp32 values throughout).
 #include "common.hpp"
 #include "launch.hpp"
 
@@ -176,6 +178,275 @@ __global__ __launch_bounds__(256) void silu_mul_generic_kernel(SiluMulParams p) 
     }
 }
 
+// ---- element access shared by the kernels that serve bf16 and fp32 tensors ----------------------
+template <typename T>
+__device__ __forceinline__ void load8(const T* p, float (&v)[8]) {
+    if constexpr (sizeof(T) == 2) {
+        const bf16x8 a = as_bf16x8(__builtin_nontemporal_load(reinterpret_cast<const u32x4*>(p)));
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = (float)a[e];
+    } else {
+        const f32x4 a = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(p));
+        const f32x4 b = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(p) + 1);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            v[e] = a[e];
+            v[4 + e] = b[e];
+        }
+    }
+}
+template <typename T>
+__device__ __forceinline__ void store8(T* p, const float (&v)[8]) {
+    if constexpr (sizeof(T) == 2) {
+        u32x4 o;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = pack_bf16(v[2 * e], v[2 * e + 1]);
+        __builtin_nontemporal_store(o, reinterpret_cast<u32x4*>(p));
+    } else {
+        __builtin_nontemporal_store(f32x4{v[0], v[1], v[2], v[3]}, reinterpret_cast<f32x4*>(p));
+        __builtin_nontemporal_store(f32x4{v[4], v[5], v[6], v[7]}, reinterpret_cast<f32x4*>(p) + 1);
+    }
+}
+// parameter vectors: small, read by every workgroup, kept in the caches; null = the given constant
+__device__ __forceinline__ void load_param8(const float* p, int col, float none, float (&v)[8]) {
+    if (p) {
+        const f32x4* q = reinterpret_cast<const f32x4*>(p + col);
+        const f32x4 a = q[0], b = q[1];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            v[e] = a[e];
+            v[4 + e] = b[e];
+        }
+    } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = none;
+    }
+}
+
+// tanh and the logistic function.  FAST (results that go to bf16, or to the residual of a bf16 model): through one
+// hardware exponential and one reciprocal, absolute error about 2e-7; both saturate cleanly (exp -> 0 or inf).
+template <bool FAST>
+__device__ __forceinline__ float tanh_of(float x) {
+    if constexpr (FAST) return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + fast_exp2(2.0f * kLog2e * x));
+    else return tanhf(x);
+}
+template <bool FAST>
+__device__ __forceinline__ float sigmoid_of(float x) {
+    if constexpr (FAST) return __builtin_amdgcn_rcpf(1.0f + fast_exp2(-kLog2e * x));
+    else return 1.0f / (1.0f + expf(-x));
+}
+
+// ---- end of a sublayer with Dynamic Tanh norms and a gated residual ------------------------------
+//   s = (sub + sub_bias) * sigmoid(gate + gate_bias)          (no gate: s = sub + sub_bias)
+//   x = resid + (post ? tanh(post_alpha * s) * post_w + post_b : s)      (no sub: x = resid)
+//   y = tanh(next_alpha * x) * next_w + next_b                (the norm in front of the next sublayer)
+// The norm has no statistics, so the whole chain is one pass over the elements.
+template <typename T>
+struct DytResidualParams {
+    const T* sub;
+    const T* gate;
+    const float *sub_bias, *gate_bias;
+    const float *post_w, *post_b;
+    const float* resid_in;
+    float* resid_out;            // may be resid_in; null: x is not kept
+    const float *next_w, *next_b;
+    T* y;
+    float post_alpha, next_alpha;
+    int64_t n_rows, sub_stride, gate_stride, y_stride;      // resid rows are contiguous
+    int n_cols, rows_per_thread;
+};
+
+template <typename T, bool FAST>
+__device__ __forceinline__ float dyt_sublayer(const DytResidualParams<T>& p, float sub, float gate, float sb, float gb, float pw,
+                                              float pb) {
+    float s = sub + sb;
+    if (p.gate) s *= sigmoid_of<FAST>(gate + gb);
+    return p.post_w ? fmaf(tanh_of<FAST>(p.post_alpha * s), pw, pb) : s;
+}
+
+// A thread owns 8 adjacent columns of rows_per_thread rows, so that the six parameter vectors -- more bytes than the
+// tensors themselves -- are fetched once for all of them.  Adjacent threads own adjacent columns.
+template <typename T>
+__global__ __launch_bounds__(256) void dyt_residual_vec8_kernel(DytResidualParams<T> p) {
+    constexpr bool FAST = sizeof(T) == 2;
+    const int groups = p.n_cols / 8;
+    const int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
+    const int64_t row0 = idx / groups * p.rows_per_thread;
+    const int col = (int)(idx % groups) * 8;
+    if (row0 >= p.n_rows) return;
+    float sb[8], gb[8], pw[8], pb[8], nw[8], nb[8];
+    load_param8(p.sub ? p.sub_bias : nullptr, col, 0.f, sb);
+    load_param8(p.gate ? p.gate_bias : nullptr, col, 0.f, gb);
+    load_param8(p.sub ? p.post_w : nullptr, col, 1.f, pw);
+    load_param8(p.sub ? p.post_b : nullptr, col, 0.f, pb);
+    load_param8(p.next_w, col, 1.f, nw);
+    load_param8(p.next_b, col, 0.f, nb);
+    const int64_t row1 = min(row0 + p.rows_per_thread, p.n_rows);
+    for (int64_t row = row0; row < row1; ++row) {
+        float x[8];
+        load8(p.resid_in + row * p.n_cols + col, x);
+        if (p.sub) {
+            float s[8], g[8] = {};
+            load8(p.sub + row * p.sub_stride + col, s);
+            if (p.gate) load8(p.gate + row * p.gate_stride + col, g);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] += dyt_sublayer<T, FAST>(p, s[e], g[e], sb[e], gb[e], pw[e], pb[e]);
+        }
+        if (p.resid_out) store8(p.resid_out + row * p.n_cols + col, x);
+        if (p.y) {
+            float y[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) y[e] = fmaf(tanh_of<FAST>(p.next_alpha * x[e]), nw[e], nb[e]);
+            store8(p.y + row * p.y_stride + col, y);
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void dyt_residual_generic_kernel(DytResidualParams<T> p) {
+    constexpr bool FAST = sizeof(T) == 2;
+    const int64_t total = p.n_rows * p.n_cols;
+    for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = idx / p.n_cols;
+        const int col = (int)(idx % p.n_cols);
+        float x = p.resid_in[idx];
+        if (p.sub)
+            x += dyt_sublayer<T, FAST>(p, (float)p.sub[row * p.sub_stride + col], p.gate ? (float)p.gate[row * p.gate_stride + col] : 0.f,
+                                       p.sub_bias ? p.sub_bias[col] : 0.f, p.gate && p.gate_bias ? p.gate_bias[col] : 0.f,
+                                       p.post_w ? p.post_w[col] : 1.f, p.post_b ? p.post_b[col] : 0.f);
+        if (p.resid_out) p.resid_out[idx] = x;
+        if (p.y)
+            p.y[row * p.y_stride + col] = (T)fmaf(tanh_of<FAST>(p.next_alpha * x), p.next_w ? p.next_w[col] : 1.f,
+                                                  p.next_b ? p.next_b[col] : 0.f);
+    }
+}
+
+// ---- PolyNorm: out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, N(v) = v / sqrt(mean(v^2) + eps) over the row ----
+template <typename T>
+struct PolyNormParams {
+    const T* z;
+    T* out;
+    int64_t n_rows, zs, os;
+    int n_cols;
+    float eps, c0, c1, c2, c3;
+};
+
+// factors of z, z^2 and z^3 from the row's sums of squares of the three powers
+template <typename T>
+__device__ __forceinline__ void polynorm_factors(const PolyNormParams<T>& p, float s1, float s2, float s3, float& f1, float& f2,
+                                                 float& f3) {
+    const float n = (float)p.n_cols;
+    f1 = p.c0 / sqrtf(s1 / n + p.eps);
+    f2 = p.c1 / sqrtf(s2 / n + p.eps);
+    f3 = p.c2 / sqrtf(s3 / n + p.eps);
+}
+
+// WAVES wavefronts per row (1: four rows per workgroup, 4: one), the row held in registers as NCHUNK chunks of
+// 512 * WAVES elements.  Requires n_cols % 8 == 0, n_cols <= 512 * WAVES * NCHUNK, 16-byte aligned rows.
+template <typename T, int WAVES, int NCHUNK>
+__global__ __launch_bounds__(256) void polynorm_rows_kernel(PolyNormParams<T> p) {
+    __shared__ float part[4][3];
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int64_t row = WAVES == 4 ? (int64_t)blockIdx.x : (int64_t)blockIdx.x * 4 + wave;
+    if (row >= p.n_rows) return;
+    const int first = (WAVES == 4 ? (int)threadIdx.x : lane) * 8;
+    const T* zr = p.z + row * p.zs;
+    float z[NCHUNK][8];
+#pragma unroll
+    for (int c = 0; c < NCHUNK; ++c) {
+        const int col = c * (512 * WAVES) + first;
+        if (col < p.n_cols) load8(zr + col, z[c]);
+        else
+#pragma unroll
+            for (int e = 0; e < 8; ++e) z[c][e] = 0.f;
+    }
+    float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+#pragma unroll
+    for (int c = 0; c < NCHUNK; ++c)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const float v2 = z[c][e] * z[c][e], v3 = v2 * z[c][e];
+            s1 += v2;
+            s2 = fmaf(v2, v2, s2);
+            s3 = fmaf(v3, v3, s3);
+        }
+    s1 = wave_sum(s1);
+    s2 = wave_sum(s2);
+    s3 = wave_sum(s3);
+    if constexpr (WAVES == 4) {
+        if (lane == 0) {
+            part[wave][0] = s1;
+            part[wave][1] = s2;
+            part[wave][2] = s3;
+        }
+        __syncthreads();
+        s1 = part[0][0] + part[1][0] + part[2][0] + part[3][0];
+        s2 = part[0][1] + part[1][1] + part[2][1] + part[3][1];
+        s3 = part[0][2] + part[1][2] + part[2][2] + part[3][2];
+    }
+    float f1, f2, f3;
+    polynorm_factors(p, s1, s2, s3, f1, f2, f3);
+    T* orow = p.out + row * p.os;
+#pragma unroll
+    for (int c = 0; c < NCHUNK; ++c) {
+        const int col = c * (512 * WAVES) + first;
+        if (col < p.n_cols) {
+            float o[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[e] = fmaf(fmaf(fmaf(f3, z[c][e], f2), z[c][e], f1), z[c][e], p.c3);
+            store8(orow + col, o);
+        }
+    }
+}
+
+// Any n_cols, any alignment: one wavefront per row, two passes.
+template <typename T>
+__global__ __launch_bounds__(256) void polynorm_generic_kernel(PolyNormParams<T> p) {
+    const int lane = threadIdx.x & 63;
+    const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (row >= p.n_rows) return;
+    const T* zr = p.z + row * p.zs;
+    float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+    for (int col = lane; col < p.n_cols; col += 64) {
+        const float v = (float)zr[col], v2 = v * v, v3 = v2 * v;
+        s1 += v2;
+        s2 = fmaf(v2, v2, s2);
+        s3 = fmaf(v3, v3, s3);
+    }
+    float f1, f2, f3;
+    polynorm_factors(p, wave_sum(s1), wave_sum(s2), wave_sum(s3), f1, f2, f3);
+    T* orow = p.out + row * p.os;
+    for (int col = lane; col < p.n_cols; col += 64) {
+        const float v = (float)zr[col];
+        orow[col] = (T)fmaf(fmaf(fmaf(f3, v, f2), v, f1), v, p.c3);
+    }
+}
+
+// ---- token embedding + learned position vector -> fp32 residual -----------------------------------
+template <typename T>
+struct EmbedPosParams {
+    const T* embed;
+    const T* pos;
+    const int64_t* tokens;
+    const int32_t* positions;
+    float* out;
+    int64_t n_rows, vocab, n_positions;
+    int n_cols;
+};
+
+// One thread per element; an id outside its table is clamped into it (the host checks what it can).
+template <typename T>
+__global__ __launch_bounds__(256) void embed_pos_kernel(EmbedPosParams<T> p) {
+    const int64_t total = p.n_rows * p.n_cols;
+    for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = idx / p.n_cols;
+        const int col = (int)(idx % p.n_cols);
+        const int64_t tok = min(max(p.tokens[row], (int64_t)0), p.vocab - 1);
+        const int64_t pos = min(max((int64_t)p.positions[row], (int64_t)0), p.n_positions - 1);
+        p.out[idx] = (float)p.embed[tok * p.n_cols + col] + (float)p.pos[pos * p.n_cols + col];
+    }
+}
+
 }  // namespace mi355
 
 using namespace mi355;
@@ -252,4 +523,150 @@ extern "C" int mi355_silu_mul_fwd(const void* gate, const void* up, void* out, i
     const int rc = (int)hipGetLastError();
     if (rc != 0) return set_error(rc, hipGetErrorString((hipError_t)rc));
     return MI355_OK;
+}
+
+static unsigned grid_1d(int64_t threads) {
+    const int64_t blocks = (threads + 255) / 256;
+    return (unsigned)(blocks < 0x7fffffffLL ? blocks : 0x7fffffffLL);
+}
+
+static int launch_status() {
+    const int rc = (int)hipGetLastError();
+    return rc != 0 ? set_error(rc, hipGetErrorString((hipError_t)rc)) : MI355_OK;
+}
+
+template <typename T>
+static int dyt_residual(const void* sub, const float* sub_bias, const void* gate, const float* gate_bias, float post_alpha,
+                        const float* post_w, const float* post_b, const float* resid_in, float* resid_out, float next_alpha,
+                        const float* next_w, const float* next_b, void* y, int64_t n_rows, int n_cols, int64_t sub_stride,
+                        int64_t gate_stride, int64_t y_stride, hipStream_t s) {
+    DytResidualParams<T> p;
+    p.sub = (const T*)sub;
+    p.gate = (const T*)gate;
+    p.sub_bias = sub_bias;
+    p.gate_bias = gate_bias;
+    p.post_w = post_w;
+    p.post_b = post_b;
+    p.resid_in = resid_in;
+    p.resid_out = resid_out;
+    p.next_w = next_w;
+    p.next_b = next_b;
+    p.y = (T*)y;
+    p.post_alpha = post_alpha;
+    p.next_alpha = next_alpha;
+    p.n_rows = n_rows;
+    p.n_cols = n_cols;
+    p.sub_stride = sub_stride;
+    p.gate_stride = gate_stride;
+    p.y_stride = y_stride;
+    bool vec = n_cols % 8 == 0 && ((sub_stride | gate_stride | y_stride) & 7) == 0;
+    for (const void* ptr : {sub, gate, (const void*)sub_bias, (const void*)gate_bias, (const void*)post_w, (const void*)post_b,
+                            (const void*)resid_in, (const void*)resid_out, (const void*)next_w, (const void*)next_b, (const void*)y})
+        vec = vec && aligned16(ptr);
+    if (vec) {
+        // rows per thread: as many as leave the GPU several workgroups per compute unit
+        const int64_t work = n_rows * (n_cols / 8);
+        int r = 1;
+        while (r < 8 && work / (2 * r) >= 256 * 2048) r *= 2;
+        p.rows_per_thread = r;
+        const int64_t threads = (n_rows + r - 1) / r * (n_cols / 8);
+        if ((threads + 255) / 256 > 0x7fffffffLL) return set_error(MI355_EINVAL, "dyt_residual: too many elements");
+        hipLaunchKernelGGL(dyt_residual_vec8_kernel<T>, dim3(grid_1d(threads)), dim3(256), 0, s, p);
+    } else {
+        p.rows_per_thread = 1;
+        hipLaunchKernelGGL(dyt_residual_generic_kernel<T>, dim3(grid_1d(n_rows * (int64_t)n_cols)), dim3(256), 0, s, p);
+    }
+    return launch_status();
+}
+
+extern "C" int mi355_dyt_residual_fwd(const void* sub, const float* sub_bias, const void* gate, const float* gate_bias,
+                                      float post_alpha, const float* post_weight, const float* post_bias,
+                                      const float* resid_in, float* resid_out, float next_alpha, const float* next_weight,
+                                      const float* next_bias, void* y, int64_t n_rows, int n_cols, int64_t sub_row_stride,
+                                      int64_t gate_row_stride, int64_t y_row_stride, int dtype, void* stream) {
+    if (!resid_in || (!resid_out && !y)) return set_error(MI355_EINVAL, "dyt_residual: null pointer argument");
+    if (!sub && (gate || post_weight || sub_bias)) return set_error(MI355_EINVAL, "dyt_residual: gate, post norm or bias given without a sublayer result");
+    if ((post_weight == nullptr) != (post_bias == nullptr) || (next_weight == nullptr) != (next_bias == nullptr))
+        return set_error(MI355_EINVAL, "dyt_residual: a norm's weight and bias go together");
+    if (gate_bias && !gate) return set_error(MI355_EINVAL, "dyt_residual: gate_bias given without a gate");
+    if (n_rows < 0 || n_cols <= 0) return set_error(MI355_EINVAL, "dyt_residual: n_rows, n_cols out of range");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32) return set_error(MI355_EDTYPE, "dyt_residual: dtype must be MI355_BF16 or MI355_FP32");
+    if (n_rows == 0) return MI355_OK;
+    hipStream_t s = (hipStream_t)stream;
+    return dtype == MI355_BF16
+               ? dyt_residual<__bf16>(sub, sub_bias, gate, gate_bias, post_alpha, post_weight, post_bias, resid_in, resid_out, next_alpha,
+                                      next_weight, next_bias, y, n_rows, n_cols, sub_row_stride, gate_row_stride, y_row_stride, s)
+               : dyt_residual<float>(sub, sub_bias, gate, gate_bias, post_alpha, post_weight, post_bias, resid_in, resid_out, next_alpha,
+                                     next_weight, next_bias, y, n_rows, n_cols, sub_row_stride, gate_row_stride, y_row_stride, s);
+}
+
+template <typename T>
+static int polynorm(const void* z, void* out, int64_t n_rows, int n_cols, int64_t zs, int64_t os, const float* c, float eps,
+                    hipStream_t s) {
+    PolyNormParams<T> p;
+    p.z = (const T*)z;
+    p.out = (T*)out;
+    p.n_rows = n_rows;
+    p.n_cols = n_cols;
+    p.zs = zs;
+    p.os = os;
+    p.eps = eps;
+    p.c0 = c[0];
+    p.c1 = c[1];
+    p.c2 = c[2];
+    p.c3 = c[3];
+    const bool vec = n_cols % 8 == 0 && n_cols <= 16384 && aligned16(z) && aligned16(out) && ((zs | os) & 7) == 0;
+    const bool wide = vec && n_cols > 1024;
+    const int64_t wgs = wide ? n_rows : (n_rows + 3) / 4;
+    if (wgs > 0x7fffffffLL) return set_error(MI355_EINVAL, "polynorm: too many rows");
+    const dim3 grid((unsigned)wgs), block(256);
+    if (!vec) hipLaunchKernelGGL(polynorm_generic_kernel<T>, grid, block, 0, s, p);
+    else if (n_cols <= 512) hipLaunchKernelGGL((polynorm_rows_kernel<T, 1, 1>), grid, block, 0, s, p);
+    else if (n_cols <= 1024) hipLaunchKernelGGL((polynorm_rows_kernel<T, 1, 2>), grid, block, 0, s, p);
+    else if (n_cols <= 2048) hipLaunchKernelGGL((polynorm_rows_kernel<T, 4, 1>), grid, block, 0, s, p);
+    else if (n_cols <= 4096) hipLaunchKernelGGL((polynorm_rows_kernel<T, 4, 2>), grid, block, 0, s, p);
+    else if (n_cols <= 8192) hipLaunchKernelGGL((polynorm_rows_kernel<T, 4, 4>), grid, block, 0, s, p);
+    else hipLaunchKernelGGL((polynorm_rows_kernel<T, 4, 8>), grid, block, 0, s, p);
+    return launch_status();
+}
+
+extern "C" int mi355_polynorm_fwd(const void* z, void* out, int64_t n_rows, int n_cols, int64_t z_row_stride,
+                                  int64_t out_row_stride, const float coeffs[4], float eps, int dtype, void* stream) {
+    if (!z || !out || !coeffs) return set_error(MI355_EINVAL, "polynorm: null pointer argument");
+    if (n_rows < 0 || n_cols <= 0) return set_error(MI355_EINVAL, "polynorm: n_rows, n_cols out of range");
+    if (!(eps >= 0.f)) return set_error(MI355_EINVAL, "polynorm: eps must be >= 0");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32) return set_error(MI355_EDTYPE, "polynorm: dtype must be MI355_BF16 or MI355_FP32");
+    if (n_rows == 0) return MI355_OK;
+    hipStream_t s = (hipStream_t)stream;
+    return dtype == MI355_BF16 ? polynorm<__bf16>(z, out, n_rows, n_cols, z_row_stride, out_row_stride, coeffs, eps, s)
+                               : polynorm<float>(z, out, n_rows, n_cols, z_row_stride, out_row_stride, coeffs, eps, s);
+}
+
+template <typename T>
+static int embed_pos(const void* embed, const void* pos, const int64_t* tokens, const int32_t* positions, float* out, int64_t n_rows,
+                     int n_cols, int64_t vocab, int64_t n_positions, hipStream_t s) {
+    EmbedPosParams<T> p;
+    p.embed = (const T*)embed;
+    p.pos = (const T*)pos;
+    p.tokens = tokens;
+    p.positions = positions;
+    p.out = out;
+    p.n_rows = n_rows;
+    p.n_cols = n_cols;
+    p.vocab = vocab;
+    p.n_positions = n_positions;
+    hipLaunchKernelGGL(embed_pos_kernel<T>, dim3(grid_1d(n_rows * (int64_t)n_cols)), dim3(256), 0, s, p);
+    return launch_status();
+}
+
+extern "C" int mi355_embed_pos_fwd(const void* embed, const void* pos, const int64_t* tokens, const int32_t* positions, float* out,
+                                   int64_t n_rows, int n_cols, int64_t vocab, int64_t n_positions, int dtype, void* stream) {
+    if (!embed || !pos || !tokens || !positions || !out) return set_error(MI355_EINVAL, "embed_pos: null pointer argument");
+    if (n_rows < 0 || n_cols <= 0 || vocab <= 0 || n_positions <= 0)
+        return set_error(MI355_EINVAL, "embed_pos: n_rows, n_cols, vocab, n_positions out of range");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32) return set_error(MI355_EDTYPE, "embed_pos: dtype must be MI355_BF16 or MI355_FP32");
+    if (n_rows == 0) return MI355_OK;
+    hipStream_t s = (hipStream_t)stream;
+    return dtype == MI355_BF16 ? embed_pos<__bf16>(embed, pos, tokens, positions, out, n_rows, n_cols, vocab, n_positions, s)
+                               : embed_pos<float>(embed, pos, tokens, positions, out, n_rows, n_cols, vocab, n_positions, s);
 }

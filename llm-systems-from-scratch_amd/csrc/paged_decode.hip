@@ -56,7 +56,17 @@ struct DecodeParams {
     int n_groups;             // ceil((Hq / Hkv) / 16): a kv head with more than 16 query heads is served 16 at a time
     int tokens_per_wave;      // 256, 512 or 1024: a long stream per wavefront amortises its start-up latency
     float scale_log2;
+    int64_t q_stride;         // elements from one sequence's query row to the next
+    // optional per-query-head terms: a factor on the scores, and a sink (a score without key or value, natural-log
+    // units, not scaled) that enters the softmax denominator once
+    const float* head_scale;
+    const float* sink;
 };
+
+// Weight of head h's sink relative to the exponent reference m (log2 domain).
+__device__ __forceinline__ float sink_weight(const DecodeParams& p, int h, float m) {
+    return p.sink ? fast_exp2(fmaf(p.sink[h], kLog2e, -m)) : 0.f;
+}
 
 template <int D, bool FP8>
 struct DecodeLds {
@@ -142,7 +152,7 @@ void paged_decode_split_kernel(DecodeParams p) {
     //             covers d = 64t + 16kg + 8e + j, so Q uses the same d order.
     bf16x8 qf[NS];
     {
-        const __bf16* qrow = p.q + ((int64_t)b * p.Hq + h0 + r) * D;
+        const __bf16* qrow = p.q + (int64_t)b * p.q_stride + (int64_t)(h0 + r) * D;
 #pragma unroll
         for (int s = 0; s < NS; ++s) {
             const int d0 = FP8 ? (64 * (s >> 1) + 16 * kg + 8 * (s & 1)) : (32 * s + 8 * kg);
@@ -151,6 +161,8 @@ void paged_decode_split_kernel(DecodeParams p) {
             qf[s] = as_bf16x8(t);
         }
     }
+
+    const float scale_log2 = p.head_scale && r < G ? p.scale_log2 * p.head_scale[h0 + r] : p.scale_log2;   // of this lane's query
 
     const int t0 = chunk_start + wave * p.tokens_per_wave;
     const int t1 = min(ctx, t0 + p.tokens_per_wave);
@@ -310,7 +322,7 @@ void paged_decode_split_kernel(DecodeParams p) {
         float mx = -INFINITY;
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
-            const float sc = p.scale_log2 * ks2[t];
+            const float sc = scale_log2 * ks2[t];
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 float v = s_acc[t][i] * sc;
@@ -401,7 +413,7 @@ void paged_decode_split_kernel(DecodeParams p) {
         }
         const int64_t row = (int64_t)b * p.Hq + h0 + qi;
         if (n_chunks == 1) {
-            p.out[row * D + d] = (__bf16)(num / den);
+            p.out[row * D + d] = (__bf16)(num / (den + sink_weight(p, h0 + qi, M)));
         } else {
             const int64_t slot = row * p.max_chunks + chunk;
             p.ws_o[slot * D + d] = num;
@@ -439,6 +451,7 @@ __global__ __launch_bounds__(kCombineThreads) void paged_decode_combine_kernel(D
         for (int i = 0; i < 4; ++i) num[i] += f * o[i];
         den += f * p.ws_l[base + c];
     }
+    den += sink_weight(p, row % p.Hq, M);
     u32x2 w;
     w[0] = pack_bf16(num[0] / den, num[1] / den);
     w[1] = pack_bf16(num[2] / den, num[3] / den);
@@ -494,6 +507,7 @@ __global__ __launch_bounds__(kCombineThreads) void paged_decode_combine_wide_ker
         for (int e = 0; e < 4; ++e) tot[e] += f * o[e];
         dtot += f * s_den[i];
     }
+    dtot += sink_weight(p, row % p.Hq, Mall);
     u32x2 w;
     w[0] = pack_bf16(tot[0] / dtot, tot[1] / dtot);
     w[1] = pack_bf16(tot[2] / dtot, tot[3] / dtot);
@@ -578,7 +592,8 @@ static int decode_common(const void* q, const void* k_cache, const void* v_cache
                          const int32_t* block_tables, int64_t bt_row_stride, const int32_t* context_lens,
                          const float* k_scale, const float* v_scale, void* workspace, size_t workspace_bytes,
                          bool static_scratch, int B, int Hq, int Hkv, int D, int block_size, int64_t num_blocks,
-                         int max_ctx, float softmax_scale, int kv_dtype, void* stream) {
+                         int max_ctx, float softmax_scale, int kv_dtype, void* stream, int64_t q_stride = 0,
+                         const float* head_scale = nullptr, const float* sink = nullptr) {
     if (!q || !k_cache || !v_cache || !out || !block_tables || !context_lens)
         return set_error(MI355_EINVAL, "paged_decode: null pointer argument");
     if (B <= 0 || Hq <= 0 || Hkv <= 0 || max_ctx <= 0)
@@ -638,6 +653,9 @@ static int decode_common(const void* q, const void* k_cache, const void* v_cache
     p.n_groups = n_groups;
     p.tokens_per_wave = chunk / kDecodeWaves;
     p.scale_log2 = softmax_scale * kLog2e;
+    p.q_stride = q_stride ? q_stride : (int64_t)Hq * D;
+    p.head_scale = head_scale;
+    p.sink = sink;
 
     hipStream_t s = (hipStream_t)stream;
     int rc;
@@ -660,6 +678,20 @@ extern "C" int mi355_paged_decode_fwd(const void* q, const void* k_cache, const 
     return decode_common(q, k_cache, v_cache, out, block_tables, bt_row_stride, context_lens, k_scale, v_scale, workspace,
                          workspace_bytes, false, B, Hq, Hkv, D, block_size, num_blocks, max_ctx, softmax_scale, kv_dtype,
                          stream);
+}
+
+extern "C" int mi355_paged_decode_fwd_headwise(const void* q, int64_t q_row_stride, const void* k_cache,
+                                               const void* v_cache, void* out, const int32_t* block_tables,
+                                               int64_t bt_row_stride, const int32_t* context_lens,
+                                               const float* k_scale, const float* v_scale, const float* head_scale,
+                                               const float* sink, void* workspace, size_t workspace_bytes, int B, int Hq,
+                                               int Hkv, int D, int block_size, int64_t num_blocks, int max_ctx,
+                                               float softmax_scale, int kv_dtype, void* stream) {
+    if (q_row_stride < (int64_t)Hq * D || (q_row_stride & 7) || ((uintptr_t)q & 15))
+        return set_error(MI355_EINVAL, "paged_decode_headwise: q must be 16-byte aligned, its row stride a multiple of 8 and at least Hq * D");
+    return decode_common(q, k_cache, v_cache, out, block_tables, bt_row_stride, context_lens, k_scale, v_scale, workspace,
+                         workspace_bytes, false, B, Hq, Hkv, D, block_size, num_blocks, max_ctx, softmax_scale, kv_dtype,
+                         stream, q_row_stride, head_scale, sink);
 }
 
 // ---- the variant that allocates nothing -------------------------------------------------------------------

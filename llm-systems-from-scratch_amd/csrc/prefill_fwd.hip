@@ -81,6 +81,7 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
     const int h = (lid / p.n_pairs) % p.Hq;
     const int b = lid / (p.n_pairs * p.Hq);
     const int hk = h / (p.Hq / p.Hkv);
+    const float scale_log2 = p.head_scale ? p.scale_log2 * p.head_scale[h] : p.scale_log2;
 
     int sq, sk;
     const __bf16 *qb, *kb, *vb;
@@ -383,8 +384,8 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
                 u32x4 pw;
 #pragma unroll
                 for (int w = 0; w < 4; ++w) {
-                    const float a0 = fast_exp2(fmaf(s_acc[t][e0 + 2 * w], p.scale_log2, neg_ref));
-                    const float a1 = fast_exp2(fmaf(s_acc[t][e0 + 2 * w + 1], p.scale_log2, neg_ref));
+                    const float a0 = fast_exp2(fmaf(s_acc[t][e0 + 2 * w], scale_log2, neg_ref));
+                    const float a1 = fast_exp2(fmaf(s_acc[t][e0 + 2 * w + 1], scale_log2, neg_ref));
                     pw[w] = pack_bf16(a0, a1);
                     const uint32_t pwv = pw[w];
                     l_run = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, pwv), ones2, l_run, false);
@@ -439,7 +440,7 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
                 bool pending = false;
                 while (tile < tile_end) {
                     if (head(masked_c, std::true_type{}, tile)) {
-                        const bool grow = !((mx - m_ref) * p.scale_log2 <= kSlack);   // also true while m_ref = -inf
+                        const bool grow = !((mx - m_ref) * scale_log2 <= kSlack);   // also true while m_ref = -inf
                         if (__builtin_amdgcn_ballot_w64(grow) != 0) {
                             pending = true;
                             break;
@@ -452,9 +453,9 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
                 if (!pending) break;
                 const float m_new = fmaxf(m_ref, mx);
                 const float m_use = (m_new == -INFINITY) ? 0.f : m_new;    // row with no key yet: keep p = 0, not NaN
-                const float alpha = fast_exp2((m_ref - m_use) * p.scale_log2);
+                const float alpha = fast_exp2((m_ref - m_use) * scale_log2);
                 m_ref = m_new;
-                neg_ref = -m_use * p.scale_log2;
+                neg_ref = -m_use * scale_log2;
                 l_run *= alpha;
 #pragma unroll
                 for (int dt = 0; dt < NDT; ++dt)
@@ -524,7 +525,10 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
             }
             continue;
         }
-        const float inv = 1.0f / l_run;          // l == 0 (no key kept) -> NaN row, like the reference softmax
+        // (a sink's weight, relative to the row's reference, joins the denominator here and nowhere else; one that
+        // outweighs every key by more than fp32's range leaves a row of zeros)
+        const float sink_w = p.sink ? fast_exp2(fmaf(p.sink[h], kLog2e, neg_ref)) : 0.f;
+        const float inv = 1.0f / (l_run + sink_w);     // l == 0 (no key kept, no sink) -> NaN row, like the reference softmax
         // sum_j exp(scale * s_j) = 2^(-neg_ref) * l  ->  lse = ln2 * (log2 l - neg_ref)
         if (lb && q_ok && kg == 0)
             lb[qi] = l_run > 0.f ? 0.69314718056f * (__log2f(l_run) - neg_ref) : -INFINITY;
@@ -592,6 +596,7 @@ static int launch_prefill(const PrefillParams& p0, hipStream_t stream) {
 struct MergeParams {
     const float* part_o;
     const float* part_lse;
+    const float* sink;                   // optional, per head: joins the denominator of the merged row
     __bf16* out;
     int64_t os[3];
     int64_t part_rows;
@@ -634,6 +639,7 @@ __global__ __launch_bounds__(256) void prefill_merge_kernel(MergeParams p) {
             }
         }
     }
+    if (p.sink) den += __expf(p.sink[h] - m);
     __bf16* dst = p.Sq_dense ? p.out + (row / p.Sq_dense) * p.os[0] + (int64_t)h * p.os[1] + (row % p.Sq_dense) * p.os[2]
                              : p.out + row * p.os[2] + (int64_t)h * p.os[1];
     const float none = __builtin_nanf("");
@@ -647,6 +653,7 @@ static int launch_merge(const PrefillParams& p, int D, hipStream_t stream) {
     MergeParams m;
     m.part_o = p.part_o;
     m.part_lse = p.part_lse;
+    m.sink = p.sink;
     m.out = p.out;
     for (int i = 0; i < 3; ++i) m.os[i] = p.os[i];
     m.part_rows = p.part_rows;
@@ -705,7 +712,7 @@ static int prefill_common(const void* q, const void* k, const void* v, void* out
                           const int64_t mask_strides[3], int B, int Hq, int Hkv, int Sq_max, int Sk_max, int D,
                           float softmax_scale, int mask_mode, int dtype, float* lse, const int64_t* lse_strides,
                           void* stream, int n_split = 1, int64_t total_q_rows = 0, void* workspace = nullptr,
-                          size_t workspace_bytes = 0) {
+                          size_t workspace_bytes = 0, const float* head_scale = nullptr, const float* sink = nullptr) {
     if (!q || !k || !v || !out || !q_strides || !k_strides || !v_strides || !o_strides)
         return set_error(MI355_EINVAL, "prefill: null pointer argument");
     if (dtype != MI355_BF16) return set_error(MI355_EDTYPE, "prefill: dtype must be MI355_BF16");
@@ -752,6 +759,8 @@ static int prefill_common(const void* q, const void* k, const void* v, void* out
     p.Sq = Sq_max;
     p.Sk = Sk_max;
     p.scale_log2 = softmax_scale * kLog2e;
+    p.head_scale = head_scale;
+    p.sink = sink;
     p.mask_mode = mask_mode;
     p.n_qtiles = (Sq_max + kBM - 1) / kBM;
     p.n_pairs = (p.n_qtiles + 1) / 2;
@@ -818,13 +827,13 @@ extern "C" int mi355_prefill_fwd_mask_lse(const void* q, const void* k, const vo
                           B, Hq, Hkv, Sq, Sk, D, softmax_scale, MI355_MASK_BOOL, dtype, lse, lse_strides, stream);
 }
 
-extern "C" int mi355_prefill_paged_fwd(const void* q, const void* k_cache, const void* v_cache, void* out,
-                                       int64_t q_token_stride, int64_t out_token_stride, const int32_t* cu_seqlens_q,
-                                       const int32_t* block_tables, int64_t table_stride, int64_t max_blocks,
-                                       const int32_t* context_lens,
-                                       int B, int Hq, int Hkv, int Sq_max, int D, int block_size, int64_t num_blocks,
-                                       float softmax_scale, int kv_dtype, int n_split, int64_t total_q_rows,
-                                       void* workspace, size_t workspace_bytes, void* stream) {
+static int prefill_paged_common(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                int64_t q_token_stride, int64_t out_token_stride, const int32_t* cu_seqlens_q,
+                                const int32_t* block_tables, int64_t table_stride, int64_t max_blocks,
+                                const int32_t* context_lens, const float* head_scale, const float* sink,
+                                int B, int Hq, int Hkv, int Sq_max, int D, int block_size, int64_t num_blocks,
+                                float softmax_scale, int kv_dtype, int n_split, int64_t total_q_rows,
+                                void* workspace, size_t workspace_bytes, void* stream) {
     if (!q || !k_cache || !v_cache || !out || !cu_seqlens_q || !block_tables || !context_lens)
         return set_error(MI355_EINVAL, "prefill_paged: null pointer argument");
     if (kv_dtype != MI355_BF16) return set_error(MI355_EDTYPE, "prefill_paged: the cache must be MI355_BF16");
@@ -858,6 +867,8 @@ extern "C" int mi355_prefill_paged_fwd(const void* q, const void* k_cache, const
     p.Sq = Sq_max;
     p.Sk = 0;
     p.scale_log2 = softmax_scale * kLog2e;
+    p.head_scale = head_scale;
+    p.sink = sink;
     p.mask_mode = MI355_MASK_CAUSAL;
     p.n_qtiles = (Sq_max + kBM - 1) / kBM;
     p.n_pairs = (p.n_qtiles + 1) / 2;
@@ -877,6 +888,31 @@ extern "C" int mi355_prefill_paged_fwd(const void* q, const void* k_cache, const
     if (rc == 0 && p.n_split > 1) rc = launch_merge(p, D, s);
     if (rc != 0) return set_error(rc, hipGetErrorString((hipError_t)rc));
     return MI355_OK;
+}
+
+extern "C" int mi355_prefill_paged_fwd(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                       int64_t q_token_stride, int64_t out_token_stride, const int32_t* cu_seqlens_q,
+                                       const int32_t* block_tables, int64_t table_stride, int64_t max_blocks,
+                                       const int32_t* context_lens,
+                                       int B, int Hq, int Hkv, int Sq_max, int D, int block_size, int64_t num_blocks,
+                                       float softmax_scale, int kv_dtype, int n_split, int64_t total_q_rows,
+                                       void* workspace, size_t workspace_bytes, void* stream) {
+    return prefill_paged_common(q, k_cache, v_cache, out, q_token_stride, out_token_stride, cu_seqlens_q, block_tables,
+                                table_stride, max_blocks, context_lens, nullptr, nullptr, B, Hq, Hkv, Sq_max, D, block_size,
+                                num_blocks, softmax_scale, kv_dtype, n_split, total_q_rows, workspace, workspace_bytes, stream);
+}
+
+extern "C" int mi355_prefill_paged_fwd_headwise(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                                int64_t q_token_stride, int64_t out_token_stride,
+                                                const int32_t* cu_seqlens_q, const int32_t* block_tables,
+                                                int64_t table_stride, int64_t max_blocks, const int32_t* context_lens,
+                                                const float* head_scale, const float* sink,
+                                                int B, int Hq, int Hkv, int Sq_max, int D, int block_size,
+                                                int64_t num_blocks, float softmax_scale, int kv_dtype, int n_split,
+                                                int64_t total_q_rows, void* workspace, size_t workspace_bytes, void* stream) {
+    return prefill_paged_common(q, k_cache, v_cache, out, q_token_stride, out_token_stride, cu_seqlens_q, block_tables,
+                                table_stride, max_blocks, context_lens, head_scale, sink, B, Hq, Hkv, Sq_max, D, block_size,
+                                num_blocks, softmax_scale, kv_dtype, n_split, total_q_rows, workspace, workspace_bytes, stream);
 }
 
 extern "C" size_t mi355_prefill_splitkv_workspace_bytes(int64_t total_q_rows, int Hq, int D, int n_split) {
@@ -969,4 +1005,20 @@ extern "C" int mi355_prefill_fwd_splitkv(const void* q, const void* k, const voi
     return prefill_common(q, k, v, out, q_strides, k_strides, v_strides, o_strides, cu_seqlens_q, cu_seqlens_k, nullptr,
                           nullptr, B, Hq, Hkv, Sq_max, Sk_max, D, softmax_scale, mask_mode, dtype, nullptr, nullptr, stream,
                           n_split, total_q_rows, workspace, workspace_bytes);
+}
+
+extern "C" int mi355_prefill_fwd_headwise(const void* q, const void* k, const void* v, void* out,
+                                          const int64_t q_strides[3], const int64_t k_strides[3],
+                                          const int64_t v_strides[3], const int64_t o_strides[3],
+                                          const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k,
+                                          const float* head_scale, const float* sink, int B, int Hq, int Hkv,
+                                          int Sq_max, int Sk_max, int D, float softmax_scale, int mask_mode, int dtype,
+                                          int n_split, int64_t total_q_rows, void* workspace, size_t workspace_bytes,
+                                          void* stream) {
+    if (mask_mode == MI355_MASK_BOOL)
+        return set_error(MI355_EINVAL, "prefill_fwd_headwise: mask_mode must be MI355_MASK_NONE or MI355_MASK_CAUSAL");
+    if (n_split < 1) return set_error(MI355_EINVAL, "prefill_fwd_headwise: n_split must be at least 1");
+    return prefill_common(q, k, v, out, q_strides, k_strides, v_strides, o_strides, cu_seqlens_q, cu_seqlens_k, nullptr,
+                          nullptr, B, Hq, Hkv, Sq_max, Sk_max, D, softmax_scale, mask_mode, dtype, nullptr, nullptr, stream,
+                          n_split, total_q_rows, workspace, workspace_bytes, head_scale, sink);
 }

@@ -220,6 +220,7 @@ __global__ __launch_bounds__(kWWaves * 64, 1) void prefill_fwd_w64_kernel(Prefil
         const int32_t* tab;              // PAGED: the sequence's row of the block table (kb, vb: block 0 of the K/V head)
         int sq, sk, q0;
         int split;                       // which share of the query tile's K/V tiles (0 when the keys are not split)
+        float scale, sink;               // the head's score scale and its sink, log2 domain (no sink: -inf, weight 0)
     };
     // Split keys (p.n_split > 1): a job works on its share of the K/V tiles and writes, instead of output rows, a
     // normalised fp32 partial row and its log-sum-exp per query, which a second kernel merges.  `ob` and `lb` of such
@@ -384,6 +385,12 @@ __global__ __launch_bounds__(kWWaves * 64, 1) void prefill_fwd_w64_kernel(Prefil
             }
         }
         j.split = share;
+        j.scale = a->scale_log2;
+        j.sink = -INFINITY;
+        if (a->head_scale)
+            j.scale *= __builtin_bit_cast(float, load_scalar_i32(reinterpret_cast<const int32_t*>(a->head_scale) + h));
+        if (a->sink)
+            j.sink = kLog2e * __builtin_bit_cast(float, load_scalar_i32(reinterpret_cast<const int32_t*>(a->sink) + h));
         job_tiles = cls;
         job_unit = unit;
         job_half = 0;
@@ -675,7 +682,7 @@ __global__ __launch_bounds__(kWWaves * 64, 1) void prefill_fwd_w64_kernel(Prefil
             float mx = -INFINITY;
 #pragma unroll
             for (int i = 0; i < 16; ++i) {
-                float x = fmaf(s_acc[i], p.scale_log2, nb[c]);
+                float x = fmaf(s_acc[i], cur.scale, nb[c]);
                 if (masked) {
                     const int key = k0 + 8 * (i >> 2) + 4 * kg + (i & 3);
                     bool keep = key < fr.sk;
@@ -851,7 +858,7 @@ __global__ __launch_bounds__(kWWaves * 64, 1) void prefill_fwd_w64_kernel(Prefil
         [n_pipe] "s"(__builtin_amdgcn_readfirstlane(min(n_plain, n_stop))),                                           \
         [n_mask] "s"(__builtin_amdgcn_readfirstlane(n_mask)), [aligned] "s"(__builtin_amdgcn_readfirstlane(aligned)), \
         [kstep] "s"(__builtin_amdgcn_readfirstlane(k_step)), [vstep] "s"(__builtin_amdgcn_readfirstlane(v_step)),     \
-        [ldsdst] "s"(lds_dst), [scale] "s"(__builtin_amdgcn_readfirstlane(__builtin_bit_cast(uint32_t, p.scale_log2))), \
+        [ldsdst] "s"(lds_dst), [scale] "s"(__builtin_amdgcn_readfirstlane(__builtin_bit_cast(uint32_t, cur.scale))), \
         [klo] "s"(__builtin_amdgcn_readfirstlane((uint32_t)kptr)),                                                    \
         [khi] "s"(__builtin_amdgcn_readfirstlane((uint32_t)(kptr >> 32))),                                            \
         [vlo] "s"(__builtin_amdgcn_readfirstlane((uint32_t)vptr)),                                                    \
@@ -956,7 +963,8 @@ __global__ __launch_bounds__(kWWaves * 64, 1) void prefill_fwd_w64_kernel(Prefil
         };
         const auto store_block = [&](auto c_c) {
             constexpr int c = decltype(c_c)::value;
-            const float inv = 1.0f / l_row[c];     // l == 0 (no key kept) -> NaN row, like the reference softmax
+            // (the sink joins the denominator only; l == 0 and no sink (no key kept) -> NaN row, like the reference softmax)
+            const float inv = 1.0f / (l_row[c] + fast_exp2(cur.sink + nb[c]));
             // sum_j exp(scale * s_j) = l * 2^(-nb)  ->  lse = ln2 * (log2 l - nb); no key kept -> -inf
             if (cur.lb && kg == 0 && qw0 + 32 * c + n < sq)
                 cur.lb[qw0 + 32 * c + n] = l_row[c] > 0.f ? 0.69314718056f * (__log2f(l_row[c]) - nb[c]) : -INFINITY;

@@ -3,6 +3,8 @@
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 
+#include "common.hpp"
+
 namespace mi355 {
 
 struct PrefillParams {
@@ -19,6 +21,10 @@ struct PrefillParams {
     int64_t ls[2];                        // its batch and head strides (elements); rows are contiguous
     int B, Hq, Hkv, Sq, Sk;
     float scale_log2;
+    // optional per-query-head terms (forward only): a factor on the scores, and a sink -- a score without key or value
+    // (natural-log units, not scaled) that only enters the softmax denominator, once per query row
+    const float* head_scale;
+    const float* sink;
     int mask_mode;
     int n_qtiles;
     int n_pairs;                          // units per (batch, head) of the 8-wavefront kernel's grid: pairs of query tiles, or ...

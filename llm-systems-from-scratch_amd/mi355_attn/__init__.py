@@ -13,6 +13,13 @@ llm-core/llm_core/model.py:308-325 and the SDPA slot at model.py:382):
     rope_and_cache_fp8(q, k, v, positions, freq_cache, k_cache8, v_cache8, k_scale, v_scale, slot_mapping)
     rms_norm(x, weight, eps, residual=None)             # RMSNorm.forward / TritonRMSNorm forward
     silu_mul(gate, up)                                  # fused kernel of FusedSwiGLU
+    paged_attention_any(q, k_cache, v_cache, block_tables, context_lens)   # any head size, bf16 or fp32
+    kv_cache_write(k, v, k_cache, v_cache, slot_mapping)                   # cache producer without RoPE
+    dyt_residual(resid, sub, gate=, post=, norm=)       # gated residual add between Dynamic Tanh norms
+    polynorm(z, coeffs, eps)                            # PolyNorm activation
+    embed_pos(embed, pos, tokens, positions)            # token + learned position embedding, fp32
+
+Models (paged cache, batched prefill and decode, sampling): load_model(folder), CachedTransformerLM, ZuzelornLM.
 
 Every function runs on the HIP library; there is no CPU or PyTorch fallback.
 """
@@ -23,6 +30,11 @@ from .ops import (  # noqa: F401
     rope_and_cache,
     rope_and_cache_fp8,
     silu_mul,
+    dyt_residual,
+    polynorm,
+    embed_pos,
+    kv_cache_write,
+    paged_attention_any,
     flash_attn_paged_prefill,
     gather_kv_fp8,
     flash_attn_prefill,
@@ -35,6 +47,8 @@ from .ops import (  # noqa: F401
     scaled_dot_product_attention,
     sdpa_slot,
 )
-from .engine import BlockAllocator, OutOfBlocks, PagedAttentionEngine  # noqa: F401
-from .model import CachedTransformerLM  # noqa: F401
+from .engine import AttentionLayer, BlockAllocator, OutOfBlocks, PagedAttentionEngine  # noqa: F401
+from .model import CachedLM, CachedTransformerLM  # noqa: F401
+from .registry import ARCHITECTURES, UnsupportedDtype, load_model, model_class  # noqa: F401
+from .zuzelorn import ZuzelornLM  # noqa: F401
 from ._lib import LIB_PATH, LibraryMissing, load  # noqa: F401

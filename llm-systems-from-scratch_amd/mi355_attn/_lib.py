@@ -6,6 +6,9 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libmi355attn.so")
+# the same library without the training kernels: what a served model needs, built by the command line tools in a fresh checkout
+SERVING_LIB_PATH = os.path.join(_HERE, "libmi355attn_serving.so")
+TRAINING_ONLY = ("mi355_prefill_bwd", "mi355_prefill_bwd_mask")
 
 MI355_BF16 = 0
 MI355_FP8_E4M3 = 1
@@ -37,6 +40,14 @@ EXPORTS = (
     "mi355_quantize_kv_fp8",
     "mi355_rms_norm_fwd",
     "mi355_silu_mul_fwd",
+    "mi355_prefill_fwd_headwise",
+    "mi355_prefill_paged_fwd_headwise",
+    "mi355_paged_decode_fwd_headwise",
+    "mi355_paged_attn_any_fwd",
+    "mi355_kv_cache_write",
+    "mi355_dyt_residual_fwd",
+    "mi355_polynorm_fwd",
+    "mi355_embed_pos_fwd",
     "mi355_calib_copy",
     "mi355_last_error",
     "mi355_version",
@@ -47,16 +58,41 @@ class LibraryMissing(RuntimeError):
     pass
 
 
+def built():
+    """Path of the library to load: the full one, else the serving one, else None."""
+    return next((p for p in (LIB_PATH, SERVING_LIB_PATH) if os.path.exists(p)), None)
+
+
+class _ServingLib:
+    """The serving library under the full one's interface: an entry point that it lacks is an error when it is called."""
+
+    class _Missing:
+        def __init__(self, name):
+            self.name = name
+
+        def __call__(self, *args):
+            raise LibraryMissing(f"{self.name} is not in {SERVING_LIB_PATH}; run `python llm-systems-from-scratch_amd/build.py`")
+
+    def __init__(self, lib):
+        self._lib = lib
+        for name in TRAINING_ONLY:
+            setattr(self, name, self._Missing(name))
+
+    def __getattr__(self, name):
+        return getattr(self._lib, name)
+
+
 def load():
     """Loads the HIP library once.  There is no fallback: a missing library is an error."""
     global _lib
     if _lib is not None:
         return _lib
-    if not os.path.exists(LIB_PATH):
+    path = built()
+    if path is None:
         raise LibraryMissing(
             f"{LIB_PATH} is not built; run `python llm-systems-from-scratch_amd/build.py` "
             "(needs hipcc, cross-compiles for gfx950 without a GPU)")
-    lib = C.CDLL(LIB_PATH)
+    lib = C.CDLL(path) if path == LIB_PATH else _ServingLib(C.CDLL(path))
     vp, i32, i64, f32, sz = C.c_void_p, C.c_int, C.c_int64, C.c_float, C.c_size_t
     lib.mi355_prefill_fwd.restype = i32
     lib.mi355_prefill_fwd.argtypes = [vp, vp, vp, vp, _i64x3, _i64x3, _i64x3, _i64x3, vp, vp, vp, _i64x3,
@@ -106,6 +142,27 @@ def load():
     lib.mi355_rms_norm_fwd.argtypes = [vp, vp, vp, vp, vp, vp, i64, i32, i64, i64, i64, i64, f32, i32, vp]
     lib.mi355_silu_mul_fwd.restype = i32
     lib.mi355_silu_mul_fwd.argtypes = [vp, vp, vp, i64, i32, i64, i64, i64, vp]
+    lib.mi355_prefill_fwd_headwise.restype = i32
+    lib.mi355_prefill_fwd_headwise.argtypes = [vp, vp, vp, vp, _i64x3, _i64x3, _i64x3, _i64x3, vp, vp, vp, vp,
+                                               i32, i32, i32, i32, i32, i32, f32, i32, i32, i32, i64, vp, sz, vp]
+    lib.mi355_prefill_paged_fwd_headwise.restype = i32
+    lib.mi355_prefill_paged_fwd_headwise.argtypes = [vp, vp, vp, vp, i64, i64, vp, vp, i64, i64, vp, vp, vp,
+                                                     i32, i32, i32, i32, i32, i32, i64, f32, i32, i32, i64, vp, sz, vp]
+    lib.mi355_paged_decode_fwd_headwise.restype = i32
+    lib.mi355_paged_decode_fwd_headwise.argtypes = [vp, i64, vp, vp, vp, vp, i64, vp, vp, vp, vp, vp, vp, sz,
+                                                    i32, i32, i32, i32, i32, i64, i32, f32, i32, vp]
+    lib.mi355_paged_attn_any_fwd.restype = i32
+    lib.mi355_paged_attn_any_fwd.argtypes = [vp, vp, vp, vp, i64, i64, i64, vp, vp, i64, i64, vp, vp, vp,
+                                             i32, i32, i32, i32, i32, i32, i64, f32, i32, vp]
+    lib.mi355_kv_cache_write.restype = i32
+    lib.mi355_kv_cache_write.argtypes = [vp, vp, vp, vp, vp, i64, i64, i32, i32, i32, i64, i64, i32, vp]
+    lib.mi355_dyt_residual_fwd.restype = i32
+    lib.mi355_dyt_residual_fwd.argtypes = [vp, vp, vp, vp, f32, vp, vp, vp, vp, f32, vp, vp, vp, i64, i32, i64, i64, i64,
+                                           i32, vp]
+    lib.mi355_polynorm_fwd.restype = i32
+    lib.mi355_polynorm_fwd.argtypes = [vp, vp, i64, i32, i64, i64, C.c_float * 4, f32, i32, vp]
+    lib.mi355_embed_pos_fwd.restype = i32
+    lib.mi355_embed_pos_fwd.argtypes = [vp, vp, vp, vp, vp, i64, i32, i64, i64, i32, vp]
     lib.mi355_calib_copy.restype = i32
     lib.mi355_calib_copy.argtypes = [vp, vp, sz, vp]
     lib.mi355_last_error.restype = C.c_char_p
@@ -120,6 +177,10 @@ def strides3(values):
 
 def strides2(values):
     return _i64x2(*[int(v) for v in values])
+
+
+def floats4(values):
+    return (C.c_float * 4)(*[float(v) for v in values])
 
 
 def check(rc: int, what: str):

@@ -5,17 +5,19 @@ which re-runs the whole forward per token at :218) needs around the attention ke
 allocator, per-sequence block tables, slot mapping for cache writes, a prefill call for newly
 admitted sequences and a decode call that serves every running sequence with one kernel launch
 per layer and step.  The bookkeeping (blocks, lengths, tables) is shared by all attention layers
-of a model; every layer has its own K/V pools.  A step is planned once (`plan_prefill`,
+of a model; every layer has its own K/V pools, of its own head count and head sizes, or reads those
+of an earlier layer (`AttentionLayer`).  A step is planned once (`plan_prefill`,
 `plan_decode`: host integers -> a few small device tensors) and then applied per layer
 (`attend_prefill`, `attend_decode`).  Projections, sampling and the scheduler policy stay with
 the caller.
 
-All tensor work runs on the HIP kernels (rope_and_cache, flash_attn_varlen_prefill,
-flash_attn_paged_prefill, paged_attention_decode); the bookkeeping here is plain Python on host integers.
+All tensor work runs on the HIP kernels (rope_and_cache, kv_cache_write, flash_attn_varlen_prefill,
+flash_attn_paged_prefill, paged_attention_decode, paged_attention_any); the bookkeeping here is plain Python on host integers.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+import math
+from dataclasses import dataclass, field
 
 import torch
 
@@ -26,6 +28,38 @@ BLOCK = 16
 
 class OutOfBlocks(RuntimeError):
     pass
+
+
+@dataclass
+class AttentionLayer:
+    """One attention layer as the cache manager sees it.  head_dim is the size of a query/key head, v_dim of a value
+    head (None: head_dim).  kv_from = i: the layer has no keys and values of its own and reads layer i's pools.
+    softmax_scale None: 1/sqrt(head_dim).  head_scale (non-negative factor per query head) and sinks (score without key
+    or value per query head) are fp32 (n_q_heads,) tensors or None.  rope: rotate q and k by the position."""
+    n_q_heads: int
+    n_kv_heads: int
+    head_dim: int
+    v_dim: int | None = None
+    kv_from: int | None = None
+    softmax_scale: float | None = None
+    head_scale: torch.Tensor | None = None
+    sinks: torch.Tensor | None = None
+    rope: bool = True
+
+
+def cache_head_dims(kv_dtype: str, head_dim: int, v_dim: int) -> tuple[int, int, bool]:
+    """(key size, value size, mfma?) of the head rows a pool holds.  The MFMA kernels take equal sizes of 32, 64 or 128
+    (fp8: 64 or 128): smaller heads are padded with zeros up to the next of these, which changes neither a score nor a
+    sum.  fp32 pools and larger heads go to the general kernel, in rows of whole 8-element pieces."""
+    if kv_dtype != "fp32":
+        for d in ((64, 128) if kv_dtype == "fp8" else (32, 64, 128)):
+            if max(head_dim, v_dim) <= d:
+                return d, d, True
+    if kv_dtype == "fp8":
+        raise ValueError("an fp8 KV cache needs head sizes up to 128")
+    if max(head_dim, v_dim) > 512:
+        raise ValueError("head sizes above 512 are not supported")
+    return (head_dim + 7) // 8 * 8, (v_dim + 7) // 8 * 8, False
 
 
 class BlockAllocator:
@@ -61,6 +95,8 @@ class PrefillPlan:
     context_lens: torch.Tensor | None = None  # (B,) int32: tokens in the cache, this chunk included
     total_context: int = 0                    # their sum (sizes the dequantised rows of an fp8 cache)
     cu_context: torch.Tensor | None = None    # (B+1,) int32: their running sum (fp8 cache: where each sequence's rows start)
+    # packed keys and values of layers that later layers share (new sequences only), by layer
+    packed: dict[int, tuple] = field(default_factory=dict)
 
 
 @dataclass
@@ -111,33 +147,75 @@ class StaticDecodeStep:
 
 
 class PagedAttentionEngine:
-    def __init__(self, num_blocks, n_q_heads, n_kv_heads, head_dim, context_length, *, rope_theta=10000.0,
-                 max_batch=256, num_layers=1, kv_dtype="bf16", device="cuda:0"):
+    def __init__(self, num_blocks, n_q_heads=None, n_kv_heads=None, head_dim=None, context_length=None, *, rope_theta=10000.0,
+                 max_batch=256, num_layers=1, kv_dtype="bf16", device="cuda:0", layers: list[AttentionLayer] | None = None):
+        """Either n_q_heads, n_kv_heads, head_dim and num_layers (equal layers with RoPE) or `layers`.  kv_dtype: "bf16",
+        "fp8" (e4m3 + scales) or "fp32" (pools, queries and outputs in fp32, general attention kernel).
+        q, k and v of layer i come with the head sizes cache_dims[i] (padded with zeros where a head is smaller)."""
         self.device = torch.device(device)
-        self.Hq, self.Hkv, self.D = n_q_heads, n_kv_heads, head_dim
+        if context_length is None:
+            raise ValueError("context_length is required")
+        if kv_dtype not in ("bf16", "fp8", "fp32"):
+            raise ValueError("kv_dtype must be 'bf16', 'fp8' or 'fp32'")
+        if layers is None:
+            if kv_dtype == "fp8" and head_dim not in (64, 128):
+                raise ValueError("an fp8 KV cache needs head_dim 64 or 128")
+            if kv_dtype == "fp32":
+                raise ValueError("an fp32 KV cache has no rotating cache write; describe layers without rope")
+            layers = [AttentionLayer(n_q_heads, n_kv_heads, head_dim) for _ in range(num_layers)]
+        self.layers = layers
+        self.num_layers = len(layers)
         self.context_length = context_length
-        self.num_layers = num_layers
-        if kv_dtype not in ("bf16", "fp8"):
-            raise ValueError("kv_dtype must be 'bf16' or 'fp8'")
-        if kv_dtype == "fp8" and head_dim not in (64, 128):
-            raise ValueError("an fp8 KV cache needs head_dim 64 or 128")
         self.kv_dtype = kv_dtype
-        cache_dtype = torch.bfloat16 if kv_dtype == "bf16" else torch.uint8      # uint8 = e4m3 bit patterns
-        self.k_caches = [torch.zeros(num_blocks, n_kv_heads, BLOCK, head_dim, dtype=cache_dtype, device=self.device)
-                         for _ in range(num_layers)]
-        self.v_caches = [torch.zeros_like(k) for k in self.k_caches]
+        self.Hq, self.Hkv, self.D = layers[0].n_q_heads, layers[0].n_kv_heads, layers[0].head_dim
+        cache_dtype = {"bf16": torch.bfloat16, "fp8": torch.uint8, "fp32": torch.float32}[kv_dtype]      # uint8 = e4m3 bit patterns
+        self.k_caches, self.v_caches, self.cache_dims, self.mfma = [], [], [], []
         # per-(block, kv head) scales of an fp8 cache, maintained by the cache write
-        self.k_scales = [torch.ones(num_blocks, n_kv_heads, dtype=torch.float32, device=self.device)
-                         for _ in range(num_layers)] if kv_dtype == "fp8" else None
-        self.v_scales = [torch.ones_like(s) for s in self.k_scales] if kv_dtype == "fp8" else None
-        self.freq_cache = ops.build_rope_cache(context_length, head_dim, rope_theta, self.device)
+        self.k_scales, self.v_scales = ([], []) if kv_dtype == "fp8" else (None, None)
+        self.shared = {ly.kv_from for ly in layers if ly.kv_from is not None}
+        rope_dims = set()
+        for i, ly in enumerate(layers):
+            if ly.n_q_heads < 1 or ly.n_kv_heads < 1 or ly.n_q_heads % ly.n_kv_heads:
+                raise ValueError(f"layer {i}: {ly.n_q_heads} query heads over {ly.n_kv_heads} kv heads")
+            kd, vd, mfma = cache_head_dims(kv_dtype, ly.head_dim, ly.v_dim or ly.head_dim)
+            if ly.rope and (not mfma or kd != ly.head_dim or (ly.v_dim or kd) != kd):
+                raise ValueError(f"layer {i}: RoPE needs equal head sizes of 32, 64 or 128 and a 16- or 8-bit cache")
+            self.cache_dims.append((kd, vd))
+            self.mfma.append(mfma)
+            src = ly.kv_from
+            if src is not None:
+                if not 0 <= src < i or layers[src].kv_from is not None:
+                    raise ValueError(f"layer {i}: kv_from {src} is not an earlier layer with keys and values of its own")
+                if layers[src].n_kv_heads != ly.n_kv_heads or self.cache_dims[src] != (kd, vd) or layers[src].rope != ly.rope:
+                    raise ValueError(f"layer {i}: kv heads, head sizes and rotation differ from those of layer {src}, whose cache it reads")
+                self.k_caches.append(self.k_caches[src])
+                self.v_caches.append(self.v_caches[src])
+            else:
+                self.k_caches.append(torch.zeros(num_blocks, ly.n_kv_heads, BLOCK, kd, dtype=cache_dtype, device=self.device))
+                self.v_caches.append(torch.zeros(num_blocks, ly.n_kv_heads, BLOCK, vd, dtype=cache_dtype, device=self.device))
+            if kv_dtype == "fp8":
+                for sc in (self.k_scales, self.v_scales):
+                    sc.append(sc[src] if src is not None else
+                              torch.ones(num_blocks, ly.n_kv_heads, dtype=torch.float32, device=self.device))
+            if ly.rope:
+                rope_dims.add(kd)
+        # layers on the general kernel read every key through the tables, also in the first chunk of a prompt
+        self.always_tables = not all(self.mfma)
+        if len(rope_dims) > 1:
+            raise ValueError("layers with RoPE must share one head size")
+        self.freq_cache = ops.build_rope_cache(context_length, rope_dims.pop(), rope_theta, self.device) if rope_dims else None
+        # rotation by the angle 0 (cos 1, sin 0, every position clamped to the one row) for layers without RoPE on an fp8 cache
+        self._no_rotation = {d: torch.stack((torch.ones(1, d // 2), torch.zeros(1, d // 2))).to(self.device)
+                             for d in {kd for kd, _ in self.cache_dims}} if kv_dtype == "fp8" else None
         self.allocator = BlockAllocator(num_blocks)
         self.blocks: dict[int, list[int]] = {}      # sequence id -> physical blocks
         self.lengths: dict[int, int] = {}           # sequence id -> tokens in the cache
         self.max_blocks_per_seq = (context_length + BLOCK - 1) // BLOCK
         # persistent step buffers: no allocation on the decode path besides the kernel outputs
         self._tables = torch.zeros(max_batch, self.max_blocks_per_seq, dtype=torch.int32, device=self.device)
-        self._workspace = ops.paged_decode_workspace(max_batch, n_q_heads, head_dim, context_length, self.device)
+        self._workspace = max((ops.paged_decode_workspace(max_batch, hq, d, context_length, self.device)
+                               for hq, d in {(ly.n_q_heads, kd) for ly, (kd, _), m in zip(layers, self.cache_dims, self.mfma) if m}),
+                              key=lambda t: t.numel(), default=None)
         self.max_batch = max_batch
 
     # the pools of layer 0 under their single-layer names
@@ -203,7 +281,7 @@ class PagedAttentionEngine:
                            torch.tensor(slots, dtype=torch.int64, device=dev),
                            torch.tensor(cu, dtype=torch.int32, device=dev), max(lens),
                            torch.tensor([c - 1 for c in cu[1:]], dtype=torch.int64, device=dev))
-        if chunked:
+        if chunked or self.always_tables:
             max_blk = max(len(self.blocks[sid]) for sid in seq_ids)
             rows = torch.zeros(len(seq_ids), max_blk, dtype=torch.int32)
             for i, sid in enumerate(seq_ids):
@@ -212,7 +290,7 @@ class PagedAttentionEngine:
             plan.tables = rows.to(dev)
             plan.context_lens = torch.tensor([self.lengths[sid] for sid in seq_ids], dtype=torch.int32, device=dev)
             plan.total_context = sum(self.lengths[sid] for sid in seq_ids)
-            if self.kv_dtype != "bf16":
+            if self.kv_dtype == "fp8":
                 run = [0]
                 for sid in seq_ids:
                     run.append(run[-1] + self.lengths[sid])
@@ -276,43 +354,69 @@ class PagedAttentionEngine:
 
     # ---- attention calls (once per layer) -----------------------------------------
     def _write_cache(self, layer: int, plan, q, k, v, k_out=None):
-        """RoPE on q and k, rotated k and v into layer `layer`'s cache (quantised when the cache is fp8);
-        returns the rotated q -- with k_out=True the pair (rotated q, rotated k in packed form)."""
+        """q and k rotated (layers with RoPE), k and v into layer `layer`'s cache (quantised when the cache is fp8);
+        returns the query to attend with -- with k_out=True the pair (query, keys in packed form).  A layer that reads
+        another layer's cache (k and v None) writes nothing."""
+        if self.layers[layer].kv_from is not None:
+            if k is not None or v is not None:
+                raise ValueError(f"layer {layer} reads the cache of layer {self.layers[layer].kv_from} and takes no keys or values")
+            return (q, None) if k_out else q
         kc, vc = self.k_caches[layer], self.v_caches[layer]
-        if self.kv_dtype == "bf16":
+        rope = self.layers[layer].rope
+        if self.kv_dtype == "fp8":
+            freq = self.freq_cache if rope else self._no_rotation[q.shape[2]]
+            return ops.rope_and_cache_fp8(q, k, v, plan.positions, freq, kc, vc, self.k_scales[layer],
+                                          self.v_scales[layer], plan.slots, k_out=k_out)
+        if rope:
             return ops.rope_and_cache(q, k, v, plan.positions, self.freq_cache, kc, vc, plan.slots, k_out=k_out)
-        return ops.rope_and_cache_fp8(q, k, v, plan.positions, self.freq_cache, kc, vc, self.k_scales[layer],
-                                      self.v_scales[layer], plan.slots, k_out=k_out)
+        ops.kv_cache_write(k, v, kc, vc, plan.slots)
+        return (q, k) if k_out else q
+
+    def _score_terms(self, layer: int):
+        ly = self.layers[layer]
+        scale = 1.0 / math.sqrt(ly.head_dim) if ly.softmax_scale is None else ly.softmax_scale        # (of the unpadded head)
+        return dict(softmax_scale=scale, head_scale=ly.head_scale, sinks=ly.sinks)
 
     def attend_prefill(self, layer: int, plan: PrefillPlan, q, k, v):
-        """q (T,Hq,D), k/v (T,Hkv,D) packed along dim 0 (token strides free, heads contiguous).  Writes
-        rotated K and V of layer `layer` into its cache and returns causal attention output (T,Hq,D).
-        New sequences attend to the packed tensors themselves (one launch rotates q and k and fills the
-        cache); when a sequence already had cached tokens, keys and values are read back through the
-        block tables, old and new alike."""
+        """q (T,Hq,D), k/v (T,Hkv,D) packed along dim 0 (token strides free, heads contiguous; k and v None for a layer
+        that reads another layer's cache).  Writes (rotated) K and V of layer `layer` into its cache and returns causal
+        attention output (T,Hq,D).  New sequences attend to the packed tensors themselves; when a sequence already had
+        cached tokens, keys and values are read back through the block tables, old and new alike."""
         if q.shape[0] != plan.positions.shape[0]:
             raise ValueError("the plan and the packed tensors disagree on the number of tokens")
+        terms = self._score_terms(layer)
         if plan.tables is not None:
-            q_rot = self._write_cache(layer, plan, q, k, v)
-            scales = {} if self.kv_dtype == "bf16" else {"k_scale": self.k_scales[layer], "v_scale": self.v_scales[layer],
-                                                         "total_context": plan.total_context,
-                                                         "cu_seqlens_k": plan.cu_context}
-            return ops.flash_attn_paged_prefill(q_rot, self.k_caches[layer], self.v_caches[layer], plan.cu_seqlens,
-                                                plan.tables, plan.context_lens, plan.max_len, **scales)
-        q_rot, k_rot = self._write_cache(layer, plan, q, k, v, k_out=True)
-        return ops.flash_attn_varlen_prefill(q_rot, k_rot, v, plan.cu_seqlens, plan.cu_seqlens, plan.max_len,
-                                             plan.max_len, causal=True)
+            q = self._write_cache(layer, plan, q, k, v)
+            kc, vc = self.k_caches[layer], self.v_caches[layer]
+            if not self.mfma[layer]:
+                return ops.paged_attention_any(q, kc, vc, plan.tables, plan.context_lens, cu_seqlens_q=plan.cu_seqlens, **terms)
+            if self.kv_dtype == "fp8":
+                terms.update(k_scale=self.k_scales[layer], v_scale=self.v_scales[layer], total_context=plan.total_context,
+                             cu_seqlens_k=plan.cu_context)
+            return ops.flash_attn_paged_prefill(q, kc, vc, plan.cu_seqlens, plan.tables, plan.context_lens, plan.max_len, **terms)
+        q, k = self._write_cache(layer, plan, q, k, v, k_out=True)
+        src = self.layers[layer].kv_from
+        if src is not None:
+            k, v = plan.packed[src]
+        elif layer in self.shared:
+            plan.packed[layer] = (k, v)
+        return ops.flash_attn_varlen_prefill(q, k, v, plan.cu_seqlens, plan.cu_seqlens, plan.max_len,
+                                             plan.max_len, causal=True, **terms)
 
     def attend_decode(self, layer: int, plan: DecodePlan, q, k, v):
-        """q (B,Hq,D), k/v (B,Hkv,D): appends the token's K/V to layer `layer`'s cache and returns its
-        attention output (B,Hq,D)."""
+        """q (B,Hq,D), k/v (B,Hkv,D) or None as in attend_prefill: appends the token's K/V to layer `layer`'s cache and
+        returns its attention output (B,Hq,D)."""
         if q.shape[0] != plan.positions.shape[0]:
             raise ValueError("one query token per sequence expected")
-        q_rot = self._write_cache(layer, plan, q, k, v)
-        scales = {} if self.kv_dtype == "bf16" else {"k_scale": self.k_scales[layer], "v_scale": self.v_scales[layer]}
-        return ops.paged_attention_decode(q_rot, self.k_caches[layer], self.v_caches[layer], plan.tables,
-                                          plan.context_lens, max_context=plan.max_context, workspace=self._workspace,
-                                          **scales)
+        q = self._write_cache(layer, plan, q, k, v)
+        terms = self._score_terms(layer)
+        kc, vc = self.k_caches[layer], self.v_caches[layer]
+        if not self.mfma[layer]:
+            return ops.paged_attention_any(q, kc, vc, plan.tables, plan.context_lens, **terms)
+        if self.kv_dtype == "fp8":
+            terms.update(k_scale=self.k_scales[layer], v_scale=self.v_scales[layer])
+        return ops.paged_attention_decode(q, kc, vc, plan.tables, plan.context_lens, max_context=plan.max_context,
+                                          workspace=self._workspace, **terms)
 
     # ---- single-layer convenience ----------------------------------------------------
     def prefill(self, seq_ids, lens, q, k, v):

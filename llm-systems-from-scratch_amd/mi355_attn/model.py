@@ -1,4 +1,7 @@
-"""KV-cached inference model with the reference decoder's parameters and call surface.
+"""KV-cached inference models: the serving base class, and the model with the reference decoder's parameters.
+
+`CachedLM` holds what every served decoder shares (sequences, prefill / decode / mixed steps, decode graphs, sampling
+loops with the reference's call surface).
 
 `CachedTransformerLM` computes what TransformerLM.forward does (llm-core/llm_core/model.py:180-185:
 embedding -> N x [RMSNorm -> causal attention with RoPE -> residual -> RMSNorm -> SwiGLU -> residual]
@@ -20,92 +23,42 @@ import torch
 
 from . import ops
 from .engine import BLOCK, PagedAttentionEngine
+from .weights import load_state_dict
 
 
-class CachedTransformerLM:
-    def __init__(self, config: dict, state_dict: dict, *, num_blocks: int | None = None, max_batch: int = 64,
-                 kv_dtype: str = "bf16", decode_graphs: bool = False, device="cuda:0"):
-        """config: the reference's constructor arguments (model.py:128-137: vocab_size, context_length,
-        d_model, num_layers, num_heads, d_ff, rope_theta); state_dict: the reference's parameter names,
-        with either the separate (ffn.gate_proj/up_proj/down_proj) or the merged (ffn.w_gate_up/w_down)
-        feed-forward weights.  num_blocks sizes the KV pool of every layer (default: max_batch full
-        contexts); kv_dtype "fp8" keeps the pool as e4m3 bytes with per-(block, head) scales (half the
-        cache bytes per decode step; d_head 64 or 128).  decode_graphs=True replays every decode step
-        after the first of a batch size from a captured HIP graph (about ten launches per layer become one
-        graph launch; the step's tensors then live at fixed addresses and tables have their full width)."""
-        self.config = dict(config)
-        self.device = torch.device(device)
-        self.vocab_size = config["vocab_size"]
-        self.context_length = config["context_length"]
-        self.d_model = d = config["d_model"]
-        self.num_layers = L = config["num_layers"]
-        self.num_heads = H = config["num_heads"]
-        self.d_ff = config["d_ff"]
-        if d % H:
-            raise ValueError("d_model must be divisible by num_heads")
-        self.d_head = d // H
-        if self.d_head not in (32, 64, 128):
-            raise ValueError("the attention kernels need d_head in {32, 64, 128}")
-        sd = {k[len("_orig_mod."):] if k.startswith("_orig_mod.") else k: v for k, v in state_dict.items()}  # model.py:247-251
+class CachedLM:
+    """What every KV-cached decoder of the package shares: sequences, prefill / decode / mixed steps, decode graphs and
+    sampling loops over a PagedAttentionEngine.  A subclass builds its weights and its engine, calls `_serve`, and
+    implements `_forward(token_ids, plan, attend, out_rows)`: (T,) token ids on the device -> fp32 logits of the packed
+    rows `out_rows` (None: all), with attend(layer, plan, q, k, v) for the attention of each layer."""
 
-        def w(name, dtype=torch.bfloat16):
-            return sd[name].detach().to(device=self.device, dtype=dtype).contiguous()
+    DTYPES = ("bfloat16",)          # compute types the class serves
 
-        self.emb = w("token_embeddings.weight")
-        self.lm_head = w("lm_head.weight")
-        self.final_norm = w("final_norm.weight", torch.float32)
-        self.layers = []
-        for i in range(L):
-            pre = f"layers.{i}."
-            wqkv = torch.cat([w(pre + f"attn.{n}.weight") for n in ("q_proj", "k_proj", "v_proj")])
-            if pre + "ffn.w_gate_up.weight" in sd:
-                wgu, wdown = w(pre + "ffn.w_gate_up.weight"), w(pre + "ffn.w_down.weight")
-            else:
-                wgu = torch.cat([w(pre + "ffn.gate_proj.weight"), w(pre + "ffn.up_proj.weight")])
-                wdown = w(pre + "ffn.down_proj.weight")
-            self.layers.append(dict(wqkv=wqkv, wo=w(pre + "attn.output_proj.weight"), wgu=wgu, wdown=wdown,
-                                    attn_norm=w(pre + "attn_norm.weight", torch.float32),
-                                    ffn_norm=w(pre + "ffn_norm.weight", torch.float32)))
-        if num_blocks is None:
-            num_blocks = max_batch * ((self.context_length + BLOCK - 1) // BLOCK)
-        self.engine = PagedAttentionEngine(num_blocks, H, H, self.d_head, self.context_length,
-                                           rope_theta=config["rope_theta"], max_batch=max_batch, num_layers=L,
-                                           kv_dtype=kv_dtype, device=self.device)
+    def _serve(self, engine: PagedAttentionEngine, vocab_size: int, decode_graphs: bool) -> None:
+        self.engine = engine
+        self.device = engine.device
+        self.vocab_size = vocab_size
+        self.context_length = engine.context_length
         self._next_id = 0
         self.decode_graphs = decode_graphs
         self._graphs = {}                      # batch size -> [static step tensors, captured graph, its logits]
 
     @classmethod
-    def from_pretrained(cls, config_path: str, checkpoint_path: str, **kwargs) -> "CachedTransformerLM":
-        """Same files as TransformerLM.from_pretrained (model.py:238-256): a JSON config and a checkpoint that is
-        a state_dict or {"model": state_dict}.  The checkpoint is read with weights_only=True."""
+    def from_pretrained(cls, config_path: str, checkpoint_path: str, **kwargs) -> "CachedLM":
+        """Same files as TransformerLM.from_pretrained (model.py:238-256): a JSON config and a checkpoint -- here a
+        .safetensors file, or a torch file (read with weights_only=True) that is a state_dict or {"model": state_dict}."""
         with open(config_path) as f:
             config = json.load(f)
-        sd = torch.load(checkpoint_path, map_location="cpu", weights_only=True)
-        if "model" in sd:
-            sd = sd["model"]
-        return cls(config, sd, **kwargs)
+        return cls(config, load_state_dict(checkpoint_path), **kwargs)
 
-    # ---- the decoder on packed tokens ------------------------------------------------------
     def _forward(self, token_ids, plan, attend, out_rows=None):
-        """token_ids (T,) int64 on the device; attend(layer, plan, q, k, v) -> (T,H,d_head).
-        Returns logits of rows `out_rows` (default: all rows), fp32."""
-        H, dh, d, ff = self.num_heads, self.d_head, self.d_model, self.d_ff
-        T = token_ids.shape[0]
-        resid = self.emb[token_ids]                                   # model.py:50
-        h = ops.rms_norm(resid, self.layers[0]["attn_norm"])
-        for i, ly in enumerate(self.layers):
-            qkv = (h @ ly["wqkv"].T).view(T, 3, H, dh)                 # model.py:361-370 in one GEMM
-            a = attend(i, plan, qkv[:, 0], qkv[:, 1], qkv[:, 2])      # model.py:372-385
-            o = a.reshape(T, d) @ ly["wo"].T                           # model.py:388-390
-            h, resid = ops.rms_norm(o, ly["ffn_norm"], residual=resid, return_sum=True)    # model.py:293-294
-            gu = h @ ly["wgu"].T
-            f = ops.silu_mul(gu[:, :ff], gu[:, ff:]) @ ly["wdown"].T   # model.py:304-305
-            nxt = self.layers[i + 1]["attn_norm"] if i + 1 < self.num_layers else self.final_norm
-            h, resid = ops.rms_norm(f, nxt, residual=resid, return_sum=True)              # model.py:294, :184
-        if out_rows is not None:
-            h = h[out_rows]
-        return (h @ self.lm_head.T).float()                            # model.py:185
+        raise NotImplementedError
+
+    def _token_ids(self, tokens):
+        ids = torch.as_tensor(tokens, dtype=torch.int64).reshape(-1)
+        if not ids.is_cuda and ids.numel() and not 0 <= int(ids.min()) <= int(ids.max()) < self.vocab_size:
+            raise ValueError(f"token ids must be in 0..{self.vocab_size - 1}")
+        return ids
 
     # ---- sequence-level API ---------------------------------------------------------------------
     def new_sequence(self) -> int:
@@ -117,25 +70,39 @@ class CachedTransformerLM:
     def free_sequence(self, seq_id: int) -> None:
         self.engine.remove_sequence(seq_id)
 
-    def prefill(self, seq_ids, prompts, *, all_logits: bool = False):
-        """Runs the prompts (lists / 1-D tensors of token ids, each 1..context_length long) of new sequences.
-        Returns next-token logits (n_seq, vocab) fp32, or the logits of every prompt position
-        (sum(len), vocab) with all_logits=True."""
-        toks = [torch.as_tensor(p, dtype=torch.int64).reshape(-1) for p in prompts]
+    def prefill(self, seq_ids, prompts, *, all_logits: bool = False, rows=None):
+        """Runs the prompts (lists / 1-D tensors of token ids, each 1..context_length long) of new sequences, or the
+        next portions of running ones.  Returns next-token logits (n_seq, vocab) fp32, the logits of every packed
+        position (sum(len), vocab) with all_logits=True, or those of the packed positions `rows`."""
+        toks = [self._token_ids(p) for p in prompts]
         plan = self.engine.plan_prefill(list(seq_ids), [int(t.numel()) for t in toks])
         ids = torch.cat(toks).to(self.device)
-        return self._forward(ids, plan, self.engine.attend_prefill, None if all_logits else plan.last_rows)
+        if rows is not None:
+            out_rows = torch.as_tensor(rows, dtype=torch.int64).reshape(-1).to(self.device)
+        else:
+            out_rows = None if all_logits else plan.last_rows
+        return self._forward(ids, plan, self.engine.attend_prefill, out_rows)
 
     def decode(self, seq_ids, tokens):
         """Appends one token to each running sequence; returns the next-token logits (n_seq, vocab) fp32."""
         seq_ids = list(seq_ids)
         if self.decode_graphs:
-            return self._decode_graphed(seq_ids, torch.as_tensor(tokens).reshape(-1).tolist())
-        ids = torch.as_tensor(tokens, dtype=torch.int64).reshape(-1).to(self.device)
+            return self._decode_graphed(seq_ids, self._token_ids(tokens).tolist())
+        ids = self._token_ids(tokens).to(self.device)
         if ids.numel() != len(seq_ids):
             raise ValueError("one token per sequence expected")
         plan = self.engine.plan_decode(seq_ids)
         return self._forward(ids, plan, self.engine.attend_decode)
+
+    def step(self, seq_ids, tokens, rows=None):
+        """One step that advances every sequence by its own tokens (lists of one or more): new prompts, further portions
+        and single decoded tokens mixed.  Returns the fp32 logits of the packed positions `rows` (default: each
+        sequence's last).  A step of one token for each of a few running sequences goes through `decode`."""
+        seq_ids = list(seq_ids)
+        if all(len(t) == 1 and self.engine.lengths[s] > 0 for s, t in zip(seq_ids, tokens)) and len(seq_ids) <= self.engine.max_batch:
+            logits = self.decode(seq_ids, [int(t[0]) for t in tokens])
+            return logits if rows is None else logits[torch.as_tensor(rows, dtype=torch.int64).to(self.device)]
+        return self.prefill(seq_ids, tokens, rows=rows)
 
     def _decode_graphed(self, seq_ids, tokens):
         """The decode step through a HIP graph.  The first step of a batch size runs eagerly on the static
@@ -259,3 +226,74 @@ class CachedTransformerLM:
                 if s is not None and s in self.engine.blocks:
                     self.free_sequence(s)
         return outs
+
+
+class CachedTransformerLM(CachedLM):
+    def __init__(self, config: dict, state_dict: dict, *, num_blocks: int | None = None, max_batch: int = 64,
+                 kv_dtype: str = "bf16", decode_graphs: bool = False, device="cuda:0"):
+        """config: the reference's constructor arguments (model.py:128-137: vocab_size, context_length,
+        d_model, num_layers, num_heads, d_ff, rope_theta); state_dict: the reference's parameter names,
+        with either the separate (ffn.gate_proj/up_proj/down_proj) or the merged (ffn.w_gate_up/w_down)
+        feed-forward weights.  num_blocks sizes the KV pool of every layer (default: max_batch full
+        contexts); kv_dtype "fp8" keeps the pool as e4m3 bytes with per-(block, head) scales (half the
+        cache bytes per decode step; d_head 64 or 128).  decode_graphs=True replays every decode step
+        after the first of a batch size from a captured HIP graph (about ten launches per layer become one
+        graph launch; the step's tensors then live at fixed addresses and tables have their full width)."""
+        self.config = dict(config)
+        self.device = torch.device(device)
+        self.context_length = config["context_length"]
+        self.d_model = d = config["d_model"]
+        self.num_layers = L = config["num_layers"]
+        self.num_heads = H = config["num_heads"]
+        self.d_ff = config["d_ff"]
+        if d % H:
+            raise ValueError("d_model must be divisible by num_heads")
+        self.d_head = d // H
+        if self.d_head not in (32, 64, 128):
+            raise ValueError("the attention kernels need d_head in {32, 64, 128}")
+        sd = {k[len("_orig_mod."):] if k.startswith("_orig_mod.") else k: v for k, v in state_dict.items()}  # model.py:247-251
+
+        def w(name, dtype=torch.bfloat16):
+            return sd[name].detach().to(device=self.device, dtype=dtype).contiguous()
+
+        self.emb = w("token_embeddings.weight")
+        self.lm_head = w("lm_head.weight")
+        self.final_norm = w("final_norm.weight", torch.float32)
+        self.layers = []
+        for i in range(L):
+            pre = f"layers.{i}."
+            wqkv = torch.cat([w(pre + f"attn.{n}.weight") for n in ("q_proj", "k_proj", "v_proj")])
+            if pre + "ffn.w_gate_up.weight" in sd:
+                wgu, wdown = w(pre + "ffn.w_gate_up.weight"), w(pre + "ffn.w_down.weight")
+            else:
+                wgu = torch.cat([w(pre + "ffn.gate_proj.weight"), w(pre + "ffn.up_proj.weight")])
+                wdown = w(pre + "ffn.down_proj.weight")
+            self.layers.append(dict(wqkv=wqkv, wo=w(pre + "attn.output_proj.weight"), wgu=wgu, wdown=wdown,
+                                    attn_norm=w(pre + "attn_norm.weight", torch.float32),
+                                    ffn_norm=w(pre + "ffn_norm.weight", torch.float32)))
+        if num_blocks is None:
+            num_blocks = max_batch * ((self.context_length + BLOCK - 1) // BLOCK)
+        self._serve(PagedAttentionEngine(num_blocks, H, H, self.d_head, self.context_length, rope_theta=config["rope_theta"],
+                                         max_batch=max_batch, num_layers=L, kv_dtype=kv_dtype, device=self.device),
+                    config["vocab_size"], decode_graphs)
+
+    # ---- the decoder on packed tokens ------------------------------------------------------
+    def _forward(self, token_ids, plan, attend, out_rows=None):
+        """token_ids (T,) int64 on the device; attend(layer, plan, q, k, v) -> (T,H,d_head).
+        Returns logits of rows `out_rows` (default: all rows), fp32."""
+        H, dh, d, ff = self.num_heads, self.d_head, self.d_model, self.d_ff
+        T = token_ids.shape[0]
+        resid = self.emb[token_ids]                                   # model.py:50
+        h = ops.rms_norm(resid, self.layers[0]["attn_norm"])
+        for i, ly in enumerate(self.layers):
+            qkv = (h @ ly["wqkv"].T).view(T, 3, H, dh)                 # model.py:361-370 in one GEMM
+            a = attend(i, plan, qkv[:, 0], qkv[:, 1], qkv[:, 2])      # model.py:372-385
+            o = a.reshape(T, d) @ ly["wo"].T                           # model.py:388-390
+            h, resid = ops.rms_norm(o, ly["ffn_norm"], residual=resid, return_sum=True)    # model.py:293-294
+            gu = h @ ly["wgu"].T
+            f = ops.silu_mul(gu[:, :ff], gu[:, ff:]) @ ly["wdown"].T   # model.py:304-305
+            nxt = self.layers[i + 1]["attn_norm"] if i + 1 < self.num_layers else self.final_norm
+            h, resid = ops.rms_norm(f, nxt, residual=resid, return_sum=True)              # model.py:294, :184
+        if out_rows is not None:
+            h = h[out_rows]
+        return (h @ self.lm_head.T).float()                            # model.py:185

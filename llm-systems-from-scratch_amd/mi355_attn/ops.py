@@ -112,9 +112,31 @@ def _split_args(kv_splits, workspace, B, Hq, D, sq_max, sk_max, total_rows, caus
     return n, workspace
 
 
+def _head_terms(head_scale, sinks, Hq, device):
+    """Data pointers of the optional per-query-head factors and sinks (fp32 (Hq,) tensors on `device`)."""
+    for n, t in (("head_scale", head_scale), ("sinks", sinks)):
+        if t is not None and (t.dtype != torch.float32 or t.shape != (Hq,) or not t.is_contiguous() or t.device != device):
+            raise ValueError(f"{n} must be a contiguous float32 ({Hq},) tensor on {device}")
+    return (None if t is None else t.data_ptr() for t in (head_scale, sinks))
+
+
 def _prefill(q, k, v, out, cu_q, cu_k, mask, B, Hq, Hkv, Sq, Sk, D, scale, mode, lse=None, n_split=1, workspace=None,
-             total_rows=0):
+             total_rows=0, head_scale=None, sinks=None):
     lib = _lib.load()
+    if head_scale is not None or sinks is not None:
+        hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
+        packed = cu_q is not None
+        qs, ks, vs, os_ = (_packed_or_dense_strides(x, packed) for x in (q, k, v, out))
+        with _on(q, k, v, out, cu_q, cu_k, workspace) as stream:
+            rc = lib.mi355_prefill_fwd_headwise(
+                q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr(),
+                _lib.strides3(qs), _lib.strides3(ks), _lib.strides3(vs), _lib.strides3(os_),
+                None if cu_q is None else cu_q.data_ptr(), None if cu_k is None else cu_k.data_ptr(), hs, sk,
+                B, Hq, Hkv, Sq, Sk, D, float(scale), mode, _lib.MI355_BF16, int(n_split), int(total_rows),
+                None if workspace is None else workspace.data_ptr(),
+                0 if workspace is None else workspace.numel() * workspace.element_size(), stream)
+        _lib.check(rc, "mi355_prefill_fwd_headwise")
+        return
     if n_split > 1:
         packed = cu_q is not None
         qs, ks, vs, os_ = (_packed_or_dense_strides(x, packed) for x in (q, k, v, out))
@@ -384,7 +406,7 @@ def scaled_dot_product_attention(Q, K, V, mask=None):
 
 
 def _varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, causal, softmax_scale, want_lse=False,
-            kv_splits=1, workspace=None):
+            kv_splits=1, workspace=None, head_scale=None, sinks=None):
     for n, t in (("q", q), ("k", k), ("v", v)):
         _require_gpu_bf16(n, t)
         if t.dim() != 3:
@@ -413,24 +435,27 @@ def _varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, cau
         n_split, workspace = (1, None) if want_lse else _split_args(
             kv_splits, workspace, B, Hq, D, max_seqlen_q, max_seqlen_k, Tq, causal, q.device)
         _prefill(q, k, v, out, cu_seqlens_q, cu_seqlens_k, None, B, Hq, Hkv, int(max_seqlen_q), int(max_seqlen_k),
-                 D, scale, _lib.MASK_CAUSAL if causal else _lib.MASK_NONE, lse, n_split, workspace, Tq)
+                 D, scale, _lib.MASK_CAUSAL if causal else _lib.MASK_NONE, lse, n_split, workspace, Tq, head_scale, sinks)
     return (out, lse) if want_lse else out
 
 
 def flash_attn_varlen_prefill(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, *,
-                              causal=True, softmax_scale=None, kv_splits=None, workspace=None):
+                              causal=True, softmax_scale=None, kv_splits=None, workspace=None, head_scale=None, sinks=None):
     """Packed ("varlen") prefill.  q (Tq,Hq,D); k, v (Tk,Hkv,D) bf16; cu_seqlens int32 (B+1,), cu[0]=0.
 
     Sequence b owns rows [cu[b], cu[b+1]).  Returns (Tq,Hq,D) bf16.  Differentiable like flash_attn_prefill;
-    kv_splits / workspace as there.
+    kv_splits / workspace as there.  head_scale, sinks (fp32 (Hq,), optional, forward only): a non-negative factor
+    on every head's scores, and a score without key or value that joins the head's softmax denominator.
     """
     q, k, v, out_dtype = _to_bf16(q, k, v)
     if _needs_grad(q, k, v):
+        if head_scale is not None or sinks is not None:
+            raise ValueError("per-head score factors and sinks are forward-only")
         out = _VarlenPrefillFn.apply(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, bool(causal),
                                      softmax_scale)
     else:
         out = _varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, causal, softmax_scale,
-                      kv_splits=kv_splits, workspace=workspace)
+                      kv_splits=kv_splits, workspace=workspace, head_scale=head_scale, sinks=sinks)
     return out if out.dtype == out_dtype else out.to(out_dtype)
 
 
@@ -448,7 +473,7 @@ def paged_decode_workspace(batch, n_q_heads, head_dim, max_context, device):
 
 def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, softmax_scale=None,
                            k_scale=None, v_scale=None, max_context=None, workspace=None, out=None,
-                           static_scratch=False):
+                           static_scratch=False, head_scale=None, sinks=None):
     """Paged-KV decode attention, one query token per sequence.
 
     q (B,Hq,D) bf16; k_cache, v_cache (num_blocks,Hkv,16,D) bf16, or fp8-e4m3
@@ -459,6 +484,9 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
     static_scratch=True (needs `out`) goes through mi355_paged_decode_fwd_static: nothing is allocated, the
     split-K partials live in the library's own device array (16 MiB per GPU; larger problems are rejected; calls
     that overlap in time on one GPU must be serialised by the caller).
+    head_scale, sinks (fp32 (Hq,), optional): a factor on every head's scores, and a score without key or value that
+    joins the head's softmax denominator.  q may have strided rows (heads contiguous, row stride a multiple of 8, e.g.
+    a view of a merged projection) unless static_scratch is set.
     """
     _require_gpu_bf16("q", q)
     if q.dim() != 3:
@@ -480,7 +508,11 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
     nb, Hkv, bs, Dc = k_cache.shape
     if bs != _BLOCK or Dc != D:
         raise ValueError(f"cache must be (num_blocks, kv_heads, {_BLOCK}, {D}), got {tuple(k_cache.shape)}")
-    for n, c in (("q", q), ("k_cache", k_cache), ("v_cache", v_cache)):
+    headwise = head_scale is not None or sinks is not None or not q.is_contiguous()
+    if headwise and (static_scratch or q.stride(2) != 1 or q.stride(1) != D or q.stride(0) % 8 or q.data_ptr() % 16):
+        raise ValueError("q must have contiguous heads, 16-byte aligned, with a row stride that is a multiple of 8 "
+                         "(and be contiguous, without per-head terms, for static_scratch)")
+    for n, c in (("k_cache", k_cache), ("v_cache", v_cache)):
         if not c.is_contiguous() or not c.is_cuda:
             raise ValueError(f"{n} must be a contiguous GPU tensor")
     if block_tables.dtype != torch.int32 or context_lens.dtype != torch.int32:
@@ -501,7 +533,7 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
     if out is None:
         if static_scratch:
             raise ValueError("static_scratch=True allocates nothing: pass `out`")
-        out = torch.empty_like(q)
+        out = torch.empty(B, Hq, D, dtype=q.dtype, device=q.device)
     if B == 0:
         return out
     lib = _lib.load()
@@ -519,6 +551,18 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
         return out
     if workspace is None:
         workspace = paged_decode_workspace(B, Hq, D, max_context, q.device)
+    if headwise:
+        hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
+        with _on(q, k_cache, v_cache, out, block_tables, context_lens, k_scale, v_scale, workspace) as stream:
+            rc = lib.mi355_paged_decode_fwd_headwise(
+                q.data_ptr(), q.stride(0) if B > 1 else Hq * D, k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(),
+                block_tables.data_ptr(), block_tables.stride(0), context_lens.data_ptr(),
+                k_scale.data_ptr() if fp8 else None, v_scale.data_ptr() if fp8 else None, hs, sk,
+                workspace.data_ptr(), workspace.numel() * workspace.element_size(),
+                B, Hq, Hkv, D, bs, k_cache.shape[0], int(max_context), float(scale),
+                _lib.MI355_FP8_E4M3 if fp8 else _lib.MI355_BF16, stream)
+        _lib.check(rc, "mi355_paged_decode_fwd_headwise")
+        return out
     with _on(q, k_cache, v_cache, out, block_tables, context_lens, k_scale, v_scale, workspace) as stream:
         rc = lib.mi355_paged_decode_fwd(
             q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(),
@@ -533,7 +577,7 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
 
 def flash_attn_paged_prefill(q, k_cache, v_cache, cu_seqlens_q, block_tables, context_lens, max_seqlen_q, *,
                              softmax_scale=None, out=None, max_context=None, kv_splits=None, workspace=None,
-                             k_scale=None, v_scale=None, total_context=None, cu_seqlens_k=None):
+                             k_scale=None, v_scale=None, total_context=None, cu_seqlens_k=None, head_scale=None, sinks=None):
     """Causal prefill of a chunk of new tokens over context that already sits in a paged cache.
 
     q (T,Hq,D) bf16, packed, contiguous heads (token stride free): sequence b owns rows
@@ -550,13 +594,14 @@ def flash_attn_paged_prefill(q, k_cache, v_cache, cu_seqlens_q, block_tables, co
     total_context (host int, optional): an upper bound on sum(context_lens) that sizes those rows (default
     batch * max_context); cu_seqlens_k (int32 (B+1,), optional): the running sum of the context lengths, if the
     caller has it on the device already (else it is computed here, a few small launches per call).
+    head_scale, sinks: per-head terms as in flash_attn_varlen_prefill.
     The mathematics is that of llm-core/llm_core/model.py:308-325 with the mask of :384; the reference
     itself would re-run the whole prefix (model.py:218)."""
     _require_gpu_bf16("q", q)
     if k_scale is not None or v_scale is not None:
         return _paged_prefill_fp8(q, k_cache, v_cache, k_scale, v_scale, cu_seqlens_q, block_tables, context_lens,
                                   max_seqlen_q, softmax_scale, out, max_context, kv_splits, workspace, total_context,
-                                  cu_seqlens_k)
+                                  cu_seqlens_k, head_scale, sinks)
     if q.dim() != 3 or q.stride(2) != 1 or q.stride(1) != q.shape[2]:
         raise ValueError("q must be (tokens, heads, d_head) with contiguous heads")
     T, Hq, D = q.shape
@@ -600,15 +645,16 @@ def flash_attn_paged_prefill(q, k_cache, v_cache, cu_seqlens_q, block_tables, co
         max_context = block_tables.shape[1] * _BLOCK
     n_split, workspace = _split_args(kv_splits, workspace, B, Hq, D, int(max_seqlen_q), int(max_context), T, True,
                                      q.device)
+    hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
     with _on(q, k_cache, v_cache, out, cu_seqlens_q, block_tables, context_lens, workspace) as stream:
-        rc = _lib.load().mi355_prefill_paged_fwd(
+        rc = _lib.load().mi355_prefill_paged_fwd_headwise(
             q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), q.stride(0), out.stride(0),
             cu_seqlens_q.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), block_tables.shape[1],
-            context_lens.data_ptr(),
+            context_lens.data_ptr(), hs, sk,
             B, Hq, Hkv, int(max_seqlen_q), D, _BLOCK, k_cache.shape[0], float(scale), _lib.MI355_BF16,
             n_split, T, None if workspace is None else workspace.data_ptr(),
             0 if workspace is None else workspace.numel() * workspace.element_size(), stream)
-    _lib.check(rc, "mi355_prefill_paged_fwd")
+    _lib.check(rc, "mi355_prefill_paged_fwd_headwise")
     return out
 
 
@@ -674,7 +720,8 @@ def gather_kv_fp8(k_cache, v_cache, k_scale, v_scale, block_tables, context_lens
 
 
 def _paged_prefill_fp8(q, k_cache, v_cache, k_scale, v_scale, cu_seqlens_q, block_tables, context_lens, max_seqlen_q,
-                       softmax_scale, out, max_context, kv_splits, workspace, total_context, cu_seqlens_k=None):
+                       softmax_scale, out, max_context, kv_splits, workspace, total_context, cu_seqlens_k=None,
+                       head_scale=None, sinks=None):
     """flash_attn_paged_prefill over an fp8 cache: gather + dequantise, then the packed prefill with more keys than
     queries per sequence (bottom-right aligned causal mask)."""
     if q.dim() != 3:
@@ -686,11 +733,92 @@ def _paged_prefill_fp8(q, k_cache, v_cache, k_scale, v_scale, cu_seqlens_q, bloc
     k_lin, v_lin, cu_k = gather_kv_fp8(k_cache, v_cache, k_scale, v_scale, block_tables, context_lens,
                                        max_context=max_context, total_context=total_context, cu_seqlens_k=cu_seqlens_k)
     res = flash_attn_varlen_prefill(q, k_lin, v_lin, cu_seqlens_q, cu_k, max_seqlen_q, max_context, causal=True,
-                                    softmax_scale=softmax_scale, kv_splits=kv_splits, workspace=workspace)
+                                    softmax_scale=softmax_scale, kv_splits=kv_splits, workspace=workspace,
+                                    head_scale=head_scale, sinks=sinks)
     if out is not None:
         out.copy_(res)
         return out
     return res
+
+
+_DTYPE_CODE = {torch.bfloat16: _lib.MI355_BF16, torch.float32: _lib.MI355_FP32}
+
+
+def _dtype_code(name, t):
+    if t.dtype not in _DTYPE_CODE:
+        raise TypeError(f"{name} must be bfloat16 or float32 (got {t.dtype})")
+    return _DTYPE_CODE[t.dtype]
+
+
+def paged_attention_any(q, k_cache, v_cache, block_tables, context_lens, *, cu_seqlens_q=None, softmax_scale=None,
+                        head_scale=None, sinks=None):
+    """Causal attention through the block tables for any head size, in bf16 or fp32 (the general path: no MFMA).
+
+    q (T,Hq,Dk), heads contiguous; k_cache (num_blocks,Hkv,16,Dk), v_cache (num_blocks,Hkv,16,Dv) of q's dtype, Dk and Dv
+    multiples of 8 up to 512; block_tables (B,max_blocks), context_lens (B,) int32.  With cu_seqlens_q (int32 (B+1,))
+    the rows are packed chunks whose keys are already cached, as in flash_attn_paged_prefill; without it sequence b owns
+    row b, as in paged_attention_decode.  head_scale, sinks as there.  Returns (T,Hq,Dv)."""
+    code = _dtype_code("q", q)
+    if q.dim() != 3 or (q.numel() and (q.stride(2) != 1 or q.stride(1) != q.shape[2])):
+        raise ValueError("q must be (tokens, heads, d_head) with contiguous heads")
+    T, Hq, Dk = q.shape
+    for n, c in (("k_cache", k_cache), ("v_cache", v_cache)):
+        if c.dtype != q.dtype or c.dim() != 4 or c.shape[2] != _BLOCK or not c.is_contiguous():
+            raise ValueError(f"{n} must be a contiguous (num_blocks, kv_heads, {_BLOCK}, d_head) tensor of q's dtype")
+    nb, Hkv, _, Dkc = k_cache.shape
+    Dv = v_cache.shape[3]
+    if Dkc != Dk or v_cache.shape[:2] != (nb, Hkv) or Hq % Hkv:
+        raise ValueError(f"shape mismatch: q {tuple(q.shape)} k_cache {tuple(k_cache.shape)} v_cache {tuple(v_cache.shape)}")
+    B = context_lens.numel()
+    for n, t in (("cu_seqlens_q", cu_seqlens_q), ("block_tables", block_tables), ("context_lens", context_lens)):
+        if t is not None and t.dtype != torch.int32:
+            raise TypeError(f"{n} must be int32")
+    if block_tables.dim() != 2 or block_tables.shape[0] != B or block_tables.stride(1) != 1:
+        raise ValueError("block_tables must be (batch, max_blocks) with unit column stride")
+    if context_lens.shape != (B,) or not context_lens.is_contiguous():
+        raise ValueError("context_lens must be a contiguous (batch,) tensor")
+    if cu_seqlens_q is None:
+        if T != B:
+            raise ValueError("one query row per sequence expected without cu_seqlens_q")
+    elif cu_seqlens_q.shape != (B + 1,) or not cu_seqlens_q.is_contiguous():
+        raise ValueError("cu_seqlens_q must be a contiguous (batch + 1,) tensor")
+    out = torch.empty(T, Hq, Dv, dtype=q.dtype, device=q.device)
+    if T == 0:
+        return out
+    scale = 1.0 / math.sqrt(Dk) if softmax_scale is None else softmax_scale
+    hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
+    with _on(q, k_cache, v_cache, out, block_tables, context_lens, cu_seqlens_q) as stream:
+        rc = _lib.load().mi355_paged_attn_any_fwd(
+            q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), q.stride(0) if T > 1 else Hq * Dk, Hq * Dv, T,
+            None if cu_seqlens_q is None else cu_seqlens_q.data_ptr(), block_tables.data_ptr(),
+            max(block_tables.stride(0), block_tables.shape[1]), block_tables.shape[1], context_lens.data_ptr(), hs, sk,
+            B, Hq, Hkv, Dk, Dv, _BLOCK, nb, float(scale), code, stream)
+    _lib.check(rc, "mi355_paged_attn_any_fwd")
+    return out
+
+
+def kv_cache_write(k, v, k_cache, v_cache, slot_mapping):
+    """Scatter of unrotated keys and values (k (T,Hkv,Dk), v (T,Hkv,Dv), heads contiguous, bf16 or fp32 like the caches)
+    into cache slots slot_mapping (T,) int64 = block*16 + offset (negative: skip)."""
+    code = _dtype_code("k", k)
+    for n, t, c in (("k", k, k_cache), ("v", v, v_cache)):
+        if t.dim() != 3 or t.stride(2) != 1 or t.stride(1) != t.shape[2]:
+            raise ValueError(f"{n} must be (tokens, heads, d_head) with contiguous heads")
+        if t.dtype != k.dtype or t.shape[:2] != k.shape[:2]:
+            raise ValueError("k and v must agree in dtype, tokens and heads")
+        if c.dtype != t.dtype or c.dim() != 4 or c.shape[1:] != (t.shape[1], _BLOCK, t.shape[2]) or not c.is_contiguous() \
+                or c.shape[0] != k_cache.shape[0]:
+            raise ValueError(f"{n}_cache must be a contiguous (num_blocks, {t.shape[1]}, {_BLOCK}, {t.shape[2]}) tensor of {n}'s dtype")
+    T, Hkv, Dk = k.shape
+    if slot_mapping.dtype != torch.int64 or slot_mapping.shape != (T,) or not slot_mapping.is_contiguous():
+        raise TypeError("slot_mapping must be a contiguous int64 (tokens,) tensor")
+    if T == 0:
+        return
+    with _on(k, v, k_cache, v_cache, slot_mapping) as stream:
+        rc = _lib.load().mi355_kv_cache_write(k.data_ptr(), v.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
+                                              slot_mapping.data_ptr(), k_cache.shape[0], T, Hkv, Dk, v.shape[2],
+                                              k.stride(0), v.stride(0), code, stream)
+    _lib.check(rc, "mi355_kv_cache_write")
 
 
 def build_rope_cache(context_length, d, theta=10000.0, device="cuda"):
@@ -911,6 +1039,93 @@ def rms_norm(x, weight, eps: float = 1e-5, *, residual=None, return_sum: bool = 
         _lib.check(rc, "mi355_rms_norm_fwd")
     extra = [t for t in (h, rstd) if t is not None]
     return (y, *extra) if extra else y
+
+
+def _matrix(name, t, dtype, shape=None):
+    if t.dtype != dtype or t.dim() != 2 or (t.stride(1) != 1 and t.shape[1] > 1) or (shape is not None and tuple(t.shape) != shape):
+        raise ValueError(f"{name} must be a {dtype} matrix with unit column stride" + (f" of shape {shape}" if shape else ""))
+    return t
+
+
+def _vector(name, t, n):
+    if t is not None and (t.dtype != torch.float32 or t.shape != (n,) or not t.is_contiguous()):
+        raise ValueError(f"{name} must be a contiguous float32 ({n},) tensor")
+    return t
+
+
+def dyt_residual(resid, sub=None, *, sub_bias=None, gate=None, gate_bias=None, post=None, norm=None, out_dtype=torch.bfloat16,
+                 keep=True):
+    """End of a sublayer with Dynamic Tanh norms and a gated residual, and the norm of the result, in one launch:
+
+        x = resid + post((sub + sub_bias) * sigmoid(gate + gate_bias)),   y = norm(x),   norm(z) = tanh(alpha z) w + b
+
+    resid (T,d) fp32, updated in place to x (keep=False: left alone); sub and gate (T,d) bf16 or fp32, rows may be strided
+    views; post and norm: (alpha float, w, b) with fp32 vectors, or None; sub_bias, gate_bias: fp32 vectors or None.
+    Without `sub` it is a plain norm of resid.  Returns y in out_dtype (which is sub's dtype when there is a sub), or None
+    when `norm` is None."""
+    _matrix("resid", resid, torch.float32)
+    if not resid.is_contiguous():
+        raise ValueError("resid must be contiguous")
+    T, d = resid.shape
+    dt = out_dtype if sub is None else sub.dtype
+    if dt not in _DTYPE_CODE or (norm is not None and out_dtype != dt):
+        raise TypeError("sub and the result must both be bfloat16 or both float32")
+    if sub is None and (gate is not None or post is not None or sub_bias is not None):
+        raise ValueError("gate, post norm and bias need a sublayer result")
+    for n, t in (("sub", sub), ("gate", gate)):
+        if t is not None:
+            _matrix(n, t, dt, (T, d))
+    pa, pw, pb = (0.0, None, None) if post is None else post
+    na, nw, nb = (0.0, None, None) if norm is None else norm
+    vecs = [_vector(n, t, d) for n, t in (("sub_bias", sub_bias), ("gate_bias", gate_bias), ("post weight", pw), ("post bias", pb),
+                                          ("norm weight", nw), ("norm bias", nb))]
+    y = None if norm is None else torch.empty(T, d, dtype=dt, device=resid.device)
+    if T == 0 or (y is None and (not keep or sub is None)):
+        return y
+    ptr = [None if t is None else t.data_ptr() for t in vecs]
+    with _on(resid, sub, gate, *vecs) as stream:
+        rc = _lib.load().mi355_dyt_residual_fwd(
+            None if sub is None else sub.data_ptr(), ptr[0], None if gate is None else gate.data_ptr(), ptr[1], float(pa), ptr[2],
+            ptr[3], resid.data_ptr(), resid.data_ptr() if keep and sub is not None else None, float(na), ptr[4], ptr[5],
+            None if y is None else y.data_ptr(), T, d, 0 if sub is None else sub.stride(0), 0 if gate is None else gate.stride(0), d,
+            _DTYPE_CODE[dt], stream)
+    _lib.check(rc, "mi355_dyt_residual_fwd")
+    return y
+
+
+def polynorm(z, coeffs, eps: float):
+    """PolyNorm activation over the last dimension of a matrix (rows may be strided): a N(z) + b N(z^2) + c N(z^3) + e with
+    N(v) = v / sqrt(mean(v^2) + eps); coeffs = (a, b, c, e) Python floats; bf16 or fp32 in and out, fp32 math."""
+    code = _dtype_code("z", z)
+    _matrix("z", z, z.dtype)
+    T, d = z.shape
+    out = torch.empty(T, d, dtype=z.dtype, device=z.device)
+    if T:
+        with _on(z) as stream:
+            rc = _lib.load().mi355_polynorm_fwd(z.data_ptr(), out.data_ptr(), T, d, z.stride(0), d, _lib.floats4(coeffs), float(eps),
+                                                code, stream)
+        _lib.check(rc, "mi355_polynorm_fwd")
+    return out
+
+
+def embed_pos(embed, pos, tokens, positions):
+    """embed[tokens] + pos[positions] as an fp32 matrix: embed (V,d) and pos (P,d) of one dtype (bf16 or fp32), tokens (T,)
+    int64, positions (T,) int32."""
+    code = _dtype_code("embed", embed)
+    for n, t in (("embed", embed), ("pos", pos)):
+        if t.dim() != 2 or not t.is_contiguous() or t.dtype != embed.dtype or t.shape[1] != embed.shape[1] or t.shape[0] < 1:
+            raise ValueError(f"{n} must be a contiguous matrix; embed and pos agree in dtype and width")
+    T = tokens.numel()
+    if tokens.dtype != torch.int64 or positions.dtype != torch.int32 or tokens.shape != (T,) or positions.shape != (T,) \
+            or not tokens.is_contiguous() or not positions.is_contiguous():
+        raise TypeError("tokens (int64) and positions (int32) must be contiguous (tokens,) tensors")
+    out = torch.empty(T, embed.shape[1], dtype=torch.float32, device=embed.device)
+    if T:
+        with _on(embed, pos, tokens, positions) as stream:
+            rc = _lib.load().mi355_embed_pos_fwd(embed.data_ptr(), pos.data_ptr(), tokens.data_ptr(), positions.data_ptr(),
+                                                 out.data_ptr(), T, embed.shape[1], embed.shape[0], pos.shape[0], code, stream)
+        _lib.check(rc, "mi355_embed_pos_fwd")
+    return out
 
 
 def silu_mul(gate, up):
