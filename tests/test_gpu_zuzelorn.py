@@ -1,0 +1,557 @@
+"""GPU parity of the Zuzelorn model and of the operators that it brought, against the plain oracle.
+
+Tolerances.  Operators: fp32 results within 1e-5 relative to the result's scale; bf16 results within one bf16 ulp of the
+oracle on the same bf16 inputs (elementwise operators), 2e-2 + 1e-2 |ref| (attention, as for the other attention tests).
+Model logits: root mean square over the vocabulary of the difference, over that of the reference: 2e-5 in fp32 (observed
+below 1e-6), 2e-2 in bf16 (observed below 9e-3: weights exact, activations bf16).
+"""
+import json
+import math
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+from oracle import zuzelorn_oracle as zo
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+DTYPES = [torch.bfloat16, torch.float32]
+
+
+@pytest.fixture(scope="module")
+def ops():
+    import mi355_attn
+    mi355_attn.load()
+    return mi355_attn
+
+
+def gen(seed):
+    return torch.Generator().manual_seed(seed)
+
+
+def rnd(*shape, seed, std=1.0, dtype=torch.float32):
+    return (torch.randn(*shape, generator=gen(seed)) * std).to(dtype)
+
+
+def close(got, ref, dtype, ulps=1.0):
+    got = got.float().cpu()
+    if dtype == torch.float32:
+        torch.testing.assert_close(got, ref, atol=1e-5 * float(ref.abs().max().clamp_min(1.0)), rtol=1e-5)
+    else:
+        torch.testing.assert_close(got, ref, atol=2e-3, rtol=ulps * 2.0 ** -7)
+
+
+# ---- elementwise operators ------------------------------------------------------------------------
+def dyt_case(T, d, dtype, seed):
+    v = lambda k, std=0.5: rnd(d, seed=seed + k, std=std)
+    wide = rnd(T, d + 3 * 8 + d, seed=seed, dtype=dtype)             # sub and gate as two views of one wide product
+    return dict(resid=rnd(T, d, seed=seed + 1, std=2.0), sub=wide[:, :d], gate=wide[:, d + 24 - (d % 8):][:, :d], sub_bias=v(2),
+                gate_bias=v(3), post=(0.7, 1 + v(4), v(5)), norm=(1.3, 1 + v(6), v(7)))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,d", [(1, 8), (5, 72), (33, 100), (64, 1024), (4099, 2056)])
+def test_dyt_residual_matches_oracle(ops, T, d, dtype):
+    print(f"case: dyt_residual {T}x{d} {dtype}", flush=True)
+    c = dyt_case(T, d, dtype, seed=d)
+    cu = lambda t: None if t is None else tuple(cu(e) if torch.is_tensor(e) else e for e in t) if isinstance(t, tuple) else t.cuda()
+    wide = torch.cat((c["sub"], c["gate"]), 1).cuda()
+    sub, gate = wide[:, :d], wide[:, d:]
+    for parts in (("sub_bias", "gate", "gate_bias", "post", "norm"), ("gate", "post", "norm"), ("post",), ("norm",), ("sub_bias", "norm")):
+        has = lambda n: c[n] if n in parts else None
+        s = c["sub"].float() + (c["sub_bias"] if has("sub_bias") is not None else 0)
+        if "gate" in parts:
+            s = s / (1 + torch.exp(-(c["gate"].float() + (c["gate_bias"] if "gate_bias" in parts else 0))))
+        x = c["resid"] + (zo.dynamic_tanh(s, *c["post"]) if "post" in parts else s)
+        r = c["resid"].cuda()
+        y = ops.dyt_residual(r, sub, sub_bias=cu(has("sub_bias")), gate=gate if "gate" in parts else None, gate_bias=cu(has("gate_bias")),
+                             post=cu(has("post")), norm=cu(has("norm")), out_dtype=dtype)
+        torch.cuda.synchronize()
+        close(r, x, torch.float32)
+        if "norm" in parts:
+            assert y.dtype == dtype
+            close(y, zo.dynamic_tanh(x, *c["norm"]), dtype)
+        else:
+            assert y is None
+    r = c["resid"].cuda()                                             # a plain norm leaves the residual alone
+    y = ops.dyt_residual(r, norm=cu(c["norm"]), out_dtype=dtype)
+    assert torch.equal(r.cpu(), c["resid"])
+    close(y, zo.dynamic_tanh(c["resid"], *c["norm"]), dtype)
+
+
+def test_dyt_residual_saturates_cleanly(ops):
+    print("case: dyt_residual saturation", flush=True)
+    big = torch.tensor([[-1e30, -200.0, -1e-4, 0.0, 1e-4, 200.0, 1e30, 3e38]])
+    for dtype in DTYPES:
+        y = ops.dyt_residual(big.cuda(), norm=(1.0, None, None), out_dtype=dtype).float().cpu()
+        close(y, torch.tanh(big), dtype)
+        s = big.to(dtype).cuda()
+        r = torch.zeros(1, 8).cuda()
+        ops.dyt_residual(r, torch.ones(1, 8, dtype=dtype).cuda(), gate=s)
+        close(r, torch.sigmoid(big.to(dtype).float()), torch.float32)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("d", [8, 56, 512, 600, 1024, 2048, 3000, 8192, 16384, 75, 20000])
+def test_polynorm_matches_oracle(ops, d, dtype):
+    print(f"case: polynorm {d} {dtype}", flush=True)
+    z = rnd(7, d + 40, seed=d, std=1.7, dtype=dtype)
+    z[3] *= 1e-3                                                       # a row where eps matters
+    cf = (0.8, -0.4, 0.3, 0.15)
+    got = ops.polynorm(z.cuda()[:, :d], cf, 1e-5)
+    torch.cuda.synchronize()
+    close(got, zo.polynorm(z[:, :d].float(), cf, 1e-5), dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_embed_pos_matches_oracle(ops, dtype):
+    print(f"case: embed_pos {dtype}", flush=True)
+    e, p = rnd(50, 37, seed=1, dtype=dtype), rnd(20, 37, seed=2, dtype=dtype)
+    tok, pos = torch.tensor([0, 49, 7, 7, 1]), torch.tensor([0, 19, 3, 4, 1], dtype=torch.int32)
+    got = ops.embed_pos(e.cuda(), p.cuda(), tok.cuda(), pos.cuda())
+    assert got.dtype == torch.float32 and torch.equal(got.cpu(), e[tok].float() + p[pos.long()].float())
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("G,dk,dv", [(1, 8, 8), (3, 24, 40), (2, 128, 128)])
+def test_kv_cache_write_is_exact_and_skips_slots_outside(ops, G, dk, dv, dtype):
+    print(f"case: kv_cache_write {G} {dk} {dv} {dtype}", flush=True)
+    T, nb = 19, 4
+    wide = rnd(T, G * (dk + dv) + 8, seed=3, dtype=dtype).cuda()
+    k, v = wide[:, :G * dk].view(T, G, dk), wide[:, G * dk:G * (dk + dv)].view(T, G, dv)
+    slots = torch.randperm(nb * 16, generator=gen(4))[:T]
+    slots[2], slots[5] = -1, nb * 16
+    kc, vc = torch.full((nb, G, 16, dk), 9.0, dtype=dtype).cuda(), torch.full((nb, G, 16, dv), 9.0, dtype=dtype).cuda()
+    rk, rv = kc.cpu(), vc.cpu()
+    ops.kv_cache_write(k, v, kc, vc, slots.cuda())
+    for t, s in enumerate(slots.tolist()):
+        if 0 <= s < nb * 16:
+            rk[s // 16, :, s % 16], rv[s // 16, :, s % 16] = k[t].cpu(), v[t].cpu()
+    assert torch.equal(kc.cpu(), rk) and torch.equal(vc.cpu(), rv)
+
+
+# ---- attention with per-head factors and sinks --------------------------------------------------------
+def planted(n, H, G, dk, dv, far, seed, dtype, n_q=None):
+    """Queries (the last n_q positions of n), keys, values, factors and sinks in which key `far` of every kv head stands out:
+    its score exceeds the others by about 6, near the sinks' size, so a wrong, missing or doubled key or sink shows."""
+    n_q = n if n_q is None else n_q
+    q, k, v = rnd(n_q, H, dk, seed=seed, std=0.5), rnd(n, G, dk, seed=seed + 1, std=0.5), rnd(n, G, dv, seed=seed + 2)
+    q[..., 0] = 2.0
+    k[..., 0] = 0.0
+    scale = 0.9 / math.sqrt(dk)
+    temp = 0.6 + torch.rand(H, generator=gen(seed + 3))
+    k[far, :, 0] = 7.0 / (2.0 * scale)
+    sink = 4.0 + torch.rand(H, generator=gen(seed + 4)) * 3
+    return q.to(dtype), k.to(dtype), v.to(dtype), scale, temp, sink
+
+
+def page(k, v, seed, extra=3):
+    """Keys and values of one sequence in a pool with a shuffled table; unused rows hold large numbers."""
+    n, G = k.shape[:2]
+    nb = (n + 15) // 16
+    perm = torch.randperm(nb + extra, generator=gen(seed))[:nb]
+    kc = torch.full((nb + extra, G, 16, k.shape[2]), 30.0, dtype=k.dtype)
+    vc = torch.full((nb + extra, G, 16, v.shape[2]), 30.0, dtype=v.dtype)
+    for t in range(n):
+        kc[perm[t // 16], :, t % 16], vc[perm[t // 16], :, t % 16] = k[t], v[t]
+    return kc.cuda(), vc.cuda(), perm.to(torch.int32)
+
+
+def attn_close(got, ref, dtype):
+    err = (got.float().cpu() - ref).abs()
+    bound = (2e-2 + 1e-2 * ref.abs()) if dtype == torch.bfloat16 else torch.full_like(ref, 3e-5)
+    assert bool((err <= bound).all()), float((err - bound).max())
+
+
+def table(rows):
+    width = max(len(r) for r in rows)
+    return torch.stack([torch.nn.functional.pad(r, (0, width - len(r))) for r in rows]).to(torch.int32).cuda()
+
+
+@pytest.mark.parametrize("D,H,G", [(32, 4, 4), (64, 6, 2), (128, 8, 2), (128, 20, 1)])
+@pytest.mark.parametrize("n", [1, 15, 16, 17, 250, 1024, 1025, 5000])
+def test_decode_with_factors_and_sinks(ops, D, H, G, n):
+    print(f"case: decode headwise D={D} H={H}/{G} ctx={n}", flush=True)
+    for far in sorted({0, min(15, n - 1), min(16, n - 1), n // 2, n - 1}):
+        q, k, v, scale, temp, sink = planted(n, H, G, D, D, far, 11 * n + far, torch.bfloat16, n_q=1)
+        kc, vc, perm = page(k, v, seed=n)
+        wide = torch.cat((q.reshape(1, -1), torch.ones(1, 8, dtype=q.dtype)), 1).repeat(3, 1).cuda()      # strided query rows
+        cl = torch.tensor([n, 1, n], dtype=torch.int32).cuda()
+        out = ops.paged_attention_decode(wide[:, :H * D].view(3, H, D), kc, vc, table([perm] * 3), cl, softmax_scale=scale,
+                                         head_scale=temp.cuda(), sinks=sink.cuda())
+        ref = zo.sink_attention(q.float(), k.float(), v.float(), scale, temp, sink, first=n - 1)[0]
+        attn_close(out[0], ref, torch.bfloat16)
+        assert torch.equal(out[0], out[2])
+        attn_close(out[1], zo.sink_attention(q.float(), k[:1].float(), v[:1].float(), scale, temp, sink)[0], torch.bfloat16)
+
+
+def test_decode_sink_alone_or_factor_alone_and_extreme_sinks(ops):
+    print("case: decode sink/factor alone", flush=True)
+    n, H, G, D = 300, 4, 2, 64
+    q, k, v, scale, temp, sink = planted(n, H, G, D, D, 77, 5, torch.bfloat16, n_q=1)
+    kc, vc, perm = page(k, v, seed=1)
+    run = lambda **kw: ops.paged_attention_decode(q.cuda(), kc, vc, table([perm]), torch.tensor([n], dtype=torch.int32).cuda(),
+                                                  softmax_scale=scale, **kw)[0]
+    ref = lambda t, s: zo.sink_attention(q.float(), k.float(), v.float(), scale, t, s, first=n - 1)[0]
+    attn_close(run(sinks=sink.cuda()), ref(None, sink), torch.bfloat16)
+    attn_close(run(head_scale=temp.cuda()), ref(temp, None), torch.bfloat16)
+    ext = torch.tensor([-200.0, 200.0, 40.0, -40.0])
+    attn_close(run(sinks=ext.cuda()), ref(None, ext), torch.bfloat16)
+
+
+@pytest.mark.parametrize("D,H,G", [(32, 4, 2), (64, 3, 1), (64, 4, 4), (128, 8, 2), (128, 3, 3)])
+@pytest.mark.parametrize("splits", [1, 3])
+def test_prefill_with_factors_and_sinks(ops, D, H, G, splits):
+    """Packed new prompts, and chunks (down to two rows) over cached keys through the block tables, in one launch each."""
+    print(f"case: prefill headwise D={D} H={H}/{G} splits={splits}", flush=True)
+    cases = [planted(n, H, G, D, D, far, 100 + n + far, torch.bfloat16) for n, far in ((1, 0), (2, 1), (70, 15), (130, 64), (300, 0))]
+    temp, sink, scale = cases[0][4], cases[0][5], cases[0][3]
+    lens = [c[0].shape[0] for c in cases]
+    cu = torch.tensor([0] + lens).cumsum(0).to(torch.int32).cuda()
+    cat = lambda i: torch.cat([c[i] for c in cases]).cuda()
+    out = ops.flash_attn_varlen_prefill(cat(0), cat(1), cat(2), cu, cu, max(lens), max(lens), softmax_scale=scale, kv_splits=splits,
+                                        head_scale=temp.cuda(), sinks=sink.cuda()).cpu()
+    refs = [zo.sink_attention(c[0].float(), c[1].float(), c[2].float(), scale, temp, sink) for c in cases]
+    attn_close(out, torch.cat(refs), torch.bfloat16)
+    # chunks: the last rows of each sequence over all of its keys
+    pools, tabs, qs, want, off = [], [], [], [], 0
+    chunk = [1, 2, 17, 2, 255]
+    for c, r, m in zip(cases, refs, chunk):
+        kc, vc, perm = page(c[1], c[2], seed=m)
+        pools.append((kc, vc))
+        tabs.append(perm + off)
+        off += kc.shape[0]
+        qs.append(c[0][-m:])
+        want.append(r[-m:])
+    cuq = torch.tensor([0] + chunk).cumsum(0).to(torch.int32).cuda()
+    out = ops.flash_attn_paged_prefill(torch.cat(qs).cuda(), torch.cat([a for a, _ in pools]), torch.cat([b for _, b in pools]), cuq,
+                                       table(tabs), torch.tensor(lens, dtype=torch.int32).cuda(), max(chunk), softmax_scale=scale,
+                                       kv_splits=splits, head_scale=temp.cuda(), sinks=sink.cuda())
+    attn_close(out, torch.cat(want), torch.bfloat16)
+
+
+@pytest.mark.parametrize("D", [64, 128])
+def test_prefill_scores_outside_the_preset_range(ops, D):
+    """Scores of several hundred: the kernels' second attempt, with references taken from the data, meets the sink too."""
+    print(f"case: prefill headwise, large scores D={D}", flush=True)
+    n, H, G = 150, 4, 1
+    q, k, v = (rnd(n, h, D, seed=30 + h + i, dtype=torch.bfloat16) for i, h in ((0, H), (1, G), (2, G)))
+    temp, sink = torch.tensor([6.0, 6.0, -0.0, 1e-30]), torch.tensor([20.0, 90.0, 1.0, -3.0])
+    cu = torch.tensor([0, n], dtype=torch.int32).cuda()
+    out = ops.flash_attn_varlen_prefill(q.cuda(), k.cuda(), v.cuda(), cu, cu, n, n, softmax_scale=1.0, head_scale=temp.abs().clamp_min(1e-30).cuda(),
+                                        sinks=sink.cuda(), kv_splits=1)
+    attn_close(out, zo.sink_attention(q.float(), k.float(), v.float(), 1.0, temp, sink), torch.bfloat16)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,dk,dv", [(4, 2, 24, 40), (3, 3, 8, 8), (6, 2, 136, 200), (2, 1, 512, 264), (1, 1, 64, 512)])
+def test_general_kernel_prefill_and_decode(ops, H, G, dk, dv, dtype):
+    print(f"case: paged_attention_any H={H}/{G} dk={dk} dv={dv} {dtype}", flush=True)
+    lens, chunk = [1, 2, 65, 64, 333], [1, 2, 65, 2, 70]
+    cases = [planted(n, H, G, dk, dv, far, 300 + n, dtype) for n, far in zip(lens, (0, 0, 16, 63, 250))]
+    scale, temp, sink = cases[0][3:]
+    temp[0] = -temp[0]                                                  # this kernel takes factors of either sign
+    refs = [zo.sink_attention(c[0].float(), c[1].float(), c[2].float(), scale, temp, sink) for c in cases]
+    kcs, vcs, tabs, off = [], [], [], 0
+    for c in cases:
+        kc, vc, perm = page(c[1], c[2], seed=c[0].shape[0])
+        kcs.append(kc), vcs.append(vc), tabs.append(perm + off)
+        off += kc.shape[0]
+    kc, vc, bt, cl = torch.cat(kcs), torch.cat(vcs), table(tabs), torch.tensor(lens, dtype=torch.int32).cuda()
+    kw = dict(softmax_scale=scale, head_scale=temp.cuda(), sinks=sink.cuda())
+    cuq = torch.tensor([0] + chunk).cumsum(0).to(torch.int32).cuda()
+    out = ops.paged_attention_any(torch.cat([c[0][-m:] for c, m in zip(cases, chunk)]).cuda(), kc, vc, bt, cl, cu_seqlens_q=cuq, **kw)
+    attn_close(out, torch.cat([r[-m:] for r, m in zip(refs, chunk)]), dtype)
+    wide = torch.cat([torch.cat((c[0][-1].reshape(1, -1), torch.ones(1, 8, dtype=dtype)), 1) for c in cases]).cuda()
+    out = ops.paged_attention_any(wide[:, :H * dk].view(len(lens), H, dk), kc, vc, bt, cl, **kw)
+    attn_close(out, torch.stack([r[-1] for r in refs]), dtype)
+
+
+# ---- the model -------------------------------------------------------------------------------------------
+def layer(ff, **m):
+    m.setdefault("vdim", m["dim"])
+    m.setdefault("scale", 1.3 / math.sqrt(m["dim"]))
+    return {"type": "attention", "mixer": m, "mlp": None if ff is None else {"kind": "dense", "ff": ff}}
+
+
+def cfg(layers, width, vocab, **kw):
+    c = dict(architecture="Zuzelorn", layers=layers, width=width, vocab=vocab, max_positions=700, logit_scale=0.8, norm={"eps": 1e-5})
+    c.update(kw)
+    return c
+
+
+CONFIGS = {
+    # value heads of another size, one source for two later layers with a layer of other heads between, a layer without feed-forward
+    "mixed": cfg([layer(104, heads=6, kv_heads=3, dim=24, vdim=40), layer(None, heads=6, kv_heads=3, dim=24, vdim=40, kv_from=0),
+                  layer(64, heads=2, kv_heads=1, dim=64), layer(88, heads=6, kv_heads=3, dim=24, vdim=40, kv_from=0)], 72, 131),
+    # sizes that are not multiples of anything, one head; logit scale and eps of their own
+    "odd": cfg([layer(75, heads=1, kv_heads=1, dim=20, vdim=12), layer(30, heads=3, kv_heads=1, dim=10),
+                layer(75, heads=3, kv_heads=1, dim=10, kv_from=1)], 100, 53, logit_scale=1.7, norm={"eps": 1e-3}),
+    # head size 128, four query heads per kv head: the 64-query prefill kernel
+    "wide": cfg([layer(256, heads=8, kv_heads=2, dim=128), layer(256, heads=4, kv_heads=2, dim=128, kv_from=0)], 128, 200),
+    # heads too large for the MFMA kernels beside one that fits
+    "large": cfg([layer(96, heads=2, kv_heads=1, dim=144, vdim=80), layer(96, heads=4, kv_heads=4, dim=32),
+                  layer(96, heads=2, kv_heads=1, dim=144, vdim=80, kv_from=0)], 64, 90),
+}
+LIMIT = {"float32": 2e-5, "bfloat16": 2e-2}
+
+
+def rel(got, ref):
+    d = got.float().cpu() - ref
+    d = d - d.mean(-1, keepdim=True)
+    r = ref - ref.mean(-1, keepdim=True)
+    return d.pow(2).mean(-1).sqrt() / r.pow(2).mean().sqrt()
+
+
+def check(got, ref, dtype, what):
+    e = rel(got, ref)
+    assert got.shape == ref.shape and got.dtype == torch.float32
+    assert bool((e <= LIMIT[dtype]).all()), f"{what}: first bad row {int((e > LIMIT[dtype]).nonzero()[0])}, worst {float(e.max()):.2e}"
+    return float(e.max())
+
+
+_cache = {}
+
+
+def oracle(name, seed, n):
+    """Parameters, tokens and oracle logits of a random sequence (computed once per (config, seed))."""
+    key = (name, seed)
+    if key not in _cache or _cache[key][1].numel() < n:
+        c = CONFIGS[name]
+        p = _cache[name] = _cache.get(name) or zo.random_params(c, len(name), sharpness=2.5)
+        toks = torch.randint(0, c["vocab"], (n,), generator=gen(seed))
+        _cache[key] = (p, toks, zo.forward(c, p, toks.tolist()))
+    p, toks, logits = _cache[key]
+    return p, toks[:n], logits[:n]
+
+
+def model(ops, name, dtype, **kw):
+    oracle(name, 0, 1)
+    kw.setdefault("max_batch", 8)
+    return ops.ZuzelornLM(CONFIGS[name], _cache[name], dtype=dtype, **kw)
+
+
+ALL = pytest.mark.parametrize("name", list(CONFIGS))
+BOTH = pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+
+
+@ALL
+@BOTH
+def test_whole_prompts(ops, name, dtype):
+    m = model(ops, name, dtype)
+    for seed, n in ((1, 1), (2, 2), (3, 17), (4, 190)):
+        p, toks, ref = oracle(name, seed, n)
+        e = check(m.forward(toks)[0], ref, dtype, f"{name} whole {n}")
+        print(f"case: {name} {dtype} whole {n}: {e:.1e}", flush=True)
+    assert m.engine.allocator.num_free == m.engine.allocator.num_blocks
+
+
+@ALL
+@BOTH
+def test_portions_of_any_size_and_single_tokens(ops, name, dtype):
+    p, toks, ref = oracle(name, 4, 190)
+    m = model(ops, name, dtype)
+    for cuts in ((2,), (1, 2), (16,), (17, 3, 1), (100, 5, 1, 1, 33), (189, 1)):
+        print(f"case: {name} {dtype} portions {cuts}", flush=True)
+        s, at, i, got = m.new_sequence(), 0, 0, []
+        while at < len(toks):
+            n = min(cuts[i % len(cuts)], len(toks) - at)
+            got.append(m.step([s], [toks[at:at + n]], rows=range(n)))
+            at, i = at + n, i + 1
+        m.free_sequence(s)
+        check(torch.cat(got), ref, dtype, f"{name} {cuts}")
+
+
+@ALL
+@BOTH
+def test_token_by_token_equals_the_prompt(ops, name, dtype):
+    print(f"case: {name} {dtype} decode from the first token, over blocks used before", flush=True)
+    p, toks, ref = oracle(name, 4, 190)
+    m = model(ops, name, dtype, num_blocks=13, max_batch=2)             # little more than one sequence needs
+    for trial in range(2):                                              # the second time on freed blocks in another order
+        s = m.new_sequence()
+        got = [m.prefill([s], [toks[:1]])]
+        got += [m.decode([s], [int(t)]) for t in toks[1:]]
+        m.free_sequence(s)
+        check(torch.cat(got), ref, dtype, f"{name} decode")
+        a, b = m.new_sequence(), m.new_sequence()
+        m.prefill([a, b], [toks[:40], toks[:90]])
+        m.free_sequence(b), m.free_sequence(a)
+
+
+@ALL
+@BOTH
+def test_unequal_requests_in_one_batch(ops, name, dtype):
+    """Prompts, portions and single tokens of unequal requests in the same steps, sequences that join and leave."""
+    print(f"case: {name} {dtype} mixed batches", flush=True)
+    m = model(ops, name, dtype, num_blocks=40)
+    seqs = {seed: oracle(name, seed, n) for seed, n in ((4, 190), (5, 64), (6, 31), (7, 2), (8, 47))}
+    sched = [{4: 100, 5: 1, 6: 16}, {4: 1, 5: 1, 6: 2}, {4: 1, 5: 30, 7: 1}, {6: 13, 7: 1, 4: 20}, {4: 1, 5: 1}, {8: 46, 4: 66},
+             {8: 1, 4: 1, 5: 31}]
+    sid, at, got = {}, {}, {s: [] for s in seqs}
+    for step in sched:
+        for s in step:
+            if s not in sid:
+                sid[s], at[s] = m.new_sequence(), 0
+        toks = [seqs[s][1][at[s]:at[s] + n] for s, n in step.items()]
+        logits = m.step([sid[s] for s in step], toks, rows=range(sum(len(t) for t in toks)))
+        for s, part in zip(step, torch.split(logits, [len(t) for t in toks])):
+            got[s].append(part)
+            at[s] += part.shape[0]
+            if at[s] == len(seqs[s][1]):
+                m.free_sequence(sid[s])
+    for s, (p, toks, ref) in seqs.items():
+        assert at[s] == len(toks)
+        check(torch.cat(got[s]), ref, dtype, f"{name} sequence {s}")
+    assert m.engine.allocator.num_free == 40
+
+
+@BOTH
+@pytest.mark.parametrize("name", ["mixed", "wide"])
+def test_long_decoding(ops, name, dtype):
+    print(f"case: {name} {dtype} long decoding", flush=True)
+    p, toks, ref = oracle(name, 9, 640)
+    m = model(ops, name, dtype, max_batch=2)
+    s = m.new_sequence()
+    got = [m.prefill([s], [toks[:301]])] + [m.decode([s], [int(t)]) for t in toks[301:]]
+    check(torch.cat(got), ref[300:], dtype, f"{name} long")
+    with pytest.raises(ValueError):
+        m.prefill([s], [toks[:61]])                                     # 700 positions and no more
+    with pytest.raises(ValueError):
+        m.decode([s], [CONFIGS[name]["vocab"]])                         # not a token
+
+
+def test_a_wrong_key_or_sink_would_show(ops):
+    """The random models are sharp enough for the comparisons above: mistakes planted in the oracle move the logits by far
+    more than the limits."""
+    print("case: sensitivity of the comparison", flush=True)
+    name = "mixed"
+    p, toks, ref = oracle(name, 3, 17)
+    for kind in ("sink", "temp", "kv_from", "alpha", "gate", "pos"):
+        c, q = json.loads(json.dumps(CONFIGS[name])), dict(p)
+        if kind == "sink":
+            q["l3.mix.sink"] = p["l3.mix.sink"] - 30
+        elif kind == "temp":
+            q["l2.mix.temp"] = torch.ones_like(p["l2.mix.temp"])
+        elif kind == "kv_from":
+            for n in ("k", "k.b", "v", "v.b"):
+                q[f"l3.mix.{n}"] = zo.random_params(dict(c, layers=c["layers"][:1]), 99)[f"l0.mix.{n}"]
+            del c["layers"][3]["mixer"]["kv_from"]
+        elif kind == "alpha":
+            q["l1.norm1b.alpha"] = p["l1.norm1b.alpha"] * 0.6
+        elif kind == "gate":
+            q["l2.rg2.b"] = p["l2.rg2.b"] + 30
+        else:
+            q["pos"] = p["pos"].roll(1, 0)
+        assert float(rel(zo.forward(c, q, toks.tolist()), ref).max()) > 3 * LIMIT["bfloat16"], kind
+
+
+# ---- generation through the framework's own entry points ----------------------------------------------------
+def greedy_oracle(name, prompt, n, margin):
+    """The oracle's greedy continuation, cut before the first step whose two best logits are closer than `margin`."""
+    ids, out = list(prompt), []
+    for _ in range(n):
+        row = zo.forward(CONFIGS[name], _cache[name], ids)[-1]
+        a, b = torch.topk(row, 2).values.tolist()
+        if a - b < margin:
+            break
+        out.append(int(row.argmax()))
+        ids.append(out[-1])
+    return out
+
+
+@pytest.mark.parametrize("name", ["mixed", "odd"])
+def test_greedy_generation(ops, name):
+    print(f"case: {name} greedy", flush=True)
+    m = model(ops, name, "float32")
+    prompts = [oracle(name, s, n)[1].tolist() for s, n in ((3, 17), (6, 31), (7, 2))]
+    want = [greedy_oracle(name, p, 12, 1e-3) for p in prompts]
+    assert sum(len(w) for w in want) >= 18
+    got = m.generate_batch(prompts, 12, temperature=0)
+    for p, w, g in zip(prompts, want, got):
+        assert g[:len(w)] == w and len(g) == 12
+        assert m.generate([p], 12, temperature=0)[0].tolist()[:len(w)] == w
+    assert m.engine.allocator.num_free == m.engine.allocator.num_blocks
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_graph_replays_equal_eager_decoding(ops, dtype):
+    print(f"case: decode graphs {dtype}", flush=True)
+    name = "mixed"
+    m, e = (model(ops, name, dtype, max_batch=2, decode_graphs=g) for g in (True, False))
+    seqs = [oracle(name, 5, 64), oracle(name, 4, 190)]
+    start = [20, 40]
+    ids = []
+    for mdl in (m, e):
+        ids.append([mdl.new_sequence() for _ in seqs])
+        mdl.prefill(ids[-1], [s[1][:n] for s, n in zip(seqs, start)])
+    for step in range(30):
+        toks = [int(s[1][n + step]) for s, n in zip(seqs, start)]
+        a, b = m.decode(ids[0], toks), e.decode(ids[1], toks)             # eager work between the replays
+        torch.cuda.synchronize()
+        assert float(rel(a, b.cpu()).max()) <= (1e-5 if dtype == "float32" else 2e-2), step
+        check(a, torch.stack([s[2][n + step] for s, n in zip(seqs, start)]), dtype, f"replay {step}")
+
+
+def test_fp8_cache(ops):
+    """An e4m3 cache under the same model: prompt, portion and decode steps within the bound stated for fp8 caches (6 % relative
+    rms of the attention result; twice that for logits after several layers)."""
+    print("case: fp8 cache", flush=True)
+    p, toks, ref = oracle("mixed", 4, 190)
+    m = model(ops, "mixed", "bfloat16", kv_dtype="fp8")
+    s = m.new_sequence()
+    got = [m.step([s], [toks[:60]], rows=range(60)), m.step([s], [toks[60:150]], rows=range(90))]
+    got += [m.decode([s], [int(t)]) for t in toks[150:]]
+    e = rel(torch.cat(got), ref)
+    assert float(e.pow(2).mean().sqrt()) <= 0.12, float(e.max())
+
+
+def save_model(tmp_path, name):
+    from safetensors.torch import save_file
+    oracle(name, 0, 1)
+    (tmp_path / "config.json").write_text(json.dumps(CONFIGS[name]))
+    save_file({k: v.contiguous() for k, v in _cache[name].items()}, str(tmp_path / "model.safetensors"))
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_run_command(ops, tmp_path, dtype):
+    print(f"case: bin/trace_run {dtype}", flush=True)
+    save_model(tmp_path, "odd")
+    p, a, ref_a = oracle("odd", 4, 190)
+    _, b, ref_b = oracle("odd", 5, 64)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:120].tolist(), "want": [0, 119, 15]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": a[120:122].tolist(), "want": []}], "end": []},
+             {"step": 2, "entries": [{"id": "a", "tokens": a[122:123].tolist(), "want": [0]}], "end": ["a"]},
+             {"step": 3, "entries": [{"id": "b", "tokens": b.tolist(), "want": [63]}], "end": ["b"]}]
+    out = tmp_path / "out"
+    res = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", dtype, "--out",
+                          str(out), "--max-tokens", "128"], input="\n".join(map(json.dumps, steps)) + "\n", capture_output=True, text=True,
+                         timeout=110)
+    assert res.returncode == 0, res.stderr[-2000:]
+    assert [ln for ln in res.stdout.splitlines() if ln.startswith("done")] == [f"done {n}" for n in range(4)]
+    read = lambda n: torch.frombuffer(bytearray((out / f"{n}.f32").read_bytes()), dtype=torch.float32).view(-1, 53)
+    assert not (out / "1.f32").exists()
+    check(read(0), ref_a[[0, 119, 15]], dtype, "step 0")
+    check(read(2), ref_a[[122]], dtype, "step 2")
+    check(read(3), ref_b[[63]], dtype, "step 3")
+
+
+def test_generate_command_and_registry(ops, tmp_path):
+    print("case: bin/generate", flush=True)
+    save_model(tmp_path, "odd")
+    m = ops.load_model(str(tmp_path), dtype="float32", max_batch=2)
+    assert isinstance(m, ops.ZuzelornLM) and m.dtype == torch.float32
+    prompts = [[3, 1, 4, 1, 5], [9, 2]]
+    want = m.generate_batch(prompts, 6, temperature=0)
+    res = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "generate"), "--model", str(tmp_path), "--dtype", "float32",
+                          "--max-new-tokens", "6", "--temperature", "0", "--prompt", "3 1 4 1 5", "--prompt", "9,2"],
+                         capture_output=True, text=True, timeout=110)
+    assert res.returncode == 0, res.stderr[-2000:]
+    assert [json.loads(ln) for ln in res.stdout.splitlines()] == want
+    # sampling: seeded runs repeat, top_k 1 is greedy
+    g = lambda: torch.Generator(device="cuda").manual_seed(7)
+    assert m.generate_batch(prompts, 6, 1.5, 20, generator=g()) == m.generate_batch(prompts, 6, 1.5, 20, generator=g())
+    assert m.generate_batch(prompts, 6, 1.5, 1) == want
