@@ -18,7 +18,7 @@ fp8 decode, then one {ms, frac} pair per auxiliary leg under "legs", and the con
 `--full` prints every leg's whole object instead; `--detail PATH` writes that verbose form to a file.
 
 usage: python bench.py [--gpus 1] [--steps K=200] [--warmup W=50] [--seed S]
-                       [--only decode|prefill|small|few|fp8|backward|producers|layer|loop] [--no-cpu] [--full] [--detail PATH]
+                       [--only decode|prefill|small|few|fp8|backward|producers|layer|loop|zuzelorn] [--no-cpu] [--full] [--detail PATH]
 """
 from __future__ import annotations
 
@@ -369,6 +369,151 @@ def bench_decode_loop(args):
         res[name] = {"ms_per_step": dt * 1e3, "tokens_per_s": B / dt}
         del model
     res["speedup"] = res["eager"]["ms_per_step"] / res["hip_graph"]["ms_per_step"]
+    return res
+
+
+def _zuzelorn_pair(d, heads, head_dim, ff, n_layers, context, seed):
+    """(config, weights) of a Zuzelorn model whose every layer has keys and values of its own, of one in which every second
+    layer reads the layer before it, and of the reference decoder of the same width, heads, layers and parameter count per
+    layer (four square projections and two gates beside two ff matrices; four and three: equal at ff = 2 d)."""
+    import torch
+    g = torch.Generator(device="cuda:0").manual_seed(seed)
+    V, att = 32000, heads * head_dim
+
+    def w(*shape, std):
+        return (torch.randn(*shape, generator=g, device="cuda:0") * std).to(torch.bfloat16)
+
+    def layer(i, shared):
+        m = {"heads": heads, "kv_heads": heads, "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5}
+        if shared and i % 2:
+            m["kv_from"] = i - 1
+        return {"type": "attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff}}
+
+    base = dict(vocab=V, width=d, max_positions=context, logit_scale=1.0, norm={"eps": 1e-5})
+    own, half = (dict(base, layers=[layer(i, s) for i in range(n_layers)]) for s in (False, True))
+    sd = {"embed": w(V, d, std=1.0), "pos": w(context, d, std=0.5), "head": w(V, d, std=d ** -0.5)}
+
+    def norm(name):
+        sd[name], sd[name + ".b"] = w(d, std=0.1) + 1, w(d, std=0.1)
+        sd[name + ".alpha"] = torch.tensor(0.6)
+
+    norm("final.norm")
+    for i in range(n_layers):
+        n = f"l{i}."
+        for s in ("norm1", "norm1b", "norm2", "norm2b"):
+            norm(n + s)
+        for s in ("q", "k", "v"):
+            sd[n + f"mix.{s}"], sd[n + f"mix.{s}.b"] = w(att, d, std=d ** -0.5), w(att, std=0.1)
+        sd[n + "mix.temp"], sd[n + "mix.sink"] = w(heads, std=0.1) + 1, w(heads, std=1.0)
+        sd[n + "mix.o"], sd[n + "mix.o.b"] = w(d, att, std=att ** -0.5), w(d, std=0.1)
+        sd[n + "mlp.up"], sd[n + "mlp.down"] = w(ff, d, std=d ** -0.5), w(d, ff, std=ff ** -0.5)
+        sd[n + "mlp.act"] = torch.tensor([0.6, 0.3, 0.3, 0.1])
+        for s in ("rg1", "rg2"):
+            sd[n + s], sd[n + s + ".b"] = w(d, d, std=d ** -0.5), w(d, std=0.1)
+    ref_cfg = dict(vocab_size=V, context_length=context, d_model=d, num_layers=n_layers, num_heads=heads, d_ff=ff, rope_theta=10000.0)
+    ref = {"token_embeddings.weight": sd["embed"], "lm_head.weight": sd["head"], "final_norm.weight": torch.ones(d)}
+    for i in range(n_layers):
+        pre = f"layers.{i}."
+        for s in ("q_proj", "k_proj", "v_proj", "output_proj"):
+            ref[pre + f"attn.{s}.weight"] = w(d, d, std=d ** -0.5)
+        for s, shape in (("gate_proj", (ff, d)), ("up_proj", (ff, d)), ("down_proj", (d, ff))):
+            ref[pre + f"ffn.{s}.weight"] = w(*shape, std=shape[1] ** -0.5)
+        ref[pre + "attn_norm.weight"] = ref[pre + "ffn_norm.weight"] = torch.ones(d)
+    return (own, sd), (half, sd), (ref_cfg, ref)
+
+
+def bench_zuzelorn(args):
+    """Prefill and decode of the Zuzelorn model beside the reference decoder at equal size (random weights, both through the
+    same engine and step functions, measured in turn), and its streaming operators beside the reference decoder's."""
+    import torch
+    import mi355_attn as ma
+
+    names = ("zuzelorn", "zuzelorn_shared_kv", "reference_decoder")
+    res = {"models": {}, "operators": {}}
+    n_prompt, prompt_len, batch, ctx = 4, 2048, 32, 2048
+    for key, d, heads, head_dim, n_layers in (("d1024", 1024, 16, 64, 8), ("d2048", 2048, 16, 128, 6), ("d4096", 4096, 32, 128, 4)):
+        context = 4096
+        g = torch.Generator().manual_seed(args.seed)
+        pairs = _zuzelorn_pair(d, heads, head_dim, 2 * d, n_layers, context, args.seed)
+        blocks = batch * (ctx + 256) // 16
+        models = [cls(c, sd, num_blocks=blocks, max_batch=batch, decode_graphs=True)
+                  for cls, (c, sd) in zip((ma.ZuzelornLM, ma.ZuzelornLM, ma.CachedTransformerLM), pairs)]
+        entry = {"workload": f"{n_layers} layers, width {d}, {heads} heads x {head_dim}, ff {2 * d}, vocab 32000; prefill: {n_prompt} new prompts "
+                             f"of {prompt_len} tokens; decode: {batch} sequences at {ctx} tokens, HIP graph, greedy tokens fed back through the host"}
+        prompts = [torch.randint(0, 32000, (prompt_len,), generator=g) for _ in range(n_prompt)]
+
+        def prefill(m):
+            s = [m.new_sequence() for _ in prompts]
+            m.prefill(s, prompts)
+            for i in s:
+                m.free_sequence(i)
+
+        best = {n: {} for n in names}
+        for rep in range(3):                                   # the sides in turn; the best of three rounds each
+            for n, m in zip(names, models):
+                ms, _ = timed(lambda: prefill(m), max(3, args.steps // 20), 2, BURN_MS)
+                best[n]["prefill_ms"] = min(ms, best[n].get("prefill_ms", 1e9))
+        state = []
+        for m in models:                                       # sequences of ctx tokens
+            sids = [m.new_sequence() for _ in range(batch)]
+            for i in range(0, batch, 8):
+                m.prefill(sids[i:i + 8], [torch.randint(0, 32000, (ctx,), generator=g) for _ in range(8)])
+            state.append([sids, [1] * batch])
+        for rep in range(3):
+            for n, m, st in zip(names, models, state):
+                def step():
+                    st[1] = m.decode(st[0], st[1]).argmax(-1).tolist()
+                ms, _ = timed(step, 30, 8)
+                best[n]["decode_ms"] = min(ms, best[n].get("decode_ms", 1e9))
+        for n in names:
+            entry[n] = {"prefill_ms": best[n]["prefill_ms"], "prefill_tokens_per_s": n_prompt * prompt_len / best[n]["prefill_ms"] * 1e3,
+                        "decode_ms": best[n]["decode_ms"], "decode_tokens_per_s": batch / best[n]["decode_ms"] * 1e3}
+        res["models"][key] = entry
+        del models, state, pairs
+        torch.cuda.empty_cache()
+
+    # the operators at prefill size (8192 rows of width 4096, ff 8192): bytes that must move over the device time
+    T, d, ff, H, D = 8192, 4096, 8192, 32, 128
+    dev = torch.device("cuda:0")
+    g = torch.Generator(device=dev).manual_seed(args.seed)
+
+    def t(*shape, dtype=torch.bfloat16):
+        return torch.randn(*shape, device=dev, generator=g).to(dtype)
+
+    vec = [t(d, dtype=torch.float32) for _ in range(6)]
+    resid, wide, u, gu, x, r = t(T, d, dtype=torch.float32), t(T, 2 * d), t(T, ff + d), t(T, 2 * ff), t(T, d), t(T, d)
+    qkv = t(T, 3, H, D)
+    pools = [torch.zeros(T // 16, H, 16, D, dtype=torch.bfloat16, device=dev) for _ in range(2)]
+    slots, pos = torch.arange(T, device=dev), torch.arange(T, dtype=torch.int32, device=dev) % 4096
+    freq, emb, ptab = ma.build_rope_cache(4096, D, 1e4, dev), t(32000, d), t(4096, d)
+    ids = torch.randint(0, 32000, (T,), device=dev, generator=g)
+    ops = {
+        "dyt_residual": (T * d * (2 + 2 + 4 + 4 + 2), lambda: ma.dyt_residual(
+            resid, wide[:, :d], sub_bias=vec[0], gate=wide[:, d:], gate_bias=vec[1], post=(0.6, vec[2], vec[3]), norm=(0.6, vec[4], vec[5]))),
+        "rms_norm_residual (reference decoder)": (T * d * 8, lambda: ma.rms_norm(x, vec[0], residual=r, return_sum=True)),
+        "polynorm": (T * ff * 4, lambda: ma.polynorm(u[:, :ff], (0.6, 0.3, 0.3, 0.1), 1e-5)),
+        "silu_mul (reference decoder)": (T * ff * 6, lambda: ma.silu_mul(gu[:, :ff], gu[:, ff:])),
+        "kv_cache_write": (T * H * D * 8, lambda: ma.kv_cache_write(qkv[:, 1], qkv[:, 2], *pools, slots)),
+        "rope_and_cache (reference decoder)": (T * H * D * 12, lambda: ma.rope_and_cache(qkv[:, 0], qkv[:, 1], qkv[:, 2], pos, freq, *pools, slots)),
+        "embed_pos": (T * d * 8, lambda: ma.embed_pos(emb, ptab, ids, pos)),
+    }
+    for n, (nbytes, fn) in ops.items():
+        _, ms = timed(fn, args.steps, args.warmup, BURN_MS)
+        res["operators"][n] = {"device_ms": ms, "algorithmic_bytes": nbytes, "frac_of_hbm_peak": nbytes / ms / 1e6 / HBM_PEAK_GBPS}
+
+    # attention with and without per-head factors and sinks, on the same tensors
+    hs, sk = torch.rand(H, device=dev) + 0.5, torch.randn(H, device=dev)
+    cu = torch.arange(0, T + 1, 2048, dtype=torch.int32, device=dev)
+    flops = 4 * (T // 2048) * H * D * 2048 * 2049 / 2
+    bt = torch.randperm(T // 16, device=dev).to(torch.int32).view(4, -1)
+    cl = torch.full((4,), 2048, dtype=torch.int32, device=dev)
+    q1 = t(4, H, D)
+    for n, kw in (("with factors and sinks", dict(head_scale=hs, sinks=sk)), ("plain (reference decoder)", {})):
+        _, ms = timed(lambda: ma.flash_attn_varlen_prefill(qkv[:, 0], qkv[:, 1], qkv[:, 2], cu, cu, 2048, 2048, **kw), args.steps, args.warmup, BURN_MS)
+        res["operators"]["prefill attention " + n] = {"device_ms": ms, "frac_of_mfma_peak": flops / ms / 1e9 / MFMA_BF16_PEAK_TFLOPS}
+        ws = ma.paged_decode_workspace(4, H, D, 2048, dev)
+        _, ms = timed(lambda: ma.paged_attention_decode(q1, *pools, bt, cl, workspace=ws, **kw), args.steps, args.warmup, BURN_MS)
+        res["operators"]["decode attention " + n] = {"device_ms": ms, "frac_of_hbm_peak": T * H * D * 4 / ms / 1e6 / HBM_PEAK_GBPS}
     return res
 
 
@@ -795,8 +940,10 @@ def main():
     ap.add_argument("--steps", type=int, default=200)
     ap.add_argument("--warmup", type=int, default=50)
     ap.add_argument("--seed", type=int, default=0)
-    ap.add_argument("--only", choices=["decode", "prefill", "small", "few", "fp8", "backward", "producers", "layer", "loop"],
-                    default=None)
+    ap.add_argument("--only", choices=["decode", "prefill", "small", "few", "fp8", "backward", "producers", "layer", "loop",
+                                       "zuzelorn"],
+                    default=None, help="one leg; `zuzelorn` (the Zuzelorn model beside the reference decoder at equal size) "
+                                       "runs only when it is named")
     ap.add_argument("--no-cpu", action="store_true")
     ap.add_argument("--full", action="store_true", help="print every leg's whole object (a line of about 10 KB)")
     ap.add_argument("--detail", default=None, metavar="PATH", help="also write the verbose form to this file")
@@ -877,6 +1024,12 @@ def main():
     if args.only in (None, "loop"):
         line["decode_few_sequences"] = bench_decode_few_sequences(args)
         line["decode_loop"] = bench_decode_loop(args)
+
+    if args.only == "zuzelorn":
+        z = line["zuzelorn"] = bench_zuzelorn(args)
+        first = z["models"]["d2048"]
+        line.update({"value": first["zuzelorn"]["prefill_tokens_per_s"], "unit": "tokens/s", "ms_per_step": first["zuzelorn"]["prefill_ms"],
+                     "dtype": "bf16", "config": {"workload": first["workload"]}})
 
     if with_cpu:
         if dec is not None:

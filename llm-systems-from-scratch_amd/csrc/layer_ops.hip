@@ -253,7 +253,7 @@ struct DytResidualParams {
     T* y;
     float post_alpha, next_alpha;
     int64_t n_rows, sub_stride, gate_stride, y_stride;      // resid rows are contiguous
-    int n_cols, rows_per_thread;
+    int n_cols;
 };
 
 template <typename T, bool FAST>
@@ -264,40 +264,51 @@ __device__ __forceinline__ float dyt_sublayer(const DytResidualParams<T>& p, flo
     return p.post_w ? fmaf(tanh_of<FAST>(p.post_alpha * s), pw, pb) : s;
 }
 
-// A thread owns 8 adjacent columns of rows_per_thread rows, so that the six parameter vectors -- more bytes than the
-// tensors themselves -- are fetched once for all of them.  Adjacent threads own adjacent columns.
-template <typename T>
+// A thread owns 8 adjacent columns of ROWS rows, so that the six parameter vectors -- more bytes than the tensors
+// themselves -- are fetched once for all of them, and asks for all of its rows before it computes.  Adjacent threads own
+// adjacent columns.
+template <typename T, int ROWS>
 __global__ __launch_bounds__(256) void dyt_residual_vec8_kernel(DytResidualParams<T> p) {
     constexpr bool FAST = sizeof(T) == 2;
     const int groups = p.n_cols / 8;
     const int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
-    const int64_t row0 = idx / groups * p.rows_per_thread;
+    const int64_t row0 = idx / groups * ROWS;
     const int col = (int)(idx % groups) * 8;
     if (row0 >= p.n_rows) return;
-    float sb[8], gb[8], pw[8], pb[8], nw[8], nb[8];
-    load_param8(p.sub ? p.sub_bias : nullptr, col, 0.f, sb);
-    load_param8(p.gate ? p.gate_bias : nullptr, col, 0.f, gb);
-    load_param8(p.sub ? p.post_w : nullptr, col, 1.f, pw);
-    load_param8(p.sub ? p.post_b : nullptr, col, 0.f, pb);
-    load_param8(p.next_w, col, 1.f, nw);
-    load_param8(p.next_b, col, 0.f, nb);
-    const int64_t row1 = min(row0 + p.rows_per_thread, p.n_rows);
-    for (int64_t row = row0; row < row1; ++row) {
-        float x[8];
-        load8(p.resid_in + row * p.n_cols + col, x);
-        if (p.sub) {
-            float s[8], g[8] = {};
-            load8(p.sub + row * p.sub_stride + col, s);
-            if (p.gate) load8(p.gate + row * p.gate_stride + col, g);
+    float x[ROWS][8], s[ROWS][8], g[ROWS][8];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) x[e] += dyt_sublayer<T, FAST>(p, s[e], g[e], sb[e], gb[e], pw[e], pb[e]);
-        }
-        if (p.resid_out) store8(p.resid_out + row * p.n_cols + col, x);
-        if (p.y) {
+    for (int r = 0; r < ROWS; ++r) {
+        const int64_t row = min(row0 + r, p.n_rows - 1);       // (rows past the end re-read the last one and store nothing)
+        load8(p.resid_in + row * p.n_cols + col, x[r]);
+        if (p.sub) load8(p.sub + row * p.sub_stride + col, s[r]);
+        if (p.gate) load8(p.gate + row * p.gate_stride + col, g[r]);
+    }
+    if (p.sub) {
+        float sb[8], gb[8], pw[8], pb[8];
+        load_param8(p.sub_bias, col, 0.f, sb);
+        load_param8(p.gate_bias, col, 0.f, gb);
+        load_param8(p.post_w, col, 1.f, pw);
+        load_param8(p.post_b, col, 0.f, pb);
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[r][e] += dyt_sublayer<T, FAST>(p, s[r][e], g[r][e], sb[e], gb[e], pw[e], pb[e]);
+    }
+    if (p.resid_out) {
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r)
+            if (row0 + r < p.n_rows) store8(p.resid_out + (row0 + r) * p.n_cols + col, x[r]);
+    }
+    if (p.y) {
+        float nw[8], nb[8];
+        load_param8(p.next_w, col, 1.f, nw);
+        load_param8(p.next_b, col, 0.f, nb);
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r) {
             float y[8];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) y[e] = fmaf(tanh_of<FAST>(p.next_alpha * x[e]), nw[e], nb[e]);
-            store8(p.y + row * p.y_stride + col, y);
+            for (int e = 0; e < 8; ++e) y[e] = fmaf(tanh_of<FAST>(p.next_alpha * x[r][e]), nw[e], nb[e]);
+            if (row0 + r < p.n_rows) store8(p.y + (row0 + r) * p.y_stride + col, y);
         }
     }
 }
@@ -434,7 +445,27 @@ struct EmbedPosParams {
     int n_cols;
 };
 
-// One thread per element; an id outside its table is clamped into it (the host checks what it can).
+// Ids outside their table are clamped into it (the host checks what it can).
+// One thread per 8 elements: n_cols % 8 == 0, aligned tables.
+template <typename T>
+__global__ __launch_bounds__(256) void embed_pos_vec8_kernel(EmbedPosParams<T> p) {
+    const int groups = p.n_cols / 8;
+    const int64_t total = p.n_rows * groups;
+    for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = idx / groups;
+        const int col = (int)(idx % groups) * 8;
+        const int64_t tok = min(max(p.tokens[row], (int64_t)0), p.vocab - 1);
+        const int64_t pos = min(max((int64_t)p.positions[row], (int64_t)0), p.n_positions - 1);
+        float a[8], b[8];
+        load8(p.embed + tok * p.n_cols + col, a);
+        load8(p.pos + pos * p.n_cols + col, b);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) a[e] += b[e];
+        store8(p.out + row * p.n_cols + col, a);
+    }
+}
+
+// One thread per element: any shape.
 template <typename T>
 __global__ __launch_bounds__(256) void embed_pos_kernel(EmbedPosParams<T> p) {
     const int64_t total = p.n_rows * p.n_cols;
@@ -565,15 +596,15 @@ static int dyt_residual(const void* sub, const float* sub_bias, const void* gate
         vec = vec && aligned16(ptr);
     if (vec) {
         // rows per thread: as many as leave the GPU several workgroups per compute unit
-        const int64_t work = n_rows * (n_cols / 8);
-        int r = 1;
-        while (r < 8 && work / (2 * r) >= 256 * 2048) r *= 2;
-        p.rows_per_thread = r;
-        const int64_t threads = (n_rows + r - 1) / r * (n_cols / 8);
+        const int64_t groups = n_cols / 8, work = n_rows * groups;
+        const int r = work >= 4 * 256 * 2048 ? 4 : work >= 2 * 256 * 2048 ? 2 : 1;
+        const int64_t threads = (n_rows + r - 1) / r * groups;
         if ((threads + 255) / 256 > 0x7fffffffLL) return set_error(MI355_EINVAL, "dyt_residual: too many elements");
-        hipLaunchKernelGGL(dyt_residual_vec8_kernel<T>, dim3(grid_1d(threads)), dim3(256), 0, s, p);
+        const dim3 grid(grid_1d(threads)), block(256);
+        if (r == 4) hipLaunchKernelGGL((dyt_residual_vec8_kernel<T, 4>), grid, block, 0, s, p);
+        else if (r == 2) hipLaunchKernelGGL((dyt_residual_vec8_kernel<T, 2>), grid, block, 0, s, p);
+        else hipLaunchKernelGGL((dyt_residual_vec8_kernel<T, 1>), grid, block, 0, s, p);
     } else {
-        p.rows_per_thread = 1;
         hipLaunchKernelGGL(dyt_residual_generic_kernel<T>, dim3(grid_1d(n_rows * (int64_t)n_cols)), dim3(256), 0, s, p);
     }
     return launch_status();
@@ -655,7 +686,10 @@ static int embed_pos(const void* embed, const void* pos, const int64_t* tokens, 
     p.n_cols = n_cols;
     p.vocab = vocab;
     p.n_positions = n_positions;
-    hipLaunchKernelGGL(embed_pos_kernel<T>, dim3(grid_1d(n_rows * (int64_t)n_cols)), dim3(256), 0, s, p);
+    if (n_cols % 8 == 0 && aligned16(embed) && aligned16(pos) && aligned16(out))
+        hipLaunchKernelGGL(embed_pos_vec8_kernel<T>, dim3(grid_1d(n_rows * (int64_t)(n_cols / 8))), dim3(256), 0, s, p);
+    else
+        hipLaunchKernelGGL(embed_pos_kernel<T>, dim3(grid_1d(n_rows * (int64_t)n_cols)), dim3(256), 0, s, p);
     return launch_status();
 }
 

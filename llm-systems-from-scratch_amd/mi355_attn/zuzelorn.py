@@ -108,7 +108,7 @@ class ZuzelornLM(CachedLM):
                     w.append(_pad_heads(raw(pre + f"mix.{n}", G * size, d).float(), G, size, to))
                     b.append(_pad_heads(raw(pre + f"mix.{n}.b", G * size).float(), G, size, to))
             w.append(raw(pre + "rg1", d, d).float())
-            b.append(torch.zeros(d))                       # (the gate's bias is added in fp32 where the gate is applied)
+            b.append(b[0].new_zeros(d))                     # (the gate's bias is added in fp32 where the gate is applied)
             w_in, starts = _stack_rows(w)
             wo = _pad_heads(raw(pre + "mix.o", d, H * dv).float().t(), H, dv, vd).t()
             ly = dict(H=H, G=G, kd=kd, vd=vd, own_kv=src is None, w_in=mat(w_in), b_in=mat(_stack_rows(b)[0]), starts=starts,

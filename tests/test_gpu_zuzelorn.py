@@ -53,7 +53,7 @@ def dyt_case(T, d, dtype, seed):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T,d", [(1, 8), (5, 72), (33, 100), (64, 1024), (4099, 2056)])
+@pytest.mark.parametrize("T,d", [(1, 8), (5, 72), (33, 100), (64, 1024), (4099, 2056), (8195, 2056)])
 def test_dyt_residual_matches_oracle(ops, T, d, dtype):
     print(f"case: dyt_residual {T}x{d} {dtype}", flush=True)
     c = dyt_case(T, d, dtype, seed=d)
@@ -107,9 +107,10 @@ def test_polynorm_matches_oracle(ops, d, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_embed_pos_matches_oracle(ops, dtype):
-    print(f"case: embed_pos {dtype}", flush=True)
-    e, p = rnd(50, 37, seed=1, dtype=dtype), rnd(20, 37, seed=2, dtype=dtype)
+@pytest.mark.parametrize("d", [37, 72, 2048])
+def test_embed_pos_matches_oracle(ops, d, dtype):
+    print(f"case: embed_pos {d} {dtype}", flush=True)
+    e, p = rnd(50, d, seed=1, dtype=dtype), rnd(20, d, seed=2, dtype=dtype)
     tok, pos = torch.tensor([0, 49, 7, 7, 1]), torch.tensor([0, 19, 3, 4, 1], dtype=torch.int32)
     got = ops.embed_pos(e.cuda(), p.cuda(), tok.cuda(), pos.cuda())
     assert got.dtype == torch.float32 and torch.equal(got.cpu(), e[tok].float() + p[pos.long()].float())
