@@ -233,6 +233,15 @@ def test_trace_run_ends_with_3_when_the_model_has_no_float32_path(tmp_path):
     assert res.returncode == 3
 
 
+def test_serving_library_reports_what_it_lacks():
+    from mi355_attn import _lib
+    lib = _lib._ServingLib(mi355_attn.load())
+    assert b"gfx950" in lib.mi355_version()
+    lib.mi355_prefill_bwd.argtypes = []
+    with pytest.raises(mi355_attn.LibraryMissing, match="mi355_prefill_bwd"):
+        lib.mi355_prefill_bwd(None)
+
+
 def test_operator_arguments_are_checked_on_the_host():
     f = torch.zeros(2, 8)
     with pytest.raises(ValueError):
