@@ -464,6 +464,130 @@ int mi355_embed_pos_fwd(const void* embed, const void* pos, const int64_t* token
                         int64_t n_rows, int n_cols, int64_t vocab, int64_t n_positions, int dtype, void* stream);
 
 /*
+ * Causal attention with a sliding window that keeps the first tokens: the query at position i sees key j when j <= i and
+ * (i - j < window or j < keep_first).  window 0: every earlier key (keep_first is then without effect).  Otherwise the
+ * headwise forms above; keys outside the window are neither read nor computed, apart from the rest of the tiles (prefill)
+ * or blocks (decode) at its lower edge.  No split keys in the prefill forms.
+ *   mi355_paged_decode_fwd_window : out rows may be strided too (out_row_stride elements, a multiple of 8); the workspace
+ *                                   of mi355_paged_decode_workspace_bytes is enough
+ */
+int mi355_prefill_fwd_window(const void* q, const void* k, const void* v, void* out, const int64_t q_strides[3],
+                             const int64_t k_strides[3], const int64_t v_strides[3], const int64_t o_strides[3],
+                             const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, const float* head_scale,
+                             const float* sink, int B, int Hq, int Hkv, int Sq_max, int Sk_max, int D,
+                             float softmax_scale, int window, int keep_first, int dtype, void* stream);
+int mi355_prefill_paged_fwd_window(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                   int64_t q_token_stride, int64_t out_token_stride, const int32_t* cu_seqlens_q,
+                                   const int32_t* block_tables, int64_t table_stride, int64_t max_blocks,
+                                   const int32_t* context_lens, const float* head_scale, const float* sink, int B,
+                                   int Hq, int Hkv, int Sq_max, int D, int block_size, int64_t num_blocks,
+                                   float softmax_scale, int window, int keep_first, int kv_dtype, void* stream);
+int mi355_paged_decode_fwd_window(const void* q, int64_t q_row_stride, const void* k_cache, const void* v_cache,
+                                  void* out, int64_t out_row_stride, const int32_t* block_tables, int64_t bt_row_stride,
+                                  const int32_t* context_lens, const float* k_scale, const float* v_scale,
+                                  const float* head_scale, const float* sink, void* workspace, size_t workspace_bytes,
+                                  int B, int Hq, int Hkv, int D, int block_size, int64_t num_blocks, int max_ctx,
+                                  float softmax_scale, int window, int keep_first, int kv_dtype, void* stream);
+int mi355_paged_attn_any_fwd_window(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                    int64_t q_row_stride, int64_t out_row_stride, int64_t n_rows,
+                                    const int32_t* cu_seqlens_q, const int32_t* block_tables, int64_t bt_row_stride,
+                                    int64_t max_blocks, const int32_t* context_lens, const float* head_scale,
+                                    const float* sink, int B, int Hq, int Hkv, int Dk, int Dv, int block_size,
+                                    int64_t num_blocks, float softmax_scale, int window, int keep_first, int dtype,
+                                    void* stream);
+
+/*
+ * Rotation in place of adjacent pairs of q (T,Hq,D) and k (T,Hkv,D) heads of any even size, MI355_BF16 or MI355_FP32, with the
+ * table layout of mi355_rope_and_cache (fp32 math).  Heads contiguous, token strides in elements; Hkv 0: q only.
+ */
+int mi355_rope_any(void* q, void* k, const float* freq_cache, const int32_t* positions, int64_t n_tokens, int Hq, int Hkv,
+                   int D, int context_length, int64_t q_token_stride, int64_t k_token_stride, int dtype, void* stream);
+
+/*
+ * Everything that is added to an fp32 residual stream, and the RMS norm of the sum, in one pass over (n_rows, n_cols):
+ *   x = resid_in + sub + sum_{k < top} routed[row * top + k] + embed[tokens[row]]
+ *   y = x / sqrt(mean(x^2) + eps) * (weight_offset + weight)
+ * Each summand is optional (NULL), as are resid_out (may be resid_in) and y (columns n_cols .. y_cols - 1 of y are set to
+ * zero).  sub, routed, embed, y: dtype MI355_BF16 or MI355_FP32; resid and weight (NULL: 0): fp32, contiguous.
+ */
+int mi355_residual_rms_fwd(const float* resid_in, float* resid_out, const void* sub, const void* routed, int top,
+                           const void* embed, const int64_t* tokens, int64_t vocab, const float* weight,
+                           float weight_offset, float eps, void* y, int64_t n_rows, int n_cols, int y_cols,
+                           int64_t sub_row_stride, int64_t routed_row_stride, int64_t y_row_stride, int dtype, void* stream);
+
+/*
+ * Feed-forward activations over (n_rows, n_cols), fp32 math: out = silu(a) * b, or with b NULL the tanh form of gelu(a);
+ * with row_gate (fp32, one per row) times sigmoid(row_gate).
+ */
+int mi355_ff_act_fwd(const void* a, const void* b, const float* row_gate, void* out, int64_t n_rows, int n_cols,
+                     int64_t a_row_stride, int64_t b_row_stride, int64_t out_row_stride, int dtype, void* stream);
+
+/*
+ * Gated norm over (n_rows, n_cols): v = y * silu(z); each of `groups` equal parts of a row divided by its own root mean square
+ * (sqrt(mean(v^2) + eps)), times weight (fp32, n_cols).
+ */
+int mi355_gated_norm_fwd(const void* y, const void* z, const float* weight, void* out, int64_t n_rows, int n_cols, int groups,
+                         int64_t y_row_stride, int64_t z_row_stride, int64_t out_row_stride, float eps, int dtype,
+                         void* stream);
+
+/*
+ * Mamba-2 mixer (state-space duality) between its projections.  Per head h of group h / (heads / groups), with
+ * [x | B | C] = silu(causal convolution of the input channels) and dt = softplus(input + dt_bias):
+ *   S_t = exp(neg_a dt_t) S_(t-1) + dt_t B_t x_t^T        y_t = S_t^T C_t + d_skip x_t        (S: state x vdim, fp32)
+ * proj rows hold the channels (heads*vdim | groups*state | groups*state) from column xbc_col and one dt per head from column
+ * dt_col.  What a sequence carries lives in slot slots[b] of
+ *   conv_state (n_slots, taps, channels) of `dtype`: the convolution's inputs, position p in row p % taps
+ *   ssm_state  (n_slots, heads, state, vdim rounded up to 4) fp32
+ * and is taken as zero when the sequence's first row of the call has position 0 (slots need no clearing).
+ *   mi355_ssm_prefill : sequence b owns rows cu_seqlens[b] .. cu_seqlens[b+1] - 1 (NULL: row b), any number of them; needs xbc
+ *                       (n_rows, channels) of `dtype` as scratch.  scan AUTO: chunks on MFMA where they apply (bf16; state
+ *                       and vdim multiples of 8, state <= 256), else token by token
+ *   mi355_ssm_decode  : one row per sequence, convolution and recurrence in one launch
+ */
+enum { MI355_SCAN_AUTO = 0, MI355_SCAN_SERIAL = 1, MI355_SCAN_CHUNKED = 2 };
+typedef struct mi355_ssm_args {
+    const void* proj;
+    const float* conv_weight;    /* (taps, channels), the last tap is the current token's */
+    const float* conv_bias;      /* (channels) */
+    const float* dt_bias;        /* (heads) */
+    const float* neg_a;          /* (heads): the decay's rate, negative */
+    const float* d_skip;         /* (heads) */
+    void* conv_state;
+    float* ssm_state;
+    const int32_t* slots;        /* (batch) */
+    const int32_t* positions;    /* (n_rows) */
+    const int32_t* cu_seqlens;   /* (batch + 1) or NULL */
+    void* xbc;
+    void* y;                     /* (n_rows, heads * vdim) of `dtype` */
+    int64_t proj_row_stride, xbc_col, dt_col, y_row_stride, n_rows;
+    int batch, heads, vdim, state, groups, taps, n_slots, dtype;
+} mi355_ssm_args;
+int mi355_ssm_prefill(const mi355_ssm_args* args, int scan, void* stream);
+int mi355_ssm_decode(const mi355_ssm_args* args, void* stream);
+
+/*
+ * Mixture-of-experts feed-forward.  A (token, choice) is a pair, numbered token * top + choice.
+ *   mi355_moe_route   : logits h W^T + bias (fp32 sums) of n_experts experts (up to 1024), the `top` (up to 64) largest and the
+ *                       softmax over them -> ids, weights (n_tokens, top).  With extra_logit (n_tokens), w and bias have one
+ *                       row more, whose logit goes there.
+ *   mi355_moe_group   : pairs sorted by expert: order (n_pairs), offsets (n_experts + 1)
+ *   mi355_moe_gate_up : act[i] = silu(Wg h) * (Wu h) for place i of the order; w (n_experts, 2 ff, k), gates first
+ *   mi355_moe_down    : out[pair] = weights[pair] * (Wd act[i]); w (n_experts, n, ff)
+ * bf16 (fp32 sums): k and ff in multiples of 64, 16-byte aligned rows.  tiling AUTO chooses by pairs per expert.
+ */
+enum { MI355_TILING_AUTO = 0, MI355_TILING_SKINNY = 1, MI355_TILING_LARGE = 2 };
+int mi355_moe_route(const void* h, const void* w, const float* bias, int32_t* ids, float* weights, float* extra_logit,
+                    int64_t n_tokens, int64_t h_row_stride, int64_t w_row_stride, int k, int n_experts, int top, int dtype,
+                    void* stream);
+int mi355_moe_group(const int32_t* ids, int64_t n_pairs, int n_experts, int32_t* offsets, int32_t* order, void* stream);
+int mi355_moe_gate_up(const void* h, const void* w, void* act, const int32_t* offsets, const int32_t* order, int64_t n_tokens,
+                      int64_t h_row_stride, int64_t act_row_stride, int n_experts, int top, int k, int ff, int dtype,
+                      int tiling, void* stream);
+int mi355_moe_down(const void* act, const void* w, const float* weights, void* out, const int32_t* offsets,
+                   const int32_t* order, int64_t n_tokens, int64_t act_row_stride, int64_t out_row_stride, int n_experts,
+                   int top, int ff, int n, int dtype, int tiling, void* stream);
+
+/*
  * Plain device-to-device copy of `bytes` bytes (16-byte aligned).  Measurement aid
  * with no counterpart in the reference: a copy of known size whose FETCH_SIZE /
  * WRITE_SIZE counter readings calibrate the HBM-traffic figures of the kernels above.

@@ -22,7 +22,7 @@ LIB_NAME = "libmi355attn.so"
 SERVING_LIB_NAME = "libmi355attn_serving.so"      # without the kernels that only training needs
 TRAINING_ONLY = ("prefill_bwd.hip",)
 SOURCES = ["api.hip", "paged_decode.hip", "prefill_fwd.hip", "prefill_fwd_w64.hip", "prefill_bwd.hip", "kv_cache_ops.hip",
-           "layer_ops.hip", "paged_attn_any.hip"]
+           "layer_ops.hip", "paged_attn_any.hip", "ssm_ops.hip", "moe_ops.hip"]
 # prefill_fwd_w64.hip keeps its output accumulators in AGPRs that only its assembly statements touch: its builtin MFMAs
 # must therefore be selected in VGPR form, so that the compiler allocates no AGPR for them.
 # It is also compiled without the machine-code hoisting of loop invariants: hoisted out of the job loop, a few dozen
@@ -190,7 +190,7 @@ def build_library(verbose: bool = True) -> str:
     srcs = [s for s in SOURCES if os.path.exists(os.path.join(CSRC, s))]
 
     # sources whose kernels issue memory instructions from inline assembly
-    asm_dma = [s for s in ("prefill_fwd.hip", "prefill_fwd_w64.hip", "prefill_bwd.hip") if s in srcs]
+    asm_dma = [s for s in ("prefill_fwd.hip", "prefill_fwd_w64.hip", "prefill_bwd.hip", "moe_ops.hip") if s in srcs]
     with ThreadPoolExecutor(max_workers=4) as ex:
         check = ex.submit(check_w64_registers)
         hazards = [ex.submit(check_scalar_address_hazards, s) for s in asm_dma]

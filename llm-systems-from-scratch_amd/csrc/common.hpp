@@ -150,6 +150,33 @@ __device__ __forceinline__ int xcd_chunked_id(int bid, int n_wg, int chunk) {
     return __builtin_amdgcn_readfirstlane(bid >= whole ? bid : id);
 }
 
+// ---- sliding window with kept first tokens ---------------------------------------
+// A query that ends a prefix of n_keys keys sees key j when j >= n_keys - window or j < keep_first (window 0: every key).
+// The blocks of 16 keys that hold visible keys -- the leading ones up to keep_first, then those from the window's first
+// key on -- are walked as one compact run of n keys: compact block b is logical block logical_block(b), and the compact
+// keys [hid0, hid1), at most 30 of them around the seam, are in those blocks without being visible.
+struct VisibleKeys {
+    int n, kept_blocks, skip_blocks, hid0, hid1;
+    __device__ __forceinline__ int logical_block(int b) const { return b < kept_blocks ? b : b + skip_blocks; }
+    __device__ __forceinline__ bool hidden(int key) const { return key >= hid0 && key < hid1; }
+};
+__device__ __forceinline__ VisibleKeys visible_keys(int n_keys, int window, int keep_first) {
+    VisibleKeys v;
+    const int lo = window > 0 ? max(0, n_keys - window) : 0;
+    v.kept_blocks = (keep_first + 15) / 16;
+    v.skip_blocks = max(0, lo / 16 - v.kept_blocks);
+    v.n = n_keys - 16 * v.skip_blocks;
+    v.hid0 = keep_first;
+    v.hid1 = max(keep_first, lo - 16 * v.skip_blocks);
+    return v;
+}
+// ... and an upper bound of n over all prefixes of up to max_keys keys
+inline int max_visible_keys(int max_keys, int window, int keep_first) {
+    if (window <= 0) return max_keys;
+    const int64_t n = (int64_t)window + 15 + ((int64_t)keep_first + 15) / 16 * 16;
+    return n < max_keys ? (int)n : max_keys;
+}
+
 __device__ __forceinline__ uint32_t lds_address(const void* lds_ptr) {
     return (uint32_t)(uintptr_t)(const MI355_LDS void*)lds_ptr;
 }

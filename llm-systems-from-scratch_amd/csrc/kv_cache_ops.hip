@@ -452,6 +452,49 @@ __global__ __launch_bounds__(256) void kv_cache_write_kernel(KvWriteParams p) {
 
 }  // namespace mi355
 
+// Rotation in place of query and key heads of any even size, bf16 or fp32: the pair (x[2i], x[2i+1]) turns by the angle of
+// (position, i), in fp32.  One thread per (token, head, pair).
+namespace mi355 {
+template <typename T>
+__global__ __launch_bounds__(256) void rope_any_kernel(T* q, T* k, const float* freq, const int32_t* positions, int64_t q_tok, int64_t k_tok,
+                                                       int64_t n_tokens, int Hq, int Hkv, int half, int ctx_len) {
+    const int64_t total = n_tokens * (Hq + Hkv) * half;
+    for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * blockDim.x) {
+        const int i = (int)(idx % half);
+        const int h = (int)((idx / half) % (Hq + Hkv));
+        const int64_t t = idx / ((int64_t)half * (Hq + Hkv));
+        const int pos = min(max(positions[t], 0), ctx_len - 1);        // a position outside the table is clamped into it
+        T* x = (h < Hq ? q + t * q_tok + (int64_t)h * 2 * half : k + t * k_tok + (int64_t)(h - Hq) * 2 * half) + 2 * i;
+        const float c = freq[(int64_t)pos * half + i], s = freq[((int64_t)ctx_len + pos) * half + i];
+        const float a = (float)x[0], b = (float)x[1];
+        x[0] = (T)(c * a - s * b);
+        x[1] = (T)(s * a + c * b);
+    }
+}
+}  // namespace mi355
+
+extern "C" int mi355_rope_any(void* q, void* k, const float* freq_cache, const int32_t* positions, int64_t n_tokens, int Hq, int Hkv,
+                              int D, int context_length, int64_t q_token_stride, int64_t k_token_stride, int dtype, void* stream) {
+    if (!q || (!k && Hkv > 0) || !freq_cache || !positions) return set_error(MI355_EINVAL, "rope_any: null pointer argument");
+    if (n_tokens < 0 || Hq <= 0 || Hkv < 0 || D <= 0 || D % 2 || context_length <= 0)
+        return set_error(MI355_EINVAL, "rope_any: n_tokens, Hq, Hkv, D, context_length out of range (D even)");
+    if (q_token_stride < (int64_t)Hq * D || k_token_stride < (int64_t)Hkv * D) return set_error(MI355_EINVAL, "rope_any: token strides shorter than a row");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32) return set_error(MI355_EDTYPE, "rope_any: dtype must be MI355_BF16 or MI355_FP32");
+    if (n_tokens == 0) return MI355_OK;
+    const int64_t wgs = (n_tokens * (Hq + Hkv) * (D / 2) + 255) / 256;
+    const dim3 grid((unsigned)(wgs < 0x7fffffffLL ? wgs : 0x7fffffffLL)), block(256);
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == MI355_BF16)
+        hipLaunchKernelGGL(rope_any_kernel<__bf16>, grid, block, 0, s, (__bf16*)q, (__bf16*)k, freq_cache, positions, q_token_stride,
+                           k_token_stride, n_tokens, Hq, Hkv, D / 2, context_length);
+    else
+        hipLaunchKernelGGL(rope_any_kernel<float>, grid, block, 0, s, (float*)q, (float*)k, freq_cache, positions, q_token_stride,
+                           k_token_stride, n_tokens, Hq, Hkv, D / 2, context_length);
+    const int rc = (int)hipGetLastError();
+    if (rc != 0) return set_error(rc, hipGetErrorString((hipError_t)rc));
+    return MI355_OK;
+}
+
 extern "C" int mi355_kv_cache_write(const void* k, const void* v, void* k_cache, void* v_cache, const int64_t* slot_mapping,
                                     int64_t num_blocks, int64_t T, int Hkv, int k_dim, int v_dim, int64_t k_token_stride,
                                     int64_t v_token_stride, int dtype, void* stream) {

@@ -1,9 +1,11 @@
 // The fused elementwise/normalisation ops that sit next to attention in a transformer
 // block: RMSNorm forward (optionally fused with the residual add in front of it),
 // silu(gate) * up, the end of a sublayer in a model with Dynamic Tanh norms and gated
-// residuals, the PolyNorm activation, and the token + position embedding.  All are
+// residuals, the PolyNorm activation, the token + position embedding, the RMS norm of an
+// fp32 residual stream with everything that is added to the stream in front of it, gated
+// and plain feed-forward activations, and the gated norm behind a recurrent mixer.  All are
 // streaming kernels: HBM-bound, 16-byte accesses, fp32 math, one rounding to bf16 per
-// stored value (the last three also exist with fp32 values throughout).
+// stored value (all but the first two also exist with fp32 values throughout).
 #include "common.hpp"
 #include "launch.hpp"
 
@@ -478,6 +480,255 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(EmbedPosParams<T> p) {
     }
 }
 
+// ---- fp32 residual stream + what a layer adds to it + RMS norm ------------------------------------
+//   x = resid + sub + sum_k routed[row * top + k] + embed[token]        (each term optional; no resid: zero)
+//   y = x / sqrt(mean(x^2) + eps) * (w_offset + w)
+// embed: the embedding output itself at the start of a model, or added again in front of a repeated pass.
+template <typename T>
+struct ResidualRmsParams {
+    const T* sub;
+    const T* routed;
+    const T* embed;
+    const int64_t* tokens;
+    const float* resid_in;
+    float* resid_out;            // may be resid_in; null: x is not kept
+    const float* w;
+    T* y;
+    int64_t n_rows, vocab, sub_stride, routed_stride, y_stride;      // resid and embed rows are contiguous
+    int n_cols, y_cols, top;     // columns n_cols .. y_cols - 1 of y are set to zero
+    float w_offset, eps;
+};
+
+template <typename T>
+__device__ __forceinline__ int64_t embed_row(const ResidualRmsParams<T>& p, int64_t row) {
+    return min(max(p.tokens[row], (int64_t)0), p.vocab - 1);           // (an id outside the table is clamped into it)
+}
+
+// WAVES wavefronts per row (1: four rows per workgroup, 4: one), the row held in registers as NCHUNK chunks of
+// 512 * WAVES elements.  Requires n_cols % 8 == 0, n_cols <= 512 * WAVES * NCHUNK, 16-byte aligned rows.
+template <typename T, int WAVES, int NCHUNK>
+__global__ __launch_bounds__(256) void residual_rms_rows_kernel(ResidualRmsParams<T> p) {
+    __shared__ float part[4];
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int64_t row = WAVES == 4 ? (int64_t)blockIdx.x : (int64_t)blockIdx.x * 4 + wave;
+    if (row >= p.n_rows) return;                                       // (uniform over the wavefronts that share a row)
+    const int first = (WAVES == 4 ? (int)threadIdx.x : lane) * 8;
+    const int64_t tok = p.embed ? embed_row(p, row) : 0;
+    float x[NCHUNK][8];
+    float ssq = 0.f;
+#pragma unroll
+    for (int c = 0; c < NCHUNK; ++c) {
+        const int col = c * (512 * WAVES) + first;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[c][e] = 0.f;
+        if (col < p.n_cols) {
+            if (p.resid_in) load8(p.resid_in + row * p.n_cols + col, x[c]);
+            float t[8];
+            if (p.sub) {
+                load8(p.sub + row * p.sub_stride + col, t);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) x[c][e] += t[e];
+            }
+            if (p.embed) {
+                load8(p.embed + tok * p.n_cols + col, t);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) x[c][e] += t[e];
+            }
+            for (int k = 0; k < (p.routed ? p.top : 0); ++k) {
+                load8(p.routed + (row * p.top + k) * p.routed_stride + col, t);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) x[c][e] += t[e];
+            }
+            if (p.resid_out) store8(p.resid_out + row * p.n_cols + col, x[c]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ssq = fmaf(x[c][e], x[c][e], ssq);
+        }
+    }
+    if (!p.y) return;
+    ssq = wave_sum(ssq);
+    if constexpr (WAVES == 4) {
+        if (lane == 0) part[wave] = ssq;
+        __syncthreads();
+        ssq = part[0] + part[1] + part[2] + part[3];
+    }
+    const float rstd = 1.0f / sqrtf(ssq / (float)p.n_cols + p.eps);
+    T* yr = p.y + row * p.y_stride;
+#pragma unroll
+    for (int c = 0; c < NCHUNK; ++c) {
+        const int col = c * (512 * WAVES) + first;
+        if (col < p.n_cols) {
+            float w[8], o[8];
+            load_param8(p.w, col, 0.f, w);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[e] = x[c][e] * rstd * (p.w_offset + w[e]);
+            store8(yr + col, o);
+        }
+    }
+    for (int col = p.n_cols + first / 8; col < p.y_cols; col += 64 * WAVES) yr[col] = (T)0.f;
+}
+
+// Any n_cols, any alignment: one wavefront per row, two passes.
+template <typename T>
+__global__ __launch_bounds__(256) void residual_rms_generic_kernel(ResidualRmsParams<T> p) {
+    const int lane = threadIdx.x & 63;
+    const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (row >= p.n_rows) return;
+    const int64_t tok = p.embed ? embed_row(p, row) : 0;
+    const auto value = [&](int col) {
+        float x = p.resid_in ? p.resid_in[row * p.n_cols + col] : 0.f;
+        if (p.sub) x += (float)p.sub[row * p.sub_stride + col];
+        if (p.embed) x += (float)p.embed[tok * p.n_cols + col];
+        for (int k = 0; k < (p.routed ? p.top : 0); ++k) x += (float)p.routed[(row * p.top + k) * p.routed_stride + col];
+        return x;
+    };
+    float ssq = 0.f;
+    for (int col = lane; col < p.n_cols; col += 64) {
+        const float x = value(col);
+        ssq = fmaf(x, x, ssq);
+    }
+    const float rstd = 1.0f / sqrtf(wave_sum(ssq) / (float)p.n_cols + p.eps);
+    for (int col = lane; col < p.n_cols; col += 64) {
+        const float x = value(col);                                    // (before resid_out, which may be resid_in, is written)
+        if (p.resid_out) p.resid_out[row * p.n_cols + col] = x;
+        if (p.y) p.y[row * p.y_stride + col] = (T)(x * rstd * (p.w_offset + (p.w ? p.w[col] : 0.f)));
+    }
+    if (p.y)
+        for (int col = p.n_cols + lane; col < p.y_cols; col += 64) p.y[row * p.y_stride + col] = (T)0.f;
+}
+
+// ---- feed-forward activations: out = silu(a) * b, or gelu(a) in its tanh form; times sigmoid(row_gate) per row ----
+template <typename T>
+struct FfActParams {
+    const T* a;
+    const T* b;                  // null: gelu(a)
+    const float* row_gate;       // optional, one logit per row
+    T* out;
+    int64_t n_rows, as, bs, os;
+    int n_cols;
+};
+
+template <bool FAST>
+__device__ __forceinline__ float gelu_tanh_of(float z) {
+    const float u = 0.7978845608028654f * fmaf(0.044715f * z * z, z, z);
+    // 1 + tanh(u) = 2 sigmoid(2u)
+    if constexpr (FAST) return z * sigmoid_of<true>(2.0f * u);
+    else return 0.5f * z * (1.0f + tanhf(u));
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void ff_act_vec8_kernel(FfActParams<T> p) {
+    constexpr bool FAST = sizeof(T) == 2;
+    const int groups = p.n_cols / 8;
+    const int64_t total = p.n_rows * groups;
+    for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = idx / groups;
+        const int col = (int)(idx % groups) * 8;
+        float a[8], b[8];
+        load8(p.a + row * p.as + col, a);
+        if (p.b) load8(p.b + row * p.bs + col, b);
+        const float f = p.row_gate ? sigmoid_of<FAST>(p.row_gate[row]) : 1.0f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) a[e] = f * (p.b ? a[e] * sigmoid_of<FAST>(a[e]) * b[e] : gelu_tanh_of<FAST>(a[e]));
+        store8(p.out + row * p.os + col, a);
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void ff_act_generic_kernel(FfActParams<T> p) {
+    constexpr bool FAST = sizeof(T) == 2;
+    const int64_t total = p.n_rows * p.n_cols;
+    for (int64_t idx = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; idx < total; idx += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = idx / p.n_cols;
+        const int col = (int)(idx % p.n_cols);
+        const float a = (float)p.a[row * p.as + col];
+        const float f = p.row_gate ? sigmoid_of<FAST>(p.row_gate[row]) : 1.0f;
+        p.out[row * p.os + col] = (T)(f * (p.b ? a * sigmoid_of<FAST>(a) * (float)p.b[row * p.bs + col] : gelu_tanh_of<FAST>(a)));
+    }
+}
+
+// ---- gated norm: v = y * silu(z); each of `groups` equal parts of a row divided by its root mean square; times w ----
+template <typename T>
+struct GatedNormParams {
+    const T* y;
+    const T* z;
+    const float* w;
+    T* out;
+    int64_t n_rows, ys, zs, os;
+    int part, groups;            // columns of a part, parts of a row
+    float eps;
+};
+
+// WAVES wavefronts per part of a row, as in residual_rms_rows_kernel.
+template <typename T, int WAVES, int NCHUNK>
+__global__ __launch_bounds__(256) void gated_norm_rows_kernel(GatedNormParams<T> p) {
+    constexpr bool FAST = sizeof(T) == 2;
+    __shared__ float sums[4];
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int64_t item = WAVES == 4 ? (int64_t)blockIdx.x : (int64_t)blockIdx.x * 4 + wave;
+    if (item >= p.n_rows * p.groups) return;
+    const int64_t row = item / p.groups;
+    const int base = (int)(item % p.groups) * p.part;
+    const int first = (WAVES == 4 ? (int)threadIdx.x : lane) * 8;
+    float v[NCHUNK][8];
+    float ssq = 0.f;
+#pragma unroll
+    for (int c = 0; c < NCHUNK; ++c) {
+        const int col = c * (512 * WAVES) + first;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[c][e] = 0.f;
+        if (col < p.part) {
+            float z[8];
+            load8(p.y + row * p.ys + base + col, v[c]);
+            load8(p.z + row * p.zs + base + col, z);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                v[c][e] *= z[e] * sigmoid_of<FAST>(z[e]);
+                ssq = fmaf(v[c][e], v[c][e], ssq);
+            }
+        }
+    }
+    ssq = wave_sum(ssq);
+    if constexpr (WAVES == 4) {
+        if (lane == 0) sums[wave] = ssq;
+        __syncthreads();
+        ssq = sums[0] + sums[1] + sums[2] + sums[3];
+    }
+    const float rstd = 1.0f / sqrtf(ssq / (float)p.part + p.eps);
+#pragma unroll
+    for (int c = 0; c < NCHUNK; ++c) {
+        const int col = c * (512 * WAVES) + first;
+        if (col < p.part) {
+            float w[8];
+            load_param8(p.w, base + col, 1.f, w);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[c][e] *= rstd * w[e];
+            store8(p.out + row * p.os + base + col, v[c]);
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void gated_norm_generic_kernel(GatedNormParams<T> p) {
+    constexpr bool FAST = sizeof(T) == 2;
+    const int lane = threadIdx.x & 63;
+    const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (item >= p.n_rows * p.groups) return;
+    const int64_t row = item / p.groups;
+    const int base = (int)(item % p.groups) * p.part;
+    const auto value = [&](int col) {
+        const float z = (float)p.z[row * p.zs + base + col];
+        return (float)p.y[row * p.ys + base + col] * (z * sigmoid_of<FAST>(z));
+    };
+    float ssq = 0.f;
+    for (int col = lane; col < p.part; col += 64) {
+        const float v = value(col);
+        ssq = fmaf(v, v, ssq);
+    }
+    const float rstd = 1.0f / sqrtf(wave_sum(ssq) / (float)p.part + p.eps);
+    for (int col = lane; col < p.part; col += 64)
+        p.out[row * p.os + base + col] = (T)(value(col) * rstd * (p.w ? p.w[base + col] : 1.f));
+}
+
 }  // namespace mi355
 
 using namespace mi355;
@@ -703,4 +954,147 @@ extern "C" int mi355_embed_pos_fwd(const void* embed, const void* pos, const int
     hipStream_t s = (hipStream_t)stream;
     return dtype == MI355_BF16 ? embed_pos<__bf16>(embed, pos, tokens, positions, out, n_rows, n_cols, vocab, n_positions, s)
                                : embed_pos<float>(embed, pos, tokens, positions, out, n_rows, n_cols, vocab, n_positions, s);
+}
+
+template <typename T>
+static int residual_rms(const ResidualRmsParams<T>& p, bool vec, hipStream_t s) {
+    const bool wide = vec && p.n_cols > 1024;
+    const int64_t wgs = wide ? p.n_rows : (p.n_rows + 3) / 4;
+    if (wgs > 0x7fffffffLL) return set_error(MI355_EINVAL, "residual_rms: too many rows");
+    const dim3 grid((unsigned)wgs), block(256);
+    if (!vec) hipLaunchKernelGGL(residual_rms_generic_kernel<T>, grid, block, 0, s, p);
+    else if (p.n_cols <= 512) hipLaunchKernelGGL((residual_rms_rows_kernel<T, 1, 1>), grid, block, 0, s, p);
+    else if (p.n_cols <= 1024) hipLaunchKernelGGL((residual_rms_rows_kernel<T, 1, 2>), grid, block, 0, s, p);
+    else if (p.n_cols <= 2048) hipLaunchKernelGGL((residual_rms_rows_kernel<T, 4, 1>), grid, block, 0, s, p);
+    else if (p.n_cols <= 4096) hipLaunchKernelGGL((residual_rms_rows_kernel<T, 4, 2>), grid, block, 0, s, p);
+    else if (p.n_cols <= 8192) hipLaunchKernelGGL((residual_rms_rows_kernel<T, 4, 4>), grid, block, 0, s, p);
+    else hipLaunchKernelGGL((residual_rms_rows_kernel<T, 4, 8>), grid, block, 0, s, p);
+    return launch_status();
+}
+
+template <typename T>
+static int residual_rms_args(const float* resid_in, float* resid_out, const void* sub, const void* routed, int top, const void* embed,
+                             const int64_t* tokens, int64_t vocab, const float* weight, float weight_offset, float eps, void* y,
+                             int64_t n_rows, int n_cols, int y_cols, int64_t sub_stride, int64_t routed_stride, int64_t y_stride,
+                             hipStream_t s) {
+    ResidualRmsParams<T> p;
+    p.sub = (const T*)sub;
+    p.routed = (const T*)routed;
+    p.embed = (const T*)embed;
+    p.tokens = tokens;
+    p.resid_in = resid_in;
+    p.resid_out = resid_out;
+    p.w = weight;
+    p.y = (T*)y;
+    p.n_rows = n_rows;
+    p.vocab = vocab;
+    p.sub_stride = sub_stride;
+    p.routed_stride = routed_stride;
+    p.y_stride = y_stride;
+    p.n_cols = n_cols;
+    p.y_cols = y_cols;
+    p.top = top;
+    p.w_offset = weight_offset;
+    p.eps = eps;
+    bool vec = n_cols % 8 == 0 && n_cols <= 16384 && ((sub_stride | routed_stride | y_stride) & 7) == 0;
+    for (const void* ptr : {sub, routed, embed, (const void*)resid_in, (const void*)resid_out, (const void*)weight, (const void*)y})
+        vec = vec && aligned16(ptr);
+    return residual_rms(p, vec, s);
+}
+
+extern "C" int mi355_residual_rms_fwd(const float* resid_in, float* resid_out, const void* sub, const void* routed, int top,
+                                      const void* embed, const int64_t* tokens, int64_t vocab, const float* weight,
+                                      float weight_offset, float eps, void* y, int64_t n_rows, int n_cols, int y_cols,
+                                      int64_t sub_row_stride, int64_t routed_row_stride, int64_t y_row_stride, int dtype,
+                                      void* stream) {
+    if (!resid_out && !y) return set_error(MI355_EINVAL, "residual_rms: no output");
+    if (!resid_in && !sub && !routed && !embed) return set_error(MI355_EINVAL, "residual_rms: no input");
+    if (embed && (!tokens || vocab <= 0)) return set_error(MI355_EINVAL, "residual_rms: an embedding table needs token ids and its row count");
+    if (routed && top <= 0) return set_error(MI355_EINVAL, "residual_rms: routed rows need top >= 1");
+    if (n_rows < 0 || n_cols <= 0 || (y && (y_cols < n_cols || y_row_stride < y_cols)))
+        return set_error(MI355_EINVAL, "residual_rms: n_rows, n_cols, y_cols out of range");
+    if (!(eps >= 0.f)) return set_error(MI355_EINVAL, "residual_rms: eps must be >= 0");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32) return set_error(MI355_EDTYPE, "residual_rms: dtype must be MI355_BF16 or MI355_FP32");
+    if (n_rows == 0) return MI355_OK;
+    hipStream_t s = (hipStream_t)stream;
+    return dtype == MI355_BF16
+               ? residual_rms_args<__bf16>(resid_in, resid_out, sub, routed, top, embed, tokens, vocab, weight, weight_offset, eps, y,
+                                           n_rows, n_cols, y_cols, sub_row_stride, routed_row_stride, y_row_stride, s)
+               : residual_rms_args<float>(resid_in, resid_out, sub, routed, top, embed, tokens, vocab, weight, weight_offset, eps, y,
+                                          n_rows, n_cols, y_cols, sub_row_stride, routed_row_stride, y_row_stride, s);
+}
+
+template <typename T>
+static int ff_act(const void* a, const void* b, const float* row_gate, void* out, int64_t n_rows, int n_cols, int64_t as, int64_t bs,
+                  int64_t os, hipStream_t s) {
+    FfActParams<T> p;
+    p.a = (const T*)a;
+    p.b = (const T*)b;
+    p.row_gate = row_gate;
+    p.out = (T*)out;
+    p.n_rows = n_rows;
+    p.as = as;
+    p.bs = bs;
+    p.os = os;
+    p.n_cols = n_cols;
+    if (n_cols % 8 == 0 && ((as | bs | os) & 7) == 0 && aligned16(a) && aligned16(b) && aligned16(out))
+        hipLaunchKernelGGL(ff_act_vec8_kernel<T>, dim3(grid_1d(n_rows * (int64_t)(n_cols / 8))), dim3(256), 0, s, p);
+    else
+        hipLaunchKernelGGL(ff_act_generic_kernel<T>, dim3(grid_1d(n_rows * (int64_t)n_cols)), dim3(256), 0, s, p);
+    return launch_status();
+}
+
+extern "C" int mi355_ff_act_fwd(const void* a, const void* b, const float* row_gate, void* out, int64_t n_rows, int n_cols,
+                                int64_t a_row_stride, int64_t b_row_stride, int64_t out_row_stride, int dtype, void* stream) {
+    if (!a || !out) return set_error(MI355_EINVAL, "ff_act: null pointer argument");
+    if (n_rows < 0 || n_cols <= 0) return set_error(MI355_EINVAL, "ff_act: n_rows, n_cols out of range");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32) return set_error(MI355_EDTYPE, "ff_act: dtype must be MI355_BF16 or MI355_FP32");
+    if (n_rows == 0) return MI355_OK;
+    hipStream_t s = (hipStream_t)stream;
+    return dtype == MI355_BF16 ? ff_act<__bf16>(a, b, row_gate, out, n_rows, n_cols, a_row_stride, b_row_stride, out_row_stride, s)
+                               : ff_act<float>(a, b, row_gate, out, n_rows, n_cols, a_row_stride, b_row_stride, out_row_stride, s);
+}
+
+template <typename T>
+static int gated_norm(const void* y, const void* z, const float* w, void* out, int64_t n_rows, int part, int groups, int64_t ys,
+                      int64_t zs, int64_t os, float eps, hipStream_t s) {
+    GatedNormParams<T> p;
+    p.y = (const T*)y;
+    p.z = (const T*)z;
+    p.w = w;
+    p.out = (T*)out;
+    p.n_rows = n_rows;
+    p.ys = ys;
+    p.zs = zs;
+    p.os = os;
+    p.part = part;
+    p.groups = groups;
+    p.eps = eps;
+    const bool vec = part % 8 == 0 && part <= 16384 && ((ys | zs | os) & 7) == 0 && aligned16(y) && aligned16(z) && aligned16(out) &&
+                     aligned16(w);
+    const bool wide = vec && part > 1024;
+    const int64_t items = n_rows * groups, wgs = wide ? items : (items + 3) / 4;
+    if (wgs > 0x7fffffffLL) return set_error(MI355_EINVAL, "gated_norm: too many rows");
+    const dim3 grid((unsigned)wgs), block(256);
+    if (!vec) hipLaunchKernelGGL(gated_norm_generic_kernel<T>, grid, block, 0, s, p);
+    else if (part <= 512) hipLaunchKernelGGL((gated_norm_rows_kernel<T, 1, 1>), grid, block, 0, s, p);
+    else if (part <= 1024) hipLaunchKernelGGL((gated_norm_rows_kernel<T, 1, 2>), grid, block, 0, s, p);
+    else if (part <= 2048) hipLaunchKernelGGL((gated_norm_rows_kernel<T, 4, 1>), grid, block, 0, s, p);
+    else if (part <= 4096) hipLaunchKernelGGL((gated_norm_rows_kernel<T, 4, 2>), grid, block, 0, s, p);
+    else if (part <= 8192) hipLaunchKernelGGL((gated_norm_rows_kernel<T, 4, 4>), grid, block, 0, s, p);
+    else hipLaunchKernelGGL((gated_norm_rows_kernel<T, 4, 8>), grid, block, 0, s, p);
+    return launch_status();
+}
+
+extern "C" int mi355_gated_norm_fwd(const void* y, const void* z, const float* weight, void* out, int64_t n_rows, int n_cols, int groups,
+                                    int64_t y_row_stride, int64_t z_row_stride, int64_t out_row_stride, float eps, int dtype,
+                                    void* stream) {
+    if (!y || !z || !out) return set_error(MI355_EINVAL, "gated_norm: null pointer argument");
+    if (n_rows < 0 || n_cols <= 0 || groups <= 0 || n_cols % groups) return set_error(MI355_EINVAL, "gated_norm: n_cols must be a positive multiple of groups");
+    if (!(eps >= 0.f)) return set_error(MI355_EINVAL, "gated_norm: eps must be >= 0");
+    if (dtype != MI355_BF16 && dtype != MI355_FP32) return set_error(MI355_EDTYPE, "gated_norm: dtype must be MI355_BF16 or MI355_FP32");
+    if (n_rows == 0) return MI355_OK;
+    hipStream_t s = (hipStream_t)stream;
+    return dtype == MI355_BF16 ? gated_norm<__bf16>(y, z, weight, out, n_rows, n_cols / groups, groups, y_row_stride, z_row_stride, out_row_stride, eps, s)
+                               : gated_norm<float>(y, z, weight, out, n_rows, n_cols / groups, groups, y_row_stride, z_row_stride, out_row_stride, eps, s);
 }

@@ -4,7 +4,7 @@
 // any token of a sequence whose keys and values already sit in the paged cache, its own included).  The keys are dealt to
 // the wavefronts in tiles of 64: a lane takes one key's dot product with the query, the wavefront runs an online softmax
 // over its tiles, and the lanes then own value columns while the tile's weights come from LDS.  The four partial results
-// meet in LDS.  Scores, weights and sums are fp32; keys and values are read as stored (bf16 or fp32).
+// meet in LDS.  With a sliding window only the blocks that hold visible keys are walked.  Scores, weights and sums are fp32; keys and values are read as stored (bf16 or fp32).
 #include "common.hpp"
 #include "launch.hpp"
 
@@ -23,6 +23,7 @@ struct PagedAnyParams {
     int64_t q_stride, out_stride, bt_stride;      // elements between query rows / output rows / table rows
     int64_t rows;
     int B, Hq, Hkv, Dk, Dv, num_blocks, max_blocks;
+    int window, keep_first;           // window 0: every earlier key is visible
     float scale_log2;
 };
 
@@ -53,7 +54,8 @@ __global__ __launch_bounds__(kAnyWaves * 64) void paged_attn_any_kernel(PagedAny
     }
     // keys 0 .. n_keys - 1 are visible: the row is token (context - chunk length + row - q_start) of its sequence
     const int ctx = min(p.context_lens[b], 16 * p.max_blocks);
-    const int n_keys = min(ctx, ctx - (q_end - q_start) + (int)(row - q_start) + 1);
+    const VisibleKeys vis = visible_keys(min(ctx, ctx - (q_end - q_start) + (int)(row - q_start) + 1), p.window, p.keep_first);
+    const int n_keys = vis.n;
     const T* q = (const T*)p.q + row * p.q_stride + (int64_t)h * p.Dk;
     for (int d = threadIdx.x; d < p.Dk; d += kAnyWaves * 64) q_lds[d] = (float)q[d];
     __syncthreads();
@@ -69,8 +71,8 @@ __global__ __launch_bounds__(kAnyWaves * 64) void paged_attn_any_kernel(PagedAny
         const int key = k0 + lane;
         float x = -INFINITY;
         // a block id outside the pool (a corrupted table) is clamped into it
-        const int my_blk = min(max(bt[min(key, n_keys - 1) >> 4], 0), p.num_blocks - 1);
-        if (key < n_keys) {
+        const int my_blk = min(max(bt[vis.logical_block(min(key, n_keys - 1) >> 4)], 0), p.num_blocks - 1);
+        if (key < n_keys && !vis.hidden(key)) {
             const T* kr = kc + (((int64_t)my_blk * p.Hkv + hk) * 16 + (key & 15)) * p.Dk;
             float dot = 0.f;
             for (int d = 0; d < p.Dk; d += 8) {             // rows are multiples of 8 elements, 16-byte aligned
@@ -95,7 +97,7 @@ __global__ __launch_bounds__(kAnyWaves * 64) void paged_attn_any_kernel(PagedAny
         float mx = x;
 #pragma unroll
         for (int off = 32; off >= 1; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
-        const float m_new = fmaxf(m, mx);                   // finite: lane 0's key is visible
+        const float m_new = fmaxf(m, mx);                   // finite: at most 30 keys of a tile are hidden, and the last key is visible
         const float alpha = fast_exp2(m - m_new);           // 0 the first time
         m = m_new;
         const float w = fast_exp2(x - m);
@@ -161,12 +163,12 @@ static int launch_any(const PagedAnyParams& p, hipStream_t s) {
 
 using namespace mi355;
 
-extern "C" int mi355_paged_attn_any_fwd(const void* q, const void* k_cache, const void* v_cache, void* out, int64_t q_row_stride,
+static int paged_attn_any_common(const void* q, const void* k_cache, const void* v_cache, void* out, int64_t q_row_stride,
                                         int64_t out_row_stride, int64_t n_rows, const int32_t* cu_seqlens_q,
                                         const int32_t* block_tables, int64_t bt_row_stride, int64_t max_blocks,
                                         const int32_t* context_lens, const float* head_scale, const float* sink, int B, int Hq,
                                         int Hkv, int Dk, int Dv, int block_size, int64_t num_blocks, float softmax_scale,
-                                        int dtype, void* stream) {
+                                        int window, int keep_first, int dtype, void* stream) {
     if (!q || !k_cache || !v_cache || !out || !block_tables || !context_lens)
         return set_error(MI355_EINVAL, "paged_attn_any: null pointer argument");
     if (dtype != MI355_BF16 && dtype != MI355_FP32)
@@ -183,6 +185,7 @@ extern "C" int mi355_paged_attn_any_fwd(const void* q, const void* k_cache, cons
         return set_error(MI355_EINVAL, "paged_attn_any: the caches must be 16-byte aligned");
     if (q_row_stride < (int64_t)Hq * Dk || out_row_stride < (int64_t)Hq * Dv)
         return set_error(MI355_EINVAL, "paged_attn_any: row strides shorter than a row");
+    if (window < 0 || keep_first < 0) return set_error(MI355_EINVAL, "paged_attn_any: window and keep_first must not be negative");
     if (n_rows * Hq > 0x7fffffffLL) return set_error(MI355_EINVAL, "paged_attn_any: too many rows");
     if (n_rows == 0) return MI355_OK;
     PagedAnyParams p;
@@ -206,8 +209,32 @@ extern "C" int mi355_paged_attn_any_fwd(const void* q, const void* k_cache, cons
     p.Dv = Dv;
     p.num_blocks = (int)num_blocks;
     p.max_blocks = (int)max_blocks;
+    p.window = window;
+    p.keep_first = keep_first;
     p.scale_log2 = softmax_scale * kLog2e;
     const int rc = dtype == MI355_BF16 ? launch_any<__bf16>(p, (hipStream_t)stream) : launch_any<float>(p, (hipStream_t)stream);
     if (rc != 0) return set_error(rc, hipGetErrorString((hipError_t)rc));
     return MI355_OK;
+}
+
+extern "C" int mi355_paged_attn_any_fwd(const void* q, const void* k_cache, const void* v_cache, void* out, int64_t q_row_stride,
+                                        int64_t out_row_stride, int64_t n_rows, const int32_t* cu_seqlens_q,
+                                        const int32_t* block_tables, int64_t bt_row_stride, int64_t max_blocks,
+                                        const int32_t* context_lens, const float* head_scale, const float* sink, int B, int Hq,
+                                        int Hkv, int Dk, int Dv, int block_size, int64_t num_blocks, float softmax_scale,
+                                        int dtype, void* stream) {
+    return paged_attn_any_common(q, k_cache, v_cache, out, q_row_stride, out_row_stride, n_rows, cu_seqlens_q, block_tables,
+                                 bt_row_stride, max_blocks, context_lens, head_scale, sink, B, Hq, Hkv, Dk, Dv, block_size, num_blocks,
+                                 softmax_scale, 0, 0, dtype, stream);
+}
+
+extern "C" int mi355_paged_attn_any_fwd_window(const void* q, const void* k_cache, const void* v_cache, void* out, int64_t q_row_stride,
+                                               int64_t out_row_stride, int64_t n_rows, const int32_t* cu_seqlens_q,
+                                               const int32_t* block_tables, int64_t bt_row_stride, int64_t max_blocks,
+                                               const int32_t* context_lens, const float* head_scale, const float* sink, int B, int Hq,
+                                               int Hkv, int Dk, int Dv, int block_size, int64_t num_blocks, float softmax_scale,
+                                               int window, int keep_first, int dtype, void* stream) {
+    return paged_attn_any_common(q, k_cache, v_cache, out, q_row_stride, out_row_stride, n_rows, cu_seqlens_q, block_tables,
+                                 bt_row_stride, max_blocks, context_lens, head_scale, sink, B, Hq, Hkv, Dk, Dv, block_size, num_blocks,
+                                 softmax_scale, window, keep_first, dtype, stream);
 }

@@ -57,6 +57,8 @@ struct DecodeParams {
     int tokens_per_wave;      // 256, 512 or 1024: a long stream per wavefront amortises its start-up latency
     float scale_log2;
     int64_t q_stride;         // elements from one sequence's query row to the next
+    int64_t out_stride;       // ... and from one output row to the next
+    int window, keep_first;   // sliding window with kept first tokens (window 0: none); the keys are then walked as one compact run
     // optional per-query-head terms: a factor on the scores, and a sink (a score without key or value, natural-log
     // units, not scaled) that enters the softmax denominator once
     const float* head_scale;
@@ -85,7 +87,7 @@ struct DecodeLds {
 // that three workgroups share a CU (3 x 52 KiB of LDS): with ragged lengths many workgroups have idle
 // wavefronts, and a third resident workgroup fills in (+1 % on a log-uniform batch, -0.7 % on equal lengths).
 // The bf16 instance needs 70 KiB of LDS per workgroup: two per CU whatever the registers.
-template <int D, bool FP8>
+template <int D, bool FP8, bool WINDOW>
 __global__ __launch_bounds__(kDecodeWaves * 64) __attribute__((amdgpu_waves_per_eu(FP8 ? 3 : 2, FP8 ? 3 : 2)))
 void paged_decode_split_kernel(DecodeParams p) {
     constexpr int NS = D / 32;                       // MFMA k-steps of K.Q^T
@@ -128,7 +130,9 @@ void paged_decode_split_kernel(DecodeParams p) {
     const int hk = item % p.Hkv;
     const int b = (item / p.Hkv) % p.B;
     const int chunk = p.max_chunks - 1 - item / (p.Hkv * p.B);
-    const int ctx = min(p.context_lens[b], p.max_ctx);     // a length beyond the promised bound is truncated, never chased
+    // a length beyond the promised bound is truncated, never chased; with a window, ctx counts the compact run of keys
+    const VisibleKeys vis = visible_keys(min(p.context_lens[b], p.max_ctx), WINDOW ? p.window : 0, WINDOW ? p.keep_first : 0);
+    const int ctx = WINDOW ? vis.n : min(p.context_lens[b], p.max_ctx);
     const int chunk_tokens = kDecodeWaves * p.tokens_per_wave;
     const int chunk_start = chunk * chunk_tokens;
     if (chunk_start >= ctx) return;
@@ -175,7 +179,7 @@ void paged_decode_split_kernel(DecodeParams p) {
     // every id is a real block.  The step loop reads them with v_readlane, so no dependent
     // table load sits between two steps.
     // a block id outside the pool (a corrupted table) is clamped into it: wrong numbers, never a wild read
-    const int my_phys = min(max(bt[min(t0 / kBlock + lane, last_blk)], 0), p.num_blocks - 1);
+    const int my_phys = min(max(bt[vis.logical_block(min(t0 / kBlock + lane, last_blk))], 0), p.num_blocks - 1);
     float my_ks = 1.0f, my_vs = 1.0f;
     if constexpr (FP8) {
         my_ks = p.k_scale[(int64_t)my_phys * p.Hkv + hk];
@@ -326,7 +330,8 @@ void paged_decode_split_kernel(DecodeParams p) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 float v = s_acc[t][i] * sc;
-                if (tail && kbase + 16 * t + 4 * kg + i >= t1) v = -INFINITY;
+                const int key = kbase + 16 * t + 4 * kg + i;
+                if (tail && (key >= t1 || (WINDOW && vis.hidden(key)))) v = -INFINITY;
                 x[4 * t + i] = v;
                 mx = fmaxf(mx, v);
             }
@@ -372,9 +377,15 @@ void paged_decode_split_kernel(DecodeParams p) {
         // the NEXT iteration, i.e. the prefetch is undone.
         asm volatile("" ::: "memory");
     };
-    for (int it = 0; it + 1 < n_iter; ++it) step(it, std::false_type{});
+    for (int it = 0; it + 1 < n_iter; ++it) {
+        // (a step that meets the hidden keys of the seam -- never all of its 32 keys -- blanks them like a tail)
+        const int kbase = t0 + it * kStage;
+        if (WINDOW && kbase < vis.hid1 && kbase + kStage > vis.hid0) step(it, std::true_type{});
+        else step(it, std::false_type{});
+    }
     if (n_iter > 0) {
-        if ((t1 - t0) % kStage == 0) step(n_iter - 1, std::false_type{});
+        if (WINDOW) step(n_iter - 1, std::true_type{});
+        else if ((t1 - t0) % kStage == 0) step(n_iter - 1, std::false_type{});
         else step(n_iter - 1, std::true_type{});
     }
 
@@ -413,7 +424,7 @@ void paged_decode_split_kernel(DecodeParams p) {
         }
         const int64_t row = (int64_t)b * p.Hq + h0 + qi;
         if (n_chunks == 1) {
-            p.out[row * D + d] = (__bf16)(num / (den + sink_weight(p, h0 + qi, M)));
+            p.out[(int64_t)b * p.out_stride + (int64_t)(h0 + qi) * D + d] = (__bf16)(num / (den + sink_weight(p, h0 + qi, M)));
         } else {
             const int64_t slot = row * p.max_chunks + chunk;
             p.ws_o[slot * D + d] = num;
@@ -434,7 +445,7 @@ __global__ __launch_bounds__(kCombineThreads) void paged_decode_combine_kernel(D
     const int row = blockIdx.x * (kCombineThreads / kLanesPerRow) + threadIdx.x / kLanesPerRow;      // b * Hq + h
     if (row >= p.B * p.Hq) return;
     const int b = row / p.Hq;
-    const int ctx = min(p.context_lens[b], p.max_ctx);
+    const int ctx = visible_keys(min(p.context_lens[b], p.max_ctx), p.window, p.keep_first).n;
     const int chunk_tokens = kDecodeWaves * p.tokens_per_wave;
     const int n_chunks = (ctx + chunk_tokens - 1) / chunk_tokens;
     if (n_chunks <= 1) return;                   // written by the split pass (or empty)
@@ -455,7 +466,7 @@ __global__ __launch_bounds__(kCombineThreads) void paged_decode_combine_kernel(D
     u32x2 w;
     w[0] = pack_bf16(num[0] / den, num[1] / den);
     w[1] = pack_bf16(num[2] / den, num[3] / den);
-    *reinterpret_cast<u32x2*>(p.out + (int64_t)row * D + d) = w;
+    *reinterpret_cast<u32x2*>(p.out + (int64_t)b * p.out_stride + (int64_t)(row % p.Hq) * D + d) = w;
 }
 
 // Combine for sequences of many chunks (a small batch of long contexts runs short chunks, see tokens_per_wave_for: one
@@ -470,7 +481,7 @@ __global__ __launch_bounds__(kCombineThreads) void paged_decode_combine_wide_ker
     __shared__ f32x4 s_num[kGroups][kLanesPerRow];
     const int row = blockIdx.x;                    // b * Hq + h
     const int b = row / p.Hq;
-    const int ctx = min(p.context_lens[b], p.max_ctx);
+    const int ctx = visible_keys(min(p.context_lens[b], p.max_ctx), p.window, p.keep_first).n;
     const int chunk_tokens = kDecodeWaves * p.tokens_per_wave;
     const int n_chunks = (ctx + chunk_tokens - 1) / chunk_tokens;
     if (n_chunks <= 1) return;                   // written by the split pass (or empty); the whole workgroup leaves
@@ -511,7 +522,7 @@ __global__ __launch_bounds__(kCombineThreads) void paged_decode_combine_wide_ker
     u32x2 w;
     w[0] = pack_bf16(tot[0] / dtot, tot[1] / dtot);
     w[1] = pack_bf16(tot[2] / dtot, tot[3] / dtot);
-    *reinterpret_cast<u32x2*>(p.out + (int64_t)row * D + d) = w;
+    *reinterpret_cast<u32x2*>(p.out + (int64_t)b * p.out_stride + (int64_t)(row % p.Hq) * D + d) = w;
 }
 
 // The wide combine serves launches of more than kWideCombineChunks chunks per sequence and at most kWideCombineRows rows
@@ -520,10 +531,17 @@ __global__ __launch_bounds__(kCombineThreads) void paged_decode_combine_wide_ker
 constexpr int kWideCombineChunks = 4;
 constexpr int kWideCombineRows = 2048;
 
+template <int D, bool FP8, bool WINDOW>
+static int launch_decode_split(const DecodeParams& p, hipStream_t stream) {
+    dim3 grid((unsigned)p.max_chunks * p.Hkv * p.n_groups * p.B);
+    hipLaunchKernelGGL((paged_decode_split_kernel<D, FP8, WINDOW>), grid, dim3(kDecodeWaves * 64), 0, stream, p);
+    return (int)hipGetLastError();
+}
+
 template <int D, bool FP8>
 static int launch_decode(const DecodeParams& p, hipStream_t stream) {
-    dim3 grid((unsigned)p.max_chunks * p.Hkv * p.n_groups * p.B);
-    hipLaunchKernelGGL((paged_decode_split_kernel<D, FP8>), grid, dim3(kDecodeWaves * 64), 0, stream, p);
+    const int rc = p.window > 0 ? launch_decode_split<D, FP8, true>(p, stream) : launch_decode_split<D, FP8, false>(p, stream);
+    if (rc != 0) return rc;
     if (p.max_chunks > kWideCombineChunks && (int64_t)p.B * p.Hq <= kWideCombineRows) {
         hipLaunchKernelGGL((paged_decode_combine_wide_kernel<D>), dim3((unsigned)(p.B * p.Hq)), dim3(kCombineThreads), 0,
                            stream, p);
@@ -593,7 +611,8 @@ static int decode_common(const void* q, const void* k_cache, const void* v_cache
                          const float* k_scale, const float* v_scale, void* workspace, size_t workspace_bytes,
                          bool static_scratch, int B, int Hq, int Hkv, int D, int block_size, int64_t num_blocks,
                          int max_ctx, float softmax_scale, int kv_dtype, void* stream, int64_t q_stride = 0,
-                         const float* head_scale = nullptr, const float* sink = nullptr) {
+                         const float* head_scale = nullptr, const float* sink = nullptr, int64_t out_stride = 0, int window = 0,
+                         int keep_first = 0) {
     if (!q || !k_cache || !v_cache || !out || !block_tables || !context_lens)
         return set_error(MI355_EINVAL, "paged_decode: null pointer argument");
     if (B <= 0 || Hq <= 0 || Hkv <= 0 || max_ctx <= 0)
@@ -603,8 +622,10 @@ static int decode_common(const void* q, const void* k_cache, const void* v_cache
     if (block_size != kBlock) return set_error(MI355_EINVAL, "paged_decode: block_size must be 16");
     if (num_blocks <= 0 || num_blocks > 0x7fffffffLL)
         return set_error(MI355_EINVAL, "paged_decode: num_blocks must be positive (and below 2^31)");
-    const int chunk = mi355_paged_decode_chunk_tokens(B, Hq, Hkv, max_ctx);
-    if ((int64_t)((max_ctx + chunk - 1) / chunk) * Hkv * n_groups * B > 0x7fffffffLL)
+    if (window < 0 || keep_first < 0) return set_error(MI355_EINVAL, "paged_decode: window and keep_first must not be negative");
+    const int max_keys = max_visible_keys(max_ctx, window, keep_first);      // what a launch walks of one sequence
+    const int chunk = mi355_paged_decode_chunk_tokens(B, Hq, Hkv, max_keys);
+    if ((int64_t)((max_keys + chunk - 1) / chunk) * Hkv * n_groups * B > 0x7fffffffLL)
         return set_error(MI355_EINVAL, "paged_decode: chunks * Hkv * B exceeds the grid limit");
     if (kv_dtype != MI355_BF16 && kv_dtype != MI355_FP8_E4M3)
         return set_error(MI355_EDTYPE, "paged_decode: kv_dtype must be MI355_BF16 or MI355_FP8_E4M3");
@@ -613,7 +634,7 @@ static int decode_common(const void* q, const void* k_cache, const void* v_cache
         return set_error(MI355_EINVAL, "paged_decode: fp8 KV cache needs k_scale and v_scale");
     if (!(D == 128 || D == 64 || (D == 32 && !fp8)))
         return set_error(MI355_EINVAL, "paged_decode: head_dim must be 64 or 128 (or 32 with a bf16 cache)");
-    const int max_chunks = (max_ctx + chunk - 1) / chunk;
+    const int max_chunks = (max_keys + chunk - 1) / chunk;
     const size_t need = workspace_layout_bytes((size_t)B * Hq * max_chunks, (size_t)D);   // <= the reported bound
     if (static_scratch) {
         if (max_chunks > 1 && need > workspace_bytes)
@@ -654,6 +675,9 @@ static int decode_common(const void* q, const void* k_cache, const void* v_cache
     p.tokens_per_wave = chunk / kDecodeWaves;
     p.scale_log2 = softmax_scale * kLog2e;
     p.q_stride = q_stride ? q_stride : (int64_t)Hq * D;
+    p.out_stride = out_stride ? out_stride : (int64_t)Hq * D;
+    p.window = window;
+    p.keep_first = keep_first;
     p.head_scale = head_scale;
     p.sink = sink;
 
@@ -692,6 +716,21 @@ extern "C" int mi355_paged_decode_fwd_headwise(const void* q, int64_t q_row_stri
     return decode_common(q, k_cache, v_cache, out, block_tables, bt_row_stride, context_lens, k_scale, v_scale, workspace,
                          workspace_bytes, false, B, Hq, Hkv, D, block_size, num_blocks, max_ctx, softmax_scale, kv_dtype,
                          stream, q_row_stride, head_scale, sink);
+}
+
+extern "C" int mi355_paged_decode_fwd_window(const void* q, int64_t q_row_stride, const void* k_cache, const void* v_cache,
+                                             void* out, int64_t out_row_stride, const int32_t* block_tables,
+                                             int64_t bt_row_stride, const int32_t* context_lens, const float* k_scale,
+                                             const float* v_scale, const float* head_scale, const float* sink, void* workspace,
+                                             size_t workspace_bytes, int B, int Hq, int Hkv, int D, int block_size,
+                                             int64_t num_blocks, int max_ctx, float softmax_scale, int window, int keep_first,
+                                             int kv_dtype, void* stream) {
+    if (q_row_stride < (int64_t)Hq * D || (q_row_stride & 7) || ((uintptr_t)q & 15) || out_row_stride < (int64_t)Hq * D ||
+        (out_row_stride & 7) || ((uintptr_t)out & 15))
+        return set_error(MI355_EINVAL, "paged_decode_window: q and out must be 16-byte aligned, their row strides multiples of 8 and at least Hq * D");
+    return decode_common(q, k_cache, v_cache, out, block_tables, bt_row_stride, context_lens, k_scale, v_scale, workspace,
+                         workspace_bytes, false, B, Hq, Hkv, D, block_size, num_blocks, max_ctx, softmax_scale, kv_dtype,
+                         stream, q_row_stride, head_scale, sink, out_row_stride, window, keep_first);
 }
 
 // ---- the variant that allocates nothing -------------------------------------------------------------------

@@ -44,7 +44,9 @@ constexpr int kBN = 64;    // keys per LDS tile
 // workgroups per compute unit, 7-8 % faster at throughput shapes and 14 % on short sequences, a handful of spilled
 // registers outside the tile loop.  Head_dim 32 has two workgroups per compute unit as it is (117 registers; a third
 // would need 85 and spills by the hundred: three to four times slower), head_dim 128 needs its 250.
-template <int D, int MODE, bool PAGED = false>
+// WINDOW (causal): a query tile walks the K/V tiles that hold the kept first tokens, then those from its window's first
+// key on, as one sequence of tiles (tile_of); keys outside are masked in the tiles at the window's lower edge.
+template <int D, int MODE, bool PAGED = false, bool WINDOW = false>
 __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_kernel(PrefillParams p) {
     constexpr int NS = D / 16;                    // MFMA k-steps of K.Q^T
     constexpr int NDT = D / 32;                   // 32-row tiles of O^T
@@ -232,7 +234,14 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
 
         int kv_end = sk;
         if (causal) kv_end = max(0, min(sk, min(sq, q0 + kBM) + coff));
-        const int n_tiles = (kv_end + kBN - 1) / kBN;
+        int n_tiles = (kv_end + kBN - 1) / kBN;
+        int kept_tiles = 0, skip = 0;              // WINDOW: tiles with kept tokens, and tiles left out behind them
+        if constexpr (WINDOW) {
+            kept_tiles = (p.keep_first + kBN - 1) / kBN;
+            skip = max(0, max(0, q0 + coff - p.window + 1) / kBN - kept_tiles);
+            n_tiles -= skip;
+        }
+        const auto tile_of = [&](int t) { return WINDOW && t >= kept_tiles ? t + skip : t; };
         int t0 = 0, t1 = n_tiles;                  // this workgroup's tiles
         if (p.n_split > 1) {
             const int per = (n_tiles + p.n_split - 1) / p.n_split;
@@ -244,7 +253,7 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
         __syncthreads();                     // the previous query tile's readers are done with the LDS buffers
 #pragma unroll
         for (int i = 0; i < kAhead; ++i)
-            if (t0 + i < t1) issue_tile(t0 + i, (t0 + i) & (NB - 1));
+            if (t0 + i < t1) issue_tile(tile_of(t0 + i), (t0 + i) & (NB - 1));
 
         // ---- Q^T fragments: step s covers d = 16s + 8kg + j ----------------------
         // rows come in whole (CPR lanes per row) and go through the wavefront's slab (private, and LDS operations
@@ -288,6 +297,12 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
         int n_plain = sk / kBN;
         if (causal) n_plain = min(n_plain, max(0, qw0 + coff + 1) / kBN);
         if (boolmask) n_plain = 0;
+        int n_low = 0;                             // WINDOW: leading tiles that may hold keys outside some query's window
+        if constexpr (WINDOW) {
+            const auto compact = [&](int t) { return t < kept_tiles ? t : max(kept_tiles, t - skip); };
+            n_low = min(n_tiles, compact((max(0, qw0 + 32 + coff - p.window) + kBN - 1) / kBN));
+            n_plain = max(n_low, compact(n_plain));
+        }
         n_plain = min(n_plain, n_tiles);
 
         f32x16 s_acc[2];
@@ -334,10 +349,11 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
             __syncthreads();                 // ... and everybody's; also: all are done reading the buffer of the tile before
 
             // The loads of the tile that takes that buffer go out first: the work of kAhead tiles hides their latency.
-            if (tile + kAhead < t1) issue_tile(tile + kAhead, (tile + kAhead) & (NB - 1));
+            if (tile + kAhead < t1) issue_tile(tile_of(tile + kAhead), (tile + kAhead) & (NB - 1));
 
-            const int k0 = tile * kBN;
+            const int k0 = tile_of(tile) * kBN;
             if (causal && MASKED && k0 > qw0 + 31 + coff) return false;
+            if (WINDOW && MASKED && k0 >= p.keep_first && k0 + kBN - 1 <= qw0 + coff - p.window) return false;    // below every window
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
 #pragma unroll
@@ -357,6 +373,7 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
                         const int key = k0 + 32 * t + 8 * (i >> 2) + 4 * kg + (i & 3);
                         bool keep = key < sk;
                         if constexpr (causal) keep = keep & (key <= qi + coff);
+                        if constexpr (WINDOW) keep = keep & ((qi + coff - key < p.window) | (key < p.keep_first));
                         // unconditional, clamped byte load: no divergent control flow around the select
                         if constexpr (boolmask) keep = keep & (mrow[min(key, sk - 1)] != 0);
                         s_acc[t][i] = keep ? s_acc[t][i] : -INFINITY;
@@ -472,20 +489,21 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
             neg_ref = -kBias;
             set_buf(t0 & (NB - 1));          // the offsets start at the first tile's buffer
             cur_tile = t0;
-            run_tiles_preset(std::false_type{}, t0, min(n_plain, t1));
+            if constexpr (WINDOW) run_tiles_preset(std::true_type{}, t0, n_low);
+            run_tiles_preset(std::false_type{}, max(n_low, t0), min(n_plain, t1));
             run_tiles_preset(std::true_type{}, max(n_plain, t0), t1);
             const float l = xor32_sum(l_run);
             // (a query that sees none of this share's keys -- causal with fewer keys than queries, or a share of split
-            // keys that lies past its diagonal -- has a sum of zero by right)
+            // keys that lies past its diagonal, or a padded lane behind the last query's window -- has a sum of zero by right)
             const int k_first = t0 * kBN;
-            const bool sees = t0 < t1 && k_first < sk && (!causal || k_first <= qi + coff);
+            const bool sees = t0 < t1 && k_first < sk && (!causal || k_first <= qi + coff) && (!WINDOW || q_ok);
             const bool bad = redo || (sees && !(l >= kUnderflow)) || !(l <= kOverflow);
             // the workgroup meets (everybody is done with the K/V buffers) and votes
             if (__syncthreads_or(bad ? 1 : 0)) {
                 tracked = true;
 #pragma unroll
                 for (int i = 0; i < kAhead; ++i)
-                    if (t0 + i < t1) issue_tile(t0 + i, (t0 + i) & (NB - 1));
+                    if (t0 + i < t1) issue_tile(tile_of(t0 + i), (t0 + i) & (NB - 1));
 #pragma unroll
                 for (int i = 0; i < NDT; ++i)
 #pragma unroll
@@ -498,7 +516,8 @@ __global__ __launch_bounds__(kPfWaves * 64, D == 64 ? 4 : 1) void prefill_fwd_ke
         if (tracked) {
             set_buf(t0 & (NB - 1));
             cur_tile = t0;
-            run_tiles(std::false_type{}, t0, min(n_plain, t1));
+            if constexpr (WINDOW) run_tiles(std::true_type{}, t0, n_low);
+            run_tiles(std::false_type{}, max(n_low, t0), min(n_plain, t1));
             run_tiles(std::true_type{}, max(n_plain, t0), t1);
         }
 
@@ -582,7 +601,9 @@ static int launch_prefill(const PrefillParams& p0, hipStream_t stream) {
     // one workgroup per PAIR of query tiles (or per tile), 1-D in x (see the id remap); y = share of the keys
     dim3 grid((unsigned)(p.n_pairs * p.Hq * p.B), (unsigned)(p.n_split > 1 ? p.n_split : 1));
     dim3 block(kPfWaves * 64);
-    if (p.mask_mode == MI355_MASK_CAUSAL)
+    if (p.mask_mode == MI355_MASK_CAUSAL && p.window > 0)
+        hipLaunchKernelGGL((prefill_fwd_kernel<D, MI355_MASK_CAUSAL, false, true>), grid, block, 0, stream, p);
+    else if (p.mask_mode == MI355_MASK_CAUSAL)
         hipLaunchKernelGGL((prefill_fwd_kernel<D, MI355_MASK_CAUSAL>), grid, block, 0, stream, p);
     else if (p.mask_mode == MI355_MASK_BOOL)
         hipLaunchKernelGGL((prefill_fwd_kernel<D, MI355_MASK_BOOL>), grid, block, 0, stream, p);
@@ -672,7 +693,10 @@ template <int D>
 static int launch_prefill_paged(const PrefillParams& p0, hipStream_t stream) {
     const PrefillParams p = with_units(p0);
     dim3 grid((unsigned)(p.n_pairs * p.Hq * p.B), (unsigned)(p.n_split > 1 ? p.n_split : 1));
-    hipLaunchKernelGGL((prefill_fwd_kernel<D, MI355_MASK_CAUSAL, true>), grid, dim3(kPfWaves * 64), 0, stream, p);
+    if (p.window > 0)
+        hipLaunchKernelGGL((prefill_fwd_kernel<D, MI355_MASK_CAUSAL, true, true>), grid, dim3(kPfWaves * 64), 0, stream, p);
+    else
+        hipLaunchKernelGGL((prefill_fwd_kernel<D, MI355_MASK_CAUSAL, true>), grid, dim3(kPfWaves * 64), 0, stream, p);
     return (int)hipGetLastError();
 }
 
@@ -712,7 +736,8 @@ static int prefill_common(const void* q, const void* k, const void* v, void* out
                           const int64_t mask_strides[3], int B, int Hq, int Hkv, int Sq_max, int Sk_max, int D,
                           float softmax_scale, int mask_mode, int dtype, float* lse, const int64_t* lse_strides,
                           void* stream, int n_split = 1, int64_t total_q_rows = 0, void* workspace = nullptr,
-                          size_t workspace_bytes = 0, const float* head_scale = nullptr, const float* sink = nullptr) {
+                          size_t workspace_bytes = 0, const float* head_scale = nullptr, const float* sink = nullptr,
+                          int window = 0, int keep_first = 0) {
     if (!q || !k || !v || !out || !q_strides || !k_strides || !v_strides || !o_strides)
         return set_error(MI355_EINVAL, "prefill: null pointer argument");
     if (dtype != MI355_BF16) return set_error(MI355_EDTYPE, "prefill: dtype must be MI355_BF16");
@@ -726,6 +751,8 @@ static int prefill_common(const void* q, const void* k, const void* v, void* out
         return set_error(MI355_EINVAL, "prefill: unknown mask_mode");
     if (mask_mode == MI355_MASK_BOOL && (!mask || !mask_strides || cu_seqlens_q))
         return set_error(MI355_EINVAL, "prefill: MI355_MASK_BOOL needs mask + mask_strides and the dense layout");
+    if (window < 0 || keep_first < 0 || (window > 0 && (mask_mode != MI355_MASK_CAUSAL || lse || n_split > 1)))
+        return set_error(MI355_EINVAL, "prefill: a window is causal, without lse and without split keys; window and keep_first must not be negative");
     for (int i = 0; i < 3; ++i) {
         if ((q_strides[i] | k_strides[i] | v_strides[i] | o_strides[i]) & 7)
             return set_error(MI355_EINVAL, "prefill: strides must be multiples of 8 elements (16-byte rows)");
@@ -762,6 +789,8 @@ static int prefill_common(const void* q, const void* k, const void* v, void* out
     p.head_scale = head_scale;
     p.sink = sink;
     p.mask_mode = mask_mode;
+    p.window = window;
+    p.keep_first = keep_first;
     p.n_qtiles = (Sq_max + kBM - 1) / kBM;
     p.n_pairs = (p.n_qtiles + 1) / 2;
     p.single_tiles = 0;
@@ -833,7 +862,9 @@ static int prefill_paged_common(const void* q, const void* k_cache, const void* 
                                 const int32_t* context_lens, const float* head_scale, const float* sink,
                                 int B, int Hq, int Hkv, int Sq_max, int D, int block_size, int64_t num_blocks,
                                 float softmax_scale, int kv_dtype, int n_split, int64_t total_q_rows,
-                                void* workspace, size_t workspace_bytes, void* stream) {
+                                void* workspace, size_t workspace_bytes, void* stream, int window = 0, int keep_first = 0) {
+    if (window < 0 || keep_first < 0 || (window > 0 && n_split > 1))
+        return set_error(MI355_EINVAL, "prefill_paged: window and keep_first must not be negative, and a window has no split keys");
     if (!q || !k_cache || !v_cache || !out || !cu_seqlens_q || !block_tables || !context_lens)
         return set_error(MI355_EINVAL, "prefill_paged: null pointer argument");
     if (kv_dtype != MI355_BF16) return set_error(MI355_EDTYPE, "prefill_paged: the cache must be MI355_BF16");
@@ -870,6 +901,8 @@ static int prefill_paged_common(const void* q, const void* k_cache, const void* 
     p.head_scale = head_scale;
     p.sink = sink;
     p.mask_mode = MI355_MASK_CAUSAL;
+    p.window = window;
+    p.keep_first = keep_first;
     p.n_qtiles = (Sq_max + kBM - 1) / kBM;
     p.n_pairs = (p.n_qtiles + 1) / 2;
     p.single_tiles = 0;
@@ -913,6 +946,27 @@ extern "C" int mi355_prefill_paged_fwd_headwise(const void* q, const void* k_cac
     return prefill_paged_common(q, k_cache, v_cache, out, q_token_stride, out_token_stride, cu_seqlens_q, block_tables,
                                 table_stride, max_blocks, context_lens, head_scale, sink, B, Hq, Hkv, Sq_max, D, block_size,
                                 num_blocks, softmax_scale, kv_dtype, n_split, total_q_rows, workspace, workspace_bytes, stream);
+}
+
+extern "C" int mi355_prefill_paged_fwd_window(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                              int64_t q_token_stride, int64_t out_token_stride, const int32_t* cu_seqlens_q,
+                                              const int32_t* block_tables, int64_t table_stride, int64_t max_blocks,
+                                              const int32_t* context_lens, const float* head_scale, const float* sink, int B,
+                                              int Hq, int Hkv, int Sq_max, int D, int block_size, int64_t num_blocks,
+                                              float softmax_scale, int window, int keep_first, int kv_dtype, void* stream) {
+    return prefill_paged_common(q, k_cache, v_cache, out, q_token_stride, out_token_stride, cu_seqlens_q, block_tables,
+                                table_stride, max_blocks, context_lens, head_scale, sink, B, Hq, Hkv, Sq_max, D, block_size,
+                                num_blocks, softmax_scale, kv_dtype, 1, 0, nullptr, 0, stream, window, keep_first);
+}
+
+extern "C" int mi355_prefill_fwd_window(const void* q, const void* k, const void* v, void* out, const int64_t q_strides[3],
+                                        const int64_t k_strides[3], const int64_t v_strides[3], const int64_t o_strides[3],
+                                        const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, const float* head_scale,
+                                        const float* sink, int B, int Hq, int Hkv, int Sq_max, int Sk_max, int D,
+                                        float softmax_scale, int window, int keep_first, int dtype, void* stream) {
+    return prefill_common(q, k, v, out, q_strides, k_strides, v_strides, o_strides, cu_seqlens_q, cu_seqlens_k, nullptr,
+                          nullptr, B, Hq, Hkv, Sq_max, Sk_max, D, softmax_scale, MI355_MASK_CAUSAL, dtype, nullptr, nullptr,
+                          stream, 1, 0, nullptr, 0, head_scale, sink, window, keep_first);
 }
 
 extern "C" size_t mi355_prefill_splitkv_workspace_bytes(int64_t total_q_rows, int Hq, int D, int n_split) {

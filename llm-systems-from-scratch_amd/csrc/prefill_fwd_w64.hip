@@ -1016,6 +1016,7 @@ __global__ __launch_bounds__(kWWaves * 64, 1) void prefill_fwd_w64_kernel(Prefil
 // The kernel multiplies head and row strides as 32-bit numbers (batch strides stay 64-bit), and keeps one number per
 // sequence of a packed batch in LDS.
 bool prefill_w64_takes(const PrefillParams& p) {
+    if (p.window > 0) return false;                  // (sliding windows: the 8-wavefront kernel)
     const int64_t strides[] = {p.qs[1], p.qs[2], p.ks[1], p.ks[2], p.vs[1], p.vs[2], p.os[1], p.os[2], p.lse ? p.ls[1] : 0};
     for (int64_t v : strides)
         if (v < 0 || v > 0x7fffffffLL) return false;

@@ -26,6 +26,7 @@ struct PrefillParams {
     const float* head_scale;
     const float* sink;
     int mask_mode;
+    int window, keep_first;               // causal only: query i sees key j when i - j < window or j < keep_first (window 0: every key j <= i)
     int n_qtiles;
     int n_pairs;                          // units per (batch, head) of the 8-wavefront kernel's grid: pairs of query tiles, or ...
     int single_tiles;                     // ... single query tiles when this is set (launches that would not fill the GPU)

@@ -18,8 +18,15 @@ llm-core/llm_core/model.py:308-325 and the SDPA slot at model.py:382):
     dyt_residual(resid, sub, gate=, post=, norm=)       # gated residual add between Dynamic Tanh norms
     polynorm(z, coeffs, eps)                            # PolyNorm activation
     embed_pos(embed, pos, tokens, positions)            # token + learned position embedding, fp32
+    rope_rotate(q, k, positions, freq_cache)            # RoPE in place, any head size, bf16 or fp32
+    residual_rms(resid, weight, sub=, routed=, embed=)  # everything added to an fp32 residual stream + RMSNorm
+    ff_act(a, b)                                        # silu(a) * b, or gelu(a)
+    gated_norm(y, z, weight, groups, eps)               # y silu(z) with a norm per group
+    ssm_mix(proj, ...)                                  # Mamba-2: causal convolution + selective state, prompts and decode
+    moe_route(h, w, bias, top), moe_experts(h, ids, weights, w_gate_up, w_down)         # mixture of experts
 
-Models (paged cache, batched prefill and decode, sampling): load_model(folder), CachedTransformerLM, ZuzelornLM.
+Models (paged cache, batched prefill and decode, sampling): load_model(folder), CachedTransformerLM, ZuzelornLM,
+ZomipelLM.
 
 Every function runs on the HIP library; there is no CPU or PyTorch fallback.
 """
@@ -33,6 +40,14 @@ from .ops import (  # noqa: F401
     dyt_residual,
     polynorm,
     embed_pos,
+    build_partial_rope_cache,
+    rope_rotate,
+    residual_rms,
+    ff_act,
+    gated_norm,
+    ssm_mix,
+    moe_route,
+    moe_experts,
     kv_cache_write,
     paged_attention_any,
     flash_attn_paged_prefill,
@@ -47,8 +62,9 @@ from .ops import (  # noqa: F401
     scaled_dot_product_attention,
     sdpa_slot,
 )
-from .engine import AttentionLayer, BlockAllocator, OutOfBlocks, PagedAttentionEngine  # noqa: F401
+from .engine import AttentionLayer, BlockAllocator, OutOfBlocks, PagedAttentionEngine, StateLayer  # noqa: F401
 from .model import CachedLM, CachedTransformerLM  # noqa: F401
 from .registry import ARCHITECTURES, UnsupportedDtype, load_model, model_class  # noqa: F401
+from .zomipel import ZomipelLM  # noqa: F401
 from .zuzelorn import ZuzelornLM  # noqa: F401
 from ._lib import LIB_PATH, LibraryMissing, load  # noqa: F401

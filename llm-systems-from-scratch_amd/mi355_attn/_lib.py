@@ -16,6 +16,9 @@ MI355_FP32 = 2
 MASK_NONE, MASK_CAUSAL, MASK_BOOL = 0, 1, 2
 STATIC_SCRATCH_BYTES = 16 << 20          # MI355_STATIC_SCRATCH_BYTES
 
+SCANS = {"auto": 0, "serial": 1, "chunked": 2}
+TILINGS = {"auto": 0, "skinny": 1, "large": 2}
+
 _i64x3 = C.c_int64 * 3
 _i64x2 = C.c_int64 * 2
 _lib = None
@@ -48,10 +51,32 @@ EXPORTS = (
     "mi355_dyt_residual_fwd",
     "mi355_polynorm_fwd",
     "mi355_embed_pos_fwd",
+    "mi355_prefill_fwd_window",
+    "mi355_prefill_paged_fwd_window",
+    "mi355_paged_decode_fwd_window",
+    "mi355_paged_attn_any_fwd_window",
+    "mi355_rope_any",
+    "mi355_residual_rms_fwd",
+    "mi355_ff_act_fwd",
+    "mi355_gated_norm_fwd",
+    "mi355_ssm_prefill",
+    "mi355_ssm_decode",
+    "mi355_moe_route",
+    "mi355_moe_group",
+    "mi355_moe_gate_up",
+    "mi355_moe_down",
     "mi355_calib_copy",
     "mi355_last_error",
     "mi355_version",
 )
+
+
+class SsmArgs(C.Structure):
+    """mi355_ssm_args"""
+    _fields_ = ([(n, C.c_void_p) for n in ("proj", "conv_weight", "conv_bias", "dt_bias", "neg_a", "d_skip", "conv_state", "ssm_state",
+                                           "slots", "positions", "cu_seqlens", "xbc", "y")] +
+                [(n, C.c_int64) for n in ("proj_row_stride", "xbc_col", "dt_col", "y_row_stride", "n_rows")] +
+                [(n, C.c_int) for n in ("batch", "heads", "vdim", "state", "groups", "taps", "n_slots", "dtype")])
 
 
 class LibraryMissing(RuntimeError):
@@ -163,6 +188,39 @@ def load():
     lib.mi355_polynorm_fwd.argtypes = [vp, vp, i64, i32, i64, i64, C.c_float * 4, f32, i32, vp]
     lib.mi355_embed_pos_fwd.restype = i32
     lib.mi355_embed_pos_fwd.argtypes = [vp, vp, vp, vp, vp, i64, i32, i64, i64, i32, vp]
+    lib.mi355_prefill_fwd_window.restype = i32
+    lib.mi355_prefill_fwd_window.argtypes = [vp, vp, vp, vp, _i64x3, _i64x3, _i64x3, _i64x3, vp, vp, vp, vp,
+                                             i32, i32, i32, i32, i32, i32, f32, i32, i32, i32, vp]
+    lib.mi355_prefill_paged_fwd_window.restype = i32
+    lib.mi355_prefill_paged_fwd_window.argtypes = [vp, vp, vp, vp, i64, i64, vp, vp, i64, i64, vp, vp, vp,
+                                                   i32, i32, i32, i32, i32, i32, i64, f32, i32, i32, i32, vp]
+    lib.mi355_paged_decode_fwd_window.restype = i32
+    lib.mi355_paged_decode_fwd_window.argtypes = [vp, i64, vp, vp, vp, i64, vp, i64, vp, vp, vp, vp, vp, vp, sz,
+                                                  i32, i32, i32, i32, i32, i64, i32, f32, i32, i32, i32, vp]
+    lib.mi355_paged_attn_any_fwd_window.restype = i32
+    lib.mi355_paged_attn_any_fwd_window.argtypes = [vp, vp, vp, vp, i64, i64, i64, vp, vp, i64, i64, vp, vp, vp,
+                                                    i32, i32, i32, i32, i32, i32, i64, f32, i32, i32, i32, vp]
+    lib.mi355_rope_any.restype = i32
+    lib.mi355_rope_any.argtypes = [vp, vp, vp, vp, i64, i32, i32, i32, i32, i64, i64, i32, vp]
+    lib.mi355_residual_rms_fwd.restype = i32
+    lib.mi355_residual_rms_fwd.argtypes = [vp, vp, vp, vp, i32, vp, vp, i64, vp, f32, f32, vp, i64, i32, i32, i64, i64, i64,
+                                           i32, vp]
+    lib.mi355_ff_act_fwd.restype = i32
+    lib.mi355_ff_act_fwd.argtypes = [vp, vp, vp, vp, i64, i32, i64, i64, i64, i32, vp]
+    lib.mi355_gated_norm_fwd.restype = i32
+    lib.mi355_gated_norm_fwd.argtypes = [vp, vp, vp, vp, i64, i32, i32, i64, i64, i64, f32, i32, vp]
+    lib.mi355_ssm_prefill.restype = i32
+    lib.mi355_ssm_prefill.argtypes = [C.POINTER(SsmArgs), i32, vp]
+    lib.mi355_ssm_decode.restype = i32
+    lib.mi355_ssm_decode.argtypes = [C.POINTER(SsmArgs), vp]
+    lib.mi355_moe_route.restype = i32
+    lib.mi355_moe_route.argtypes = [vp, vp, vp, vp, vp, vp, i64, i64, i64, i32, i32, i32, i32, vp]
+    lib.mi355_moe_group.restype = i32
+    lib.mi355_moe_group.argtypes = [vp, i64, i32, vp, vp, vp]
+    lib.mi355_moe_gate_up.restype = i32
+    lib.mi355_moe_gate_up.argtypes = [vp, vp, vp, vp, vp, i64, i64, i64, i32, i32, i32, i32, i32, i32, vp]
+    lib.mi355_moe_down.restype = i32
+    lib.mi355_moe_down.argtypes = [vp, vp, vp, vp, vp, vp, i64, i64, i64, i32, i32, i32, i32, i32, i32, vp]
     lib.mi355_calib_copy.restype = i32
     lib.mi355_calib_copy.argtypes = [vp, vp, sz, vp]
     lib.mi355_last_error.restype = C.c_char_p

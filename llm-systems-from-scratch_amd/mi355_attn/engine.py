@@ -6,13 +6,14 @@ allocator, per-sequence block tables, slot mapping for cache writes, a prefill c
 admitted sequences and a decode call that serves every running sequence with one kernel launch
 per layer and step.  The bookkeeping (blocks, lengths, tables) is shared by all attention layers
 of a model; every layer has its own K/V pools, of its own head count and head sizes, or reads those
-of an earlier layer (`AttentionLayer`).  A step is planned once (`plan_prefill`,
+of an earlier layer (`AttentionLayer`); a recurrent layer has a fixed-size state per sequence instead, in the sequence's
+state slot (`StateLayer`).  A step is planned once (`plan_prefill`,
 `plan_decode`: host integers -> a few small device tensors) and then applied per layer
-(`attend_prefill`, `attend_decode`).  Projections, sampling and the scheduler policy stay with
+(`attend_prefill`, `attend_decode`, `advance_state`).  Projections, sampling and the scheduler policy stay with
 the caller.
 
-All tensor work runs on the HIP kernels (rope_and_cache, kv_cache_write, flash_attn_varlen_prefill,
-flash_attn_paged_prefill, paged_attention_decode, paged_attention_any); the bookkeeping here is plain Python on host integers.
+All tensor work runs on the HIP kernels (rope_and_cache, rope_rotate, kv_cache_write, flash_attn_varlen_prefill,
+flash_attn_paged_prefill, paged_attention_decode, paged_attention_any, ssm_mix); the bookkeeping here is plain Python on host integers.
 """
 from __future__ import annotations
 
@@ -35,7 +36,10 @@ class AttentionLayer:
     """One attention layer as the cache manager sees it.  head_dim is the size of a query/key head, v_dim of a value
     head (None: head_dim).  kv_from = i: the layer has no keys and values of its own and reads layer i's pools.
     softmax_scale None: 1/sqrt(head_dim).  head_scale (non-negative factor per query head) and sinks (score without key
-    or value per query head) are fp32 (n_q_heads,) tensors or None.  rope: rotate q and k by the position."""
+    or value per query head) are fp32 (n_q_heads,) tensors or None.  rope: rotate adjacent pairs of q and k by the position;
+    rope_base None: with the engine's rope_theta over the whole head, else the first rope_dims (None: all) entries of a head
+    turn, pair i by rope_base^(-2i/rope_dims) per position.  window > 0: the token at position i sees position j when i - j <
+    window or j < keep_first."""
     n_q_heads: int
     n_kv_heads: int
     head_dim: int
@@ -45,6 +49,26 @@ class AttentionLayer:
     head_scale: torch.Tensor | None = None
     sinks: torch.Tensor | None = None
     rope: bool = True
+    rope_base: float | None = None
+    rope_dims: int | None = None
+    window: int = 0
+    keep_first: int = 0
+
+
+@dataclass
+class StateLayer:
+    """One Mamba-2 mixer as the state manager sees it: per sequence the last `taps` inputs of its convolution and, in fp32, a
+    (state x vdim) matrix per head.  params: the fp32 tensors that ops.ssm_mix takes."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    taps: int
+    params: dict
+
+    @property
+    def channels(self) -> int:
+        return self.heads * self.vdim + 2 * self.groups * self.state
 
 
 def cache_head_dims(kv_dtype: str, head_dim: int, v_dim: int) -> tuple[int, int, bool]:
@@ -95,6 +119,7 @@ class PrefillPlan:
     context_lens: torch.Tensor | None = None  # (B,) int32: tokens in the cache, this chunk included
     total_context: int = 0                    # their sum (sizes the dequantised rows of an fp8 cache)
     cu_context: torch.Tensor | None = None    # (B+1,) int32: their running sum (fp8 cache: where each sequence's rows start)
+    state_slots: torch.Tensor | None = None   # (B,) int32: where each sequence's recurrent state lives
     # packed keys and values of layers that later layers share (new sequences only), by layer
     packed: dict[int, tuple] = field(default_factory=dict)
 
@@ -106,18 +131,19 @@ class DecodePlan:
     tables: torch.Tensor         # (B, max_blocks) int32
     context_lens: torch.Tensor   # (B,) int32, the new token included
     max_context: int
+    state_slots: torch.Tensor | None = None      # (B,) int32
 
 
 class StaticDecodeStep:
     """Device tensors of one decode step at fixed addresses, refreshed from the host by one copy.
 
     Layout of the int32 buffer: token ids (int64), slots (int64), positions, context lengths,
-    block tables (batch x max_blocks)."""
+    state slots, block tables (batch x max_blocks)."""
 
     def __init__(self, batch: int, max_blocks: int, device):
         B, M = batch, max_blocks
         self.batch, self.max_blocks = B, M
-        n = 6 * B + B * M
+        n = 7 * B + B * M
         self._dev = torch.zeros(n, dtype=torch.int32, device=device)
         self._host = torch.zeros(n, dtype=torch.int32, pin_memory=True)
         self._copied = torch.cuda.Event()
@@ -126,19 +152,21 @@ class StaticDecodeStep:
         slots = self._dev[2 * B:4 * B].view(torch.int64)
         positions = self._dev[4 * B:5 * B]
         context_lens = self._dev[5 * B:6 * B]
-        tables = self._dev[6 * B:].view(B, M)
-        self.plan = DecodePlan(positions, slots, tables, context_lens, M * BLOCK)
+        tables = self._dev[7 * B:].view(B, M)
+        self.plan = DecodePlan(positions, slots, tables, context_lens, M * BLOCK, self._dev[6 * B:7 * B])
         h = self._host
         self._h_tokens, self._h_slots = h[0:2 * B].view(torch.int64), h[2 * B:4 * B].view(torch.int64)
-        self._h_positions, self._h_ctx, self._h_tables = h[4 * B:5 * B], h[5 * B:6 * B], h[6 * B:].view(B, M)
+        self._h_positions, self._h_ctx, self._h_state = h[4 * B:5 * B], h[5 * B:6 * B], h[6 * B:7 * B]
+        self._h_tables = h[7 * B:].view(B, M)
 
-    def fill(self, tokens, slots, positions, context_lens, block_lists) -> None:
+    def fill(self, tokens, slots, positions, context_lens, block_lists, state_slots) -> None:
         if self._pending:
             self._copied.synchronize()              # the previous copy has left the staging buffer
         self._h_tokens.copy_(torch.tensor(tokens, dtype=torch.int64))
         self._h_slots.copy_(torch.tensor(slots, dtype=torch.int64))
         self._h_positions.copy_(torch.tensor(positions, dtype=torch.int32))
         self._h_ctx.copy_(torch.tensor(context_lens, dtype=torch.int32))
+        self._h_state.copy_(torch.tensor(state_slots, dtype=torch.int32))
         for i, blocks in enumerate(block_lists):
             self._h_tables[i, :len(blocks)] = torch.tensor(blocks, dtype=torch.int32)
         self._dev.copy_(self._host, non_blocking=True)
@@ -148,10 +176,12 @@ class StaticDecodeStep:
 
 class PagedAttentionEngine:
     def __init__(self, num_blocks, n_q_heads=None, n_kv_heads=None, head_dim=None, context_length=None, *, rope_theta=10000.0,
-                 max_batch=256, num_layers=1, kv_dtype="bf16", device="cuda:0", layers: list[AttentionLayer] | None = None):
+                 max_batch=256, num_layers=1, kv_dtype="bf16", device="cuda:0",
+                 layers: list[AttentionLayer | StateLayer] | None = None):
         """Either n_q_heads, n_kv_heads, head_dim and num_layers (equal layers with RoPE) or `layers`.  kv_dtype: "bf16",
         "fp8" (e4m3 + scales) or "fp32" (pools, queries and outputs in fp32, general attention kernel).
-        q, k and v of layer i come with the head sizes cache_dims[i] (padded with zeros where a head is smaller)."""
+        q, k and v of layer i come with the head sizes cache_dims[i] (padded with zeros where a head is smaller).  With state
+        layers at most max_batch sequences exist at a time."""
         self.device = torch.device(device)
         if context_length is None:
             raise ValueError("context_length is required")
@@ -167,26 +197,44 @@ class PagedAttentionEngine:
         self.num_layers = len(layers)
         self.context_length = context_length
         self.kv_dtype = kv_dtype
-        self.Hq, self.Hkv, self.D = layers[0].n_q_heads, layers[0].n_kv_heads, layers[0].head_dim
+        attention = [ly for ly in layers if isinstance(ly, AttentionLayer)]
+        if attention:
+            self.Hq, self.Hkv, self.D = attention[0].n_q_heads, attention[0].n_kv_heads, attention[0].head_dim
         cache_dtype = {"bf16": torch.bfloat16, "fp8": torch.uint8, "fp32": torch.float32}[kv_dtype]      # uint8 = e4m3 bit patterns
         self.k_caches, self.v_caches, self.cache_dims, self.mfma = [], [], [], []
         # per-(block, kv head) scales of an fp8 cache, maintained by the cache write
         self.k_scales, self.v_scales = ([], []) if kv_dtype == "fp8" else (None, None)
-        self.shared = {ly.kv_from for ly in layers if ly.kv_from is not None}
-        rope_dims = set()
+        self.shared = {ly.kv_from for ly in attention if ly.kv_from is not None}
+        self.conv_states, self.ssm_states = {}, {}        # by state layer
+        rope_dims, tables = set(), {}
+        self.freq_caches = []                             # by layer: its cos/sin table or None
         for i, ly in enumerate(layers):
+            if isinstance(ly, StateLayer):
+                act = torch.float32 if kv_dtype == "fp32" else torch.bfloat16
+                self.conv_states[i] = torch.zeros(max_batch, ly.taps, ly.channels, dtype=act, device=self.device)
+                self.ssm_states[i] = torch.zeros(max_batch, ly.heads, ly.state, (ly.vdim + 3) // 4 * 4, dtype=torch.float32,
+                                                 device=self.device)
+                for per_layer in (self.k_caches, self.v_caches, self.cache_dims, self.mfma, self.freq_caches):
+                    per_layer.append(None)
+                if kv_dtype == "fp8":
+                    self.k_scales.append(None)
+                    self.v_scales.append(None)
+                continue
             if ly.n_q_heads < 1 or ly.n_kv_heads < 1 or ly.n_q_heads % ly.n_kv_heads:
                 raise ValueError(f"layer {i}: {ly.n_q_heads} query heads over {ly.n_kv_heads} kv heads")
             kd, vd, mfma = cache_head_dims(kv_dtype, ly.head_dim, ly.v_dim or ly.head_dim)
-            if ly.rope and (not mfma or kd != ly.head_dim or (ly.v_dim or kd) != kd):
+            if ly.rope and ly.rope_base is None and (not mfma or kd != ly.head_dim or (ly.v_dim or kd) != kd):
                 raise ValueError(f"layer {i}: RoPE needs equal head sizes of 32, 64 or 128 and a 16- or 8-bit cache")
+            if ly.window < 0 or ly.keep_first < 0:
+                raise ValueError(f"layer {i}: window and keep_first must not be negative")
             self.cache_dims.append((kd, vd))
             self.mfma.append(mfma)
             src = ly.kv_from
             if src is not None:
-                if not 0 <= src < i or layers[src].kv_from is not None:
+                if not 0 <= src < i or not isinstance(layers[src], AttentionLayer) or layers[src].kv_from is not None:
                     raise ValueError(f"layer {i}: kv_from {src} is not an earlier layer with keys and values of its own")
-                if layers[src].n_kv_heads != ly.n_kv_heads or self.cache_dims[src] != (kd, vd) or layers[src].rope != ly.rope:
+                if layers[src].n_kv_heads != ly.n_kv_heads or self.cache_dims[src] != (kd, vd) \
+                        or any(getattr(layers[src], n) != getattr(ly, n) for n in ("rope", "rope_base", "rope_dims")):
                     raise ValueError(f"layer {i}: kv heads, head sizes and rotation differ from those of layer {src}, whose cache it reads")
                 self.k_caches.append(self.k_caches[src])
                 self.v_caches.append(self.v_caches[src])
@@ -197,24 +245,35 @@ class PagedAttentionEngine:
                 for sc in (self.k_scales, self.v_scales):
                     sc.append(sc[src] if src is not None else
                               torch.ones(num_blocks, ly.n_kv_heads, dtype=torch.float32, device=self.device))
-            if ly.rope:
+            key = None
+            if ly.rope and ly.rope_base is None:
                 rope_dims.add(kd)
+                key = kd
+                if key not in tables:
+                    tables[key] = ops.build_rope_cache(context_length, kd, rope_theta, self.device)
+            elif ly.rope:
+                key = (kd, ly.head_dim if ly.rope_dims is None else ly.rope_dims, float(ly.rope_base))
+                if key not in tables:
+                    tables[key] = ops.build_partial_rope_cache(context_length, *key, self.device)
+            self.freq_caches.append(tables.get(key))
         # layers on the general kernel read every key through the tables, also in the first chunk of a prompt
-        self.always_tables = not all(self.mfma)
+        self.always_tables = any(m is False for m in self.mfma)
         if len(rope_dims) > 1:
             raise ValueError("layers with RoPE must share one head size")
-        self.freq_cache = ops.build_rope_cache(context_length, rope_dims.pop(), rope_theta, self.device) if rope_dims else None
+        self.freq_cache = next((t for t in self.freq_caches if t is not None), None)
         # rotation by the angle 0 (cos 1, sin 0, every position clamped to the one row) for layers without RoPE on an fp8 cache
         self._no_rotation = {d: torch.stack((torch.ones(1, d // 2), torch.zeros(1, d // 2))).to(self.device)
-                             for d in {kd for kd, _ in self.cache_dims}} if kv_dtype == "fp8" else None
+                             for d in {dims[0] for dims in self.cache_dims if dims}} if kv_dtype == "fp8" else None
         self.allocator = BlockAllocator(num_blocks)
         self.blocks: dict[int, list[int]] = {}      # sequence id -> physical blocks
         self.lengths: dict[int, int] = {}           # sequence id -> tokens in the cache
+        self.state_slots: dict[int, int] = {}       # sequence id -> state slot (models with state layers)
+        self._free_slots = list(range(max_batch - 1, -1, -1))
         self.max_blocks_per_seq = (context_length + BLOCK - 1) // BLOCK
         # persistent step buffers: no allocation on the decode path besides the kernel outputs
         self._tables = torch.zeros(max_batch, self.max_blocks_per_seq, dtype=torch.int32, device=self.device)
         self._workspace = max((ops.paged_decode_workspace(max_batch, hq, d, context_length, self.device)
-                               for hq, d in {(ly.n_q_heads, kd) for ly, (kd, _), m in zip(layers, self.cache_dims, self.mfma) if m}),
+                               for hq, d in {(ly.n_q_heads, dims[0]) for ly, dims, m in zip(layers, self.cache_dims, self.mfma) if m}),
                               key=lambda t: t.numel(), default=None)
         self.max_batch = max_batch
 
@@ -231,12 +290,21 @@ class PagedAttentionEngine:
     def add_sequence(self, seq_id: int) -> None:
         if seq_id in self.blocks:
             raise ValueError(f"sequence {seq_id} already exists")
+        if self.conv_states:
+            if not self._free_slots:
+                raise OutOfBlocks(f"all {self.max_batch} state slots are taken")
+            self.state_slots[seq_id] = self._free_slots.pop()
         self.blocks[seq_id] = []
         self.lengths[seq_id] = 0
 
     def remove_sequence(self, seq_id: int) -> None:
         self.allocator.free(self.blocks.pop(seq_id))
         del self.lengths[seq_id]
+        if seq_id in self.state_slots:
+            self._free_slots.append(self.state_slots.pop(seq_id))       # (a new sequence starts from zero whatever the slot holds)
+
+    def _slots_of(self, seq_ids) -> torch.Tensor | None:
+        return torch.tensor([self.state_slots[s] for s in seq_ids], dtype=torch.int32, device=self.device) if self.conv_states else None
 
     def _reserve(self, seq_id: int, n_new: int) -> list[int]:
         """Slots for the next n_new tokens of a sequence (allocates blocks as needed)."""
@@ -280,7 +348,8 @@ class PagedAttentionEngine:
         plan = PrefillPlan(torch.tensor(positions, dtype=torch.int32, device=dev),
                            torch.tensor(slots, dtype=torch.int64, device=dev),
                            torch.tensor(cu, dtype=torch.int32, device=dev), max(lens),
-                           torch.tensor([c - 1 for c in cu[1:]], dtype=torch.int64, device=dev))
+                           torch.tensor([c - 1 for c in cu[1:]], dtype=torch.int64, device=dev),
+                           state_slots=self._slots_of(seq_ids))
         if chunked or self.always_tables:
             max_blk = max(len(self.blocks[sid]) for sid in seq_ids)
             rows = torch.zeros(len(seq_ids), max_blk, dtype=torch.int32)
@@ -331,7 +400,8 @@ class PagedAttentionEngine:
         tables.copy_(rows, non_blocking=False)
         return DecodePlan(torch.tensor(positions, dtype=torch.int32, device=dev),
                           torch.tensor(slots, dtype=torch.int64, device=dev), tables,
-                          torch.tensor([p + 1 for p in positions], dtype=torch.int32, device=dev), max_blk * BLOCK)
+                          torch.tensor([p + 1 for p in positions], dtype=torch.int32, device=dev), max_blk * BLOCK,
+                          self._slots_of(seq_ids))
 
     def make_static_decode(self, batch: int) -> "StaticDecodeStep":
         """Fixed device tensors for decode steps of `batch` sequences (what a captured HIP graph needs:
@@ -349,7 +419,7 @@ class PagedAttentionEngine:
             raise ValueError("seq_ids, tokens and the static buffers disagree on the batch size")
         positions, slots = self._reserve_decode(seq_ids)
         static.fill([int(t) for t in tokens], slots, positions, [p + 1 for p in positions],
-                    [self.blocks[s] for s in seq_ids])
+                    [self.blocks[s] for s in seq_ids], [self.state_slots.get(s, 0) for s in seq_ids])
         return static.plan
 
     # ---- attention calls (once per layer) -----------------------------------------
@@ -363,28 +433,32 @@ class PagedAttentionEngine:
             return (q, None) if k_out else q
         kc, vc = self.k_caches[layer], self.v_caches[layer]
         rope = self.layers[layer].rope
+        if rope and (not self.mfma[layer] or self.cache_dims[layer][0] != self.cache_dims[layer][1]):
+            ops.rope_rotate(q, k, plan.positions, self.freq_caches[layer])          # (in place)
+            rope = False
         if self.kv_dtype == "fp8":
-            freq = self.freq_cache if rope else self._no_rotation[q.shape[2]]
+            freq = self.freq_caches[layer] if rope else self._no_rotation[q.shape[2]]
             return ops.rope_and_cache_fp8(q, k, v, plan.positions, freq, kc, vc, self.k_scales[layer],
                                           self.v_scales[layer], plan.slots, k_out=k_out)
         if rope:
-            return ops.rope_and_cache(q, k, v, plan.positions, self.freq_cache, kc, vc, plan.slots, k_out=k_out)
+            return ops.rope_and_cache(q, k, v, plan.positions, self.freq_caches[layer], kc, vc, plan.slots, k_out=k_out)
         ops.kv_cache_write(k, v, kc, vc, plan.slots)
         return (q, k) if k_out else q
 
     def _score_terms(self, layer: int):
         ly = self.layers[layer]
         scale = 1.0 / math.sqrt(ly.head_dim) if ly.softmax_scale is None else ly.softmax_scale        # (of the unpadded head)
-        return dict(softmax_scale=scale, head_scale=ly.head_scale, sinks=ly.sinks)
+        return dict(softmax_scale=scale, head_scale=ly.head_scale, sinks=ly.sinks, window=ly.window, keep_first=ly.keep_first)
 
-    def attend_prefill(self, layer: int, plan: PrefillPlan, q, k, v):
+    def attend_prefill(self, layer: int, plan: PrefillPlan, q, k, v, out=None):
         """q (T,Hq,D), k/v (T,Hkv,D) packed along dim 0 (token strides free, heads contiguous; k and v None for a layer
         that reads another layer's cache).  Writes (rotated) K and V of layer `layer` into its cache and returns causal
         attention output (T,Hq,D).  New sequences attend to the packed tensors themselves; when a sequence already had
-        cached tokens, keys and values are read back through the block tables, old and new alike."""
+        cached tokens, keys and values are read back through the block tables, old and new alike.  out: where to write (rows may
+        be strided)."""
         if q.shape[0] != plan.positions.shape[0]:
             raise ValueError("the plan and the packed tensors disagree on the number of tokens")
-        terms = self._score_terms(layer)
+        terms = dict(self._score_terms(layer), out=out)
         if plan.tables is not None:
             q = self._write_cache(layer, plan, q, k, v)
             kc, vc = self.k_caches[layer], self.v_caches[layer]
@@ -403,13 +477,13 @@ class PagedAttentionEngine:
         return ops.flash_attn_varlen_prefill(q, k, v, plan.cu_seqlens, plan.cu_seqlens, plan.max_len,
                                              plan.max_len, causal=True, **terms)
 
-    def attend_decode(self, layer: int, plan: DecodePlan, q, k, v):
+    def attend_decode(self, layer: int, plan: DecodePlan, q, k, v, out=None):
         """q (B,Hq,D), k/v (B,Hkv,D) or None as in attend_prefill: appends the token's K/V to layer `layer`'s cache and
-        returns its attention output (B,Hq,D)."""
+        returns its attention output (B,Hq,D), written into `out` when given (rows may be strided)."""
         if q.shape[0] != plan.positions.shape[0]:
             raise ValueError("one query token per sequence expected")
         q = self._write_cache(layer, plan, q, k, v)
-        terms = self._score_terms(layer)
+        terms = dict(self._score_terms(layer), out=out)
         kc, vc = self.k_caches[layer], self.v_caches[layer]
         if not self.mfma[layer]:
             return ops.paged_attention_any(q, kc, vc, plan.tables, plan.context_lens, **terms)
@@ -417,6 +491,16 @@ class PagedAttentionEngine:
             terms.update(k_scale=self.k_scales[layer], v_scale=self.v_scales[layer])
         return ops.paged_attention_decode(q, kc, vc, plan.tables, plan.context_lens, max_context=plan.max_context,
                                           workspace=self._workspace, **terms)
+
+    def advance_state(self, layer: int, plan: PrefillPlan | DecodePlan, proj, xbc_col: int, dt_col: int, out=None):
+        """State layer `layer` over the plan's tokens: the columns of proj (T,*) that hold its convolution inputs and step sizes
+        (see ops.ssm_mix), each sequence's state read from its slot and left there.  Returns y (T, heads * vdim)."""
+        ly = self.layers[layer]
+        if proj.shape[0] != plan.positions.shape[0]:
+            raise ValueError("the plan and the projection disagree on the number of tokens")
+        return ops.ssm_mix(proj, xbc_col, dt_col, ly.params, self.conv_states[layer], self.ssm_states[layer], plan.state_slots,
+                           plan.positions, plan.cu_seqlens if isinstance(plan, PrefillPlan) else None, heads=ly.heads, vdim=ly.vdim,
+                           state=ly.state, groups=ly.groups, out=out)
 
     # ---- single-layer convenience ----------------------------------------------------
     def prefill(self, seq_ids, lens, q, k, v):

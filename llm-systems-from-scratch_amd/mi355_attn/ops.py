@@ -121,8 +121,20 @@ def _head_terms(head_scale, sinks, Hq, device):
 
 
 def _prefill(q, k, v, out, cu_q, cu_k, mask, B, Hq, Hkv, Sq, Sk, D, scale, mode, lse=None, n_split=1, workspace=None,
-             total_rows=0, head_scale=None, sinks=None):
+             total_rows=0, head_scale=None, sinks=None, window=0, keep_first=0):
     lib = _lib.load()
+    if window:
+        hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
+        packed = cu_q is not None
+        qs, ks, vs, os_ = (_packed_or_dense_strides(x, packed) for x in (q, k, v, out))
+        with _on(q, k, v, out, cu_q, cu_k) as stream:
+            rc = lib.mi355_prefill_fwd_window(
+                q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr(),
+                _lib.strides3(qs), _lib.strides3(ks), _lib.strides3(vs), _lib.strides3(os_),
+                None if cu_q is None else cu_q.data_ptr(), None if cu_k is None else cu_k.data_ptr(), hs, sk,
+                B, Hq, Hkv, Sq, Sk, D, float(scale), int(window), int(keep_first), _lib.MI355_BF16, stream)
+        _lib.check(rc, "mi355_prefill_fwd_window")
+        return
     if head_scale is not None or sinks is not None:
         hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
         packed = cu_q is not None
@@ -405,8 +417,25 @@ def scaled_dot_product_attention(Q, K, V, mask=None):
     return out.reshape(*lead, nq, d).to(out_dtype)
 
 
+def _window(window, keep_first):
+    """A sliding window with kept first tokens as two non-negative ints (0: no window)."""
+    window, keep_first = int(window or 0), int(keep_first or 0)
+    if window < 0 or keep_first < 0:
+        raise ValueError("window and keep_first must not be negative")
+    return window, keep_first
+
+
+def _out_rows(out, T, H, D, dtype):
+    """An output (T,H,D) given by the caller: contiguous heads, rows may be strided (a view of a wider matrix)."""
+    align = 16 // out.element_size()
+    if out.dtype != dtype or tuple(out.shape) != (T, H, D) or (out.numel() and (
+            out.stride(2) != 1 or (H > 1 and out.stride(1) != D) or (T > 1 and out.stride(0) % align) or out.data_ptr() % 16)):
+        raise ValueError(f"out must be a {dtype} ({T}, {H}, {D}) tensor with contiguous heads, 16-byte aligned rows")
+    return out
+
+
 def _varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, causal, softmax_scale, want_lse=False,
-            kv_splits=1, workspace=None, head_scale=None, sinks=None):
+            kv_splits=1, workspace=None, head_scale=None, sinks=None, window=0, keep_first=0, out=None):
     for n, t in (("q", q), ("k", k), ("v", v)):
         _require_gpu_bf16(n, t)
         if t.dim() != 3:
@@ -429,33 +458,41 @@ def _varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, cau
     if (Tq and max_seqlen_q < 1) or (Tk and max_seqlen_k < 1):
         raise ValueError("max_seqlen_q and max_seqlen_k must be at least 1 when there are tokens")
     scale = 1.0 / math.sqrt(D) if softmax_scale is None else softmax_scale
-    out = torch.empty(Tq, Hq, D, dtype=q.dtype, device=q.device)
+    out = torch.empty(Tq, Hq, D, dtype=q.dtype, device=q.device) if out is None else _out_rows(out, Tq, Hq, D, q.dtype)
     lse = torch.empty(Hq, Tq, dtype=torch.float32, device=q.device) if want_lse else None
     if Tq and max_seqlen_q:
-        n_split, workspace = (1, None) if want_lse else _split_args(
+        n_split, workspace = (1, None) if want_lse or window else _split_args(
             kv_splits, workspace, B, Hq, D, max_seqlen_q, max_seqlen_k, Tq, causal, q.device)
         _prefill(q, k, v, out, cu_seqlens_q, cu_seqlens_k, None, B, Hq, Hkv, int(max_seqlen_q), int(max_seqlen_k),
-                 D, scale, _lib.MASK_CAUSAL if causal else _lib.MASK_NONE, lse, n_split, workspace, Tq, head_scale, sinks)
+                 D, scale, _lib.MASK_CAUSAL if causal else _lib.MASK_NONE, lse, n_split, workspace, Tq, head_scale, sinks,
+                 window, keep_first)
     return (out, lse) if want_lse else out
 
 
 def flash_attn_varlen_prefill(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, *,
-                              causal=True, softmax_scale=None, kv_splits=None, workspace=None, head_scale=None, sinks=None):
+                              causal=True, softmax_scale=None, kv_splits=None, workspace=None, head_scale=None, sinks=None,
+                              window=0, keep_first=0, out=None):
     """Packed ("varlen") prefill.  q (Tq,Hq,D); k, v (Tk,Hkv,D) bf16; cu_seqlens int32 (B+1,), cu[0]=0.
 
     Sequence b owns rows [cu[b], cu[b+1]).  Returns (Tq,Hq,D) bf16.  Differentiable like flash_attn_prefill;
     kv_splits / workspace as there.  head_scale, sinks (fp32 (Hq,), optional, forward only): a non-negative factor
     on every head's scores, and a score without key or value that joins the head's softmax denominator.
+    window, keep_first (causal, forward only): query i sees key j when i - j < window or j < keep_first (window 0: every
+    earlier key).  out: (Tq,Hq,D) bf16 to write into, rows may be strided.
     """
     q, k, v, out_dtype = _to_bf16(q, k, v)
+    window, keep_first = _window(window, keep_first)
+    if window and not causal:
+        raise ValueError("a window is causal")
     if _needs_grad(q, k, v):
-        if head_scale is not None or sinks is not None:
-            raise ValueError("per-head score factors and sinks are forward-only")
+        if head_scale is not None or sinks is not None or window or out is not None:
+            raise ValueError("per-head score factors, sinks, windows and a given output are forward-only")
         out = _VarlenPrefillFn.apply(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, bool(causal),
                                      softmax_scale)
     else:
         out = _varlen(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k, causal, softmax_scale,
-                      kv_splits=kv_splits, workspace=workspace, head_scale=head_scale, sinks=sinks)
+                      kv_splits=kv_splits, workspace=workspace, head_scale=head_scale, sinks=sinks, window=window,
+                      keep_first=keep_first, out=out)
     return out if out.dtype == out_dtype else out.to(out_dtype)
 
 
@@ -473,7 +510,7 @@ def paged_decode_workspace(batch, n_q_heads, head_dim, max_context, device):
 
 def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, softmax_scale=None,
                            k_scale=None, v_scale=None, max_context=None, workspace=None, out=None,
-                           static_scratch=False, head_scale=None, sinks=None):
+                           static_scratch=False, head_scale=None, sinks=None, window=0, keep_first=0):
     """Paged-KV decode attention, one query token per sequence.
 
     q (B,Hq,D) bf16; k_cache, v_cache (num_blocks,Hkv,16,D) bf16, or fp8-e4m3
@@ -487,7 +524,10 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
     head_scale, sinks (fp32 (Hq,), optional): a factor on every head's scores, and a score without key or value that
     joins the head's softmax denominator.  q may have strided rows (heads contiguous, row stride a multiple of 8, e.g.
     a view of a merged projection) unless static_scratch is set.
+    window, keep_first: the token at position i sees key j when i - j < window or j < keep_first (window 0: every earlier
+    key); not with static_scratch.  `out` may have strided rows like q unless static_scratch is set.
     """
+    window, keep_first = _window(window, keep_first)
     _require_gpu_bf16("q", q)
     if q.dim() != 3:
         raise ValueError(f"q must be (batch, heads, d_head), got {tuple(q.shape)}")
@@ -534,6 +574,13 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
         if static_scratch:
             raise ValueError("static_scratch=True allocates nothing: pass `out`")
         out = torch.empty(B, Hq, D, dtype=q.dtype, device=q.device)
+    windowed = window > 0 or not out.is_contiguous()
+    if windowed:
+        if static_scratch:
+            raise ValueError("static_scratch has no windows and no strided output")
+        if not headwise and q.data_ptr() % 16:
+            raise ValueError("q must be 16-byte aligned")
+        _out_rows(out, B, Hq, D, q.dtype)
     if B == 0:
         return out
     lib = _lib.load()
@@ -551,6 +598,18 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
         return out
     if workspace is None:
         workspace = paged_decode_workspace(B, Hq, D, max_context, q.device)
+    if windowed:
+        hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
+        with _on(q, k_cache, v_cache, out, block_tables, context_lens, k_scale, v_scale, workspace) as stream:
+            rc = lib.mi355_paged_decode_fwd_window(
+                q.data_ptr(), q.stride(0) if B > 1 else Hq * D, k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(),
+                out.stride(0) if B > 1 else Hq * D, block_tables.data_ptr(), block_tables.stride(0), context_lens.data_ptr(),
+                k_scale.data_ptr() if fp8 else None, v_scale.data_ptr() if fp8 else None, hs, sk,
+                workspace.data_ptr(), workspace.numel() * workspace.element_size(),
+                B, Hq, Hkv, D, bs, k_cache.shape[0], int(max_context), float(scale), window, keep_first,
+                _lib.MI355_FP8_E4M3 if fp8 else _lib.MI355_BF16, stream)
+        _lib.check(rc, "mi355_paged_decode_fwd_window")
+        return out
     if headwise:
         hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
         with _on(q, k_cache, v_cache, out, block_tables, context_lens, k_scale, v_scale, workspace) as stream:
@@ -577,7 +636,8 @@ def paged_attention_decode(q, k_cache, v_cache, block_tables, context_lens, *, s
 
 def flash_attn_paged_prefill(q, k_cache, v_cache, cu_seqlens_q, block_tables, context_lens, max_seqlen_q, *,
                              softmax_scale=None, out=None, max_context=None, kv_splits=None, workspace=None,
-                             k_scale=None, v_scale=None, total_context=None, cu_seqlens_k=None, head_scale=None, sinks=None):
+                             k_scale=None, v_scale=None, total_context=None, cu_seqlens_k=None, head_scale=None, sinks=None,
+                             window=0, keep_first=0):
     """Causal prefill of a chunk of new tokens over context that already sits in a paged cache.
 
     q (T,Hq,D) bf16, packed, contiguous heads (token stride free): sequence b owns rows
@@ -594,14 +654,15 @@ def flash_attn_paged_prefill(q, k_cache, v_cache, cu_seqlens_q, block_tables, co
     total_context (host int, optional): an upper bound on sum(context_lens) that sizes those rows (default
     batch * max_context); cu_seqlens_k (int32 (B+1,), optional): the running sum of the context lengths, if the
     caller has it on the device already (else it is computed here, a few small launches per call).
-    head_scale, sinks: per-head terms as in flash_attn_varlen_prefill.
+    head_scale, sinks: per-head terms, window, keep_first: sliding window, as in flash_attn_varlen_prefill.
     The mathematics is that of llm-core/llm_core/model.py:308-325 with the mask of :384; the reference
     itself would re-run the whole prefix (model.py:218)."""
     _require_gpu_bf16("q", q)
+    window, keep_first = _window(window, keep_first)
     if k_scale is not None or v_scale is not None:
         return _paged_prefill_fp8(q, k_cache, v_cache, k_scale, v_scale, cu_seqlens_q, block_tables, context_lens,
                                   max_seqlen_q, softmax_scale, out, max_context, kv_splits, workspace, total_context,
-                                  cu_seqlens_k, head_scale, sinks)
+                                  cu_seqlens_k, head_scale, sinks, window, keep_first)
     if q.dim() != 3 or q.stride(2) != 1 or q.stride(1) != q.shape[2]:
         raise ValueError("q must be (tokens, heads, d_head) with contiguous heads")
     T, Hq, D = q.shape
@@ -641,6 +702,16 @@ def flash_attn_paged_prefill(q, k_cache, v_cache, cu_seqlens_q, block_tables, co
     if T == 0 or B == 0:
         return out
     scale = 1.0 / math.sqrt(D) if softmax_scale is None else softmax_scale
+    if window:
+        hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
+        with _on(q, k_cache, v_cache, out, cu_seqlens_q, block_tables, context_lens) as stream:
+            rc = _lib.load().mi355_prefill_paged_fwd_window(
+                q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), q.stride(0), out.stride(0),
+                cu_seqlens_q.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), block_tables.shape[1],
+                context_lens.data_ptr(), hs, sk, B, Hq, Hkv, int(max_seqlen_q), D, _BLOCK, k_cache.shape[0], float(scale),
+                window, keep_first, _lib.MI355_BF16, stream)
+        _lib.check(rc, "mi355_prefill_paged_fwd_window")
+        return out
     if max_context is None:
         max_context = block_tables.shape[1] * _BLOCK
     n_split, workspace = _split_args(kv_splits, workspace, B, Hq, D, int(max_seqlen_q), int(max_context), T, True,
@@ -721,7 +792,7 @@ def gather_kv_fp8(k_cache, v_cache, k_scale, v_scale, block_tables, context_lens
 
 def _paged_prefill_fp8(q, k_cache, v_cache, k_scale, v_scale, cu_seqlens_q, block_tables, context_lens, max_seqlen_q,
                        softmax_scale, out, max_context, kv_splits, workspace, total_context, cu_seqlens_k=None,
-                       head_scale=None, sinks=None):
+                       head_scale=None, sinks=None, window=0, keep_first=0):
     """flash_attn_paged_prefill over an fp8 cache: gather + dequantise, then the packed prefill with more keys than
     queries per sequence (bottom-right aligned causal mask)."""
     if q.dim() != 3:
@@ -732,13 +803,9 @@ def _paged_prefill_fp8(q, k_cache, v_cache, k_scale, v_scale, cu_seqlens_q, bloc
     max_context = width if max_context is None else min(int(max_context), width)
     k_lin, v_lin, cu_k = gather_kv_fp8(k_cache, v_cache, k_scale, v_scale, block_tables, context_lens,
                                        max_context=max_context, total_context=total_context, cu_seqlens_k=cu_seqlens_k)
-    res = flash_attn_varlen_prefill(q, k_lin, v_lin, cu_seqlens_q, cu_k, max_seqlen_q, max_context, causal=True,
-                                    softmax_scale=softmax_scale, kv_splits=kv_splits, workspace=workspace,
-                                    head_scale=head_scale, sinks=sinks)
-    if out is not None:
-        out.copy_(res)
-        return out
-    return res
+    return flash_attn_varlen_prefill(q, k_lin, v_lin, cu_seqlens_q, cu_k, max_seqlen_q, max_context, causal=True,
+                                     softmax_scale=softmax_scale, kv_splits=kv_splits, workspace=workspace,
+                                     head_scale=head_scale, sinks=sinks, window=window, keep_first=keep_first, out=out)
 
 
 _DTYPE_CODE = {torch.bfloat16: _lib.MI355_BF16, torch.float32: _lib.MI355_FP32}
@@ -751,13 +818,15 @@ def _dtype_code(name, t):
 
 
 def paged_attention_any(q, k_cache, v_cache, block_tables, context_lens, *, cu_seqlens_q=None, softmax_scale=None,
-                        head_scale=None, sinks=None):
+                        head_scale=None, sinks=None, window=0, keep_first=0, out=None):
     """Causal attention through the block tables for any head size, in bf16 or fp32 (the general path: no MFMA).
 
     q (T,Hq,Dk), heads contiguous; k_cache (num_blocks,Hkv,16,Dk), v_cache (num_blocks,Hkv,16,Dv) of q's dtype, Dk and Dv
     multiples of 8 up to 512; block_tables (B,max_blocks), context_lens (B,) int32.  With cu_seqlens_q (int32 (B+1,))
     the rows are packed chunks whose keys are already cached, as in flash_attn_paged_prefill; without it sequence b owns
-    row b, as in paged_attention_decode.  head_scale, sinks as there.  Returns (T,Hq,Dv)."""
+    row b, as in paged_attention_decode.  head_scale, sinks, window, keep_first as there.  Returns (T,Hq,Dv), written into
+    `out` (rows may be strided) when given."""
+    window, keep_first = _window(window, keep_first)
     code = _dtype_code("q", q)
     if q.dim() != 3 or (q.numel() and (q.stride(2) != 1 or q.stride(1) != q.shape[2])):
         raise ValueError("q must be (tokens, heads, d_head) with contiguous heads")
@@ -782,18 +851,19 @@ def paged_attention_any(q, k_cache, v_cache, block_tables, context_lens, *, cu_s
             raise ValueError("one query row per sequence expected without cu_seqlens_q")
     elif cu_seqlens_q.shape != (B + 1,) or not cu_seqlens_q.is_contiguous():
         raise ValueError("cu_seqlens_q must be a contiguous (batch + 1,) tensor")
-    out = torch.empty(T, Hq, Dv, dtype=q.dtype, device=q.device)
+    out = torch.empty(T, Hq, Dv, dtype=q.dtype, device=q.device) if out is None else _out_rows(out, T, Hq, Dv, q.dtype)
     if T == 0:
         return out
     scale = 1.0 / math.sqrt(Dk) if softmax_scale is None else softmax_scale
     hs, sk = _head_terms(head_scale, sinks, Hq, q.device)
     with _on(q, k_cache, v_cache, out, block_tables, context_lens, cu_seqlens_q) as stream:
-        rc = _lib.load().mi355_paged_attn_any_fwd(
-            q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), q.stride(0) if T > 1 else Hq * Dk, Hq * Dv, T,
+        rc = _lib.load().mi355_paged_attn_any_fwd_window(
+            q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), q.stride(0) if T > 1 else Hq * Dk,
+            out.stride(0) if T > 1 else Hq * Dv, T,
             None if cu_seqlens_q is None else cu_seqlens_q.data_ptr(), block_tables.data_ptr(),
             max(block_tables.stride(0), block_tables.shape[1]), block_tables.shape[1], context_lens.data_ptr(), hs, sk,
-            B, Hq, Hkv, Dk, Dv, _BLOCK, nb, float(scale), code, stream)
-    _lib.check(rc, "mi355_paged_attn_any_fwd")
+            B, Hq, Hkv, Dk, Dv, _BLOCK, nb, float(scale), window, keep_first, code, stream)
+    _lib.check(rc, "mi355_paged_attn_any_fwd_window")
     return out
 
 
@@ -827,6 +897,41 @@ def build_rope_cache(context_length, d, theta=10000.0, device="cuda"):
     inv_freq = theta ** -(torch.arange(0, d, 2, dtype=torch.float32) / d)
     angles = torch.arange(context_length, dtype=torch.float32)[:, None] * inv_freq[None, :]
     return torch.stack((torch.cos(angles), torch.sin(angles))).to(device)
+
+
+def build_partial_rope_cache(context_length, d, dims, base, device="cuda"):
+    """The same table for heads of size d whose first `dims` entries turn, the pair i by base^(-2i/dims) per position; the
+    remaining pairs have the angle 0.  Angles are taken in double precision and rounded once."""
+    if dims % 2 or not 0 <= dims <= d or d % 2:
+        raise ValueError("dims must be even and at most d, d even")
+    angles = torch.zeros(context_length, d // 2, dtype=torch.float64)
+    inv_freq = float(base) ** -(torch.arange(0, dims, 2, dtype=torch.float64) / max(dims, 1))
+    angles[:, :dims // 2] = torch.arange(context_length, dtype=torch.float64)[:, None] * inv_freq[None, :]
+    return torch.stack((torch.cos(angles), torch.sin(angles))).to(device=device, dtype=torch.float32)
+
+
+def rope_rotate(q, k, positions, freq_cache):
+    """Rotation in place of adjacent pairs of q (T,Hq,D) and k (T,Hkv,D) (or None), bf16 or fp32, any even D; heads contiguous,
+    rows may be strided; positions (T,) int32; freq_cache as in rope_and_cache."""
+    code = _dtype_code("q", q)
+    T, Hq, D = q.shape
+    for n, t in (("q", q), ("k", k)):
+        if t is not None and (t.dtype != q.dtype or t.dim() != 3 or (t.shape[0], t.shape[2]) != (T, D)
+                              or (t.numel() and (t.stride(2) != 1 or (t.shape[1] > 1 and t.stride(1) != D)))):
+            raise ValueError(f"{n} must be (tokens, heads, d_head) with contiguous heads; q and k agree in dtype, tokens and d_head")
+    if freq_cache.dtype != torch.float32 or freq_cache.dim() != 3 or freq_cache.shape[0] != 2 or freq_cache.shape[2] * 2 != D \
+            or not freq_cache.is_contiguous():
+        raise ValueError("freq_cache must be a contiguous float32 tensor (2, context_length, d_head/2)")
+    if positions.dtype != torch.int32 or positions.shape != (T,) or not positions.is_contiguous():
+        raise TypeError("positions must be a contiguous int32 (tokens,) tensor")
+    if T == 0:
+        return
+    Hkv = 0 if k is None else k.shape[1]
+    with _on(q, k, positions, freq_cache) as stream:
+        rc = _lib.load().mi355_rope_any(q.data_ptr(), None if k is None else k.data_ptr(), freq_cache.data_ptr(), positions.data_ptr(),
+                                        T, Hq, Hkv, D, freq_cache.shape[1], q.stride(0) if T > 1 else Hq * D,
+                                        0 if k is None else k.stride(0) if T > 1 else Hkv * D, code, stream)
+    _lib.check(rc, "mi355_rope_any")
 
 
 def _packed_k_out(k_out, k):
@@ -1143,4 +1248,194 @@ def silu_mul(gate, up):
             rc = _lib.load().mi355_silu_mul_fwd(g2.data_ptr(), u2.data_ptr(), out.data_ptr(), n_rows, d,
                                                 g2.stride(0), u2.stride(0), d, stream)
         _lib.check(rc, "mi355_silu_mul_fwd")
+    return out
+
+
+def residual_rms(resid, weight, *, sub=None, routed=None, top=1, embed=None, tokens=None, weight_offset=0.0, eps=1e-6,
+                 out_dtype=torch.bfloat16, y_cols=None):
+    """Everything that is added to an fp32 residual stream, and the RMS norm of the sum, in one launch:
+
+        x = resid + sub + sum_k routed[row * top + k] + embed[tokens[row]],   y = x / sqrt(mean(x^2) + eps) * (weight_offset + weight)
+
+    resid (T,d) fp32, updated in place, or None (the stream starts here: returned as a new tensor); sub (T,d) and routed
+    (T * top,d), rows may be strided, embed (vocab,d) with tokens (T,) int64: all of out_dtype, each optional.  weight (d,) fp32,
+    or None: no norm.  y has y_cols >= d columns, zero beyond d.  Returns (x, y)."""
+    parts = [t for t in (sub, routed, embed) if t is not None]
+    code = _dtype_code("the result", torch.empty(0, dtype=out_dtype))
+    if any(t.dtype != out_dtype for t in parts):
+        raise TypeError(f"sub, routed and embed must be {out_dtype}")
+    if resid is not None:
+        T, d = _matrix("resid", resid, torch.float32).shape
+        if not resid.is_contiguous():
+            raise ValueError("resid must be contiguous")
+    elif sub is not None:
+        T, d = sub.shape
+    elif embed is not None:
+        T, d = tokens.numel(), embed.shape[1]
+    else:
+        raise ValueError("resid, sub or embed is needed")
+    if sub is not None:
+        _matrix("sub", sub, out_dtype, (T, d))
+    if routed is not None:
+        _matrix("routed", routed, out_dtype, (T * top, d))
+    if embed is not None:
+        if embed.dim() != 2 or embed.shape[1] != d or not embed.is_contiguous():
+            raise ValueError(f"embed must be a contiguous matrix of {d} columns")
+        if tokens is None or tokens.dtype != torch.int64 or tokens.shape != (T,) or not tokens.is_contiguous():
+            raise TypeError("tokens must be a contiguous int64 (tokens,) tensor")
+    _vector("weight", weight, d)
+    y_cols = d if y_cols is None else y_cols
+    device = (resid if resid is not None else parts[0]).device
+    x = torch.empty(T, d, dtype=torch.float32, device=device) if resid is None else resid
+    y = None if weight is None else torch.empty(T, y_cols, dtype=out_dtype, device=device)
+    if T:
+        with _on(resid, weight, tokens, *parts) as stream:
+            rc = _lib.load().mi355_residual_rms_fwd(
+                None if resid is None else resid.data_ptr(), x.data_ptr() if parts else None,
+                None if sub is None else sub.data_ptr(), None if routed is None else routed.data_ptr(), int(top),
+                None if embed is None else embed.data_ptr(), None if tokens is None else tokens.data_ptr(),
+                0 if embed is None else embed.shape[0], None if weight is None else weight.data_ptr(), float(weight_offset),
+                float(eps), None if y is None else y.data_ptr(), T, d, y_cols, 0 if sub is None else sub.stride(0),
+                0 if routed is None else routed.stride(0), y_cols, code, stream)
+        _lib.check(rc, "mi355_residual_rms_fwd")
+    return x, y
+
+
+def ff_act(a, b=None, *, row_gate=None, out=None):
+    """silu(a) * b, or without b the tanh form of gelu(a), in fp32 with one rounding; with row_gate (rows,) fp32 times
+    sigmoid(row_gate).  a, b, out: matrices (rows may be strided) of bf16 or fp32."""
+    code = _dtype_code("a", a)
+    T, d = _matrix("a", a, a.dtype).shape
+    if b is not None:
+        _matrix("b", b, a.dtype, (T, d))
+    _vector("row_gate", row_gate, T)
+    out = torch.empty(T, d, dtype=a.dtype, device=a.device) if out is None else _matrix("out", out, a.dtype, (T, d))
+    if T and d:
+        with _on(a, b, row_gate, out) as stream:
+            rc = _lib.load().mi355_ff_act_fwd(a.data_ptr(), None if b is None else b.data_ptr(),
+                                              None if row_gate is None else row_gate.data_ptr(), out.data_ptr(), T, d, a.stride(0),
+                                              0 if b is None else b.stride(0), out.stride(0), code, stream)
+        _lib.check(rc, "mi355_ff_act_fwd")
+    return out
+
+
+def gated_norm(y, z, weight, groups: int, eps: float, *, out=None):
+    """v = y * silu(z), each of `groups` equal parts of a row divided by its own root mean square, times weight (fp32).  y, z,
+    out: matrices (rows may be strided) of bf16 or fp32; out may be y."""
+    code = _dtype_code("y", y)
+    T, d = _matrix("y", y, y.dtype).shape
+    _matrix("z", z, y.dtype, (T, d))
+    _vector("weight", weight, d)
+    if groups < 1 or d % groups:
+        raise ValueError("groups must divide the number of columns")
+    out = torch.empty(T, d, dtype=y.dtype, device=y.device) if out is None else _matrix("out", out, y.dtype, (T, d))
+    if T:
+        with _on(y, z, weight, out) as stream:
+            rc = _lib.load().mi355_gated_norm_fwd(y.data_ptr(), z.data_ptr(), None if weight is None else weight.data_ptr(),
+                                                  out.data_ptr(), T, d, int(groups), y.stride(0), z.stride(0), out.stride(0),
+                                                  float(eps), code, stream)
+        _lib.check(rc, "mi355_gated_norm_fwd")
+    return out
+
+
+def ssm_mix(proj, xbc_col, dt_col, params, conv_state, ssm_state, slots, positions, cu_seqlens=None, *, heads, vdim, state, groups,
+            out=None, scan="auto"):
+    """Mamba-2 mixer between its projections: causal convolution + silu of the channels (x | B | C) at column xbc_col of proj's
+    rows, then S <- exp(A dt) S + dt B x^T, y = S^T C + D x with dt = softplus(columns dt_col .. + dt_bias).
+
+    proj (T,*) bf16 or fp32, rows may be strided; params: dict of fp32 tensors conv (taps,channels), conv_b (channels,), dt_bias,
+    neg_a, d_skip (heads,); conv_state (n_slots,taps,channels) of proj's dtype and ssm_state (n_slots,heads,state,vdim rounded up
+    to 4) fp32, updated in place at slots (B,) int32; positions (T,) int32 (a sequence whose first row has position 0 starts from
+    zero).  With cu_seqlens (int32 (B+1,)) sequence b owns those rows; without it each owns one and everything is one launch.
+    scan: "auto", "serial" or "chunked" (see mi355_ssm_prefill).  Returns y (T, heads * vdim), into `out` when given."""
+    code = _dtype_code("proj", proj)
+    T, width = _matrix("proj", proj, proj.dtype).shape
+    channels, inner = heads * vdim + 2 * groups * state, heads * vdim
+    taps = params["conv"].shape[0]
+    for n, shape in (("conv", (taps, channels)), ("conv_b", (channels,)), ("dt_bias", (heads,)), ("neg_a", (heads,)), ("d_skip", (heads,))):
+        t = params[n]
+        if t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous():
+            raise ValueError(f"{n} must be a contiguous float32 {shape} tensor")
+    n_slots = conv_state.shape[0]
+    if conv_state.dtype != proj.dtype or tuple(conv_state.shape) != (n_slots, taps, channels) or not conv_state.is_contiguous():
+        raise ValueError(f"conv_state must be a contiguous {proj.dtype} (n_slots, {taps}, {channels}) tensor")
+    if ssm_state.dtype != torch.float32 or tuple(ssm_state.shape) != (n_slots, heads, state, (vdim + 3) // 4 * 4) or not ssm_state.is_contiguous():
+        raise ValueError(f"ssm_state must be a contiguous float32 ({n_slots}, {heads}, {state}, {(vdim + 3) // 4 * 4}) tensor")
+    B = slots.numel()
+    for n, t, k in (("slots", slots, B), ("positions", positions, T), ("cu_seqlens", cu_seqlens, B + 1)):
+        if t is not None and (t.dtype != torch.int32 or t.shape != (k,) or not t.is_contiguous()):
+            raise TypeError(f"{n} must be a contiguous int32 ({k},) tensor")
+    if cu_seqlens is None and T != B:
+        raise ValueError("one row per sequence expected without cu_seqlens")
+    if not 0 <= xbc_col <= width - channels or not 0 <= dt_col <= width - heads:
+        raise ValueError("columns outside the rows of proj")
+    out = torch.empty(T, inner, dtype=proj.dtype, device=proj.device) if out is None else _matrix("out", out, proj.dtype, (T, inner))
+    if T == 0:
+        return out
+    xbc = None if cu_seqlens is None else torch.empty(T, channels, dtype=proj.dtype, device=proj.device)
+    with _on(proj, conv_state, ssm_state, slots, positions, cu_seqlens, out, *params.values()) as stream:
+        args = _lib.SsmArgs(proj.data_ptr(), *(params[n].data_ptr() for n in ("conv", "conv_b", "dt_bias", "neg_a", "d_skip")),
+                            conv_state.data_ptr(), ssm_state.data_ptr(), slots.data_ptr(), positions.data_ptr(),
+                            None if cu_seqlens is None else cu_seqlens.data_ptr(), None if xbc is None else xbc.data_ptr(),
+                            out.data_ptr(), proj.stride(0) if T > 1 else width, xbc_col, dt_col, out.stride(0) if T > 1 else inner, T,
+                            B, heads, vdim, state, groups, taps, n_slots, code)
+        if cu_seqlens is None:
+            rc = _lib.load().mi355_ssm_decode(args, stream)
+        else:
+            rc = _lib.load().mi355_ssm_prefill(args, _lib.SCANS[scan], stream)
+    _lib.check(rc, "mi355_ssm_prefill" if cu_seqlens is not None else "mi355_ssm_decode")
+    return out
+
+
+def moe_route(h, w, bias, top: int, *, extra_row: bool = False):
+    """Router: logits h W^T + bias in fp32, the `top` largest per row and the softmax over them.  h (T,k), w (experts,k) of one
+    dtype (bf16: k a multiple of 8), bias fp32.  extra_row: w and bias have one row more that is no expert.  Returns
+    (ids (T,top) int32, weights (T,top) fp32, the extra row's logits (T,) fp32 or None)."""
+    code = _dtype_code("h", h)
+    T, k = _matrix("h", h, h.dtype).shape
+    n_experts = w.shape[0] - int(extra_row)
+    _matrix("w", w, h.dtype, (w.shape[0], k))
+    _vector("bias", bias, w.shape[0])
+    ids = torch.empty(T, top, dtype=torch.int32, device=h.device)
+    weights = torch.empty(T, top, dtype=torch.float32, device=h.device)
+    extra = torch.empty(T, dtype=torch.float32, device=h.device) if extra_row else None
+    with _on(h, w, bias) as stream:
+        rc = _lib.load().mi355_moe_route(h.data_ptr(), w.data_ptr(), bias.data_ptr(), ids.data_ptr(), weights.data_ptr(),
+                                         None if extra is None else extra.data_ptr(), T, h.stride(0) if T > 1 else k,
+                                         w.stride(0) if w.shape[0] > 1 else k, k, n_experts, int(top), code, stream)
+    _lib.check(rc, "mi355_moe_route")
+    return ids, weights, extra
+
+
+def moe_experts(h, ids, weights, w_gate_up, w_down, *, tiling="auto"):
+    """Gated feed-forward of each row's chosen experts: weights[t, c] * Wd (silu(Wg h_t) * (Wu h_t)) of expert ids[t, c] as row
+    t * top + c of the result (T * top, n); their sum is left to the reader (residual_rms).  h (T,k), w_gate_up
+    (experts, 2 ff, k) with the gates first, w_down (experts, n, ff), all bf16 (k and ff multiples of 64) or fp32."""
+    code = _dtype_code("h", h)
+    T, k = _matrix("h", h, h.dtype).shape
+    E, n, ff = w_down.shape
+    if w_gate_up.dtype != h.dtype or w_down.dtype != h.dtype or tuple(w_gate_up.shape) != (E, 2 * ff, k) \
+            or not w_gate_up.is_contiguous() or not w_down.is_contiguous():
+        raise ValueError("w_gate_up (experts, 2 ff, k) and w_down (experts, n, ff) must be contiguous tensors of h's dtype")
+    top = ids.shape[1]
+    for name, t, dt in (("ids", ids, torch.int32), ("weights", weights, torch.float32)):
+        if t.dtype != dt or tuple(t.shape) != (T, top) or not t.is_contiguous():
+            raise ValueError(f"{name} must be a contiguous {dt} ({T}, {top}) tensor")
+    dev = h.device
+    out = torch.empty(T * top, n, dtype=h.dtype, device=dev)
+    if T == 0:
+        return out
+    offsets = torch.empty(E + 1, dtype=torch.int32, device=dev)
+    order = torch.empty(T * top, dtype=torch.int32, device=dev)
+    act = torch.empty(T * top, ff, dtype=h.dtype, device=dev)
+    lib, tl = _lib.load(), _lib.TILINGS[tiling]
+    with _on(h, ids, weights, w_gate_up, w_down) as stream:
+        rc = lib.mi355_moe_group(ids.data_ptr(), T * top, E, offsets.data_ptr(), order.data_ptr(), stream)
+        _lib.check(rc, "mi355_moe_group")
+        rc = lib.mi355_moe_gate_up(h.data_ptr(), w_gate_up.data_ptr(), act.data_ptr(), offsets.data_ptr(), order.data_ptr(), T,
+                                   h.stride(0) if T > 1 else k, ff, E, top, k, ff, code, tl, stream)
+        _lib.check(rc, "mi355_moe_gate_up")
+        rc = lib.mi355_moe_down(act.data_ptr(), w_down.data_ptr(), weights.data_ptr(), out.data_ptr(), offsets.data_ptr(),
+                                order.data_ptr(), T, ff, n, E, top, ff, n, code, tl, stream)
+        _lib.check(rc, "mi355_moe_down")
     return out

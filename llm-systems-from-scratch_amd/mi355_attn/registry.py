@@ -6,11 +6,13 @@ import os
 
 from .model import CachedLM, CachedTransformerLM
 from .weights import load_state_dict
+from .zomipel import ZomipelLM
 from .zuzelorn import ZuzelornLM
 
 # config.json's "architecture" -> class; a configuration without the key is the reference decoder's
 # (llm-core/llm_core/model.py:238-256 stores only the constructor arguments)
-ARCHITECTURES: dict[str, type[CachedLM]] = {"TransformerLM": CachedTransformerLM, "Zuzelorn": ZuzelornLM}
+ARCHITECTURES: dict[str, type[CachedLM]] = {"TransformerLM": CachedTransformerLM, "Zuzelorn": ZuzelornLM,
+                                          "Zomipel": ZomipelLM}
 CHECKPOINT_NAMES = ("model.safetensors", "model.pt", "checkpoint.pt")
 
 

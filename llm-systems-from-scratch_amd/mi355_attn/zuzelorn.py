@@ -23,26 +23,7 @@ import torch
 from . import ops
 from .engine import BLOCK, AttentionLayer, PagedAttentionEngine, cache_head_dims
 from .model import CachedLM
-
-
-def _pad_heads(t, heads, size, to):
-    """(heads * size, ...) -> (heads * to, ...) with zero rows behind every head."""
-    if size == to:
-        return t
-    t = t.view(heads, size, *t.shape[1:])
-    return torch.cat((t, t.new_zeros(heads, to - size, *t.shape[2:])), 1).flatten(0, 1)
-
-
-def _stack_rows(parts):
-    """Rows of several matrices (or entries of vectors), each part starting at a multiple of 8 rows (zero rows between),
-    so that every part of a product's row is 16-byte aligned.  Returns the stack and the parts' first rows."""
-    out, starts, at = [], [], 0
-    for t in parts:
-        starts.append(at)
-        pad = -t.shape[0] % 8
-        out += [t, t.new_zeros(pad, *t.shape[1:])] if pad else [t]
-        at += t.shape[0] + pad
-    return torch.cat(out).contiguous(), starts
+from .weights import Checkpoint, pad_heads, stack_rows
 
 
 class ZuzelornLM(CachedLM):
@@ -66,21 +47,8 @@ class ZuzelornLM(CachedLM):
         self.eps = float(config["norm"]["eps"])
         self.logit_scale = float(config.get("logit_scale", 1.0))
         context_length = config["max_positions"]
-        sd = state_dict
-
-        def raw(name, *shape):
-            if name not in sd:
-                raise KeyError(f"the checkpoint has no tensor {name}")
-            t = sd[name].detach()
-            if tuple(t.shape) != shape:
-                raise ValueError(f"{name} is {tuple(t.shape)}, the configuration says {shape}")
-            return t
-
-        def mat(t):
-            return t.to(device=dev, dtype=self.dtype).contiguous()
-
-        def vec(name, *shape):
-            return raw(name, *shape).to(device=dev, dtype=torch.float32).contiguous()
+        ckpt = Checkpoint(state_dict, self.dtype, dev)
+        raw, mat, vec = ckpt.raw, ckpt.matrix, ckpt.vector
 
         def norm(name):
             return float(raw(name + ".alpha").float()), vec(name, d), vec(name + ".b", d)
@@ -100,25 +68,25 @@ class ZuzelornLM(CachedLM):
             # temp_head: its size scales the scores in the kernels; its sign moves into the head's query (exact)
             temp = raw(pre + "mix.temp", H).float()
             sign = torch.where(temp < 0, -1.0, 1.0).repeat_interleave(dk)
-            w = [_pad_heads(raw(pre + "mix.q", H * dk, d).float() * sign[:, None], H, dk, kd)]
-            b = [_pad_heads(raw(pre + "mix.q.b", H * dk).float() * sign, H, dk, kd)]
+            w = [pad_heads(raw(pre + "mix.q", H * dk, d).float() * sign[:, None], H, dk, kd)]
+            b = [pad_heads(raw(pre + "mix.q.b", H * dk).float() * sign, H, dk, kd)]
             src = m.get("kv_from")
             if src is None:
                 for n, size, to in (("k", dk, kd), ("v", dv, vd)):
-                    w.append(_pad_heads(raw(pre + f"mix.{n}", G * size, d).float(), G, size, to))
-                    b.append(_pad_heads(raw(pre + f"mix.{n}.b", G * size).float(), G, size, to))
+                    w.append(pad_heads(raw(pre + f"mix.{n}", G * size, d).float(), G, size, to))
+                    b.append(pad_heads(raw(pre + f"mix.{n}.b", G * size).float(), G, size, to))
             w.append(raw(pre + "rg1", d, d).float())
             b.append(b[0].new_zeros(d))                     # (the gate's bias is added in fp32 where the gate is applied)
-            w_in, starts = _stack_rows(w)
-            wo = _pad_heads(raw(pre + "mix.o", d, H * dv).float().t(), H, dv, vd).t()
-            ly = dict(H=H, G=G, kd=kd, vd=vd, own_kv=src is None, w_in=mat(w_in), b_in=mat(_stack_rows(b)[0]), starts=starts,
+            w_in, starts = stack_rows(w)
+            wo = pad_heads(raw(pre + "mix.o", d, H * dv).float().t(), H, dv, vd).t()
+            ly = dict(H=H, G=G, kd=kd, vd=vd, own_kv=src is None, w_in=mat(w_in), b_in=mat(stack_rows(b)[0]), starts=starts,
                       wo=mat(wo), bo=vec(pre + "mix.o.b", d), rg1_b=vec(pre + "rg1.b", d), norm1=norm(pre + "norm1"),
                       norm1b=norm(pre + "norm1b"), ff=None)
             if mlp is not None:
                 if mlp["kind"] != "dense":
                     raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
                 ff = mlp["ff"]
-                w_up, (_, gate_at) = _stack_rows([raw(pre + "mlp.up", ff, d), raw(pre + "rg2", d, d)])
+                w_up, (_, gate_at) = stack_rows([raw(pre + "mlp.up", ff, d), raw(pre + "rg2", d, d)])
                 ly.update(ff=ff, w_up=mat(w_up), gate_at=gate_at, wdown=mat(raw(pre + "mlp.down", d, ff)),
                           act=raw(pre + "mlp.act", 4).float().tolist(), rg2_b=vec(pre + "rg2.b", d), norm2=norm(pre + "norm2"),
                           norm2b=norm(pre + "norm2b"))
