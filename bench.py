@@ -18,7 +18,7 @@ fp8 decode, then one {ms, frac} pair per auxiliary leg under "legs", and the con
 `--full` prints every leg's whole object instead; `--detail PATH` writes that verbose form to a file.
 
 usage: python bench.py [--gpus 1] [--steps K=200] [--warmup W=50] [--seed S]
-                       [--only decode|prefill|small|few|fp8|backward|producers|layer|loop|zuzelorn] [--no-cpu] [--full] [--detail PATH]
+                       [--only decode|prefill|small|few|fp8|backward|producers|layer|loop|zuzelorn|zomipel] [--no-cpu] [--full] [--detail PATH]
 """
 from __future__ import annotations
 
@@ -372,6 +372,40 @@ def bench_decode_loop(args):
     return res
 
 
+def _serve_side_by_side(names, models, args, n_prompt, prompt_len, batch, ctx):
+    """Prefill of n_prompt new prompts and decode steps of `batch` sequences at ctx tokens (greedy tokens fed back through the
+    host) of several models with a vocabulary of 32000, measured in turn: the best of three rounds each."""
+    import torch
+    g = torch.Generator().manual_seed(args.seed)
+    prompts = [torch.randint(0, 32000, (prompt_len,), generator=g) for _ in range(n_prompt)]
+
+    def prefill(m):
+        s = [m.new_sequence() for _ in prompts]
+        m.prefill(s, prompts)
+        for i in s:
+            m.free_sequence(i)
+
+    best = {n: {} for n in names}
+    for rep in range(3):
+        for n, m in zip(names, models):
+            ms, _ = timed(lambda: prefill(m), max(3, args.steps // 20), 2, BURN_MS)
+            best[n]["prefill_ms"] = min(ms, best[n].get("prefill_ms", 1e9))
+    state = []
+    for m in models:                                       # sequences of ctx tokens
+        sids = [m.new_sequence() for _ in range(batch)]
+        for i in range(0, batch, 8):
+            m.prefill(sids[i:i + 8], [torch.randint(0, 32000, (ctx,), generator=g) for _ in range(8)])
+        state.append([sids, [1] * batch])
+    for rep in range(3):
+        for n, m, st in zip(names, models, state):
+            def step():
+                st[1] = m.decode(st[0], st[1]).argmax(-1).tolist()
+            ms, _ = timed(step, 30, 8)
+            best[n]["decode_ms"] = min(ms, best[n].get("decode_ms", 1e9))
+    return {n: {"prefill_ms": best[n]["prefill_ms"], "prefill_tokens_per_s": n_prompt * prompt_len / best[n]["prefill_ms"] * 1e3,
+                "decode_ms": best[n]["decode_ms"], "decode_tokens_per_s": batch / best[n]["decode_ms"] * 1e3} for n in names}
+
+
 def _zuzelorn_pair(d, heads, head_dim, ff, n_layers, context, seed):
     """(config, weights) of a Zuzelorn model whose every layer has keys and values of its own, of one in which every second
     layer reads the layer before it, and of the reference decoder of the same width, heads, layers and parameter count per
@@ -433,43 +467,15 @@ def bench_zuzelorn(args):
     n_prompt, prompt_len, batch, ctx = 4, 2048, 32, 2048
     for key, d, heads, head_dim, n_layers in (("d1024", 1024, 16, 64, 8), ("d2048", 2048, 16, 128, 6), ("d4096", 4096, 32, 128, 4)):
         context = 4096
-        g = torch.Generator().manual_seed(args.seed)
         pairs = _zuzelorn_pair(d, heads, head_dim, 2 * d, n_layers, context, args.seed)
         blocks = batch * (ctx + 256) // 16
         models = [cls(c, sd, num_blocks=blocks, max_batch=batch, decode_graphs=True)
                   for cls, (c, sd) in zip((ma.ZuzelornLM, ma.ZuzelornLM, ma.CachedTransformerLM), pairs)]
         entry = {"workload": f"{n_layers} layers, width {d}, {heads} heads x {head_dim}, ff {2 * d}, vocab 32000; prefill: {n_prompt} new prompts "
                              f"of {prompt_len} tokens; decode: {batch} sequences at {ctx} tokens, HIP graph, greedy tokens fed back through the host"}
-        prompts = [torch.randint(0, 32000, (prompt_len,), generator=g) for _ in range(n_prompt)]
-
-        def prefill(m):
-            s = [m.new_sequence() for _ in prompts]
-            m.prefill(s, prompts)
-            for i in s:
-                m.free_sequence(i)
-
-        best = {n: {} for n in names}
-        for rep in range(3):                                   # the sides in turn; the best of three rounds each
-            for n, m in zip(names, models):
-                ms, _ = timed(lambda: prefill(m), max(3, args.steps // 20), 2, BURN_MS)
-                best[n]["prefill_ms"] = min(ms, best[n].get("prefill_ms", 1e9))
-        state = []
-        for m in models:                                       # sequences of ctx tokens
-            sids = [m.new_sequence() for _ in range(batch)]
-            for i in range(0, batch, 8):
-                m.prefill(sids[i:i + 8], [torch.randint(0, 32000, (ctx,), generator=g) for _ in range(8)])
-            state.append([sids, [1] * batch])
-        for rep in range(3):
-            for n, m, st in zip(names, models, state):
-                def step():
-                    st[1] = m.decode(st[0], st[1]).argmax(-1).tolist()
-                ms, _ = timed(step, 30, 8)
-                best[n]["decode_ms"] = min(ms, best[n].get("decode_ms", 1e9))
-        for n in names:
-            entry[n] = {"prefill_ms": best[n]["prefill_ms"], "prefill_tokens_per_s": n_prompt * prompt_len / best[n]["prefill_ms"] * 1e3,
-                        "decode_ms": best[n]["decode_ms"], "decode_tokens_per_s": batch / best[n]["decode_ms"] * 1e3}
+        entry.update(_serve_side_by_side(names, models, args, n_prompt, prompt_len, batch, ctx))
         res["models"][key] = entry
-        del models, state, pairs
+        del models, pairs
         torch.cuda.empty_cache()
 
     # the operators at prefill size (8192 rows of width 4096, ff 8192): bytes that must move over the device time
@@ -514,6 +520,170 @@ def bench_zuzelorn(args):
         ws = ma.paged_decode_workspace(4, H, D, 2048, dev)
         _, ms = timed(lambda: ma.paged_attention_decode(q1, *pools, bt, cl, workspace=ws, **kw), args.steps, args.warmup, BURN_MS)
         res["operators"]["decode attention " + n] = {"device_ms": ms, "frac_of_hbm_peak": T * H * D * 4 / ms / 1e6 / HBM_PEAK_GBPS}
+    return res
+
+
+ZOMIPEL_SIZES = (("d1024", 1024, 8), ("d2048", 2048, 8), ("d4096", 4096, 4))        # name, width, layers
+
+
+def _zomipel_pair(d, n_layers, context, seed):
+    """(config, weights) of a Zomipel model -- per four layers: windowed attention with a dense feed-forward, two Mamba-2 and one
+    windowed attention with mixtures of 16 experts of which a token uses 4, and a shared one -- and of the reference decoder
+    of the same width and layers whose layers hold as many parameters as a token uses here on average (12 d^2)."""
+    import torch
+    g = torch.Generator(device="cuda:0").manual_seed(seed)
+    V, hd = 32000, 128 if d >= 2048 else 64
+    heads, kv, ssm_heads, N = d // hd, d // hd // 4, 2 * d // 64, 128
+    ff = d // 2
+
+    def w(*shape, std):
+        return (torch.randn(*shape, generator=g, device="cuda:0") * std).to(torch.bfloat16)
+
+    attention = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv, "dim": hd, "vdim": hd, "scale": hd ** -0.5,
+                                                "rot": {"base": 10000.0, "dims": hd}, "mask": {"size": 1024, "keep_first": 64}}}
+    mamba = {"type": "mamba2", "mixer": {"heads": ssm_heads, "vdim": 64, "state": N, "groups": 1, "norm_groups": 1, "conv": 4}}
+    dense = {"kind": "dense", "ff": 4 * d}
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 4}, "expert": {"ff": ff}, "shared": {"ff": ff}}
+    kinds = [(attention, dense), (mamba, moe), (mamba, moe), (attention, moe)]
+    cfg = dict(architecture="Zomipel", vocab=V, width=d, norm={"eps": 1e-6}, loop=None,
+               layers=[dict(kinds[i % 4][0], mlp=kinds[i % 4][1]) for i in range(n_layers)])
+    sd = {"embed": w(V, d, std=d ** -0.5), "final.norm": w(d, std=0.1)}
+    for i, layer in enumerate(cfg["layers"]):
+        n = f"l{i}."
+        sd[n + "norm1"] = w(d, std=0.1)
+        if layer["type"] == "attention":
+            for s, size in (("q", heads * hd), ("k", kv * hd), ("v", kv * hd)):
+                sd[n + f"mix.{s}"], sd[n + f"mix.{s}.b"] = w(size, d, std=d ** -0.5), w(size, std=0.1)
+            sd[n + "mix.o"] = w(d, heads * hd, std=d ** -0.5)
+        else:
+            inner, C = 2 * d, 2 * d + 2 * N
+            sd.update({n + "mix.in": w(inner + C + ssm_heads, d, std=d ** -0.5), n + "mix.conv": w(C, 4, std=0.5),
+                       n + "mix.conv.b": w(C, std=0.1), n + "mix.dt_bias": w(ssm_heads, std=0.5) - 3, n + "mix.A_log": w(ssm_heads, std=1.0),
+                       n + "mix.D": w(ssm_heads, std=0.5), n + "mix.norm": w(inner, std=0.1) + 1, n + "mix.o": w(d, inner, std=inner ** -0.5)})
+        if layer["mlp"] is dense:
+            sd[n + "mlp.up"], sd[n + "mlp.down"] = w(4 * d, d, std=d ** -0.5), w(d, 4 * d, std=(4 * d) ** -0.5)
+        else:
+            for e in [f"e{j}" for j in range(16)] + ["shared"]:
+                for s, shape in (("gate", (ff, d)), ("up", (ff, d)), ("down", (d, ff))):
+                    sd[n + f"mlp.{e}.{s}"] = w(*shape, std=shape[1] ** -0.5)
+            sd[n + "mlp.router"], sd[n + "mlp.router.b"] = w(16, d, std=d ** -0.5), w(16, std=0.1)
+            sd[n + "mlp.shared.sg"] = w(1, d, std=d ** -0.5)
+    rff = 21 * d // 8
+    ref_cfg = dict(vocab_size=V, context_length=context, d_model=d, num_layers=n_layers, num_heads=heads, d_ff=rff, rope_theta=10000.0)
+    ref = {"token_embeddings.weight": sd["embed"], "lm_head.weight": sd["embed"], "final_norm.weight": torch.ones(d)}
+    for i in range(n_layers):
+        pre = f"layers.{i}."
+        for s in ("q_proj", "k_proj", "v_proj", "output_proj"):
+            ref[pre + f"attn.{s}.weight"] = w(d, d, std=d ** -0.5)
+        for s, shape in (("gate_proj", (rff, d)), ("up_proj", (rff, d)), ("down_proj", (d, rff))):
+            ref[pre + f"ffn.{s}.weight"] = w(*shape, std=shape[1] ** -0.5)
+        ref[pre + "attn_norm.weight"] = ref[pre + "ffn_norm.weight"] = torch.ones(d)
+    return (cfg, sd), (ref_cfg, ref)
+
+
+def bench_zomipel(args):
+    """Prefill and decode of the Zomipel model beside the reference decoder at equal size (random weights, both through the same
+    engine and step functions, measured in turn), and its operators beside the like ones of the reference decoder."""
+    import torch
+    import mi355_attn as ma
+
+    names = ("zomipel", "reference_decoder")
+    res = {"models": {}, "operators": {}}
+    n_prompt, prompt_len, batch, ctx, context = 4, 2048, 32, 2048, 4096
+    for key, d, n_layers in ZOMIPEL_SIZES:
+        pairs = _zomipel_pair(d, n_layers, context, args.seed)
+        blocks = batch * (ctx + 256) // 16
+        models = [ma.ZomipelLM(*pairs[0], num_blocks=blocks, max_batch=batch, context_length=context, decode_graphs=True),
+                  ma.CachedTransformerLM(*pairs[1], num_blocks=blocks, max_batch=batch, decode_graphs=True)]
+        entry = {"workload": f"{n_layers} layers, width {d}, half Mamba-2 (state 128), half attention (window 1024 + 64 first tokens), 16 experts top 4, "
+                             f"vocab 32000; prefill: {n_prompt} new prompts of {prompt_len} tokens; decode: {batch} sequences at {ctx} tokens, HIP "
+                             "graph, greedy tokens fed back through the host"}
+        entry.update(_serve_side_by_side(names, models, args, n_prompt, prompt_len, batch, ctx))
+        res["models"][key] = entry
+        del models, pairs
+        torch.cuda.empty_cache()
+
+    dev = torch.device("cuda:0")
+    g = torch.Generator(device=dev).manual_seed(args.seed)
+
+    def t(*shape, dtype=torch.bfloat16, std=1.0):
+        return (torch.randn(*shape, device=dev, generator=g) * std).to(dtype)
+
+    def op(name, fn, nbytes=None, flops=None):
+        _, ms = timed(fn, args.steps, args.warmup, BURN_MS)
+        r = res["operators"][name] = {"device_ms": ms}
+        if nbytes:
+            r.update(algorithmic_bytes=nbytes, frac_of_hbm_peak=nbytes / ms / 1e6 / HBM_PEAK_GBPS)
+        if flops:
+            r.update(algorithmic_flops=flops, frac_of_mfma_peak=flops / ms / 1e9 / MFMA_BF16_PEAK_TFLOPS)
+
+    # streaming operators, 8192 rows of width 4096
+    T, d = 8192, 4096
+    w, resid, x, r, wide = t(d, dtype=torch.float32), t(T, d, dtype=torch.float32), t(T, d), t(T, d), t(T, 2 * d)
+    routed = t(T * 4, d)
+    op("residual_rms", lambda: ma.residual_rms(resid, w, sub=x, weight_offset=1.0), T * d * 12)
+    op("residual_rms with 4 routed rows", lambda: ma.residual_rms(resid, w, sub=x, routed=routed, top=4, weight_offset=1.0), T * d * 20)
+    op("rms_norm_residual (reference decoder)", lambda: ma.rms_norm(x, w, residual=r, return_sum=True), T * d * 8)
+    op("gelu", lambda: ma.ff_act(x), T * d * 4)
+    op("silu_mul with row gate", lambda: ma.ff_act(wide[:, :d], wide[:, d:], row_gate=resid[:, 0].contiguous()), T * d * 6)
+    op("silu_mul (reference decoder)", lambda: ma.silu_mul(wide[:, :d], wide[:, d:]), T * d * 6)
+    op("gated_norm", lambda: ma.gated_norm(x, r, w, 1, 1e-6), T * d * 6)
+    del routed
+
+    # Mamba-2 between its projections, inner 4096: 64 heads x 64, state 128
+    H, P, N, K = 64, 64, 128, 4
+    C = H * P + 2 * N
+    pr = dict(conv=t(K, C, dtype=torch.float32, std=0.5), conv_b=t(C, dtype=torch.float32), dt_bias=t(H, dtype=torch.float32) - 3,
+              neg_a=-torch.exp(t(H, dtype=torch.float32)), d_skip=t(H, dtype=torch.float32))
+    kw = dict(heads=H, vdim=P, state=N, groups=1)
+    conv, state = torch.zeros(32, K, C, dtype=torch.bfloat16, device=dev), torch.zeros(32, H, N, P, dtype=torch.float32, device=dev)
+    for n_seq, length in ((4, 2048), (1, 8192), (16, 512)):
+        proj = t(n_seq * length, C + H)
+        cu = torch.arange(0, n_seq * length + 1, length, dtype=torch.int32, device=dev)
+        pos = torch.arange(length, dtype=torch.int32, device=dev).repeat(n_seq)
+        slots = torch.arange(n_seq, dtype=torch.int32, device=dev)
+        # a token's outer product and read-out: 4 N P per head
+        op(f"ssm prefill {n_seq} x {length}", lambda: ma.ssm_mix(proj, 0, C, pr, conv, state, slots, pos, cu, **kw),
+           n_seq * length * 2 * (C + H + H * P), n_seq * length * 4 * N * P * H)
+    proj, slots = t(32, C + H), torch.arange(32, dtype=torch.int32, device=dev)
+    pos = torch.full((32,), 2048, dtype=torch.int32, device=dev)
+    op("ssm decode, 32 sequences", lambda: ma.ssm_mix(proj, 0, C, pr, conv, state, slots, pos, **kw), 32 * H * N * P * 8)
+
+    # experts: width 2048, 16 experts of 1024, 4 per token, beside library GEMMs of the same size
+    E, top, k, ff = 16, 4, 2048, 1024
+    wg, wd = t(E, 2 * ff, k, std=k ** -0.5), t(E, k, ff, std=ff ** -0.5)
+    router, bias = t(E, k, std=k ** -0.5), t(E, dtype=torch.float32)
+    for T in (8192, 32):
+        h = t(T, k)
+        ids, wt, _ = ma.moe_route(h, router, bias, top)
+        flops = T * top * 6 * k * ff if T > 1000 else None
+        nbytes = None if flops else E * 3 * k * ff * 2
+        op(f"router, {T} tokens", lambda: ma.moe_route(h, router, bias, top), T * k * 2)
+        op(f"experts, {T} tokens", lambda: ma.moe_experts(h, ids, wt, wg, wd), nbytes, flops)
+        if flops:
+            a, b = t(T * top, k), t(T * top, ff)
+            op("library GEMMs of the experts' size (reference decoder)", lambda: (a @ wg[0].T, b @ wd[0].T), None, flops)
+        else:
+            a, b = t(T, k), t(T, E * ff)
+            wu, wo = wg.view(E * 2 * ff, k), t(k, E * ff)
+            op("library GEMMs over the same weights, 32 tokens (reference decoder)", lambda: (a @ wu.T, b @ wo.T), nbytes)
+
+    # attention over a window of 1024 and 64 first tokens, and over every key, on the same tensors
+    H, G, D, S = 32, 8, 128, 4096
+    q, k, v = t(S, H, D), t(S, G, D), t(S, G, D)
+    cu = torch.tensor([0, S], dtype=torch.int32, device=dev)
+    seen = sum(min(i + 1, 1024 + min(64, max(0, i + 1 - 1024))) for i in range(S))
+    op("prefill attention, window", lambda: ma.flash_attn_varlen_prefill(q, k, v, cu, cu, S, S, window=1024, keep_first=64), None, 4 * H * D * seen)
+    op("prefill attention, every key (reference decoder)", lambda: ma.flash_attn_varlen_prefill(q, k, v, cu, cu, S, S), None, 4 * H * D * S * (S + 1) // 2)
+    B = 32
+    pools = [t(B * S // 16, G, 16, D) for _ in range(2)]
+    bt = torch.randperm(B * S // 16, device=dev).to(torch.int32).view(B, -1)
+    cl, q1 = torch.full((B,), S, dtype=torch.int32, device=dev), t(B, H, D)
+    ws = ma.paged_decode_workspace(B, H, D, S, dev)
+    op("decode attention, window", lambda: ma.paged_attention_decode(q1, *pools, bt, cl, workspace=ws, window=1024, keep_first=64), B * 1088 * G * D * 4)
+    cl1 = torch.full((B,), 1088, dtype=torch.int32, device=dev)
+    op("decode attention, every key of as many (reference decoder)", lambda: ma.paged_attention_decode(
+        q1, *pools, bt[:, :68], cl1, workspace=ws), B * 1088 * G * D * 4)
     return res
 
 
@@ -941,9 +1111,9 @@ def main():
     ap.add_argument("--warmup", type=int, default=50)
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--only", choices=["decode", "prefill", "small", "few", "fp8", "backward", "producers", "layer", "loop",
-                                       "zuzelorn"],
-                    default=None, help="one leg; `zuzelorn` (the Zuzelorn model beside the reference decoder at equal size) "
-                                       "runs only when it is named")
+                                       "zuzelorn", "zomipel"],
+                    default=None, help="one leg; `zuzelorn` and `zomipel` (these models beside the reference decoder at equal size) "
+                                       "run only when they are named")
     ap.add_argument("--no-cpu", action="store_true")
     ap.add_argument("--full", action="store_true", help="print every leg's whole object (a line of about 10 KB)")
     ap.add_argument("--detail", default=None, metavar="PATH", help="also write the verbose form to this file")
@@ -1025,10 +1195,10 @@ def main():
         line["decode_few_sequences"] = bench_decode_few_sequences(args)
         line["decode_loop"] = bench_decode_loop(args)
 
-    if args.only == "zuzelorn":
-        z = line["zuzelorn"] = bench_zuzelorn(args)
+    if args.only in ("zuzelorn", "zomipel"):
+        z = line[args.only] = {"zuzelorn": bench_zuzelorn, "zomipel": bench_zomipel}[args.only](args)
         first = z["models"]["d2048"]
-        line.update({"value": first["zuzelorn"]["prefill_tokens_per_s"], "unit": "tokens/s", "ms_per_step": first["zuzelorn"]["prefill_ms"],
+        line.update({"value": first[args.only]["prefill_tokens_per_s"], "unit": "tokens/s", "ms_per_step": first[args.only]["prefill_ms"],
                      "dtype": "bf16", "config": {"workload": first["workload"]}})
 
     if with_cpu:

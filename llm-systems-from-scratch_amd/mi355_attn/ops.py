@@ -1422,7 +1422,7 @@ def moe_experts(h, ids, weights, w_gate_up, w_down, *, tiling="auto"):
         if t.dtype != dt or tuple(t.shape) != (T, top) or not t.is_contiguous():
             raise ValueError(f"{name} must be a contiguous {dt} ({T}, {top}) tensor")
     dev = h.device
-    out = torch.empty(T * top, n, dtype=h.dtype, device=dev)
+    out = torch.empty(T * top, n + (-n % 8), dtype=h.dtype, device=dev)[:, :n]            # (16-byte aligned rows)
     if T == 0:
         return out
     offsets = torch.empty(E + 1, dtype=torch.int32, device=dev)
@@ -1436,6 +1436,6 @@ def moe_experts(h, ids, weights, w_gate_up, w_down, *, tiling="auto"):
                                    h.stride(0) if T > 1 else k, ff, E, top, k, ff, code, tl, stream)
         _lib.check(rc, "mi355_moe_gate_up")
         rc = lib.mi355_moe_down(act.data_ptr(), w_down.data_ptr(), weights.data_ptr(), out.data_ptr(), offsets.data_ptr(),
-                                order.data_ptr(), T, ff, n, E, top, ff, n, code, tl, stream)
+                                order.data_ptr(), T, ff, out.stride(0), E, top, ff, n, code, tl, stream)
         _lib.check(rc, "mi355_moe_down")
     return out

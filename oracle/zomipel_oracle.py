@@ -194,3 +194,52 @@ def forward(config, params, tokens, dtype=torch.float32, want_layers=False):
         after.append(x)
     logits = offset_rms_norm(x, p["final.norm"], eps) @ p["embed"].T
     return (logits, torch.stack(after)) if want_layers else logits
+
+
+def random_params(config, seed):
+    """bf16 parameters of a configuration, of sizes that keep the residual stream near one, let the attention prefer single keys and
+    give the recurrences memories between a few and a few hundred tokens."""
+    g = torch.Generator().manual_seed(seed)
+    r = lambda *s, std=1.0, mean=0.0: (torch.randn(*s, generator=g) * std + mean).to(torch.bfloat16)
+    d, p = config["width"], {}
+    w = lambda name, rows, cols, gain=1.0: p.__setitem__(name, r(rows, cols, std=gain / math.sqrt(cols)))
+
+    def gated(n, ff):
+        w(n + ".gate", ff, d, 1.5)
+        w(n + ".up", ff, d, 1.5)
+        w(n + ".down", d, ff, 1.0)
+
+    p["embed"] = r(config["vocab"], d, std=0.7)
+    p["final.norm"] = r(d, std=0.2)
+    for i, layer in enumerate(config["layers"]):
+        n, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        p[n + "norm1"] = r(d, std=0.2)
+        if layer["type"] == "attention":
+            for name, size, gain in (("q", m["heads"] * m["dim"], 1.6), ("k", m["kv_heads"] * m["dim"], 1.6), ("v", m["kv_heads"] * m["vdim"], 1.0)):
+                w(f"{n}mix.{name}", size, d, gain)
+                p[f"{n}mix.{name}.b"] = r(size, std=0.3)
+            w(n + "mix.o", d, m["heads"] * m["vdim"])
+        else:
+            inner, bc = m["heads"] * m["vdim"], m["groups"] * m["state"]
+            w(n + "mix.in", 2 * inner + 2 * bc + m["heads"], d)
+            p[n + "mix.conv"] = r(inner + 2 * bc, m["conv"], std=0.6)
+            p[n + "mix.conv.b"] = r(inner + 2 * bc, std=0.2)
+            p[n + "mix.dt_bias"] = r(m["heads"], std=0.5, mean=-2.0)
+            p[n + "mix.A_log"] = r(m["heads"], std=1.5, mean=-1.0)
+            p[n + "mix.D"] = r(m["heads"], std=0.5, mean=0.5)
+            p[n + "mix.norm"] = r(inner, std=0.2, mean=1.0)
+            w(n + "mix.o", d, inner)
+        if f is None:
+            continue
+        if f["kind"] == "dense":
+            w(n + "mlp.up", f["ff"], d, 1.5)
+            w(n + "mlp.down", d, f["ff"])
+            continue
+        for e in range(f["router"]["experts"]):
+            gated(f"{n}mlp.e{e}", f["expert"]["ff"])
+        w(n + "mlp.router", f["router"]["experts"], d, 2.0)
+        p[n + "mlp.router.b"] = r(f["router"]["experts"], std=0.3)
+        if f.get("shared") is not None:
+            gated(n + "mlp.shared", f["shared"]["ff"])
+            w(n + "mlp.shared.sg", 1, d, 1.5)
+    return p

@@ -1,0 +1,732 @@
+"""GPU parity of the Zomipel model and of the operators that it brought, against the plain oracle.
+
+Tolerances.  Operators: fp32 results within 1e-5 relative to the result's scale (2e-5 where a recurrence or a long sum is behind
+them); bf16 elementwise operators within one bf16 ulp of the oracle on the same inputs; bf16 attention, products and recurrences
+by the root mean square per row of the difference over that of the reference: 1e-2 (bf16 rounding of weights or results is 4e-3).
+Model logits: the same measure over the vocabulary, 2e-5 in fp32, 3e-2 in bf16.  Rows in which a router's choice is closer than
+bf16 can tell are left out of the bf16 model comparisons, and what the model's own rounding of h decides stays decided: nothing
+rests on a close call.
+"""
+import json
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+from oracle import zomipel_oracle as zo
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+DTYPES = [torch.bfloat16, torch.float32]
+
+
+@pytest.fixture(scope="module")
+def ops():
+    import mi355_attn
+    mi355_attn.load()
+    return mi355_attn
+
+
+def gen(seed):
+    return torch.Generator().manual_seed(seed)
+
+
+def rnd(*shape, seed, std=1.0, dtype=torch.float32):
+    return (torch.randn(*shape, generator=gen(seed)) * std).to(dtype)
+
+
+def close(got, ref, dtype):
+    got = got.float().cpu()
+    if dtype == torch.float32:
+        torch.testing.assert_close(got, ref, atol=1e-5 * float(ref.abs().max().clamp_min(1.0)), rtol=1e-5)
+    else:
+        torch.testing.assert_close(got, ref, atol=2e-3, rtol=2.0 ** -7)
+
+
+def rel(got, ref):
+    got, ref = got.float().cpu().flatten(1), ref.float().flatten(1)
+    return (got - ref).pow(2).mean(1).sqrt() / ref.pow(2).mean(1).sqrt().clamp_min(1e-6)
+
+
+def rows_close(got, ref, dtype, limit=1e-2, what=""):
+    assert got.shape == ref.shape
+    e = rel(got, ref)
+    worst = int(e.argmax())
+    assert bool(torch.isfinite(got).all()), what
+    assert float(e.max()) <= (2e-5 if dtype == torch.float32 else limit), f"{what}: row {worst} is off by {float(e.max()):.3g}"
+
+
+# ---- sliding window with kept first tokens -------------------------------------------------------------
+def edge_case(n, H, G, dk, dv, seed, dtype, loud):
+    """Queries, keys and values of n tokens in which the keys `loud` draw nearly all of the weight of every query that sees them
+    (scores above the others' by about 8): a window that is one key off replaces most of a result."""
+    q, k, v = rnd(n, H, dk, seed=seed), rnd(n, G, dk, seed=seed + 1, std=0.5), rnd(n, G, dv, seed=seed + 2)
+    q[:, :, 0] = 8.0
+    k[:, :, 0] = 0.0
+    for j in loud:
+        k[j, :, 0] = 1.0 + 0.02 * (j % 7)
+    return tuple(t.to(dtype) for t in (q, k, v))
+
+
+def cached(k, v, block_order, dk, dv, dtype):
+    """Keys and values in a pool whose blocks are handed out in a scrambled order."""
+    n, G = k.shape[:2]
+    nb = len(block_order)
+    kc, vc = (torch.full((nb, G, 16, d), 7.0, dtype=dtype) for d in (dk, dv))
+    for j in range(n):
+        kc[block_order[j // 16], :, j % 16], vc[block_order[j // 16], :, j % 16] = k[j], v[j]
+    return kc.cuda(), vc.cuda(), torch.tensor([block_order], dtype=torch.int32).cuda()
+
+
+WINDOWS = [(1, 0), (1, 3), (16, 16), (17, 1), (40, 20), (64, 70), (100, 0), (129, 33), (37, 200)]
+
+
+@pytest.mark.parametrize("D,H,G", [(32, 4, 4), (64, 6, 2), (128, 8, 1)])
+@pytest.mark.parametrize("window,keep", WINDOWS)
+def test_window_in_decoding(ops, D, H, G, window, keep):
+    for n in (1, 2, keep + 1, window + keep, window + keep + 1, 272, 273, 300, 1500):
+        print(f"case: decode D {D} window {window} keep {keep} n {n}", flush=True)
+        last = n - 1
+        loud = {j for j in (last - window, last - window + 1, keep - 1, keep, keep + 1) if 0 <= j < n}
+        q, k, v = edge_case(n, H, G, D, D, n + D, torch.bfloat16, loud)
+        kc, vc, bt = cached(k, v, torch.randperm((n + 15) // 16, generator=gen(n)).tolist(), D, D, torch.bfloat16)
+        cl = torch.tensor([n], dtype=torch.int32).cuda()
+        ref = zo.window_attention(q[-1:].float(), k.float(), v.float(), 1.0, window, keep, first=last)
+        got = ops.paged_attention_decode(q[-1:].cuda(), kc, vc, bt, cl, softmax_scale=1.0, window=window, keep_first=keep)
+        rows_close(got, ref, torch.bfloat16, what=f"decode n {n}")
+        wide = torch.full((1, H * D + 24), 3.0, dtype=torch.bfloat16).cuda()               # into the rows of a wider matrix
+        ops.paged_attention_decode(q[-1:].cuda(), kc, vc, bt, cl, softmax_scale=1.0, window=window, keep_first=keep,
+                                   out=wide[:, :H * D].view(1, H, D))
+        assert torch.equal(wide[:, :H * D].view(1, H, D), got) and bool((wide[:, H * D:] == 3.0).all())
+        for dtype in DTYPES:
+            qa, kca, vca = (t.to(dtype) for t in (q[-1:].cuda(), kc, vc))
+            got = ops.paged_attention_any(qa, kca, vca, bt, cl, softmax_scale=1.0, window=window, keep_first=keep)
+            rows_close(got, ref, dtype, what=f"general decode n {n} {dtype}")
+
+
+@pytest.mark.parametrize("D,H,G", [(32, 2, 2), (64, 4, 2), (128, 3, 1)])
+@pytest.mark.parametrize("window,keep", WINDOWS)
+def test_window_in_prompts(ops, D, H, G, window, keep):
+    n = 330
+    print(f"case: prefill D {D} window {window} keep {keep}", flush=True)
+    loud = {0, 5, 63, 64, 120, 200, 255, 256, 257, 311} | {j for j in (keep - 1, keep) if 0 <= j < n}
+    q, k, v = edge_case(n, H, G, D, D, D + window, torch.bfloat16, loud)
+    ref = zo.window_attention(q.float(), k.float(), v.float(), 1.0, window, keep)
+    cu = torch.tensor([0, n], dtype=torch.int32).cuda()
+    qc, kd, vd = q.cuda(), k.cuda(), v.cuda()
+    wide = torch.full((n, H * D + 8), 3.0, dtype=torch.bfloat16).cuda()
+    got = ops.flash_attn_varlen_prefill(qc, kd, vd, cu, cu, n, n, softmax_scale=1.0, window=window, keep_first=keep,
+                                        out=wide[:, :H * D].view(n, H, D))
+    rows_close(got, ref, torch.bfloat16, what="packed")
+    assert bool((wide[:, H * D:] == 3.0).all())
+    order = torch.randperm((n + 15) // 16, generator=gen(5)).tolist()
+    kc, vc, bt = cached(k, v, order, D, D, torch.bfloat16)
+    for a, b in ((0, 2), (2, 70), (70, 263), (263, 330), (328, 330), (17, 330)):          # portions of a prompt
+        cq, cl = torch.tensor([0, b - a], dtype=torch.int32).cuda(), torch.tensor([b], dtype=torch.int32).cuda()
+        got = ops.flash_attn_paged_prefill(qc[a:b], kc, vc, cq, bt, cl, b - a, softmax_scale=1.0, window=window, keep_first=keep)
+        rows_close(got, ref[a:b], torch.bfloat16, what=f"portion {a}..{b}")
+        for dtype in DTYPES:
+            got = ops.paged_attention_any(qc[a:b].to(dtype), kc.to(dtype), vc.to(dtype), bt, cl, cu_seqlens_q=cq, softmax_scale=1.0,
+                                          window=window, keep_first=keep)
+            rows_close(got, ref[a:b], dtype, what=f"general portion {a}..{b} {dtype}")
+
+
+def test_window_prefill_scores_outside_the_preset_range(ops):
+    """Scores that the kernel's first attempt cannot represent: the tile is computed again with tracked maxima."""
+    n, H, D, window, keep = 300, 2, 64, 70, 9
+    print("case: window prefill, large scores", flush=True)
+    q, k, v = edge_case(n, H, H, D, D, 3, torch.bfloat16, {4, 130, 200})
+    for scale in (30.0, 0.3):
+        q2 = q.clone()
+        q2[:, :, 0] = -60.0 if scale > 1 else 8.0
+        ref = zo.window_attention(q2.float(), k.float(), v.float(), scale, window, keep)
+        cu = torch.tensor([0, n], dtype=torch.int32).cuda()
+        got = ops.flash_attn_varlen_prefill(q2.cuda(), k.cuda(), v.cuda(), cu, cu, n, n, softmax_scale=scale, window=window, keep_first=keep)
+        rows_close(got, ref, torch.bfloat16, limit=2e-2, what=f"scale {scale}")
+
+
+def test_window_with_unequal_sequences(ops):
+    print("case: window, batch", flush=True)
+    H, G, D, window, keep = 4, 2, 64, 50, 7
+    lens = [1, 200, 33, 450]
+    parts = [edge_case(n, H, G, D, D, n, torch.bfloat16, {3, 20, n - 1, max(0, n - 60)} & set(range(n))) for n in lens]
+    q, k, v = (torch.cat([p[i] for p in parts]) for i in range(3))
+    ref = torch.cat([zo.window_attention(*(t.float() for t in p), 1.0, window, keep) for p in parts])
+    cu = torch.tensor([0] + lens).cumsum(0).int().cuda()
+    got = ops.flash_attn_varlen_prefill(q.cuda(), k.cuda(), v.cuda(), cu, cu, 450, 450, softmax_scale=1.0, window=window, keep_first=keep)
+    rows_close(got, ref, torch.bfloat16, what="packed batch")
+
+
+# ---- rotation --------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("D,dims", [(20, 20), (40, 16), (64, 64), (128, 32), (48, 2)])
+def test_partial_rotation(ops, D, dims, dtype):
+    print(f"case: rotation {D} {dims} {dtype}", flush=True)
+    from mi355_attn.weights import pair_halves
+    T, H, G = 9, 3, 2
+    q, k = rnd(T, H, D, seed=1, dtype=dtype), rnd(T, G, D, seed=2, dtype=dtype)
+    pos = torch.tensor([0, 1, 2, 63, 64, 500, 4095, 17, 3], dtype=torch.int32)
+    table = ops.build_partial_rope_cache(4096, D, dims, 700.0, "cuda")
+    adj = lambda t, h: pair_halves(t.permute(1, 2, 0).reshape(h * D, T), h, D, dims).view(h, D, T).permute(2, 0, 1).contiguous()
+    qa, ka = adj(q, H).cuda(), adj(k, G).cuda()
+    ops.rope_rotate(qa, ka, pos.cuda(), table)
+    for got, x, h in ((qa, q, H), (ka, k, G)):
+        ref = torch.stack([zo.rotate(x[t].double(), int(pos[t]), 700.0, dims) for t in range(T)]).float()
+        got, want = got.float().cpu(), adj(ref, h)
+        torch.testing.assert_close(got, want, atol=2e-5 if dtype == torch.float32 else 2e-2, rtol=2e-5 if dtype == torch.float32 else 2 ** -7)
+
+
+# ---- elementwise operators -----------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,d", [(1, 8), (5, 72), (7, 100), (33, 1024), (9, 2056), (3, 8200)])
+def test_residual_rms(ops, T, d, dtype):
+    print(f"case: residual_rms {T}x{d} {dtype}", flush=True)
+    top, eps = 3, 1e-3
+    resid, w = rnd(T, d, seed=1, std=2.0), rnd(d, seed=2, std=0.4)
+    sub, routed, emb = rnd(T, d + 8, seed=3, dtype=dtype), rnd(T * top, d, seed=4, dtype=dtype), rnd(11, d, seed=5, dtype=dtype)
+    tok = torch.randint(0, 11, (T,), generator=gen(6))
+    for parts in (("sub", "routed", "embed"), ("sub",), ("embed",), ("routed",), ()):
+        x = resid.clone()
+        if "sub" in parts:
+            x = x + sub[:, :d].float()
+        if "embed" in parts:
+            x = x + emb[tok].float()
+        if "routed" in parts:
+            x = x + routed.float().view(T, top, d).sum(1)
+        r = resid.cuda()
+        cols = d + (-d % 64)
+        out, y = ops.residual_rms(r, w.cuda(), sub=sub.cuda()[:, :d] if "sub" in parts else None, routed=routed.cuda() if "routed" in parts else None,
+                                  top=top, embed=emb.cuda() if "embed" in parts else None, tokens=tok.cuda() if "embed" in parts else None,
+                                  weight_offset=1.0, eps=eps, out_dtype=dtype, y_cols=cols)
+        assert out is r
+        close(r, x, torch.float32)
+        close(y[:, :d], zo.offset_rms_norm(x, w, eps), dtype)
+        assert bool((y[:, d:] == 0).all())
+    x, y = ops.residual_rms(None, w.cuda(), embed=emb.cuda(), tokens=tok.cuda(), weight_offset=1.0, eps=eps, out_dtype=dtype)
+    assert torch.equal(x.cpu(), emb[tok].float())
+    close(y, zo.offset_rms_norm(emb[tok].float(), w, eps), dtype)
+    x, y = ops.residual_rms(x, None, sub=sub.cuda()[:, :d], out_dtype=dtype)
+    assert y is None
+    close(x, emb[tok].float() + sub[:, :d].float(), torch.float32)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("d", [8, 30, 1000])
+def test_activations(ops, d, dtype):
+    print(f"case: ff_act {d} {dtype}", flush=True)
+    wide = rnd(6, 2 * d + 16, seed=d, std=3.0, dtype=dtype)
+    wide[0, :4] = torch.tensor([0.0, 60.0, -60.0, -3.0])
+    a, b = wide[:, :d], wide[:, d:2 * d]
+    gate = rnd(6, seed=2, std=2.0)
+    wc = wide.cuda()
+    close(ops.ff_act(wc[:, :d]), zo.gelu_tanh(a.float()), dtype)
+    close(ops.ff_act(wc[:, :d], wc[:, d:2 * d]), zo.silu(a.float()) * b.float(), dtype)
+    close(ops.ff_act(wc[:, :d], wc[:, d:2 * d], row_gate=gate.cuda()), zo.silu(a.float()) * b.float() * torch.sigmoid(gate)[:, None], dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("d,groups", [(24, 3), (64, 1), (90, 2), (1536, 1), (4096, 4), (5000, 1)])
+def test_gated_norm(ops, d, groups, dtype):
+    print(f"case: gated_norm {d} {groups} {dtype}", flush=True)
+    wide, w = rnd(5, 2 * d + 8, seed=d, dtype=dtype), rnd(d, seed=1)
+    wide[2] *= 1e-3
+    wc = wide.cuda()
+    ref = zo.gated_group_norm(wide[:, :d].float(), wide[:, d:2 * d].float(), w, groups, 1e-4)
+    close(ops.gated_norm(wc[:, :d], wc[:, d:2 * d], w.cuda(), groups, 1e-4), ref, dtype)
+    ops.gated_norm(wc[:, :d], wc[:, d:2 * d], w.cuda(), groups, 1e-4, out=wc[:, :d])             # in place
+    close(wc[:, :d], ref, dtype)
+
+
+# ---- Mamba-2 ------------------------------------------------------------------------------------------------------
+SSM = [dict(heads=4, vdim=16, state=32, groups=2, taps=4), dict(heads=3, vdim=6, state=10, groups=1, taps=2),
+       dict(heads=2, vdim=64, state=128, groups=1, taps=3), dict(heads=2, vdim=72, state=200, groups=2, taps=5),
+       dict(heads=2, vdim=8, state=256, groups=1, taps=1), dict(heads=1, vdim=136, state=24, groups=1, taps=16)]
+
+
+def ssm_case(m, T, seed, dtype):
+    H, P, N, G, K = (m[k] for k in ("heads", "vdim", "state", "groups", "taps"))
+    C = H * P + 2 * G * N
+    pad = -C % 8
+    proj = rnd(T, 8 + C + pad + H + (-H % 8), seed=seed, dtype=dtype)                # 8 columns of something else in front
+    f = lambda *s, k, std, mean=0.0: rnd(*s, seed=seed + k, std=std) + mean
+    params = dict(conv=f(K, C, k=1, std=0.6), conv_b=f(C, k=2, std=0.2), dt_bias=f(H, k=3, std=0.5, mean=-2.5), neg_a=-torch.exp(f(H, k=4, std=1.0, mean=-2.0)),
+                  d_skip=f(H, k=5, std=0.5))
+    return proj, params, 8, 8 + C + pad
+
+
+def ssm_oracle(m, proj, params, xbc_at, dt_at, round_conv):
+    H, P, N, G = (m[k] for k in ("heads", "vdim", "state", "groups"))
+    T, C = proj.shape[0], H * P + 2 * G * N
+    u = zo.causal_conv_silu(proj[:, xbc_at:xbc_at + C].float(), params["conv"].t(), params["conv_b"])
+    if round_conv:
+        u = u.bfloat16().float()
+    x, B, Cc = torch.split(u, [H * P, G * N, G * N], -1)
+    y, S = zo.selective_state(x.reshape(T, H, P), B.reshape(T, G, N), Cc.reshape(T, G, N),
+                              zo.softplus(proj[:, dt_at:dt_at + H].float() + params["dt_bias"]), params["neg_a"], params["d_skip"])
+    return y.reshape(T, H * P), S
+
+
+def ssm_pools(m, n_slots, dtype):
+    C = m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"]           # slots start with rubbish: a first token must not see it
+    return (torch.full((n_slots, m["taps"], C), 50.0, dtype=dtype).cuda(),
+            torch.full((n_slots, m["heads"], m["state"], (m["vdim"] + 3) // 4 * 4), 1e6).cuda())
+
+
+@pytest.mark.parametrize("scan,dtype", [("serial", torch.float32), ("serial", torch.bfloat16), ("chunked", torch.bfloat16)])
+@pytest.mark.parametrize("m", SSM, ids=lambda m: "-".join(str(v) for v in m.values()))
+def test_state_space_mixer(ops, m, scan, dtype):
+    if scan == "chunked" and (m["state"] % 8 or m["vdim"] % 8):
+        scan = "auto"
+    T = 203
+    proj, params, xbc_at, dt_at = ssm_case(m, T, 7, dtype)
+    ref, S = ssm_oracle(m, proj, params, xbc_at, dt_at, dtype == torch.bfloat16)
+    kw = {k: m[k] for k in ("heads", "vdim", "state", "groups")}
+    pc = {k: v.cuda() for k, v in params.items()}
+    slots = torch.tensor([2], dtype=torch.int32).cuda()
+    for cuts in ((203,), (64, 128, 203), (1, 2, 4, 66, 67, 130, 131, 203), (100, 101, 102, 103, 203)):
+        print(f"case: ssm {m} {scan} {dtype} cuts {cuts}", flush=True)
+        conv, state = ssm_pools(m, 4, dtype)
+        got, a = [], 0
+        for b in cuts:
+            pos = torch.arange(a, b, dtype=torch.int32).cuda()
+            if b - a == 1:
+                got.append(ops.ssm_mix(proj[a:b].cuda(), xbc_at, dt_at, pc, conv, state, slots, pos, **kw))
+            else:
+                cu = torch.tensor([0, b - a], dtype=torch.int32).cuda()
+                got.append(ops.ssm_mix(proj[a:b].cuda(), xbc_at, dt_at, pc, conv, state, slots, pos, cu, scan=scan, **kw))
+            a = b
+        rows_close(torch.cat(got), ref, dtype, what=f"{cuts}")
+        s = state[2, :, :, :m["vdim"]].cpu()
+        e = float((s - S).pow(2).mean().sqrt() / S.pow(2).mean().sqrt())
+        assert e <= (1e-5 if dtype == torch.float32 else 1.5e-3), e
+        assert bool((state[[0, 1, 3]] == 1e6).all()) and bool((conv[[0, 1, 3]] == 50.0).all())            # nobody else's slot
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_state_space_batches(ops, dtype):
+    """Unequal sequences in one call, at scattered slots, then a decode step of all of them; every sequence against itself alone."""
+    m = SSM[0]
+    kw = {k: m[k] for k in ("heads", "vdim", "state", "groups")}
+    lens, slots = [65, 1, 2, 130, 17], [4, 0, 6, 1, 3]
+    print(f"case: ssm batch {dtype}", flush=True)
+    cases = [ssm_case(m, n + 1, 30, dtype) for n in lens]
+    params, xbc_at, dt_at = cases[0][1], cases[0][2], cases[0][3]
+    projs = [rnd(n + 1, cases[0][0].shape[1], seed=n, dtype=dtype) for n in lens]
+    conv, state = ssm_pools(m, 7, dtype)
+    pc, sl = {k: v.cuda() for k, v in params.items()}, torch.tensor(slots, dtype=torch.int32).cuda()
+    cu = torch.tensor([0] + lens).cumsum(0).int().cuda()
+    got = ops.ssm_mix(torch.cat([p[:-1] for p in projs]).cuda(), xbc_at, dt_at, pc, conv, state, sl,
+                      torch.cat([torch.arange(n) for n in lens]).int().cuda(), cu, **kw)
+    step = ops.ssm_mix(torch.cat([p[-1:] for p in projs]).cuda(), xbc_at, dt_at, pc, conv, state, sl, torch.tensor(lens).int().cuda(), **kw)
+    for i, (p, n) in enumerate(zip(projs, lens)):
+        ref, _ = ssm_oracle(m, p, params, xbc_at, dt_at, dtype == torch.bfloat16)
+        rows_close(torch.cat((got[cu[i]:cu[i + 1]], step[i:i + 1])), ref, dtype, what=f"sequence {i}")
+
+
+def test_chunked_scan_forgets_and_remembers(ops):
+    """Decays from almost none to complete within a token: chunks agree with the token-by-token form."""
+    m = SSM[2]
+    print("case: ssm extreme decays", flush=True)
+    kw = {k: m[k] for k in ("heads", "vdim", "state", "groups")}
+    proj, params, xbc_at, dt_at = ssm_case(m, 300, 3, torch.bfloat16)
+    params["neg_a"] = torch.tensor([-1e-4, -400.0])
+    params["dt_bias"] = torch.tensor([-1.0, 2.0])
+    ref, _ = ssm_oracle(m, proj, params, xbc_at, dt_at, True)
+    conv, state = ssm_pools(m, 1, torch.bfloat16)
+    got = ops.ssm_mix(proj.cuda(), xbc_at, dt_at, {k: v.cuda() for k, v in params.items()}, conv, state,
+                      torch.zeros(1, dtype=torch.int32).cuda(), torch.arange(300).int().cuda(), torch.tensor([0, 300], dtype=torch.int32).cuda(),
+                      scan="chunked", **kw)
+    rows_close(got, ref, torch.bfloat16)
+
+
+# ---- mixture of experts -------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("E,top", [(1, 1), (8, 2), (17, 17), (64, 6), (200, 3)])
+def test_router(ops, E, top, dtype):
+    T, k = 37, 72
+    print(f"case: route {E} {top} {dtype}", flush=True)
+    h, w, b = rnd(T, k + 8, seed=1, dtype=dtype), rnd(E + 1, k, seed=2, std=0.3, dtype=dtype), rnd(E + 1, seed=3)
+    ids, wt, extra = ops.moe_route(h.cuda()[:, :k], w.cuda(), b.cuda(), top, extra_row=True)
+    z = h[:, :k].float() @ w.float().t() + b
+    close(extra, z[:, E], torch.float32)
+    for t in range(T):
+        chosen, weight = zo.route(h[t, :k].float(), w[:E].float(), b[:E], top)
+        gap = torch.sort(z[t, :E], descending=True).values.diff().abs().min() if E > 1 else 1.0
+        if gap > 1e-4:
+            assert ids[t].tolist() == chosen, t
+        torch.testing.assert_close(wt[t].cpu(), weight, atol=1e-5, rtol=1e-4)
+    ids2, _, none = ops.moe_route(h.cuda()[:, :k], w[:E].contiguous().cuda(), b[:E].contiguous().cuda(), top)
+    assert none is None and torch.equal(ids, ids2)
+    ids, wt, _ = ops.moe_route(torch.zeros_like(h[:2, :k]).cuda(), w.cuda(), torch.zeros(E + 1).cuda(), top, extra_row=True)      # ties
+    assert ids.tolist() == [list(range(top))] * 2 and bool(((wt - 1.0 / top).abs() < 1e-6).all())
+
+
+@pytest.mark.parametrize("tiling,dtype", [("skinny", torch.bfloat16), ("large", torch.bfloat16), ("auto", torch.float32)])
+@pytest.mark.parametrize("T,E,top,k,ff,n", [(1, 4, 2, 64, 64, 40), (50, 8, 3, 128, 192, 72), (300, 5, 2, 192, 64, 200), (700, 2, 1, 64, 128, 130)])
+def test_experts(ops, T, E, top, k, ff, n, tiling, dtype):
+    print(f"case: experts {T} {E} {top} {k} {ff} {n} {tiling} {dtype}", flush=True)
+    h, wg = rnd(T, k + 8, seed=1, dtype=dtype), rnd(E, 2 * ff, k, seed=2, std=k ** -0.5, dtype=dtype)
+    wd, wt = rnd(E, n, ff, seed=3, std=ff ** -0.5, dtype=dtype), torch.rand(T, top, generator=gen(4))
+    scattered = torch.stack([torch.randperm(E, generator=gen(t))[:top] for t in range(T)]).int()
+    crowded = torch.arange(top).repeat(T, 1).int()                         # everybody with the first experts, the others idle
+    for ids in (scattered, crowded):
+        got = ops.moe_experts(h.cuda()[:, :k], ids.cuda(), wt.cuda(), wg.cuda(), wd.cuda(), tiling=tiling)
+        ref = torch.zeros(T * top, n)
+        for t in range(T):
+            for c in range(top):
+                e = int(ids[t, c])
+                a = zo.silu(wg[e, :ff].float() @ h[t, :k].float()) * (wg[e, ff:].float() @ h[t, :k].float())
+                ref[t * top + c] = wt[t, c] * (wd[e].float() @ a)
+        rows_close(got, ref, dtype, what=f"{tiling}")
+
+
+# ---- the model ---------------------------------------------------------------------------------------------------------
+def attn(window, keep, **kw):
+    return {"type": "attention", "mixer": dict(dict(heads=4, kv_heads=2, dim=24, vdim=24, rot={"base": 300.0, "dims": 24}, scale=0.25,
+                                                    mask={"size": window, "keep_first": keep}), **kw)}
+
+
+def mamba(**kw):
+    return {"type": "mamba2", "mixer": dict(dict(heads=4, vdim=16, state=24, groups=2, norm_groups=2, conv=4), **kw)}
+
+
+def dense(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe(experts, top, ff, shared=None):
+    return {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}, "shared": shared and {"ff": shared}}
+
+
+def net(layers, **kw):
+    return dict(dict(architecture="Zomipel", norm={"eps": 1e-5}, layers=[dict(ly, mlp=f) for ly, f in layers], loop=None), **kw)
+
+
+CONFIGS = {
+    # unequal head sizes and partial rotation, every kind of feed-forward, a loop that leaves layers on both sides
+    "mixed": net([(attn(20, 5, heads=6, dim=40, vdim=24, rot={"base": 100.0, "dims": 16}), moe(6, 2, 40, 56)), (mamba(), dense(72)),
+                  (mamba(heads=6, groups=3, norm_groups=1, conv=2), None), (attn(33, 18), moe(4, 3, 24))],
+                 vocab=53, width=72, loop={"start": 1, "stop": 4, "times": 3}),
+    # nothing a multiple of 8, a first kept stretch longer than the window, one expert, one pass
+    "odd": net([(mamba(heads=3, vdim=6, state=10, groups=1, norm_groups=3, conv=3), moe(1, 1, 18, 10)),
+                (attn(9, 30, heads=3, kv_heads=1, dim=20, vdim=36, rot={"base": 10.0, "dims": 12}), dense(30)),
+                (mamba(heads=5, vdim=10, state=7, groups=5, norm_groups=5, conv=1), moe(3, 3, 26)), (attn(1, 0, heads=2, kv_heads=2), None)],
+               vocab=61, width=50, norm={"eps": 1e-3}),
+    # MFMA head sizes as they are, attention in front, everything looped twice
+    "plain": net([(attn(48, 0, heads=8, kv_heads=2, dim=64, vdim=64, rot={"base": 10000.0, "dims": 64}, scale=0.1), dense(128)),
+                  (mamba(heads=2, vdim=64, state=64, groups=1, norm_groups=1), moe(16, 4, 64, 64))], vocab=80, width=128,
+                 loop={"start": 0, "stop": 2, "times": 2}),
+    # attention only, heads for the general kernel; and no attention at all
+    "general": net([(attn(25, 3, heads=2, kv_heads=1, dim=136, vdim=72, rot={"base": 50.0, "dims": 136}, scale=0.08), dense(40))] * 2, vocab=40, width=64),
+    "stateful": net([(mamba(), moe(5, 2, 32, 24)), (mamba(heads=8, vdim=8), dense(48))], vocab=47, width=56, loop={"start": 1, "stop": 2, "times": 2}),
+}
+LIMIT = {"float32": 2e-5, "bfloat16": 3e-2}
+BOTH = pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+NAMES = pytest.mark.parametrize("name", list(CONFIGS))
+_params, _runs = {}, {}
+
+
+def params(name):
+    if name not in _params:
+        _params[name] = zo.random_params(CONFIGS[name], 11)
+    return _params[name]
+
+
+def router_gap(cfg, p, toks):
+    """Per position, how close the closest call of any router was (and of any router on earlier positions, which states and keys
+    carry on): the smallest distance between the last chosen and the first left-out logit, over the logits' spread."""
+    gaps = torch.full((len(toks),), 9.0)
+    real = zo.route
+    calls = []
+
+    def spy(h, w, b, top):
+        z = w @ h + b
+        s = torch.sort(z, descending=True).values
+        calls.append(float(s[top - 1] - s[top]) if top < len(z) else 9.0)
+        return real(h, w, b, top)
+    zo.route = spy
+    try:
+        ref = zo.forward(cfg, p, toks)
+    finally:
+        zo.route = real
+    for r in range(0, len(calls), len(toks)):
+        gaps = torch.minimum(gaps, torch.tensor(calls[r:r + len(toks)]))
+    return ref, gaps
+
+
+def oracle(name, seed, n):
+    """(tokens, logits, positions fit for a bf16 comparison).  A position is fit when no router of it had a close call."""
+    if (name, seed, n) not in _runs:
+        toks = torch.randint(0, CONFIGS[name]["vocab"], (n,), generator=gen(seed)).tolist()
+        ref, gaps = router_gap(CONFIGS[name], params(name), toks)
+        _runs[name, seed, n] = (toks, ref, gaps > 0.1)
+    return _runs[name, seed, n]
+
+
+def model(ops, name, dtype, **kw):
+    kw.setdefault("num_blocks", 60)
+    kw.setdefault("max_batch", 4)
+    return ops.ZomipelLM(CONFIGS[name], params(name), dtype=dtype, **kw)
+
+
+def check(got, ref, fit, dtype, what):
+    e = rel(got, ref)
+    assert bool(torch.isfinite(got).all()), what
+    if dtype == "float32":
+        assert float(e.max()) <= LIMIT[dtype], f"{what}: row {int(e.argmax())} is off by {float(e.max()):.3g}"
+        return
+    # bf16: a router's close call at an earlier position may have moved what later ones read, a little; the bulk must be within
+    # rounding, and no row of its own far off
+    e = e[fit]
+    if e.numel():
+        assert float(e.median()) <= LIMIT[dtype] and float(e.max()) <= 6 * LIMIT[dtype], f"{what}: median {float(e.median()):.3g}, worst {float(e.max()):.3g}"
+
+
+@BOTH
+@NAMES
+def test_whole_prompts(ops, name, dtype):
+    m = model(ops, name, dtype)
+    for seed, n in ((1, 1), (2, 2), (3, 17), (4, 150)):
+        print(f"case: {name} {dtype} prompt of {n}", flush=True)
+        toks, ref, fit = oracle(name, seed, n)
+        check(m.forward(torch.tensor(toks))[0], ref, fit, dtype, f"{name} {n}")
+    assert m.engine.allocator.num_free == 60 and len(m.engine._free_slots) == 4
+
+
+@BOTH
+@NAMES
+def test_layers_one_by_one(ops, name, dtype):
+    """The residual stream after every layer run."""
+    print(f"case: {name} {dtype} layers", flush=True)
+    m = model(ops, name, dtype)
+    toks = oracle(name, 3, 17)[0]
+    _, want = zo.forward(CONFIGS[name], params(name), toks, want_layers=True)
+    s, got = m.new_sequence(), []
+    plan = m.engine.plan_prefill([s], [17])
+    m._run(torch.tensor(toks).cuda(), plan, m.engine.attend_prefill, after_layer=lambda x: got.append(x.clone()))
+    assert len(got) == want.shape[0]
+    for i, (g, w) in enumerate(zip(got, want)):
+        e = rel(g, w)
+        assert float(e.median()) <= LIMIT[dtype] and (dtype == "bfloat16" or float(e.max()) <= LIMIT[dtype]), f"run {i}: {float(e.max()):.3g}"
+
+
+@BOTH
+@NAMES
+def test_portions_and_single_tokens(ops, name, dtype):
+    toks, ref, fit = oracle(name, 4, 150)
+    m = model(ops, name, dtype)
+    for cuts in ((2, 4, 6, 8, 48, 50, 150), (15, 16, 17, 20, 21, 64, 129, 150), (75, 150), (1, 149, 150)):
+        print(f"case: {name} {dtype} cuts {cuts}", flush=True)
+        s, got, a = m.new_sequence(), [], 0
+        for b in cuts:
+            got.append(m.step([s], [toks[a:b]], rows=range(b - a)))
+            a = b
+        m.free_sequence(s)                                                    # blocks and slot are used again by the next
+        check(torch.cat(got), ref, fit, dtype, f"{name} {cuts}")
+
+
+@BOTH
+@NAMES
+def test_token_by_token(ops, name, dtype):
+    print(f"case: {name} {dtype} token by token", flush=True)
+    toks, ref, fit = oracle(name, 4, 150)
+    m = model(ops, name, dtype)
+    s = m.new_sequence()
+    got = torch.cat([m.prefill([s], [toks[:1]])] + [m.decode([s], [t]) for t in toks[1:]])
+    check(got, ref, fit, dtype, name)
+    if dtype == "float32":
+        check(m.forward(torch.tensor(toks))[0], got.cpu(), fit, dtype, f"{name} prompt against decoding")
+
+
+@BOTH
+@NAMES
+def test_unequal_requests_in_one_batch(ops, name, dtype):
+    """Prompts, portions and single tokens of different sequences in one step, with sequences that end and whose blocks and slots
+    later ones take over."""
+    print(f"case: {name} {dtype} mixed batches", flush=True)
+    m = model(ops, name, dtype, num_blocks=26, max_batch=3)
+    seqs = {i: oracle(name, 20 + i, n) for i, n in enumerate((70, 9, 120, 33, 64))}
+    at, sid, got = {i: 0 for i in seqs}, {}, {i: [] for i in seqs}
+    plan = [{0: 31, 1: 5}, {0: 1, 1: 1, 2: 64}, {0: 1, 1: 1, 2: 1}, {0: 20, 1: 2, 2: 2}, {0: 17, 3: 3, 2: 40}, {3: 30, 2: 1, 4: 15},
+            {2: 12, 4: 1}, {4: 48}]
+    for step in plan:
+        for i in step:
+            if i not in sid:
+                sid[i] = m.new_sequence()
+        toks = [seqs[i][0][at[i]:at[i] + n] for i, n in step.items()]
+        logits = m.step([sid[i] for i in step], toks, rows=range(sum(map(len, toks))))
+        for i, part in zip(step, torch.split(logits, [len(t) for t in toks])):
+            got[i].append(part)
+            at[i] += part.shape[0]
+            if at[i] == len(seqs[i][0]):
+                m.free_sequence(sid[i])
+    for i, (toks, ref, fit) in seqs.items():
+        assert at[i] == len(toks)
+        check(torch.cat(got[i]), ref, fit, dtype, f"{name} sequence {i}")
+    assert m.engine.allocator.num_free == 26 and len(m.engine._free_slots) == 3
+
+
+@BOTH
+@pytest.mark.parametrize("name", ["mixed", "plain"])
+def test_long_decoding(ops, name, dtype):
+    print(f"case: {name} {dtype} long decoding", flush=True)
+    toks, ref, fit = oracle(name, 9, 420)
+    m = model(ops, name, dtype, max_batch=2)
+    s = m.new_sequence()
+    got = [m.prefill([s], [toks[:101]])] + [m.decode([s], [t]) for t in toks[101:]]
+    check(torch.cat(got), ref[100:], fit[100:], dtype, f"{name} long")
+    with pytest.raises(ValueError):
+        m.prefill([s], [[0] * 2000])
+    with pytest.raises(ValueError):
+        m.decode([s], [CONFIGS[name]["vocab"]])
+
+
+def test_a_wrong_mechanism_would_show(ops):
+    """The random models are sharp enough for the comparisons above: mistakes planted in the oracle move the logits of most
+    positions by far more than the limits."""
+    print("case: sensitivity of the comparison", flush=True)
+    name = "mixed"
+    toks, ref, _ = oracle(name, 4, 150)
+    for kind in ("window", "keep", "dims", "base", "groups", "taps", "norm_groups", "top", "loop", "again", "sg", "D", "eps"):
+        c, q = json.loads(json.dumps(CONFIGS[name])), dict(params(name))
+        a, s = c["layers"][0]["mixer"], c["layers"][1]["mixer"]
+        if kind == "window":
+            a["mask"]["size"] += 1
+        elif kind == "keep":
+            a["mask"]["keep_first"] -= 1
+        elif kind == "dims":
+            a["rot"]["dims"] = 14
+        elif kind == "base":
+            a["rot"]["base"] = 120.0
+        elif kind == "groups":
+            q["l1.mix.in"] = q["l1.mix.in"].clone()
+            q["l1.mix.in"][128:152], q["l1.mix.in"][152:176] = params(name)["l1.mix.in"][152:176], params(name)["l1.mix.in"][128:152]
+        elif kind == "taps":
+            q["l1.mix.conv"] = q["l1.mix.conv"].roll(1, 1)
+        elif kind == "norm_groups":
+            s["norm_groups"] = 1
+        elif kind == "top":
+            c["layers"][3]["mlp"]["router"]["top"] = 2
+        elif kind == "loop":
+            c["loop"]["times"] = 2
+        elif kind == "again":
+            c["loop"] = None
+            c["layers"] = [c["layers"][i] for i in (0, 1, 2, 3, 1, 2, 3, 1, 2, 3)]
+            q = dict(params(name))
+            for new, old in enumerate((0, 1, 2, 3, 1, 2, 3, 1, 2, 3)):
+                q.update({f"l{new}." + k.split(".", 1)[1]: v for k, v in params(name).items() if k.startswith(f"l{old}.")})
+        elif kind == "sg":
+            q["l0.mlp.shared.sg"] = torch.zeros_like(q["l0.mlp.shared.sg"])
+        elif kind == "D":
+            q["l2.mix.D"] = torch.zeros_like(q["l2.mix.D"])
+        else:
+            c["norm"]["eps"] = 0.05
+        e = rel(zo.forward(c, q, toks), ref)
+        assert float(e.max()) > 3 * LIMIT["bfloat16"] and float(e.median()) > 50 * LIMIT["float32"], (kind, float(e.max()), float(e.median()))
+
+
+# ---- generation through the framework's own entry points ------------------------------------------------------------------
+def greedy_oracle(name, prompt, n, margin):
+    """The oracle's greedy continuation, cut before the first step whose two best logits are closer than `margin`."""
+    ids, out = list(prompt), []
+    for _ in range(n):
+        row = zo.forward(CONFIGS[name], params(name), ids)[-1]
+        a, b = torch.topk(row, 2).values.tolist()
+        if a - b < margin:
+            break
+        out.append(int(row.argmax()))
+        ids.append(out[-1])
+    return out
+
+
+@pytest.mark.parametrize("name", ["mixed", "odd"])
+def test_greedy_generation(ops, name):
+    print(f"case: {name} greedy", flush=True)
+    m = model(ops, name, "float32")
+    prompts = [oracle(name, s, n)[0] for s, n in ((3, 17), (6, 31), (7, 2))]
+    want = [greedy_oracle(name, p, 12, 1e-3) for p in prompts]
+    assert sum(len(w) for w in want) >= 18
+    got = m.generate_batch(prompts, 12, temperature=0)
+    for p, w, g in zip(prompts, want, got):
+        assert g[:len(w)] == w and len(g) == 12
+        assert m.generate([p], 12, temperature=0)[0].tolist()[:len(w)] == w
+    assert m.engine.allocator.num_free == m.engine.allocator.num_blocks and len(m.engine._free_slots) == 4
+
+
+@BOTH
+@pytest.mark.parametrize("name", ["mixed", "plain"])
+def test_graph_replays_equal_eager_decoding(ops, name, dtype):
+    print(f"case: decode graphs {name} {dtype}", flush=True)
+    m, e = (model(ops, name, dtype, max_batch=2, decode_graphs=g) for g in (True, False))
+    seqs = [oracle(name, 5, 64), oracle(name, 4, 150)]
+    start, ids = [20, 40], []
+    for mdl in (m, e):
+        ids.append([mdl.new_sequence() for _ in seqs])
+        mdl.prefill(ids[-1], [s[0][:n] for s, n in zip(seqs, start)])
+    eager, graphed = [], []
+    for step in range(30):
+        toks = [s[0][n + step] for s, n in zip(seqs, start)]
+        graphed.append(m.decode(ids[0], toks).cpu())
+        eager.append(e.decode(ids[1], toks).cpu())                          # eager work between the replays
+        torch.cuda.synchronize()
+        assert float(rel(graphed[-1], eager[-1]).max()) <= (1e-5 if dtype == "float32" else 2e-2), step
+    for i, (s, n) in enumerate(zip(seqs, start)):
+        check(torch.stack([g[i] for g in graphed]), s[1][n:n + 30], s[2][n:n + 30], dtype, f"sequence {i}")
+
+
+def test_fp8_cache(ops):
+    """An e4m3 cache under the same model: within twice the 6 % relative rms that is stated for the attention over fp8 caches."""
+    print("case: fp8 cache", flush=True)
+    toks, ref, fit = oracle("plain", 4, 150)
+    m = model(ops, "plain", "bfloat16", kv_dtype="fp8")
+    s = m.new_sequence()
+    got = [m.step([s], [toks[:60]], rows=range(60)), m.step([s], [toks[60:120]], rows=range(60))]
+    got += [m.decode([s], [t]) for t in toks[120:]]
+    e = rel(torch.cat(got), ref)[fit]
+    assert float(e.median()) <= 0.12, float(e.median())
+
+
+def save_model(tmp_path, name):
+    from safetensors.torch import save_file
+    (tmp_path / "config.json").write_text(json.dumps(CONFIGS[name]))
+    save_file({k: v.contiguous() for k, v in params(name).items()}, str(tmp_path / "model.safetensors"))
+
+
+@BOTH
+def test_trace_run_command(ops, tmp_path, dtype):
+    print(f"case: bin/trace_run {dtype}", flush=True)
+    save_model(tmp_path, "mixed")
+    a, ref_a, fit_a = oracle("mixed", 4, 150)
+    b, ref_b, fit_b = oracle("mixed", 5, 64)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:120], "want": [0, 119, 15]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": a[120:122], "want": []}], "end": []},
+             {"step": 2, "entries": [{"id": "a", "tokens": a[122:123], "want": [0]}], "end": ["a"]},
+             {"step": 3, "entries": [{"id": "b", "tokens": b, "want": [63]}], "end": ["b"]}]
+    out = tmp_path / "out"
+    res = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", dtype, "--out",
+                          str(out), "--max-tokens", "128"], input="\n".join(map(json.dumps, steps)) + "\n", capture_output=True, text=True,
+                         timeout=110)
+    assert res.returncode == 0, res.stderr[-2000:]
+    assert [ln for ln in res.stdout.splitlines() if ln.startswith("done")] == [f"done {n}" for n in range(4)]
+    read = lambda n: torch.frombuffer(bytearray((out / f"{n}.f32").read_bytes()), dtype=torch.float32).view(-1, 53)
+    assert not (out / "1.f32").exists()
+    for n, ref, fit, at in ((0, ref_a, fit_a, [0, 119, 15]), (2, ref_a, fit_a, [122]), (3, ref_b, fit_b, [63])):
+        check(read(n), ref[at], fit[at], dtype, f"step {n}")
+
+
+def test_generate_command_and_registry(ops, tmp_path):
+    print("case: bin/generate", flush=True)
+    save_model(tmp_path, "odd")
+    m = ops.load_model(str(tmp_path), dtype="float32", max_batch=2, num_blocks=20)
+    assert isinstance(m, ops.ZomipelLM) and m.dtype == torch.float32
+    prompts = [[3, 1, 4, 1, 5], [9, 2]]
+    want = m.generate_batch(prompts, 6, temperature=0)
+    res = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "generate"), "--model", str(tmp_path), "--dtype", "float32",
+                          "--max-new-tokens", "6", "--temperature", "0", "--prompt", "3 1 4 1 5", "--prompt", "9,2"],
+                         capture_output=True, text=True, timeout=110)
+    assert res.returncode == 0, res.stderr[-2000:]
+    assert [json.loads(ln) for ln in res.stdout.splitlines()] == want
+    g = lambda: torch.Generator(device="cuda").manual_seed(7)
+    assert m.generate_batch(prompts, 6, 1.5, 20, generator=g()) == m.generate_batch(prompts, 6, 1.5, 20, generator=g())
