@@ -541,7 +541,9 @@ int mi355_gated_norm_fwd(const void* y, const void* z, const float* weight, void
  * and is taken as zero when the sequence's first row of the call has position 0 (slots need no clearing).
  *   mi355_ssm_prefill : sequence b owns rows cu_seqlens[b] .. cu_seqlens[b+1] - 1 (NULL: row b), any number of them; needs xbc
  *                       (n_rows, channels) of `dtype` as scratch.  scan AUTO: chunks on MFMA where they apply (bf16; state
- *                       and vdim multiples of 8, state <= 256), else token by token
+ *                       and vdim multiples of 8, state <= 256), else token by token.  seg_len > 0 (a multiple of 64) lets the
+ *                       chunked scan run the segments of a sequence side by side, with scratch for them: seg_state
+ *                       (n_rows / seg_len + batch, heads, state, vdim) and seg_decay (n_rows / seg_len + batch, heads), fp32
  *   mi355_ssm_decode  : one row per sequence, convolution and recurrence in one launch
  */
 enum { MI355_SCAN_AUTO = 0, MI355_SCAN_SERIAL = 1, MI355_SCAN_CHUNKED = 2 };
@@ -561,6 +563,8 @@ typedef struct mi355_ssm_args {
     void* y;                     /* (n_rows, heads * vdim) of `dtype` */
     int64_t proj_row_stride, xbc_col, dt_col, y_row_stride, n_rows;
     int batch, heads, vdim, state, groups, taps, n_slots, dtype;
+    float *seg_state, *seg_decay; /* chunked scan in segments: scratch */
+    int seg_len;                 /* tokens per segment, 0: none */
 } mi355_ssm_args;
 int mi355_ssm_prefill(const mi355_ssm_args* args, int scan, void* stream);
 int mi355_ssm_decode(const mi355_ssm_args* args, void* stream);

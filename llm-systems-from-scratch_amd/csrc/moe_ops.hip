@@ -76,12 +76,13 @@ __device__ __forceinline__ void choose_experts(const RouteParams& p, float* z, i
     }
 }
 
-// 16 tokens per workgroup; the four wavefronts take the 32-wide steps of k in turn and meet in LDS.
-__global__ __launch_bounds__(256) void moe_route_kernel(RouteParams p) {
+// 16 tokens per workgroup; the wavefronts take the 32-wide steps of k in turn and meet in LDS.
+constexpr int kRouteWaves = 8;
+__global__ __launch_bounds__(64 * kRouteWaves) void moe_route_kernel(RouteParams p) {
     extern __shared__ __attribute__((aligned(16))) float route_lds[];
-    constexpr int kTiles = 4;                     // 16 logits each
+    constexpr int kTiles = 4, kBatch = 4;         // 16 logits each
     f32x4* part = reinterpret_cast<f32x4*>(route_lds);                         // [wave][tile][lane]
-    float* z = route_lds + 4 * kTiles * 64 * 4;                                // [16][n_logits]
+    float* z = route_lds + kRouteWaves * kTiles * 64 * 4;                              // [16][n_logits]
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int r = lane & 15, kg = lane >> 4;
     const int64_t t0 = (int64_t)blockIdx.x * 16;
@@ -94,36 +95,44 @@ __global__ __launch_bounds__(256) void moe_route_kernel(RouteParams p) {
             acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
             w[j] = (const __bf16*)p.w + (int64_t)min(l0 + 16 * j + r, p.n_logits - 1) * p.w_stride;
         }
-        for (int k0 = 32 * wave; k0 < p.k; k0 += 128) {
-            const int col = k0 + 8 * kg;
-            const bool in = col < p.k;
-            u32x4 hv = {0u, 0u, 0u, 0u};
-            if (in) hv = *reinterpret_cast<const u32x4*>(h + col);
+        for (int k0 = 32 * wave; k0 < p.k; k0 += 32 * kRouteWaves * kBatch) {       // kBatch steps' loads, then their products
+            u32x4 hv[kBatch], wv[kTiles][kBatch];
 #pragma unroll
-            for (int j = 0; j < kTiles; ++j) {
-                if (l0 + 16 * j < p.n_logits) {
-                    u32x4 wv = {0u, 0u, 0u, 0u};
-                    if (in) wv = *reinterpret_cast<const u32x4*>(w[j] + col);
-                    acc[j] = mfma16(as_bf16x8(wv), as_bf16x8(hv), acc[j]);         // column r: token, rows 4 kg + i: logits
+            for (int i = 0; i < kBatch; ++i) {
+                const int col = k0 + 32 * kRouteWaves * i + 8 * kg;
+                const bool in = col < p.k;
+                hv[i] = u32x4{0u, 0u, 0u, 0u};
+                if (in) hv[i] = *reinterpret_cast<const u32x4*>(h + col);
+#pragma unroll
+                for (int j = 0; j < kTiles; ++j) {
+                    wv[j][i] = u32x4{0u, 0u, 0u, 0u};
+                    if (in && l0 + 16 * j < p.n_logits) wv[j][i] = *reinterpret_cast<const u32x4*>(w[j] + col);
                 }
             }
+#pragma unroll
+            for (int j = 0; j < kTiles; ++j)
+                if (l0 + 16 * j < p.n_logits)
+#pragma unroll
+                    for (int i = 0; i < kBatch; ++i) acc[j] = mfma16(as_bf16x8(wv[j][i]), as_bf16x8(hv[i]), acc[j]);      // column r: token, rows 4 kg + i: logits
         }
         __syncthreads();
 #pragma unroll
         for (int j = 0; j < kTiles; ++j) part[(wave * kTiles + j) * 64 + lane] = acc[j];
         __syncthreads();
         // wavefront j sums tile j
-        f32x4 s = {0.f, 0.f, 0.f, 0.f};
+        if (wave < kTiles) {
+            f32x4 s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int w4 = 0; w4 < 4; ++w4) s += part[(w4 * kTiles + wave) * 64 + lane];
+            for (int w8 = 0; w8 < kRouteWaves; ++w8) s += part[(w8 * kTiles + wave) * 64 + lane];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int l = l0 + 16 * wave + 4 * kg + i;
-            if (l < p.n_logits) z[r * p.n_logits + l] = s[i] + p.bias[l];
+            for (int i = 0; i < 4; ++i) {
+                const int l = l0 + 16 * wave + 4 * kg + i;
+                if (l < p.n_logits) z[r * p.n_logits + l] = s[i] + p.bias[l];
+            }
         }
     }
     __syncthreads();
-    for (int t = wave; t < 16; t += 4) {
+    for (int t = wave; t < 16; t += kRouteWaves) {
         if (t0 + t >= p.T) break;
         float* zt = z + t * p.n_logits;
         if (p.extra_logit && lane == 0) p.extra_logit[t0 + t] = zt[p.E];
@@ -324,7 +333,7 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(MoeParams p, int n_til
 // their operands straight from memory and meet in LDS.
 template <bool GATE_UP>
 __global__ __launch_bounds__(256) void moe_skinny_kernel(MoeParams p, int n_tiles, int m_tiles) {
-    constexpr int BM = 16, NW = GATE_UP ? 2 : 1, kSteps = 2;
+    constexpr int BM = 16, NW = GATE_UP ? 2 : 1, kBatch = 4;        // steps of k whose loads are in flight together
     __shared__ f32x4 part[4][NW][64];
     const int id = xcd_chunked_id(blockIdx.x, n_tiles * m_tiles, n_tiles);
     const int n0 = id % n_tiles * 16;
@@ -338,19 +347,28 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(MoeParams p, int n_tile
     f32x4 acc[NW];
 #pragma unroll
     for (int i = 0; i < NW; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-    for (int k0 = 64 * wave; k0 < p.k; k0 += 256) {
-        u32x4 av[kSteps], wv[NW][kSteps];
+    for (int k0 = 64 * wave; k0 < p.k; k0 += 256 * kBatch) {
+        u32x4 av[kBatch][2], wv[NW][kBatch][2];
 #pragma unroll
-        for (int s = 0; s < kSteps; ++s) {
+        for (int t = 0; t < kBatch; ++t)
 #pragma unroll
-            for (int i = 0; i < NW; ++i) wv[i][s] = *reinterpret_cast<const u32x4*>(w + i * up + k0 + 32 * s);
-            av[s] = *reinterpret_cast<const u32x4*>(a + k0 + 32 * s);
-        }
+            for (int s = 0; s < 2; ++s) {
+                const int col = k0 + 256 * t + 32 * s;
+                av[t][s] = u32x4{0u, 0u, 0u, 0u};
 #pragma unroll
-        for (int s = 0; s < kSteps; ++s)
+                for (int i = 0; i < NW; ++i) wv[i][t][s] = av[t][s];
+                if (k0 + 256 * t < p.k) {
 #pragma unroll
-            for (int i = 0; i < NW; ++i) acc[i] = mfma16(as_bf16x8(wv[i][s]), as_bf16x8(av[s]), acc[i]);
+                    for (int i = 0; i < NW; ++i) wv[i][t][s] = *reinterpret_cast<const u32x4*>(w + i * up + col);
+                    av[t][s] = *reinterpret_cast<const u32x4*>(a + col);
+                }
+            }
+#pragma unroll
+        for (int t = 0; t < kBatch; ++t)
+#pragma unroll
+            for (int s = 0; s < 2; ++s)
+#pragma unroll
+                for (int i = 0; i < NW; ++i) acc[i] = mfma16(as_bf16x8(wv[i][t][s]), as_bf16x8(av[t][s]), acc[i]);
     }
 #pragma unroll
     for (int i = 0; i < NW; ++i) part[wave][i][lane] = acc[i];
@@ -514,7 +532,8 @@ extern "C" int mi355_moe_route(const void* h, const void* w, const float* bias, 
     p.top = top;
     hipStream_t s = (hipStream_t)stream;
     if (dtype == MI355_BF16)
-        hipLaunchKernelGGL(moe_route_kernel, dim3((unsigned)((n_tokens + 15) / 16)), dim3(256), (4 * 4 * 64 * 4 + 16 * p.n_logits) * sizeof(float), s, p);
+        hipLaunchKernelGGL(moe_route_kernel, dim3((unsigned)((n_tokens + 15) / 16)), dim3(64 * kRouteWaves),
+                           (kRouteWaves * 4 * 64 * 4 + 16 * p.n_logits) * sizeof(float), s, p);
     else
         hipLaunchKernelGGL(moe_route_f32_kernel, dim3((unsigned)((n_tokens + 3) / 4)), dim3(256), 4 * p.n_logits * sizeof(float), s, p);
     const int rc = (int)hipGetLastError();

@@ -11,7 +11,8 @@
 // A sequence's first token is at position 0: its history is zero whatever the slot holds, so slots are never cleared.
 //
 // Three kernels besides the convolution:
-//   ssd_chunk_kernel   bf16 prompts: chunks of 64 tokens on MFMA, the state in accumulators from chunk to chunk
+//   ssd_chunk_kernel   bf16 prompts: chunks of 64 tokens on MFMA, the state in accumulators from chunk to chunk; where
+//                      that walk leaves the chip idle, segments of a sequence side by side (ssd_carry_kernel between them)
 //   ssm_scan_kernel    any sizes and fp32: token by token, the state in registers
 //   ... the same kernel with the convolution inside: one decode step of every sequence
 #include "common.hpp"
@@ -37,11 +38,24 @@ struct SsmParams {
     int64_t y_stride, n_rows;
     int B, H, P, Pp, N, G, taps, channels, n_slots;
     int np4, slices;                 // scan: 4-wide pieces of vdim per workgroup, and workgroups per head
+    float *seg_state, *seg_decay;    // segments: (segment, head) states (N x Pp), log2 of the decay across a segment
+    int seg_len, n_segs;
 };
 
 template <typename T>
 __device__ __forceinline__ int state_slot(const SsmParams<T>& p, int b) {
     return min(max(p.slots[b], 0), p.n_slots - 1);
+}
+// the sequence that unit `unit` of `size` tokens lies in: units of sequence b start at number first_row / size + b
+template <typename T>
+__device__ __forceinline__ int seq_of_unit(const SsmParams<T>& p, int unit, int size) {
+    int lo = 0, hi = p.B - 1;
+    while (lo < hi) {
+        const int mid = (lo + hi + 1) / 2;
+        if ((p.cu ? p.cu[mid] : mid) / size + mid <= unit) lo = mid;
+        else hi = mid - 1;
+    }
+    return lo;
 }
 // rows of sequence b
 template <typename T>
@@ -102,14 +116,7 @@ __global__ __launch_bounds__(256) void causal_conv_silu_kernel(SsmParams<T> p) {
     const int g_blocks = (ch_groups + 255) / 256;
     const int tile = blockIdx.x / g_blocks;
     const int cg = (blockIdx.x % g_blocks) * 256 + threadIdx.x;
-    // tiles of sequence b start at tile number first_row / kConvTile + b
-    int lo = 0, hi = p.B - 1;
-    while (lo < hi) {
-        const int mid = (lo + hi + 1) / 2;
-        if ((p.cu ? p.cu[mid] : mid) / kConvTile + mid <= tile) lo = mid;
-        else hi = mid - 1;
-    }
-    const int b = lo;
+    const int b = seq_of_unit(p, tile, kConvTile);
     int first, len;
     seq_rows(p, b, first, len);
     const int t0 = (tile - (first / kConvTile + b)) * kConvTile;
@@ -308,7 +315,12 @@ __device__ __forceinline__ void split_bf16(float a, float b, uint32_t& hi, uint3
 //   S   (n x p)  += B^T (w x)     B^T through the transposed read; w x: the X^T fragments again, weighted in registers
 // x, B and C are bf16 (the convolution's output); what is computed in fp32 -- S, the bracketed factors, the weighted x -- enters
 // the MFMAs as a bf16 pair of leading part and remainder, so nothing of the recurrence is rounded to 8 bits.
-template <int NT>
+//
+// kWhole: a workgroup walks its whole sequence.  Few sequences and heads leave most of the chip idle then, so their segments
+// of seg_len tokens go side by side: kSegState leaves what each segment but the last adds to the state, ssd_carry_kernel turns
+// these into the states in front of the segments, and kSegOut computes every segment's outputs from there.
+enum { kWhole, kSegState, kSegOut };
+template <int NT, int MODE>
 __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
     constexpr int Q = 64, NP = 32 * NT;
     constexpr int kBRow = NP * 2 + 32, kCRow = NP * 2 + 16, kXRow = 64 * 2 + 32, kFRow = Q * 2 + 16;
@@ -320,10 +332,20 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
 
     const int h = blockIdx.x / p.slices % p.H;
     const int col0 = (blockIdx.x % p.slices) * 64;
-    const int b = blockIdx.x / (p.slices * p.H);
+    const int unit = blockIdx.x / (p.slices * p.H);
+    const int b = MODE == kWhole ? unit : seq_of_unit(p, unit, p.seg_len);
     int first, len;
     seq_rows(p, b, first, len);
     if (len <= 0) return;
+    bool last = true;
+    if constexpr (MODE != kWhole) {
+        const int s0 = (unit - (first / p.seg_len + b)) * p.seg_len;
+        if (s0 < 0 || s0 >= len) return;
+        last = s0 + p.seg_len >= len;
+        if (MODE == kSegState && last) return;           // nobody comes after it
+        first += s0;
+        len = min(p.seg_len, len - s0);
+    }
     const int g = h / (p.H / p.G), inner = p.H * p.P;
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -332,6 +354,7 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
     const bool has_cols = pc < p.P;
     const int slot = state_slot(p, b);
     float* st = p.ssm_state + ((int64_t)slot * p.H + h) * p.N * p.Pp + pc + r;
+    float* seg_st = MODE == kWhole ? nullptr : p.seg_state + ((int64_t)unit * p.H + h) * p.N * p.Pp + pc + r;
     const float bias = p.dt_bias[h], na2 = p.neg_a[h] * kLog2e, skip = p.d_skip[h];
     const __bf16* xsrc = p.xbc + h * p.P + col0;
     const __bf16* bsrc = p.xbc + inner + g * p.N;
@@ -339,18 +362,19 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
 
     // S: lane holds column pc + r, rows 16 j + 4 kg + i
     f32x4 S[2 * NT];
-    const bool resumed = p.positions[first] > 0;
+    const float* from = MODE == kWhole ? st : seg_st;
+    const bool resumed = MODE == kSegOut || (MODE == kWhole && p.positions[first] > 0);
 #pragma unroll
     for (int j = 0; j < 2 * NT; ++j)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int n = 16 * j + 4 * kg + i;
-            S[j][i] = resumed && n < p.N && pc + r < p.P ? st[(int64_t)n * p.Pp] : 0.f;
+            S[j][i] = resumed && n < p.N && pc + r < p.P ? from[(int64_t)n * p.Pp] : 0.f;
         }
 
     // one chunk's loads: NT 16-byte pieces of B and C and two of x per thread, dt of token `lane`
     u32x4 rb[NT], rc[NT], rx[2];
-    float rdt = 0.f;
+    float rdt = 0.f, total = 0.f;                        // total: log2 of the decay so far
     const auto fetch = [&](int t0) {
 #pragma unroll
         for (int j = 0; j < NT; ++j) {
@@ -359,7 +383,7 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
             if (t0 + row < len && col < p.N) {
                 const int64_t at = (int64_t)(first + t0 + row) * p.channels + col;
                 rb[j] = *reinterpret_cast<const u32x4*>(bsrc + at);
-                rc[j] = *reinterpret_cast<const u32x4*>(csrc + at);
+                if constexpr (MODE != kSegState) rc[j] = *reinterpret_cast<const u32x4*>(csrc + at);
             }
         }
 #pragma unroll
@@ -381,12 +405,13 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
             if (lane >= off) cum += up;
         }
         const float cum_last = __shfl(cum, 63, 64);
+        total += cum_last;
         __syncthreads();                                 // everybody has read the chunk before
 #pragma unroll
         for (int j = 0; j < NT; ++j) {
             const int idx = j * 256 + tid, row = idx / (4 * NT), col = idx % (4 * NT) * 8;
             *reinterpret_cast<u32x4*>(b_lds + row * kBRow + col * 2) = rb[j];
-            *reinterpret_cast<u32x4*>(c_lds + row * kCRow + col * 2) = rc[j];
+            if constexpr (MODE != kSegState) *reinterpret_cast<u32x4*>(c_lds + row * kCRow + col * 2) = rc[j];
         }
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
@@ -401,38 +426,35 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
         __syncthreads();
 
         // ---- bracketed factors of tokens 16 wave + r ------------------------------------------
-        {
+        if constexpr (MODE != kSegState) {
             const int t = 16 * wave + r;
             const float ct = cum_lds[t];
             bf16x8 cf[NT];
 #pragma unroll
             for (int u = 0; u < NT; ++u)
                 cf[u] = as_bf16x8(*reinterpret_cast<const u32x4*>(c_lds + t * kCRow + (32 * u + 8 * kg) * 2));
-            for (int s0 = 0; s0 <= (wave | 1); ++s0) {
-                u32x2 hi = {0u, 0u}, lo = {0u, 0u};
-                if (s0 <= wave) {
-                    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+            // (tiles behind the wavefront's own come out as zeros: four independent chains are shorter than a branch per tile)
 #pragma unroll
-                    for (int u = 0; u < NT; ++u)
-                        acc = mfma16(as_bf16x8(*reinterpret_cast<const u32x4*>(b_lds + (16 * s0 + r) * kBRow + (32 * u + 8 * kg) * 2)),
-                                     cf[u], acc);
-                    float f[4];
+            for (int s0 = 0; s0 < 4; ++s0) {
+                f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) {
-                        const int s = 16 * s0 + 4 * kg + i;
-                        f[i] = s <= t ? acc[i] * (fast_exp2(ct - cum_lds[s]) * dt_lds[s]) : 0.f;
-                    }
-                    uint32_t h0, h1, l0, l1;
-                    split_bf16(f[0], f[1], h0, l0);
-                    split_bf16(f[2], f[3], h1, l1);
-                    hi = u32x2{h0, h1};
-                    lo = u32x2{l0, l1};
+                for (int u = 0; u < NT; ++u)
+                    acc = mfma16(as_bf16x8(*reinterpret_cast<const u32x4*>(b_lds + (16 * s0 + r) * kBRow + (32 * u + 8 * kg) * 2)),
+                                 cf[u], acc);
+                float f[4];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int s = 16 * s0 + 4 * kg + i;
+                    f[i] = s <= t ? acc[i] * (fast_exp2(ct - cum_lds[s]) * dt_lds[s]) : 0.f;
                 }
-                *reinterpret_cast<u32x2*>(f_lds[0] + t * kFRow + (16 * s0 + 4 * kg) * 2) = hi;
-                *reinterpret_cast<u32x2*>(f_lds[1] + t * kFRow + (16 * s0 + 4 * kg) * 2) = lo;
+                uint32_t h0, h1, l0, l1;
+                split_bf16(f[0], f[1], h0, l0);
+                split_bf16(f[2], f[3], h1, l1);
+                *reinterpret_cast<u32x2*>(f_lds[0] + t * kFRow + (16 * s0 + 4 * kg) * 2) = u32x2{h0, h1};
+                *reinterpret_cast<u32x2*>(f_lds[1] + t * kFRow + (16 * s0 + 4 * kg) * 2) = u32x2{l0, l1};
             }
+            __syncthreads();
         }
-        __syncthreads();
         if (!has_cols) continue;
 
         // X^T fragments: row p = r, k = token 32 u + 8 kg + j
@@ -444,7 +466,7 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
             xf[u] = join_bf16x8(lds_read_tr16(src), lds_read_tr16(src + 4 * kXRow));
         }
         // ---- Y^T -------------------------------------------------------------------------------
-        {
+        if constexpr (MODE != kSegState) {
             bf16x8 sh[NT], sl[NT];
 #pragma unroll
             for (int u = 0; u < NT; ++u) {
@@ -521,13 +543,54 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsmParams<__bf16> p) {
             }
         }
     }
+    if constexpr (MODE == kSegState) {
+        if (tid == 0 && col0 == 0) p.seg_decay[(int64_t)unit * p.H + h] = total;
+    }
+    if (MODE == kSegOut && !last) return;
+    float* to = MODE == kSegState ? seg_st : st;
 #pragma unroll
     for (int j = 0; j < 2 * NT; ++j)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int n = 16 * j + 4 * kg + i;
-            if (n < p.N && pc + r < p.P) st[(int64_t)n * p.Pp] = S[j][i];
+            if (n < p.N && pc + r < p.P) to[(int64_t)n * p.Pp] = S[j][i];
         }
+}
+
+// What the segments of a sequence add -> the states in front of them, in place: a thread owns four columns of one row.
+__global__ __launch_bounds__(256) void ssd_carry_kernel(SsmParams<__bf16> p) {
+    constexpr int kAhead = 4;
+    const int h = blockIdx.x % p.H, b = blockIdx.x / p.H;
+    const int64_t size = (int64_t)p.N * p.Pp, at = 4 * (blockIdx.y * 256LL + threadIdx.x);
+    int first, len;
+    seq_rows(p, b, first, len);
+    if (len <= 0 || at >= size) return;
+    f32x4 S = {0.f, 0.f, 0.f, 0.f};
+    if (p.positions[first] > 0) S = *reinterpret_cast<const f32x4*>(p.ssm_state + ((int64_t)state_slot(p, b) * p.H + h) * size + at);
+    const int64_t seg0 = first / p.seg_len + b;
+    const int n = (len + p.seg_len - 1) / p.seg_len;
+    float* seg = p.seg_state + (seg0 * p.H + h) * size + at;
+    const float* decay = p.seg_decay + seg0 * p.H + h;
+    for (int i = 0; i < n; i += kAhead) {
+        f32x4 add[kAhead];
+        float d[kAhead];
+#pragma unroll
+        for (int j = 0; j < kAhead; ++j)
+            if (i + j < n - 1) {                         // (the last segment's state is nobody's start)
+                add[j] = *reinterpret_cast<const f32x4*>(seg + (i + j) * p.H * size);
+                d[j] = decay[(i + j) * p.H];
+            }
+#pragma unroll
+        for (int j = 0; j < kAhead; ++j)
+            if (i + j < n) {
+                *reinterpret_cast<f32x4*>(seg + (i + j) * p.H * size) = S;
+                if (i + j < n - 1) {
+                    const float f = fast_exp2(d[j]);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) S[e] = fmaf(f, S[e], add[j][e]);
+                }
+            }
+    }
 }
 
 template <typename T>
@@ -573,16 +636,28 @@ static bool chunked_takes(const SsmParams<__bf16>& p) {
            (reinterpret_cast<uintptr_t>(p.y) & 7) == 0;
 }
 
-static int launch_chunked(SsmParams<__bf16> p, hipStream_t s) {
-    p.slices = (p.P + 63) / 64;
-    const int64_t wgs = (int64_t)p.B * p.H * p.slices;
+template <int MODE>
+static int launch_chunks(const SsmParams<__bf16>& p, int64_t units, hipStream_t s) {
+    const int64_t wgs = units * p.H * p.slices;
     if (wgs > 0x7fffffffLL) return (int)hipErrorInvalidValue;
     const dim3 grid((unsigned)wgs), block(256);
-    if (p.N <= 32) hipLaunchKernelGGL(ssd_chunk_kernel<1>, grid, block, 0, s, p);
-    else if (p.N <= 64) hipLaunchKernelGGL(ssd_chunk_kernel<2>, grid, block, 0, s, p);
-    else if (p.N <= 128) hipLaunchKernelGGL(ssd_chunk_kernel<4>, grid, block, 0, s, p);
-    else hipLaunchKernelGGL(ssd_chunk_kernel<8>, grid, block, 0, s, p);
+    if (p.N <= 32) hipLaunchKernelGGL((ssd_chunk_kernel<1, MODE>), grid, block, 0, s, p);
+    else if (p.N <= 64) hipLaunchKernelGGL((ssd_chunk_kernel<2, MODE>), grid, block, 0, s, p);
+    else if (p.N <= 128) hipLaunchKernelGGL((ssd_chunk_kernel<4, MODE>), grid, block, 0, s, p);
+    else hipLaunchKernelGGL((ssd_chunk_kernel<8, MODE>), grid, block, 0, s, p);
     return (int)hipGetLastError();
+}
+
+static int launch_chunked(SsmParams<__bf16> p, hipStream_t s) {
+    p.slices = (p.P + 63) / 64;
+    if (p.seg_len == 0) return launch_chunks<kWhole>(p, p.B, s);
+    p.n_segs = (int)(p.n_rows / p.seg_len) + p.B;
+    if (int e = launch_chunks<kSegState>(p, p.n_segs, s)) return e;
+    const int64_t pieces = ((int64_t)p.N * p.Pp / 4 + 255) / 256, heads = (int64_t)p.B * p.H;
+    if (pieces > 65535 || heads > 0x7fffffffLL) return (int)hipErrorInvalidValue;
+    hipLaunchKernelGGL(ssd_carry_kernel, dim3((unsigned)heads, (unsigned)pieces), dim3(256), 0, s, p);
+    if (int e = (int)hipGetLastError()) return e;
+    return launch_chunks<kSegOut>(p, p.n_segs, s);
 }
 
 template <typename T>
@@ -615,6 +690,9 @@ static SsmParams<T> ssm_params(const mi355_ssm_args& a) {
     p.taps = a.taps;
     p.channels = a.heads * a.vdim + 2 * a.groups * a.state;
     p.n_slots = a.n_slots;
+    p.seg_state = a.seg_state;
+    p.seg_decay = a.seg_decay;
+    p.seg_len = a.seg_len;
     return p;
 }
 
@@ -645,6 +723,9 @@ extern "C" int mi355_ssm_prefill(const mi355_ssm_args* args, int scan, void* str
     if (!args->xbc) return set_error(MI355_EINVAL, "ssm_prefill: null xbc buffer");
     if (!args->cu_seqlens && args->n_rows != args->batch) return set_error(MI355_EINVAL, "ssm_prefill: one row per sequence without cu_seqlens");
     if (scan < MI355_SCAN_AUTO || scan > MI355_SCAN_CHUNKED) return set_error(MI355_EINVAL, "ssm_prefill: unknown scan");
+    if (args->seg_len < 0 || args->seg_len % 64 ||
+        (args->seg_len > 0 && (!args->seg_state || !args->seg_decay || (reinterpret_cast<uintptr_t>(args->seg_state) & 15))))
+        return set_error(MI355_EINVAL, "ssm_prefill: segments are multiples of 64 tokens and need their buffers");
     if (args->n_rows == 0) return MI355_OK;
     hipStream_t s = (hipStream_t)stream;
     int rc;

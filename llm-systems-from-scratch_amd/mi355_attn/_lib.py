@@ -76,7 +76,8 @@ class SsmArgs(C.Structure):
     _fields_ = ([(n, C.c_void_p) for n in ("proj", "conv_weight", "conv_bias", "dt_bias", "neg_a", "d_skip", "conv_state", "ssm_state",
                                            "slots", "positions", "cu_seqlens", "xbc", "y")] +
                 [(n, C.c_int64) for n in ("proj_row_stride", "xbc_col", "dt_col", "y_row_stride", "n_rows")] +
-                [(n, C.c_int) for n in ("batch", "heads", "vdim", "state", "groups", "taps", "n_slots", "dtype")])
+                [(n, C.c_int) for n in ("batch", "heads", "vdim", "state", "groups", "taps", "n_slots", "dtype")] +
+                [("seg_state", C.c_void_p), ("seg_decay", C.c_void_p), ("seg_len", C.c_int)])
 
 
 class LibraryMissing(RuntimeError):

@@ -1338,8 +1338,16 @@ def gated_norm(y, z, weight, groups: int, eps: float, *, out=None):
     return out
 
 
+def ssm_segment_length(n_tokens: int, n_sequences: int, heads: int, vdim: int) -> int:
+    """Tokens per segment of the chunked scan (0: whole sequences): enough workgroups to fill the chip, of 256 tokens or more."""
+    per_unit = heads * ((vdim + 63) // 64)
+    if n_sequences * per_unit >= 1024 or n_tokens < 768 * n_sequences:
+        return 0
+    return max(256, -(-n_tokens * per_unit // 1024) // 64 * 64)
+
+
 def ssm_mix(proj, xbc_col, dt_col, params, conv_state, ssm_state, slots, positions, cu_seqlens=None, *, heads, vdim, state, groups,
-            out=None, scan="auto"):
+            out=None, scan="auto", segment: int | None = None):
     """Mamba-2 mixer between its projections: causal convolution + silu of the channels (x | B | C) at column xbc_col of proj's
     rows, then S <- exp(A dt) S + dt B x^T, y = S^T C + D x with dt = softplus(columns dt_col .. + dt_bias).
 
@@ -1347,7 +1355,8 @@ def ssm_mix(proj, xbc_col, dt_col, params, conv_state, ssm_state, slots, positio
     neg_a, d_skip (heads,); conv_state (n_slots,taps,channels) of proj's dtype and ssm_state (n_slots,heads,state,vdim rounded up
     to 4) fp32, updated in place at slots (B,) int32; positions (T,) int32 (a sequence whose first row has position 0 starts from
     zero).  With cu_seqlens (int32 (B+1,)) sequence b owns those rows; without it each owns one and everything is one launch.
-    scan: "auto", "serial" or "chunked" (see mi355_ssm_prefill).  Returns y (T, heads * vdim), into `out` when given."""
+    scan: "auto", "serial" or "chunked" (see mi355_ssm_prefill); segment: tokens per segment of the chunked scan (0: whole
+    sequences, None: chosen by size).  Returns y (T, heads * vdim), into `out` when given."""
     code = _dtype_code("proj", proj)
     T, width = _matrix("proj", proj, proj.dtype).shape
     channels, inner = heads * vdim + 2 * groups * state, heads * vdim
@@ -1373,12 +1382,20 @@ def ssm_mix(proj, xbc_col, dt_col, params, conv_state, ssm_state, slots, positio
     if T == 0:
         return out
     xbc = None if cu_seqlens is None else torch.empty(T, channels, dtype=proj.dtype, device=proj.device)
+    seg_len, seg_state, seg_decay = 0, None, None
+    if cu_seqlens is not None and scan != "serial" and proj.dtype == torch.bfloat16 and state % 8 == 0 and vdim % 8 == 0 and state <= 256:
+        seg_len = ssm_segment_length(T, B, heads, vdim) if segment is None else int(segment)
+    if seg_len:
+        units = T // seg_len + B
+        seg_state = torch.empty(units, heads, state, vdim, dtype=torch.float32, device=proj.device)
+        seg_decay = torch.empty(units, heads, dtype=torch.float32, device=proj.device)
     with _on(proj, conv_state, ssm_state, slots, positions, cu_seqlens, out, *params.values()) as stream:
         args = _lib.SsmArgs(proj.data_ptr(), *(params[n].data_ptr() for n in ("conv", "conv_b", "dt_bias", "neg_a", "d_skip")),
                             conv_state.data_ptr(), ssm_state.data_ptr(), slots.data_ptr(), positions.data_ptr(),
                             None if cu_seqlens is None else cu_seqlens.data_ptr(), None if xbc is None else xbc.data_ptr(),
                             out.data_ptr(), proj.stride(0) if T > 1 else width, xbc_col, dt_col, out.stride(0) if T > 1 else inner, T,
-                            B, heads, vdim, state, groups, taps, n_slots, code)
+                            B, heads, vdim, state, groups, taps, n_slots, code, None if seg_state is None else seg_state.data_ptr(),
+                            None if seg_decay is None else seg_decay.data_ptr(), seg_len)
         if cu_seqlens is None:
             rc = _lib.load().mi355_ssm_decode(args, stream)
         else:

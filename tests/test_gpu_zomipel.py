@@ -325,6 +325,42 @@ def test_state_space_batches(ops, dtype):
         rows_close(torch.cat((got[cu[i]:cu[i + 1]], step[i:i + 1])), ref, dtype, what=f"sequence {i}")
 
 
+@pytest.mark.parametrize("m", [m for m in SSM if m["state"] % 8 == 0 and m["vdim"] % 8 == 0], ids=lambda m: "-".join(str(v) for v in m.values()))
+def test_segments_side_by_side(ops, m):
+    """Unequal sequences -- shorter than a segment, exactly one, a token more, many -- resumed once, against whole sequences and
+    the oracle."""
+    kw = {k: m[k] for k in ("heads", "vdim", "state", "groups")}
+    lens, slots, dtype = [130, 1, 64, 65, 400, 2], [4, 0, 6, 1, 3, 2], torch.bfloat16
+    case, params, xbc_at, dt_at = ssm_case(m, 1, 30, dtype)
+    params["neg_a"] = params["neg_a"] * 0.1                               # long memories: what crosses a segment's edge shows
+    projs = [rnd(n, case.shape[1], seed=n, dtype=dtype) for n in lens]
+    pc, sl = {k: v.cuda() for k, v in params.items()}, torch.tensor(slots, dtype=torch.int32).cuda()
+    refs = [ssm_oracle(m, p, params, xbc_at, dt_at, True) for p in projs]
+    cut = [n // 3 for n in lens]                                          # two of them are still empty after the first call
+    for segment in (0, 64, 128, 256):
+        print(f"case: ssm segments {m} {segment}", flush=True)
+        conv, state = ssm_pools(m, 7, dtype)
+        parts = []
+        for a, b in ((([0] * 6), cut), (cut, lens)):
+            n = [y - x for x, y in zip(a, b)]
+            cu = torch.tensor([0] + n).cumsum(0).int().cuda()
+            pos = torch.cat([torch.arange(x, y) for x, y in zip(a, b)]).int().cuda()
+            got = ops.ssm_mix(torch.cat([p[x:y] for p, x, y in zip(projs, a, b)]).cuda(), xbc_at, dt_at, pc, conv, state, sl, pos, cu,
+                              segment=segment, **kw)
+            parts.append(torch.split(got, n))
+        for i, (ref, S) in enumerate(refs):
+            rows_close(torch.cat([p[i] for p in parts]), ref, dtype, what=f"segment {segment} sequence {i}")
+            s = state[slots[i], :, :, :m["vdim"]].cpu()
+            assert float((s - S).pow(2).mean().sqrt() / S.pow(2).mean().sqrt()) <= 1.5e-3
+        assert bool((state[5] == 1e6).all())
+
+
+def test_segment_lengths(ops):
+    length = ops.ops.ssm_segment_length
+    assert length(8192, 1, 64, 64) == 512 and length(8192, 4, 64, 64) == 512 and length(8192, 16, 64, 64) == 0
+    assert length(700, 1, 8, 48) == 0 and length(1100, 1, 8, 48) == 256 and length(10 ** 6, 1, 24, 200) % 64 == 0
+
+
 def test_chunked_scan_forgets_and_remembers(ops):
     """Decays from almost none to complete within a token: chunks agree with the token-by-token form."""
     m = SSM[2]
@@ -343,7 +379,7 @@ def test_chunked_scan_forgets_and_remembers(ops):
 
 # ---- mixture of experts -------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("E,top", [(1, 1), (8, 2), (17, 17), (64, 6), (200, 3)])
+@pytest.mark.parametrize("E,top", [(1, 1), (8, 2), (17, 17), (64, 6), (200, 3), (1024, 64)])
 def test_router(ops, E, top, dtype):
     T, k = 37, 72
     print(f"case: route {E} {top} {dtype}", flush=True)
