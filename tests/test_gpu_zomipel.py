@@ -358,7 +358,7 @@ def test_segments_side_by_side(ops, m):
 def test_segment_lengths(ops):
     length = ops.ops.ssm_segment_length
     assert length(8192, 1, 64, 64) == 512 and length(8192, 4, 64, 64) == 512 and length(8192, 16, 64, 64) == 0
-    assert length(700, 1, 8, 48) == 0 and length(1100, 1, 8, 48) == 256 and length(10 ** 6, 1, 24, 200) % 64 == 0
+    assert length(700, 1, 6, 40) == 0 and length(1100, 1, 6, 40) == 256 and length(10 ** 6, 1, 24, 200) % 64 == 0
 
 
 def test_chunked_scan_forgets_and_remembers(ops):
